@@ -296,6 +296,7 @@ typedef struct shainet_llama_block shainet_llama_block;
 int shainet_llama_block_create(shainet_llama_block **out, int d_model, int num_heads, int ff_hidden, double eps,
                                double rope_theta, int num_kv_heads, int head_dim);
 int shainet_llama_block_destroy(shainet_llama_block *block);
+/* null for a block whose mixer is not the attention above (see shainet_llama_block_latent_config) */
 shainet_llama_attn *shainet_llama_block_attn(shainet_llama_block *block);
 /* gamma of @norm1 and @norm2, host [d_model] each; null = ones (rms_norm.cr:10). */
 int shainet_llama_block_set_norms(shainet_llama_block *block, const float *norm1_gamma, const float *norm2_gamma);
@@ -310,6 +311,21 @@ int shainet_llama_block_forward_cached(shainet_llama_block *block, const float *
                                        int mem);
 /* LlamaBlock#forward (179-186): the whole sequence without the cache (Network#run with use_kv_cache off). */
 int shainet_llama_block_forward(shainet_llama_block *block, const float *x, int seq_len, float *out, int mem);
+
+/* Latent attention, the other mixer a block can have (made by shainet_hf_load_model): queries, keys and
+ * values go through low-rank latents and the cache holds one row per position that all heads share,
+ * [RMS-normed latent of kv_rank | rotated key part of rot_dim | zeros to a multiple of 16].  Per head, dim
+ * unrotated and rot_dim rotated query / key dimensions (pairs (2i, 2i + 1) of the first rot_dims turn by
+ * position * rot_base^(-2i / rot_dims)) and vdim value dimensions; scores times `scale`; a learned sink per
+ * head in the softmax's denominator; the head's output times a sigmoid gate.  window > 0: a position sees
+ * itself and the window - 1 before it, and the cache drops the rows nobody can see any more; 0: all before it. */
+typedef struct {
+  int heads, dim, rot_dim, vdim, kv_rank, q_rank, window, rot_dims;
+  double rot_base, scale;
+} shainet_latent_config;
+int shainet_llama_block_latent_config(shainet_llama_block *block, shainet_latent_config *cfg);
+/* the block's cache, owned by the block (null before a grouped-query block's first call) */
+shainet_kv_cache *shainet_llama_block_cache(shainet_llama_block *block);
 
 /* ---- the model around the blocks ----------------------------------------------
  *
@@ -328,6 +344,10 @@ int shainet_llama_model_create(shainet_llama_model **out, int vocab, int d_model
                                int num_kv_heads, int head_dim, int ff_hidden, double eps, double rope_theta);
 int shainet_llama_model_destroy(shainet_llama_model *model);
 int shainet_llama_model_layers(const shainet_llama_model *model);
+int shainet_llama_model_vocab(const shainet_llama_model *model);
+int shainet_llama_model_d_model(const shainet_llama_model *model);
+/* makes room for `positions` positions in every block's cache ahead of time (they grow on demand otherwise) */
+int shainet_llama_model_reserve(shainet_llama_model *model, int positions);
 shainet_llama_block *shainet_llama_model_block(shainet_llama_model *model, int layer);
 /* host [vocab, d_model] */
 int shainet_llama_model_set_embedding(shainet_llama_model *model, const float *table);
@@ -340,6 +360,10 @@ int shainet_llama_model_cache_len(const shainet_llama_model *model);
 /* tokens: host ids [n_tokens], appended to every block's cache.  logits: host [vocab], or null to leave
  * them on the device (the call is then asynchronous; the sampling calls and _sync wait). */
 int shainet_llama_model_run(shainet_llama_model *model, const int *tokens, int n_tokens, float *logits);
+/* shainet_llama_model_run, and the logits of any of the run's rows: rows[n_rows] are places among `tokens`,
+ * logits is host [n_rows, vocab] in their order.  The last row's logits are left for the sampling calls as usual. */
+int shainet_llama_model_run_rows(shainet_llama_model *model, const int *tokens, int n_tokens, const int *rows,
+                                 int n_rows, float *logits);
 /* The same with the network's use_kv_cache switched off (network_setup.cr:32, network_run.cr:199-204:
  * LlamaBlock#forward instead of forward_cached in every block): the n_tokens rows attend among
  * themselves from position 0, every block's cache and cache length stay as they are.  The logits of
@@ -436,6 +460,9 @@ int shainet_hf_rope_freqs(const shainet_hf_llama_config *cfg, float *out, int n)
  * "mistral", "qwen2", "qwen3"): every tensor goes to the GPU in its stored type and is converted
  * to fp32 and transposed to [in, out] there.  The model is ready for shainet_llama_model_run. */
 int shainet_hf_load_llama(const char *model_dir, shainet_llama_model **out);
+/* Any model this library has, by its config.json: a design named under "architecture" ("Tutilorn": latent
+ * attention, Dynamic Tanh norms, dense SwiGLU, its layers listed one by one), else shainet_hf_load_llama. */
+int shainet_hf_load_model(const char *model_dir, shainet_llama_model **out);
 
 /* Kernel timing for benchmarks: while enabled, every shainet_attn_forward call
  * times its attention kernel (the split-K decode kernel, the MFMA prefill kernel

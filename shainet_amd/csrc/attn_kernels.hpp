@@ -170,6 +170,10 @@ hipError_t launch_generic(const float *q_rot, const float *kc, const float *vc, 
 
 // y[T,N] = epilogue(norm(x)[T,K] * W[K,N]), T <= 16, N % 4 == 0: the projections of a
 // decode step with what surrounds them fused in.
+// What happens to the rows of x on their way into a product:
+//   kNormRms      x / sqrt(mean(x^2) + eps) * gamma (gamma null: ones)
+//   kNormDynTanh  tanh(alpha x) * gamma + beta, element by element, no statistics (gamma, beta not null)
+enum { kNormNone = 0, kNormRms = 1, kNormDynTanh = 2 };
 enum { kGemvPlain = 0, kGemvResidual = 1, kGemvSwiglu = 2, kGemvQkvPrep = 3 };
 // kGemvQkvPrep: W = W_q | W_k | W_v and the product's rows never go to memory as
 // they are: each head row gets its bias, QK-norm and rotation where it is summed up
@@ -188,8 +192,10 @@ struct GemvPrep {
 struct GemvArgs {
   const float *x;        // [T, K], rows x_stride floats apart
   long long x_stride;
-  int norm;              // != 0: RMSNorm the rows of x first (gamma may be null = ones)
+  int norm;              // kNorm*: applied to the rows of x first
   const float *gamma;    // [K]
+  const float *beta;     // [K]; kNormDynTanh only
+  float alpha;           // kNormDynTanh only
   double eps;
   const float *w;        // [K, N]; kGemvSwiglu: [K, 2N] = gate_proj | up_proj
   const float *res;      // kGemvResidual: [T, N], y = res + x W
@@ -218,7 +224,7 @@ hipError_t launch_gemv(const GemvArgs &a, const GemvPlan &p, hipStream_t stream)
 // gate | up for kGemvSwiglu): a wavefront per output, nothing shared between wavefronts.
 // gemvt_takes: what it serves (one row; K 1024, 2048, 4096, or 8192 without norm and SwiGLU; the
 // kGemvQkvPrep epilogue, a.w: [(H + 2 KV) hd, K], where *prep asks for no QK-norm).
-bool gemvt_takes(int T, int K, int N, int epilogue, bool norm, const GemvPrep *prep = nullptr);
+bool gemvt_takes(int T, int K, int N, int epilogue, int norm, const GemvPrep *prep = nullptr);
 hipError_t launch_gemvt(const GemvArgs &a, hipStream_t stream);
 
 // A pinned host int per context (block, model) that its kernels set when they give up a

@@ -103,10 +103,26 @@ __global__ __launch_bounds__(256) void swiglu_act_kernel(const float *__restrict
 }
 
 __global__ __launch_bounds__(256) void embed_kernel(const float *__restrict__ table, const int *__restrict__ tokens,
-                                                    float *__restrict__ out, int d_model) {
+                                                    float *__restrict__ out, int d_model, float scale) {
   const float *src = table + (long long)tokens[blockIdx.x] * d_model;
   float *dst = out + (long long)blockIdx.x * d_model;
-  for (int j = threadIdx.x; j < d_model; j += 256) dst[j] = src[j];
+  for (int j = threadIdx.x; j < d_model; j += 256) dst[j] = src[j] * scale;
+}
+
+// Dynamic Tanh: no statistics over the row, so a workgroup takes 1024 columns of one row.
+__global__ __launch_bounds__(256) void dyn_tanh_kernel(const float *__restrict__ x, long long x_stride,
+                                                       const float *__restrict__ gamma, const float *__restrict__ beta,
+                                                       float alpha, float *__restrict__ out, int cols) {
+  const float *xr = x + (long long)blockIdx.x * x_stride;
+  float *orow = out + (long long)blockIdx.x * cols;
+  const int j = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (j + 3 < cols && ((cols | x_stride) & 3) == 0) {
+    const f32x4 v = *(const f32x4 *)(xr + j), g = *(const f32x4 *)(gamma + j), b = *(const f32x4 *)(beta + j);
+    *(f32x4 *)(orow + j) = f32x4{tanhf(alpha * v.x) * g.x + b.x, tanhf(alpha * v.y) * g.y + b.y,
+                                 tanhf(alpha * v.z) * g.z + b.z, tanhf(alpha * v.w) * g.w + b.w};
+  } else {
+    for (int k = j; k < cols && k < j + 4; ++k) orow[k] = tanhf(alpha * xr[k]) * gamma[k] + beta[k];
+  }
 }
 
 __global__ __launch_bounds__(256) void add_bias_row_kernel(float *__restrict__ logits, const float *__restrict__ bias,
@@ -340,6 +356,22 @@ hipError_t launch_rmsnorm(const float *x, long long x_stride, const float *gamma
   return hipGetLastError();
 }
 
+hipError_t launch_dyn_tanh(const float *x, long long x_stride, const float *gamma, const float *beta, float alpha,
+                           float *out, int rows, int cols, hipStream_t stream) {
+  if (!x || !gamma || !beta || !out || rows < 1 || cols < 1 || x_stride < cols || (cols + 1023) / 1024 > 65535)
+    return hipErrorInvalidValue;
+  hipLaunchKernelGGL(dyn_tanh_kernel, dim3((unsigned)rows, (unsigned)((cols + 1023) / 1024)), dim3(256), 0, stream, x,
+                     x_stride, gamma, beta, alpha, out, cols);
+  return hipGetLastError();
+}
+
+hipError_t launch_gather_rows(const float *x, const int *rows, float *out, int n, int cols, hipStream_t stream) {
+  if (!x || !rows || !out || n < 1 || cols < 1) return hipErrorInvalidValue;
+  // (a row gather is what the embedding lookup is)
+  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n), dim3(256), 0, stream, x, rows, out, cols, 1.f);
+  return hipGetLastError();
+}
+
 hipError_t launch_add(const float *a, const float *b, float *out, long long n, hipStream_t stream) {
   if (n < 1) return hipErrorInvalidValue;
   const long long blocks = (n + 1023) / 1024;
@@ -356,9 +388,9 @@ hipError_t launch_swiglu_act(const float *gate_up, float *hidden, int rows, int 
 }
 
 hipError_t launch_embed(const float *table, const int *tokens, float *out, int n_tokens, int d_model,
-                        hipStream_t stream) {
+                        hipStream_t stream, float scale) {
   if (n_tokens < 1 || d_model < 1) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n_tokens), dim3(256), 0, stream, table, tokens, out, d_model);
+  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n_tokens), dim3(256), 0, stream, table, tokens, out, d_model, scale);
   return hipGetLastError();
 }
 

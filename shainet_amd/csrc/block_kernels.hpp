@@ -10,6 +10,9 @@ namespace shainet {
 // the rows of x are x_stride floats apart, those of out are dense
 hipError_t launch_rmsnorm(const float *x, long long x_stride, const float *gamma, float *out, int rows, int cols,
                           double eps, hipStream_t stream);
+// out[r, j] = tanh(alpha x[r, j]) * gamma[j] + beta[j], fp32; rows as for launch_rmsnorm
+hipError_t launch_dyn_tanh(const float *x, long long x_stride, const float *gamma, const float *beta, float alpha,
+                           float *out, int rows, int cols, hipStream_t stream);
 // dst[c, r] = src[r, c]: src is [rows, cols], dst [cols, rows], both dense
 hipError_t launch_transpose(const float *src, float *dst, int rows, int cols, hipStream_t stream,
                             const float *row_scale = nullptr);
@@ -20,9 +23,11 @@ hipError_t launch_transposed_differ(const float *a, const float *b, int rows, in
 hipError_t launch_add(const float *a, const float *b, float *out, long long n, hipStream_t stream);
 // hidden[r, j] = silu(gate_up[r, j]) * gate_up[r, ff + j];  gate_up is [rows, 2*ff]
 hipError_t launch_swiglu_act(const float *gate_up, float *hidden, int rows, int ff, hipStream_t stream);
-// out[t, :] = table[tokens[t], :];  the caller has checked 0 <= tokens[t] < vocab
+// out[t, :] = table[tokens[t], :] * scale;  the caller has checked 0 <= tokens[t] < vocab
 hipError_t launch_embed(const float *table, const int *tokens, float *out, int n_tokens, int d_model,
-                        hipStream_t stream);
+                        hipStream_t stream, float scale = 1.f);
+// out[i, :] = x[rows[i], :], n rows of `cols` floats
+hipError_t launch_gather_rows(const float *x, const int *rows, float *out, int n, int cols, hipStream_t stream);
 // logits[j] += bias[j]
 hipError_t launch_add_bias_row(float *logits, const float *bias, int n, hipStream_t stream);
 // Sampler#apply_repetition_penalty! : ids in order, duplicates penalised once per occurrence

@@ -11,6 +11,7 @@
 #include <vector>
 
 #include "../../include/shainet_hip_attn.h"
+#include "attn_context.hpp"
 #include "attn_kernels.hpp"
 #include "block_kernels.hpp"
 
@@ -77,106 +78,47 @@ int hip_fail(hipError_t e, const char *what) {
     if (e_ != hipSuccess) return hip_fail(e_, #expr);  \
   } while (0)
 
-// Grow-only device buffer.
-struct DevBuf {
-  float *p = nullptr;
-  size_t cap = 0;  // floats
-  int reserve(size_t n) {
-    if (n <= cap) return SHAINET_HIP_OK;
-    size_t want = cap ? cap : 1024;
-    while (want < n) want *= 2;
-    float *np = nullptr;
-    hipError_t e = hipMalloc((void **)&np, want * sizeof(float));
-    if (e != hipSuccess) {  // try the exact size before giving up
-      want = n;
-      e = hipMalloc((void **)&np, want * sizeof(float));
-    }
-    if (e != hipSuccess) return hip_fail(e, "hipMalloc");
-    if (p) (void)hipFree(p);
-    p = np;
-    cap = want;
-    return SHAINET_HIP_OK;
-  }
-  void release() {
-    if (p) (void)hipFree(p);
-    p = nullptr;
-    cap = 0;
-  }
-};
-
-// Grow-only pinned host buffer: host-pointer calls stage their rows through it, so that each
-// copy to or from the device is one asynchronous DMA instead of the runtime's staged copy of
-// pageable memory.
-struct PinBuf {
-  float *p = nullptr;
-  size_t cap = 0;  // floats
-  int reserve(size_t n) {
-    if (n <= cap) return SHAINET_HIP_OK;
-    size_t want = cap ? cap : 4096;
-    while (want < n) want *= 2;
-    float *np = nullptr;
-    hipError_t e = hipHostMalloc((void **)&np, want * sizeof(float), hipHostMallocDefault);
-    if (e != hipSuccess) return hip_fail(e, "hipHostMalloc");
-    if (p) (void)hipHostFree(p);
-    p = np;
-    cap = want;
-    return SHAINET_HIP_OK;
-  }
-  void release() {
-    if (p) (void)hipHostFree(p);
-    p = nullptr;
-    cap = 0;
-  }
-};
 
 }  // namespace
 
-struct shainet_attn_ctx {
-  int H, KV, g, hd;
-  double eps;
-  float scale;  // (float)(1.0 / sqrt((double)hd)), llama_block.cr:249
-  std::vector<float> inv_freq;
-  float *d_q_norm = nullptr, *d_k_norm = nullptr;
-  float *d_bq = nullptr, *d_bk = nullptr, *d_bv = nullptr;
-  float2 *d_rope = nullptr;
-  int rope_positions = 0;
-  // DecodeArgs::ahead_* of the next decode launch (shainet_attn_read_ahead); forgotten after it
-  const float *ahead_w = nullptr;
-  int ahead_k = 0, ahead_n = 0, ahead_wgs = 0;
-  hipStream_t stream = nullptr;      // where work is issued
-  hipStream_t own_stream = nullptr;  // created with the context, destroyed with it
-  DevBuf q_rot, partials, in_q, in_k, in_v, out;
-  PinBuf pin_in, pin_out;  // host-pointer calls: q | k | v rows on their way in, the result on its way out
-  // decode split: a word per partial slot that says when it is complete (zero between launches)
-  unsigned *part_flag = nullptr;
-  size_t part_flag_cap = 0;
-  bool test_lose_marks = false;  // SHAINET_HIP_TEST_LOSE_PARTIAL_MARKS: exercises the give-up path
-  // pinned host word this context's kernels set when they give up a bounded wait; `error` is
-  // the one in use: the context's own, or the one of the block or model that owns the context
-  int *error = nullptr, *own_error = nullptr;
-  int last_rows = 0;
-  int decode_wgs_override = 0;  // 0 = default workgroup count of the decode split
-  int prefill_wgs_per_cu = 0;   // 0 = default occupancy of the prefill kernel
-  int prefill_splits_override = 0;  // 0 = default number of key splits of the prefill kernel
-  int prefill_groups_override = 0;  // 0 = default number of wavefront groups of the prefill kernel
-  bool profiling = false;
-  std::vector<hipEvent_t> prof_events;  // start, stop, start, stop, ...
-};
-
-// What shainet_attn_decode_step works with: all of it allocated by shainet_kv_cache_lengths_to_device,
-// none of it by the step.
-struct StepState {
-  int *d_len = nullptr;               // [batch] cached rows per slot, as the device counts them
-  int *pin_len = nullptr;             // [batch] pinned staging for both directions
-  DecodeDevicePlan *d_plan = nullptr; // rewritten by every step
-  float *q_rot = nullptr;             // [batch, H, hd]
-  float *partials = nullptr;          // device_plan_slots(batch, KV) slots of g columns
-  unsigned *flags = nullptr;          // zero between launches
-  int cap = 0;                        // the capacity the buffers above were laid out for
-  // Between shainet_kv_cache_lengths_to_device and _from_device the device's lengths are the ones that count
-  // (decode steps advance only those): every entry point that reads or writes the host's copy is refused.
-  bool lengths_on_device = false;
-};
+int shainet::DevBuf::reserve(size_t n) {
+  if (n <= cap) return SHAINET_HIP_OK;
+  size_t want = cap ? cap : 1024;
+  while (want < n) want *= 2;
+  float *np = nullptr;
+  hipError_t e = hipMalloc((void **)&np, want * sizeof(float));
+  if (e != hipSuccess) {  // try the exact size before giving up
+    want = n;
+    e = hipMalloc((void **)&np, want * sizeof(float));
+  }
+  if (e != hipSuccess) return hip_fail(e, "hipMalloc");
+  if (p) (void)hipFree(p);
+  p = np;
+  cap = want;
+  return SHAINET_HIP_OK;
+}
+void shainet::DevBuf::release() {
+  if (p) (void)hipFree(p);
+  p = nullptr;
+  cap = 0;
+}
+int shainet::PinBuf::reserve(size_t n) {
+  if (n <= cap) return SHAINET_HIP_OK;
+  size_t want = cap ? cap : 4096;
+  while (want < n) want *= 2;
+  float *np = nullptr;
+  hipError_t e = hipHostMalloc((void **)&np, want * sizeof(float), hipHostMallocDefault);
+  if (e != hipSuccess) return hip_fail(e, "hipHostMalloc");
+  if (p) (void)hipHostFree(p);
+  p = np;
+  cap = want;
+  return SHAINET_HIP_OK;
+}
+void shainet::PinBuf::release() {
+  if (p) (void)hipHostFree(p);
+  p = nullptr;
+  cap = 0;
+}
 
 static void release_step_state(StepState &s) {
   if (s.d_len) (void)hipFree(s.d_len);
@@ -187,14 +129,6 @@ static void release_step_state(StepState &s) {
   if (s.flags) (void)hipFree(s.flags);
   s = StepState();
 }
-
-struct shainet_kv_cache {
-  shainet_attn_ctx *ctx;
-  int batch, cap;
-  float *k = nullptr, *v = nullptr;
-  std::vector<int> len;
-  StepState step;
-};
 
 namespace {
 int refuse_while_lengths_on_device(const shainet_kv_cache *kc, const char *what) {
@@ -216,13 +150,15 @@ int upload(float **dst, const float *src, size_t n) {
   return SHAINET_HIP_OK;
 }
 
+}  // namespace
+
 // cos/sin of (float)pos * inv_freq[i], computed with the host's libm exactly as
-// llama_block.cr:274-277 does, for pos in [0, positions).
-int ensure_rope_table(shainet_attn_ctx *c, int positions) {
+// llama_block.cr:274-277 does, for pos in [0, positions); rope_fp64: of pos * inv_freq64[i] instead.
+int shainet::ensure_rope_table(shainet_attn_ctx *c, int positions) {
   if (positions <= c->rope_positions) return SHAINET_HIP_OK;
   int want = c->rope_positions ? c->rope_positions : 1024;
   while (want < positions) want *= 2;
-  const int half = c->hd / 2;
+  const int half = (int)c->inv_freq.size();
   if (half == 0) {
     c->rope_positions = want;
     return SHAINET_HIP_OK;
@@ -230,8 +166,13 @@ int ensure_rope_table(shainet_attn_ctx *c, int positions) {
   std::vector<float2> tab((size_t)want * half);
   for (int pos = 0; pos < want; ++pos)
     for (int i = 0; i < half; ++i) {
-      const float angle = (float)pos * c->inv_freq[i];
-      tab[(size_t)pos * half + i] = float2{cosf(angle), sinf(angle)};
+      if (c->rope_fp64) {
+        const double angle = (double)pos * c->inv_freq64[i];
+        tab[(size_t)pos * half + i] = float2{(float)cos(angle), (float)sin(angle)};
+      } else {
+        const float angle = (float)pos * c->inv_freq[i];
+        tab[(size_t)pos * half + i] = float2{cosf(angle), sinf(angle)};
+      }
     }
   float2 *np = nullptr;
   HIP_TRY(hipMalloc((void **)&np, tab.size() * sizeof(float2)));
@@ -249,6 +190,8 @@ int ensure_rope_table(shainet_attn_ctx *c, int positions) {
   c->rope_positions = want;
   return SHAINET_HIP_OK;
 }
+
+namespace {
 
 Shape shape_of(const shainet_attn_ctx *c, int cap) {
   Shape sh;
@@ -479,7 +422,7 @@ int shainet_attn_create(shainet_attn_ctx **out, int num_heads, int num_kv_heads,
   c->H = num_heads;
   c->KV = num_kv_heads;
   c->g = num_heads / num_kv_heads;
-  c->hd = head_dim;
+  c->hd = c->v_hd = head_dim;
   c->eps = qk_norm_eps;
   c->scale = (float)(1.0 / sqrt((double)head_dim));
   c->inv_freq.resize(head_dim / 2);
@@ -513,6 +456,44 @@ int shainet_attn_create(shainet_attn_ctx **out, int num_heads, int num_kv_heads,
   *out = c;
   return SHAINET_HIP_OK;
 }
+
+}  // extern "C"
+
+int shainet_attn_create_rows(shainet_attn_ctx **out, int num_heads, int row_width, int window, double rope_base,
+                             int rope_dims, float scale, int max_positions) {
+  *out = nullptr;
+  if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
+  shainet_attn_ctx *c = new (std::nothrow) shainet_attn_ctx();
+  if (!c) return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
+  c->H = c->g = num_heads;
+  c->KV = 1;
+  c->hd = row_width;
+  c->v_hd = 0;
+  c->window = window;
+  c->rope_fp64 = true;
+  c->scale = scale;
+  c->inv_freq64.resize(rope_dims / 2);
+  c->inv_freq.resize(rope_dims / 2);
+  for (int i = 0; i < rope_dims / 2; ++i) {
+    c->inv_freq64[i] = pow(rope_base, -2.0 * i / rope_dims);
+    c->inv_freq[i] = (float)c->inv_freq64[i];
+  }
+  int rc = SHAINET_HIP_OK;
+  const hipError_t e = hipStreamCreateWithFlags(&c->own_stream, hipStreamNonBlocking);
+  if (e != hipSuccess) rc = hip_fail(e, "hipStreamCreate");
+  c->stream = c->own_stream;
+  c->error = c->own_error = alloc_error_word();
+  if (!rc && !c->error) rc = fail(SHAINET_HIP_ERR_ALLOC, "hipHostMalloc failed");
+  if (!rc) rc = ensure_rope_table(c, max_positions > 0 ? max_positions : 1024);
+  if (rc) {
+    shainet_attn_destroy(c);
+    return rc;
+  }
+  *out = c;
+  return SHAINET_HIP_OK;
+}
+
+extern "C" {
 
 int shainet_attn_set_bias(shainet_attn_ctx *c, const float *b_q, int b_q_len, const float *b_k, int b_k_len,
                           const float *b_v, int b_v_len) {
@@ -583,14 +564,16 @@ int shainet_kv_cache_create(shainet_kv_cache **out, shainet_attn_ctx *ctx, int b
   kc->batch = batch;
   kc->cap = capacity;
   kc->len.assign(batch, 0);
+  kc->base.assign(batch, 0);
   const size_t bytes = (size_t)batch * ctx->KV * capacity * ctx->hd * sizeof(float);
+  const bool has_v = ctx->v_hd > 0;
   hipError_t e = hipMalloc((void **)&kc->k, bytes);
-  if (e == hipSuccess) e = hipMalloc((void **)&kc->v, bytes);
+  if (e == hipSuccess && has_v) e = hipMalloc((void **)&kc->v, bytes);
   // zero-fill: rows never appended must hold finite values.  On the context's stream and
   // waited for: a fill on the null stream is not ordered with the kernels that append rows
   // (the stream is non-blocking) and could wipe rows written right after this call.
   if (e == hipSuccess) e = hipMemsetAsync(kc->k, 0, bytes, ctx->stream);
-  if (e == hipSuccess) e = hipMemsetAsync(kc->v, 0, bytes, ctx->stream);
+  if (e == hipSuccess && has_v) e = hipMemsetAsync(kc->v, 0, bytes, ctx->stream);
   if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
   if (e != hipSuccess) {
     int rc = hip_fail(e, "kv cache allocation");
@@ -614,10 +597,12 @@ int shainet_kv_cache_destroy(shainet_kv_cache *kc) {
 int shainet_kv_cache_clear(shainet_kv_cache *kc, int seq) {
   if (!kc || seq >= kc->batch) return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid sequence");
   if (int rc = refuse_while_lengths_on_device(kc, "shainet_kv_cache_clear")) return rc;
-  if (seq < 0)
+  if (seq < 0) {
     kc->len.assign(kc->batch, 0);
-  else
-    kc->len[seq] = 0;
+    kc->base.assign(kc->batch, 0);
+  } else {
+    kc->len[seq] = kc->base[seq] = 0;
+  }
   return SHAINET_HIP_OK;
 }
 
@@ -626,6 +611,15 @@ int shainet_kv_cache_truncate(shainet_kv_cache *kc, int seq, int len) {
   if (int rc = refuse_while_lengths_on_device(kc, "shainet_kv_cache_truncate")) return rc;
   if (len < 0 || len > kc->len[seq])
     return fail(SHAINET_HIP_ERR_ARGUMENT, "truncate to %d outside 0..%d", len, kc->len[seq]);
+  if (len == 0) {
+    kc->base[seq] = 0;
+  } else if (kc->base[seq] > 0) {
+    // the next position sees window - 1 rows before it
+    const int first = len - (kc->ctx->window - 1);
+    if (kc->base[seq] > (first > 0 ? first : 0))
+      return fail(SHAINET_HIP_ERR_ARGUMENT, "truncate to %d: the rows before position %d have been dropped", len,
+                  kc->base[seq]);
+  }
   kc->len[seq] = len;
   return SHAINET_HIP_OK;
 }
@@ -649,15 +643,16 @@ int shainet_kv_cache_reserve(shainet_kv_cache *kc, int capacity) {
   const size_t row = (size_t)c->hd * sizeof(float);
   const size_t bytes = (size_t)kc->batch * c->KV * capacity * row;
   float *nk = nullptr, *nv = nullptr;
+  const bool has_v = c->v_hd > 0;
   hipError_t e = hipMalloc((void **)&nk, bytes);
-  if (e == hipSuccess) e = hipMalloc((void **)&nv, bytes);
+  if (e == hipSuccess && has_v) e = hipMalloc((void **)&nv, bytes);
   if (e == hipSuccess) e = hipMemsetAsync(nk, 0, bytes, c->stream);
-  if (e == hipSuccess) e = hipMemsetAsync(nv, 0, bytes, c->stream);
+  if (e == hipSuccess && has_v) e = hipMemsetAsync(nv, 0, bytes, c->stream);
   // one strided copy per tensor: [batch*KV] runs of cap rows into runs of capacity rows
   if (e == hipSuccess)
     e = hipMemcpy2DAsync(nk, (size_t)capacity * row, kc->k, (size_t)kc->cap * row, (size_t)kc->cap * row,
                          (size_t)kc->batch * c->KV, hipMemcpyDeviceToDevice, c->stream);
-  if (e == hipSuccess)
+  if (e == hipSuccess && has_v)
     e = hipMemcpy2DAsync(nv, (size_t)capacity * row, kc->v, (size_t)kc->cap * row, (size_t)kc->cap * row,
                          (size_t)kc->batch * c->KV, hipMemcpyDeviceToDevice, c->stream);
   if (e == hipSuccess) e = hipStreamSynchronize(c->stream);
@@ -667,7 +662,7 @@ int shainet_kv_cache_reserve(shainet_kv_cache *kc, int capacity) {
     return hip_fail(e, "kv cache growth");
   }
   (void)hipFree(kc->k);
-  (void)hipFree(kc->v);
+  if (kc->v) (void)hipFree(kc->v);
   kc->k = nk;
   kc->v = nv;
   kc->cap = capacity;
@@ -675,7 +670,7 @@ int shainet_kv_cache_reserve(shainet_kv_cache *kc, int capacity) {
 }
 
 int shainet_kv_cache_fill(shainet_kv_cache *kc, int seq, const float *k_rows, const float *v_rows, int n, int mem) {
-  if (!kc || seq < 0 || seq >= kc->batch || n < 0 || !k_rows || !v_rows)
+  if (!kc || seq < 0 || seq >= kc->batch || n < 0 || !k_rows || (!v_rows && kc->v))
     return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid fill arguments");
   if (int rc = refuse_while_lengths_on_device(kc, "shainet_kv_cache_fill")) return rc;
   if (n > kc->cap) return fail(SHAINET_HIP_ERR_CAPACITY, "fill of %d rows exceeds capacity %d", n, kc->cap);
@@ -684,28 +679,71 @@ int shainet_kv_cache_fill(shainet_kv_cache *kc, int seq, const float *k_rows, co
   const hipMemcpyKind kind = mem == SHAINET_HIP_MEM_HOST ? hipMemcpyHostToDevice : hipMemcpyDeviceToDevice;
   if (n > 0) {
     float *dk = kc->k + (size_t)seq * c->KV * kc->cap * c->hd;
-    float *dv = kc->v + (size_t)seq * c->KV * kc->cap * c->hd;
     HIP_TRY(hipMemcpy2DAsync(dk, (size_t)kc->cap * row, k_rows, (size_t)n * row, (size_t)n * row, c->KV, kind,
                              c->stream));
-    HIP_TRY(hipMemcpy2DAsync(dv, (size_t)kc->cap * row, v_rows, (size_t)n * row, (size_t)n * row, c->KV, kind,
-                             c->stream));
+    if (kc->v)
+      HIP_TRY(hipMemcpy2DAsync(kc->v + (size_t)seq * c->KV * kc->cap * c->hd, (size_t)kc->cap * row, v_rows,
+                               (size_t)n * row, (size_t)n * row, c->KV, kind, c->stream));
     HIP_TRY(hipStreamSynchronize(c->stream));
   }
   kc->len[seq] = n;
+  kc->base[seq] = 0;
   return ensure_rope_table(c, n + 1);
 }
 
 int shainet_kv_cache_read(shainet_kv_cache *kc, int seq, int kv_head, int pos0, int n, float *k_out, float *v_out) {
-  if (!kc || seq < 0 || seq >= kc->batch || kv_head < 0 || kv_head >= kc->ctx->KV || pos0 < 0 || n < 0 ||
-      pos0 + n > kc->cap)
+  if (!kc || seq < 0 || seq >= kc->batch || kv_head < 0 || kv_head >= kc->ctx->KV || pos0 < kc->base[seq] || n < 0 ||
+      pos0 - kc->base[seq] + n > kc->cap || (v_out && !kc->v))
     return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid read arguments");
   shainet_attn_ctx *c = kc->ctx;
-  const size_t off = (((size_t)seq * c->KV + kv_head) * kc->cap + pos0) * c->hd;
+  const size_t off = (((size_t)seq * c->KV + kv_head) * kc->cap + (pos0 - kc->base[seq])) * c->hd;
   HIP_TRY(hipStreamSynchronize(c->stream));
   if (k_out && n) HIP_TRY(hipMemcpy(k_out, kc->k + off, (size_t)n * c->hd * sizeof(float), hipMemcpyDeviceToHost));
   if (v_out && n) HIP_TRY(hipMemcpy(v_out, kc->v + off, (size_t)n * c->hd * sizeof(float), hipMemcpyDeviceToHost));
   return SHAINET_HIP_OK;
 }
+
+}  // extern "C"
+
+int shainet_kv_cache_make_room(shainet_kv_cache *kc, int seq, int new_rows, int keep_back) {
+  if (!kc || seq < 0 || seq >= kc->batch || new_rows < 1 || keep_back < 0)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid arguments");
+  if (int rc = refuse_while_lengths_on_device(kc, "shainet_kv_cache_make_room")) return rc;
+  shainet_attn_ctx *c = kc->ctx;
+  const int held = kc->len[seq] - kc->base[seq];
+  if (held + new_rows <= kc->cap) return SHAINET_HIP_OK;
+  // what the next positions, and those a truncate may go back to, can still see
+  const long long wanted = (long long)c->window - 1 + keep_back;
+  const int keep = c->window > 0 && wanted < held ? (int)wanted : held;
+  if (keep == held || (long long)keep + new_rows > kc->cap) {
+    // (room for the rows to come besides those that stay, so that the next move is not due at once)
+    const long long want = keep == held ? (long long)held + new_rows : 2LL * keep + new_rows;
+    const long long cap = want > 2LL * kc->cap ? want : 2LL * kc->cap;
+    if (cap > 0x7fffffffLL) return fail(SHAINET_HIP_ERR_CAPACITY, "a cache of %lld rows", cap);
+    if (int rc = shainet_kv_cache_reserve(kc, (int)cap)) return rc;
+    if (held + new_rows <= kc->cap) return SHAINET_HIP_OK;
+  }
+  // the rows that stay move to the front; through a buffer of their own where the ranges overlap
+  const int drop = held - keep;
+  const size_t row_floats = (size_t)c->hd, bytes = (size_t)keep * row_floats * sizeof(float);
+  if (keep > drop)
+    if (int rc = c->in_k.reserve((size_t)keep * row_floats)) return rc;
+  for (float *p : {kc->k, kc->v}) {
+    for (int h = 0; p && h < c->KV && keep > 0; ++h) {
+      float *first = p + ((size_t)seq * c->KV + h) * kc->cap * c->hd;
+      const float *from = first + (size_t)drop * c->hd;
+      if (keep > drop) {
+        HIP_TRY(hipMemcpyAsync(c->in_k.p, from, bytes, hipMemcpyDeviceToDevice, c->stream));
+        from = c->in_k.p;
+      }
+      HIP_TRY(hipMemcpyAsync(first, from, bytes, hipMemcpyDeviceToDevice, c->stream));
+    }
+  }
+  kc->base[seq] += drop;
+  return SHAINET_HIP_OK;
+}
+
+extern "C" {
 
 int shainet_attn_forward(shainet_attn_ctx *c, shainet_kv_cache *kc, const int *seq_ids, const int *new_tokens,
                          int n_seqs, const float *q, const float *k, const float *v, float *out, int mem) {
@@ -739,6 +777,7 @@ int forward_core(shainet_attn_ctx *c, shainet_kv_cache *kc, const int *seq_ids, 
                  const float *q, const float *k, const float *v, long long q_stride, long long k_stride,
                  long long v_stride, float *out, int mem, const Workspace *ws) {
   if (!c || !kc || kc->ctx != c) return fail(SHAINET_HIP_ERR_ARGUMENT, "context and cache do not belong together");
+  if (!kc->v) return fail(SHAINET_HIP_ERR_ARGUMENT, "this cache holds latent rows: there is no V array to attend over");
   if (int rc = refuse_while_lengths_on_device(kc, "shainet_attn_forward")) return rc;
   if (ws && mem != SHAINET_HIP_MEM_DEVICE)
     return fail(SHAINET_HIP_ERR_ARGUMENT, "the entry point that allocates nothing takes device pointers only");
@@ -938,7 +977,7 @@ DecodePlan step_launch_plan(const shainet_attn_ctx *c, int n_seqs) {
 extern "C" int shainet_kv_cache_lengths_to_device(shainet_kv_cache *kc) {
   if (!kc) return fail(SHAINET_HIP_ERR_ARGUMENT, "cache is null");
   shainet_attn_ctx *c = kc->ctx;
-  if (!decode_tile_head_dim(c->hd) || c->hd > 128 || c->g > 16)  // (the step's prep kernel: a wavefront per row of at most 128)
+  if (!kc->v || !decode_tile_head_dim(c->hd) || c->hd > 128 || c->g > 16)  // (the step's prep kernel: a wavefront per row of at most 128)
     return fail(SHAINET_HIP_ERR_ARGUMENT,
                 "decode steps need a head_dim that is a multiple of 4 up to 128 and at most 16 query heads per kv head");
   if (kc->batch > SHAINET_HIP_MAX_BATCH)

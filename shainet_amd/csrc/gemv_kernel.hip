@@ -11,7 +11,8 @@
 // the flags of the others, adds the partials in a fixed order, so results do not
 // depend on scheduling, and applies the epilogue.  Everything a decode step does around a product rides along:
 //   * prologue: RMSNorm of the x rows (rms_norm.cr:18-37, fp64 as there), so the
-//     normalised activations never go to memory;
+//     normalised activations never go to memory, or Dynamic Tanh (fp32; an element at a time, so
+//     a workgroup only touches the values of its own K range);
 //   * epilogue: residual add (simple_matrix.cr:39-48), the SwiGLU gate
 //     (swiglu_ff.cr:84-89) over a [K, 2*ff] matrix holding gate_proj | up_proj, or,
 //     for the q | k | v product, bias -> QK-norm -> RoPE -> cache append
@@ -34,6 +35,11 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 // written through to memory (sc1 = device scope), 16 bytes at a time.
 __device__ __forceinline__ void coherent_store4(float *p, f32x4 v) {
   asm volatile("global_store_dwordx4 %0, %1, off sc1" : : "v"(p), "v"(v) : "memory");
+}
+
+__device__ __forceinline__ f32x4 dyn_tanh4(f32x4 x, float alpha, f32x4 g, f32x4 b) {
+  return f32x4{tanhf(alpha * x.x) * g.x + b.x, tanhf(alpha * x.y) * g.y + b.y, tanhf(alpha * x.z) * g.z + b.z,
+               tanhf(alpha * x.w) * g.w + b.w};
 }
 
 __device__ __forceinline__ float swiglu1(float gate, float up) {
@@ -181,7 +187,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(GemvArgs a) {
 
   // ---- prologue: the x values of this workgroup's K range, normalised if asked;
   // zero beyond K and beyond T, so that clamped loads below contribute nothing
-  if (a.norm) {
+  if (a.norm == kNormRms) {
     for (int t = 0; t < T; ++t) {
       const float *xr = a.x + (long long)t * a.x_stride;
       double sq = 0.0;
@@ -207,7 +213,8 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(GemvArgs a) {
     float v = 0.f;
     if (t < T && k < K) {
       v = a.x[(long long)t * a.x_stride + k];
-      if (a.norm) v = (float)(((double)v / rms_s[t]) * (double)(a.gamma ? a.gamma[k] : 1.f));
+      if (a.norm == kNormRms) v = (float)(((double)v / rms_s[t]) * (double)(a.gamma ? a.gamma[k] : 1.f));
+      if (a.norm == kNormDynTanh) v = tanhf(a.alpha * v) * a.gamma[k] + a.beta[k];
     }
     smem[idx] = v;
   }
@@ -421,9 +428,12 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(GemvArgs a) {
 // the pair need (llama_block.cr:256-286, 332-344), so the head rows never go through memory either.
 // A workgroup takes two pairs: wavefronts 0 and 1 their lower rows, 2 and 3 their upper rows, and
 // the sums meet in LDS (a wavefront per pair, two rows each, took 0.85 us longer for 3072 rows).
-template <int KV4, int NACC, int SP, bool MULTI, bool PREP = false>
+// DYT: the prologue is Dynamic Tanh instead: x becomes tanh(alpha x) gamma + beta where it is staged.
+template <int KV4, int NACC, int SP, bool MULTI, bool PREP = false, bool DYT = false>
 __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
   static_assert(!PREP || (NACC == 1 && SP == 1 && !MULTI), "the q | k | v epilogue: one row per wavefront");
+  static_assert(!DYT || (SP == 1 && !PREP), "rows shared by two wavefronts come without a norm");
+  const bool rms_norm = !DYT && a.norm;
   // x: up to 2048 values stay in registers.  Longer (half) rows: a wavefront with one output reads
   // them again from memory (the L2), eight 16-byte pieces at a time, where they are used; one with
   // several outputs keeps its own normed copy in LDS
@@ -466,6 +476,7 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
   f32x4 wa[NACC][KV4], wb[MULTI ? NACC : 1][MULTI ? KV4 : 1];
   float rms = 1.0f;  // 1 / the root mean square
   constexpr bool NORMS = SP == 1;  // (rows shared by two wavefronts come without the norm: gemvt_takes)
+  f32x4 b_own[XSH && DYT ? K / 1024 : 1];  // its share of beta
   f32x4 x_own[XSH ? K / 1024 : 1], g_own[XSH && NORMS ? K / 1024 : 1];  // this thread's share of x (and gamma) on its way to LDS
   if constexpr (XSH) {
 #pragma unroll
@@ -474,10 +485,18 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
 #pragma unroll
       for (int i = 0; i < K / 1024; ++i) g_own[i] = *(const f32x4 *)(a.gamma + 4 * threadIdx.x + 1024 * i);
     }
+    if constexpr (DYT) {
+#pragma unroll
+      for (int i = 0; i < K / 1024; ++i) b_own[i] = *(const f32x4 *)(a.beta + 4 * threadIdx.x + 1024 * i);
+    }
   }
   if (live || PREP) load_row(wa, n0);
   if constexpr (XSH) {
-    if (NORMS && a.norm) {
+    if constexpr (DYT) {
+#pragma unroll
+      for (int i = 0; i < K / 1024; ++i) x_own[i] = dyn_tanh4(x_own[i], a.alpha, g_own[i], b_own[i]);
+    }
+    if (NORMS && rms_norm) {
       // squares, their sums and the root in fp32 (a reciprocal square root and one Newton step):
       // within a few 1e-7 of the fp64 factor of rms_norm.cr:18-37
       f32x4 q = {0.f, 0.f, 0.f, 0.f};
@@ -496,7 +515,7 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
     for (int i = 0; i < K / 1024; ++i) *(f32x4 *)(xsh + 4 * threadIdx.x + 1024 * i) = x_own[i];
     __syncthreads();
     if (!PREP && !live) return;
-    if (NORMS && a.norm) {
+    if (NORMS && rms_norm) {
       const float m = ((sq_s[0] + sq_s[1]) + (sq_s[2] + sq_s[3])) / (float)K + (float)a.eps;
       float r = rsqrtf(m);
       rms = r * (1.5f - 0.5f * m * r * r);
@@ -518,7 +537,7 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
 #pragma unroll
     for (int i = 0; i < KV4; ++i) xv[i] = *(const f32x4 *)(xp + 256 * i);
   }
-  if (!XSH && a.norm) {
+  if (!XSH && rms_norm) {
     // every wavefront of the launch runs this, so it is kept short: squares, their sums and the
     // root in fp32 (a reciprocal square root and one Newton step; all of it in fp64 as
     // rms_norm.cr does cost 0.4 us of a 3072-row product for the sums and as much for the root);
@@ -544,7 +563,13 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
   auto x_pieces = [&](f32x4 (&t)[XC], int c0) {
 #pragma unroll
     for (int i = 0; i < XC; ++i) t[i] = *(const f32x4 *)(xp + 256 * (c0 + i));
-    if (a.norm) {
+    if constexpr (DYT) {
+#pragma unroll
+      for (int i = 0; i < XC; ++i) {
+        const int o = seg * KW + 4 * lane + 256 * (c0 + i);
+        t[i] = dyn_tanh4(t[i], a.alpha, *(const f32x4 *)(a.gamma + o), *(const f32x4 *)(a.beta + o));
+      }
+    } else if (a.norm) {
 #pragma unroll
       for (int i = 0; i < XC; ++i) {
         f32x4 g = {1.f, 1.f, 1.f, 1.f};
@@ -553,7 +578,11 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
       }
     }
   };
-  if constexpr (XREG) {
+  if constexpr (XREG && DYT) {
+#pragma unroll
+    for (int i = 0; i < KV4; ++i)
+      xv[i] = dyn_tanh4(xv[i], a.alpha, *(const f32x4 *)(a.gamma + 4 * lane + 256 * i), *(const f32x4 *)(a.beta + 4 * lane + 256 * i));
+  } else if constexpr (XREG) {
     if (a.norm && a.gamma) {
 #pragma unroll
       for (int i = 0; i < KV4; ++i) xv[i] = xv[i] * *(const f32x4 *)(a.gamma + 4 * lane + 256 * i);
@@ -604,7 +633,7 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
       s[0] = half_s[wave & ~1] + half_s[wave | 1];
       if (seg) return;
     }
-    if (a.norm) {
+    if (rms_norm) {
 #pragma unroll
       for (int c = 0; c < NACC; ++c) s[c] = s[c] * rms;
     }
@@ -684,6 +713,7 @@ hipError_t launch_gemv(const GemvArgs &args, const GemvPlan &p, hipStream_t stre
   if (p.rows_per_wave < 8 * p.rows_per_instr || p.rows_per_wave % (8 * p.rows_per_instr)) return hipErrorInvalidValue;
   if (p.splits > 1 && (!a.partials || !a.flags || !a.error)) return hipErrorInvalidValue;
   if (a.epilogue == kGemvResidual && !a.res) return hipErrorInvalidValue;
+  if (a.norm == kNormDynTanh && (!a.gamma || !a.beta)) return hipErrorInvalidValue;
   if (a.epilogue != kGemvResidual) a.res = nullptr;
   const bool prep = a.epilogue == kGemvQkvPrep;
   if (prep) {
@@ -729,10 +759,10 @@ hipError_t launch_gemv(const GemvArgs &args, const GemvPlan &p, hipStream_t stre
   return hipGetLastError();
 }
 
-bool gemvt_takes(int T, int K, int N, int epilogue, bool norm, const GemvPrep *prep) {
+bool gemvt_takes(int T, int K, int N, int epilogue, int norm, const GemvPrep *prep) {
   if (T != 1 || N < 1) return false;
   if (epilogue == kGemvQkvPrep) {
-    if (!prep || prep->q_norm || prep->k_norm || prep->hd < 2 || (prep->hd & (prep->hd - 1))) return false;
+    if (norm == kNormDynTanh || !prep || prep->q_norm || prep->k_norm || prep->hd < 2 || (prep->hd & (prep->hd - 1))) return false;
     return (K == 1024 || K == 2048 || K == 4096) && N == (prep->H + 2 * prep->KV) * prep->hd;
   }
   // rows of 8192: two wavefronts per output, which leaves out the norm prologue and SwiGLU
@@ -744,9 +774,11 @@ bool gemvt_takes(int T, int K, int N, int epilogue, bool norm, const GemvPrep *p
 hipError_t launch_gemvt(const GemvArgs &args, hipStream_t stream) {
   GemvArgs a = args;
   const bool prep = a.epilogue == kGemvQkvPrep;
-  if (!gemvt_takes(a.T, a.K, a.N, a.epilogue, a.norm != 0, &a.prep) || !a.x || !a.w || (!a.y && !prep)) return hipErrorInvalidValue;
+  if (!gemvt_takes(a.T, a.K, a.N, a.epilogue, a.norm, &a.prep) || !a.x || !a.w || (!a.y && !prep)) return hipErrorInvalidValue;
   if (a.epilogue == kGemvResidual && !a.res) return hipErrorInvalidValue;
-  if (((uintptr_t)a.x | (uintptr_t)a.w | (uintptr_t)a.gamma) & 15) return hipErrorInvalidValue;
+  if (((uintptr_t)a.x | (uintptr_t)a.w | (uintptr_t)a.gamma | (uintptr_t)a.beta) & 15) return hipErrorInvalidValue;
+  const bool dyt = a.norm == kNormDynTanh;
+  if (dyt && (!a.gamma || !a.beta)) return hipErrorInvalidValue;
   if (prep) {
     const GemvPrep &q = a.prep;
     if (q.H < 1 || q.KV < 1 || !q.rope_tab || !q.q_rot || !q.kc || !q.vc || q.start_pos < 0 || q.start_pos + 1 > q.cap)
@@ -774,16 +806,23 @@ hipError_t launch_gemvt(const GemvArgs &args, hipStream_t stream) {
   a.rows_per_wave = rpw;
   const int per_wg = (4 / sp) * rpw;
   const dim3 grid((unsigned)((a.N + per_wg - 1) / per_wg));
-#define SHAINET_LAUNCH_GEMVT(KV4_)                                                            \
-  do {                                                                                        \
-    if (two && rpw > 1)                                                                       \
-      hipLaunchKernelGGL((gemvt_kernel<KV4_, 2, 1, true>), grid, dim3(256), 0, stream, a);    \
-    else if (two)                                                                             \
-      hipLaunchKernelGGL((gemvt_kernel<KV4_, 2, 1, false>), grid, dim3(256), 0, stream, a);   \
-    else if (rpw > 1)                                                                         \
-      hipLaunchKernelGGL((gemvt_kernel<KV4_, 1, 1, true>), grid, dim3(256), 0, stream, a);    \
-    else                                                                                      \
-      hipLaunchKernelGGL((gemvt_kernel<KV4_, 1, 1, false>), grid, dim3(256), 0, stream, a);   \
+#define SHAINET_LAUNCH_GEMVT_N(KV4_, DYT_)                                                               \
+  do {                                                                                                   \
+    if (two && rpw > 1)                                                                                  \
+      hipLaunchKernelGGL((gemvt_kernel<KV4_, 2, 1, true, false, DYT_>), grid, dim3(256), 0, stream, a);  \
+    else if (two)                                                                                        \
+      hipLaunchKernelGGL((gemvt_kernel<KV4_, 2, 1, false, false, DYT_>), grid, dim3(256), 0, stream, a); \
+    else if (rpw > 1)                                                                                    \
+      hipLaunchKernelGGL((gemvt_kernel<KV4_, 1, 1, true, false, DYT_>), grid, dim3(256), 0, stream, a);  \
+    else                                                                                                 \
+      hipLaunchKernelGGL((gemvt_kernel<KV4_, 1, 1, false, false, DYT_>), grid, dim3(256), 0, stream, a); \
+  } while (0)
+#define SHAINET_LAUNCH_GEMVT(KV4_)           \
+  do {                                       \
+    if (dyt)                                 \
+      SHAINET_LAUNCH_GEMVT_N(KV4_, true);    \
+    else                                     \
+      SHAINET_LAUNCH_GEMVT_N(KV4_, false);   \
   } while (0)
   switch (a.K) {
     case 1024: SHAINET_LAUNCH_GEMVT(4); break;
@@ -797,6 +836,7 @@ hipError_t launch_gemvt(const GemvArgs &args, hipStream_t stream) {
       break;
   }
 #undef SHAINET_LAUNCH_GEMVT
+#undef SHAINET_LAUNCH_GEMVT_N
   return hipGetLastError();
 }
 

@@ -14,6 +14,8 @@
 #include <vector>
 
 #include "../../include/shainet_hip_attn.h"
+#include "attn_kernels.hpp"
+#include "latent_attn.hpp"
 #include "llama_internal.hpp"
 #include "mini_json.hpp"
 #include "safetensors.hpp"
@@ -161,6 +163,16 @@ bool as_double(const Json *j, double &v) {
   return true;
 }
 
+// config.json of a model directory, parsed
+int read_text(const std::string &path, std::string &out);
+int read_config(const char *model_dir, Json &j) {
+  std::string text, err;
+  if (int rc = read_text(std::string(model_dir) + "/config.json", text)) return rc;
+  if (!JsonParser(text.data(), text.size()).parse(j, err) || j.kind != Json::kObject)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + (err.empty() ? std::string("not a JSON object") : err));
+  return SHAINET_HIP_OK;
+}
+
 int read_text(const std::string &path, std::string &out) {
   FILE *f = fopen(path.c_str(), "rb");
   if (!f) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json not found in " + path.substr(0, path.rfind('/')));
@@ -179,12 +191,8 @@ extern "C" {
 int shainet_hf_read_llama_config(const char *model_dir, shainet_hf_llama_config *cfg) {
   if (!model_dir || !cfg) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
   memset(cfg, 0, sizeof *cfg);
-  std::string text, err;
-  int rc = read_text(std::string(model_dir) + "/config.json", text);
-  if (rc) return rc;
   Json j;
-  if (!JsonParser(text.data(), text.size()).parse(j, err) || j.kind != Json::kObject)
-    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + (err.empty() ? std::string("not a JSON object") : err));
+  if (int rc = read_config(model_dir, j)) return rc;
   const Json *mt = j.get("model_type");
   if (!mt || mt->kind != Json::kString) return fail(SHAINET_HIP_ERR_ARGUMENT, "No model_type in config.json");
   strncpy(cfg->model_type, mt->str.c_str(), sizeof cfg->model_type - 1);
@@ -303,8 +311,8 @@ int shainet_hf_load_llama(const char *model_dir, shainet_llama_model **out) {
     if ((rc = load_transposed(st, stage, p + ".mlp.up_proj.weight", ff, d, bb.gate_up, 2LL * ff, ff))) break;
     if ((rc = load_transposed(st, stage, p + ".mlp.down_proj.weight", d, ff, bb.down, d, 0))) break;
     // RMSNorm (349-350)
-    if ((rc = load_plain(st, stage, p + ".input_layernorm.weight", 1, d, bb.norm1))) break;
-    if ((rc = load_plain(st, stage, p + ".post_attention_layernorm.weight", 1, d, bb.norm2))) break;
+    if ((rc = load_plain(st, stage, p + ".input_layernorm.weight", 1, d, bb.norm1->gamma))) break;
+    if ((rc = load_plain(st, stage, p + ".post_attention_layernorm.weight", 1, d, bb.norm2->gamma))) break;
     // optional Q/K/V biases, a complete set or none (352-363)
     const bool hq = st->find(p + ".self_attn.q_proj.bias"), hk = st->find(p + ".self_attn.k_proj.bias"),
                hv = st->find(p + ".self_attn.v_proj.bias");
@@ -337,7 +345,7 @@ int shainet_hf_load_llama(const char *model_dir, shainet_llama_model **out) {
     }
   }
   // final RMSNorm and the output head (393-404)
-  if (!rc) rc = load_plain(st, stage, "model.norm.weight", 1, d, mb.final_norm);
+  if (!rc) rc = load_plain(st, stage, "model.norm.weight", 1, d, mb.final_norm->gamma);
   if (!rc) {
     if (cfg.tie_word_embeddings) {  // embed.transpose: [d, vocab] from the rows already on the device
       dim3 grid((unsigned)((d + 31) / 32), (unsigned)((V + 31) / 32));
@@ -356,6 +364,247 @@ int shainet_hf_load_llama(const char *model_dir, shainet_llama_model **out) {
   }
   *out = m;
   return SHAINET_HIP_OK;
+}
+
+}  // extern "C"
+
+// ---- designs whose config.json lists their layers one by one ---------------------------------
+namespace {
+
+// Numbers of an object that must be there; the first one that is not is named in the error.
+struct Fields {
+  const Json *obj;
+  std::string where, missing;
+  int integer(const char *key) {
+    int v = 0;
+    if (!obj || !as_int(obj->get(key), v) || !obj->get(key)->is_int) note(key);
+    return v;
+  }
+  double real(const char *key) {
+    double v = 0.0;
+    if (!obj || !as_double(obj->get(key), v)) note(key);
+    return v;
+  }
+  const Json *object(const char *key) {
+    const Json *o = obj ? obj->get(key) : nullptr;
+    if (!o || o->kind != Json::kObject) note(key);
+    return o && o->kind == Json::kObject ? o : nullptr;
+  }
+  void note(const char *key) {
+    if (missing.empty()) missing = where + key;
+  }
+  int status() const {
+    return missing.empty() ? SHAINET_HIP_OK : fail(SHAINET_HIP_ERR_ARGUMENT, "config.json lacks " + missing);
+  }
+};
+
+struct LayerConfig {
+  shainet_latent_config mixer = {};
+  int ff = 0;           // 0: no feed-forward
+  int weights_of = -1;  // the layer whose weights it uses
+};
+struct TutilornConfig {
+  int vocab = 0, width = 0;
+  double eps = 0.0, embedding_scale = 1.0;
+  std::vector<LayerConfig> layers;
+};
+
+int read_layer(const Json &j, int index, LayerConfig &out) {
+  const std::string where = "layers[" + std::to_string(index) + "].";
+  const Json *type = j.get("type");
+  if (!type || type->kind != Json::kString) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json lacks " + where + "type");
+  if (type->str != "latent_attention")
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "type '" + type->str + "' is not a mixer this library has");
+  Fields top = {&j, where, ""};
+  const Json *mixer = top.object("mixer");
+  if (int rc = top.status()) return rc;
+  Fields f = {mixer, where + "mixer.", ""};
+  shainet_latent_config &m = out.mixer;
+  m.heads = f.integer("heads");
+  m.dim = f.integer("dim");
+  m.rot_dim = f.integer("rot_dim");
+  m.vdim = f.integer("vdim");
+  m.kv_rank = f.integer("kv_rank");
+  m.q_rank = f.integer("q_rank");
+  m.scale = f.real("scale");
+  Fields rot = {f.object("rot"), where + "mixer.rot.", ""};
+  m.rot_dims = rot.integer("dims");
+  m.rot_base = rot.real("base");
+  const Json *mask = mixer->get("mask");
+  Fields win = {mask, where + "mixer.mask.", ""};
+  if (mask && !mask->is_null()) {  // without a mask: every position up to its own
+    m.window = win.integer("size");
+    if (win.missing.empty() && m.window < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + win.where + "size must be positive");
+  }
+  for (const Fields *x : {&f, &rot, &win})
+    if (int rc = x->status()) return rc;
+  const Json *mlp = j.get("mlp");
+  if (mlp && !mlp->is_null()) {
+    const Json *kind = mlp->get("kind");
+    if (!kind || kind->kind != Json::kString || kind->str != "dense")
+      return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "mlp.kind must be \"dense\"");
+    Fields g = {mlp, where + "mlp.", ""};
+    out.ff = g.integer("ff");
+    if (int rc = g.status()) return rc;
+    if (out.ff < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "mlp.ff must be positive");
+  }
+  const Json *of = j.get("weights_of");
+  if (of && !of->is_null() && !as_int(of, out.weights_of)) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "weights_of is not a layer");
+  return SHAINET_HIP_OK;
+}
+
+int read_tutilorn_config(const Json &j, TutilornConfig &c) {
+  Fields f = {&j, "", ""};
+  c.vocab = f.integer("vocab");
+  c.width = f.integer("width");
+  Fields norm = {f.object("norm"), "norm.", ""}, emb = {f.object("embedding"), "embedding.", ""};
+  c.eps = norm.real("eps");
+  c.embedding_scale = emb.real("scale");
+  for (const Fields *x : {&f, &norm, &emb})
+    if (int rc = x->status()) return rc;
+  if (c.vocab < 1 || c.width < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: vocab and width must be positive");
+  const Json *layers = j.get("layers");
+  if (!layers || layers->kind != Json::kArray || layers->arr.empty())
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json lacks layers");
+  const int n = (int)layers->arr.size();
+  c.layers.resize(n);
+  for (int i = 0; i < n; ++i)
+    if (int rc = read_layer(layers->arr[i], i, c.layers[i])) return rc;
+  for (int i = 0; i < n; ++i) {  // a layer that borrows may lend what it borrowed
+    int owner = i, steps = 0;
+    while (c.layers[owner].weights_of >= 0 && steps++ <= n) {
+      owner = c.layers[owner].weights_of;
+      if (owner >= n) break;
+    }
+    if (owner >= n || steps > n)
+      return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: layers[" + std::to_string(i) + "].weights_of leads to no layer with weights");
+    if (owner != i) {
+      const LayerConfig &a = c.layers[i], &b = c.layers[owner];
+      const shainet_latent_config &p = a.mixer, &q = b.mixer;
+      if (p.heads != q.heads || p.dim != q.dim || p.rot_dim != q.rot_dim || p.vdim != q.vdim || p.kv_rank != q.kv_rank ||
+          p.q_rank != q.q_rank || p.window != q.window || p.rot_dims != q.rot_dims || p.rot_base != q.rot_base ||
+          p.scale != q.scale || a.ff != b.ff)
+        return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: layers[" + std::to_string(i) + "] differs from the layer whose weights it uses");
+    }
+  }
+  for (int i = 0; i < n; ++i)  // (only now: the walk above follows the links as they are written)
+    while (c.layers[i].weights_of >= 0 && c.layers[c.layers[i].weights_of].weights_of >= 0)
+      c.layers[i].weights_of = c.layers[c.layers[i].weights_of].weights_of;
+  return SHAINET_HIP_OK;
+}
+
+int load_norm(const shainet_safetensors *st, Stager &stage, const std::string &name, int d, NormWeights &n) {
+  int rc = load_plain(st, stage, name, 1, d, n.gamma);
+  if (rc || n.kind != kNormDynTanh) return rc;
+  if ((rc = load_plain(st, stage, name + ".b", 1, d, n.beta))) return rc;
+  std::vector<float> alpha;
+  if ((rc = read_host_vector(st, name + ".alpha", alpha))) return rc;
+  if (alpha.size() != 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "tensor '" + name + ".alpha' is not a scalar");
+  n.alpha = alpha[0];
+  return SHAINET_HIP_OK;
+}
+
+int load_latent_mixer(const shainet_safetensors *st, Stager &stage, const std::string &p, int d, const shainet_latent_config &c,
+                      LatentWeights &w) {
+  const int qw = c.heads * (c.dim + c.rot_dim), kw = c.heads * c.dim, vw = c.heads * c.vdim;
+  int rc;
+  if ((rc = load_transposed(st, stage, p + "dq", c.q_rank, d, w.w_in, w.n_in, 0))) return rc;
+  if ((rc = load_transposed(st, stage, p + "dkv", c.kv_rank + c.rot_dim, d, w.w_in, w.n_in, c.q_rank))) return rc;
+  if ((rc = load_transposed(st, stage, p + "g", c.heads, d, w.w_in, w.n_in, c.q_rank + c.kv_rank + c.rot_dim))) return rc;
+  if ((rc = load_plain(st, stage, p + "dq.norm", 1, c.q_rank, w.dq_norm))) return rc;
+  if ((rc = load_plain(st, stage, p + "dkv.norm", 1, c.kv_rank, w.dkv_norm))) return rc;
+  if ((rc = load_transposed(st, stage, p + "uq", qw, c.q_rank, w.w_uq, qw, 0))) return rc;
+  // W_uk and W_uv twice: a row per output (absorbed), and side by side as a product's matrix (expanded)
+  if ((rc = load_plain(st, stage, p + "uk", kw, c.kv_rank, w.u_kv))) return rc;
+  if ((rc = load_plain(st, stage, p + "uv", vw, c.kv_rank, w.u_kv + (size_t)kw * c.kv_rank))) return rc;
+  if ((rc = load_transposed(st, stage, p + "uk", kw, c.kv_rank, w.w_ukv, kw + vw, 0))) return rc;
+  if ((rc = load_transposed(st, stage, p + "uv", vw, c.kv_rank, w.w_ukv, kw + vw, kw))) return rc;
+  if ((rc = load_plain(st, stage, p + "sink", 1, c.heads, w.sink))) return rc;
+  if ((rc = load_transposed(st, stage, p + "o", d, vw, w.w_o, d, 0))) return rc;
+  w.w_in_t_stale = w.w_uq_t_stale = w.w_o_t_stale = true;
+  return SHAINET_HIP_OK;
+}
+
+// Tutilorn: latent attention with sliding windows, sinks and output gates, Dynamic Tanh norms, dense SwiGLU
+// feed-forwards, layers that may use another layer's weights.
+int load_tutilorn(const char *model_dir, const Json &j, shainet_llama_model **out) {
+  TutilornConfig cfg;
+  int rc = read_tutilorn_config(j, cfg);
+  if (rc) return rc;
+  if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
+  const int d = cfg.width, n = (int)cfg.layers.size();
+  shainet_safetensors *st = nullptr;
+  if ((rc = shainet_safetensors_open(model_dir, &st))) return rc;
+  shainet_llama_model *m = nullptr;
+  Stager stage;
+  rc = shainet_llama_model_create_empty(&m, cfg.vocab, d, cfg.eps, cfg.embedding_scale, kNormDynTanh);
+  std::vector<shainet_llama_block *> blocks(n, nullptr);
+  for (int pass = 0; pass < 2; ++pass)  // layers with weights first: the others may come before them
+    for (int i = 0; i < n && !rc; ++i) {
+      const LayerConfig &lc = cfg.layers[i];
+      if ((lc.weights_of >= 0) != (pass == 1)) continue;
+      rc = shainet_llama_block_create_latent(&blocks[i], d, lc.mixer, lc.ff, kNormDynTanh, cfg.eps,
+                                             pass ? blocks[lc.weights_of] : nullptr);
+    }
+  for (int i = 0; i < n && !rc; ++i) {
+    const LayerConfig &lc = cfg.layers[i];
+    if (lc.weights_of >= 0) continue;
+    const std::string p = "l" + std::to_string(i) + ".";
+    LlamaBlockBuffers bb;
+    if ((rc = shainet_llama_block_buffers(blocks[i], &bb))) break;
+    if ((rc = load_norm(st, stage, p + "norm1", d, *bb.norm1))) break;
+    if ((rc = load_latent_mixer(st, stage, p + "mix.", d, lc.mixer, latent_attn_weights(shainet_llama_block_latent_mixer(blocks[i]))))) break;
+    if (!lc.ff) continue;
+    if ((rc = load_norm(st, stage, p + "norm2", d, *bb.norm2))) break;
+    if ((rc = load_transposed(st, stage, p + "mlp.gate", lc.ff, d, bb.gate_up, 2LL * lc.ff, 0))) break;
+    if ((rc = load_transposed(st, stage, p + "mlp.up", lc.ff, d, bb.gate_up, 2LL * lc.ff, lc.ff))) break;
+    if ((rc = load_transposed(st, stage, p + "mlp.down", d, lc.ff, bb.down, d, 0))) break;
+  }
+  // the model owns the blocks from here on, in the order of the layers
+  for (int i = 0; i < n; ++i)
+    if (blocks[i]) {
+      if (m)
+        shainet_llama_model_add_block(m, blocks[i]);
+      else
+        shainet_llama_block_destroy(blocks[i]);
+    }
+  LlamaModelBuffers mb;
+  if (!rc) rc = shainet_llama_model_buffers(m, &mb);
+  if (!rc) rc = load_plain(st, stage, "embed", cfg.vocab, d, mb.embedding);
+  if (!rc) rc = load_norm(st, stage, "final.norm", d, *mb.final_norm);
+  if (!rc) rc = load_transposed(st, stage, "head", cfg.vocab, d, mb.lm_head, cfg.vocab, 0);
+  shainet_safetensors_close(st);
+  if (rc) {
+    shainet_llama_model_destroy(m);
+    return rc;
+  }
+  *out = m;
+  return SHAINET_HIP_OK;
+}
+
+// Designs by the name their config.json gives under "architecture".
+struct Design {
+  const char *name;
+  int (*load)(const char *model_dir, const Json &config, shainet_llama_model **out);
+};
+constexpr Design kDesigns[] = {{"Tutilorn", load_tutilorn}};
+
+}  // namespace
+
+extern "C" {
+
+int shainet_hf_load_model(const char *model_dir, shainet_llama_model **out) {
+  if (!model_dir || !out) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
+  *out = nullptr;
+  Json j;
+  if (int rc = read_config(model_dir, j)) return rc;
+  const Json *arch = j.get("architecture");
+  if (!arch || arch->kind != Json::kString) return shainet_hf_load_llama(model_dir, out);  // goes by model_type
+  for (const Design &d : kDesigns)
+    if (arch->str == d.name) return d.load(model_dir, j, out);
+  std::string known;
+  for (const Design &d : kDesigns) known += std::string(known.empty() ? "" : ", ") + d.name;
+  return fail(SHAINET_HIP_ERR_ARGUMENT, "Unsupported architecture: '" + arch->str + "'. Supported: " + known);
 }
 
 }  // extern "C"

@@ -9,19 +9,25 @@
 // The second half of this file adds what LlamaBlock#forward_cached
 // (llama_block.cr:189-196) does around attention: the two RMSNorms, the two
 // residual adds and the dense SwiGLU feed-forward, again all on the device.
+// A block's parts are parameters: its mixer is the attention above or latent
+// attention (latent_attn.hip), its norms RMSNorm or Dynamic Tanh, its feed-forward
+// may be missing, and its weights may be another block's.
 #include <hip/hip_runtime.h>
 #include <math.h>
 #include <stdio.h>
 #include <stdlib.h>
 #include <string.h>
 
+#include <memory>
 #include <new>
 #include <string>
 #include <vector>
 
 #include "../../include/shainet_hip_attn.h"
 #include "attn_kernels.hpp"
+#include "attn_context.hpp"
 #include "block_kernels.hpp"
+#include "latent_attn.hpp"
 #include "llama_internal.hpp"
 #include "step_kernel.hpp"
 
@@ -312,54 +318,91 @@ static int attn_forward_host(shainet_llama_attn *l, const float *x, int new_toke
 // ---------------------------------------------------------------------------
 // The whole block: LlamaBlock#forward_cached (llama_block.cr:189-196) with a dense
 // SwiGLU feed-forward (swiglu_ff.cr:76-91).
-struct shainet_llama_block {
-  shainet_llama_attn *attn = nullptr;
-  int d_model = 0, ff_hidden = 0;
-  double eps = 1e-6;                                // RMSNorm eps of @norm1 / @norm2 (llama_block.cr:93-94)
-  float *norm1 = nullptr, *norm2 = nullptr;         // device gamma [d_model]; null = ones (rms_norm.cr:10)
+
+// What blocks that use the same weights share.
+struct BlockWeights {
+  NormWeights norm1, norm2;
   float *gate_up = nullptr, *down = nullptr;        // device [d_model, 2*ff] (gate | up) and [ff, d_model]
   float *gate_up_t = nullptr, *down_t = nullptr;    // the same transposed ([2*ff, d_model], [d_model, ff]), like w_o_t
   bool gate_up_t_stale = true, down_t_stale = true;
+  ~BlockWeights() {
+    for (float *p : {norm1.gamma, norm1.beta, norm2.gamma, norm2.beta, gate_up, down, gate_up_t, down_t})
+      if (p) (void)hipFree(p);
+  }
+};
+
+struct shainet_llama_block {
+  shainet_llama_attn *attn = nullptr;  // the mixer: one of the two
+  LatentAttn *latent = nullptr;
+  int d_model = 0, ff_hidden = 0;                   // ff_hidden 0: no feed-forward
+  double eps = 1e-6;                                // RMSNorm eps of @norm1 / @norm2 (llama_block.cr:93-94)
+  std::shared_ptr<BlockWeights> w = std::make_shared<BlockWeights>();
   DevF x, h, hidden, out;
   PinnedF x_pin, out_pin;  // host-pointer calls stage their rows here
 };
 
 namespace {
 
+// the context behind the block's mixer: stream, error word
+int block_context(shainet_llama_block *b, shainet_attn_ctx **ctx) {
+  if (b->latent) {
+    *ctx = latent_attn_context(b->latent);
+    return SHAINET_HIP_OK;
+  }
+  const int rc = ensure_context(b->attn);
+  *ctx = b->attn->ctx;
+  return rc;
+}
+
+int latent_only(const shainet_llama_block *b, const char *what) {
+  if (b->latent) return fail(SHAINET_HIP_ERR_ARGUMENT, std::string(what) + ": this block's mixer is latent attention");
+  return SHAINET_HIP_OK;
+}
+
+}  // namespace
+
+namespace {
+
 // x and out on the device; asynchronous on the block's stream.
 int block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache = false) {
-  if (!b->gate_up || !b->down) return fail(SHAINET_HIP_ERR_ARGUMENT, "feed-forward weights not set");
-  shainet_llama_attn *l = b->attn;
-  int rc = ensure_context(l);
-  if (rc) return rc;
-  hipStream_t stream = (hipStream_t)shainet_attn_stream(l->ctx);
+  BlockWeights &w = *b->w;
   const int d = b->d_model, ff = b->ff_hidden;
-  if (!b->h.reserve((size_t)T * d) || !b->hidden.reserve((size_t)T * ff))
+  if (ff && (!w.gate_up || !w.down)) return fail(SHAINET_HIP_ERR_ARGUMENT, "feed-forward weights not set");
+  shainet_attn_ctx *ctx = nullptr;
+  int rc = block_context(b, &ctx);
+  if (rc) return rc;
+  hipStream_t stream = (hipStream_t)shainet_attn_stream(ctx);
+  Projector &proj = b->latent ? latent_attn_projector(b->latent) : b->attn->proj;
+  if (ff && (!b->h.reserve((size_t)T * d) || !b->hidden.reserve((size_t)T * ff)))
     return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+  float *h = ff ? b->h.p : out;  // without a feed-forward the mixer's sum is the block's result
   // h = x + attention_cached_cpu(@norm1.forward(x))
   Fused n1;
-  n1.norm = true;
-  n1.gamma = b->norm1;
-  n1.eps = b->eps;
+  w.norm1.apply(n1, b->eps);
   Fused gate;
-  gate.norm = true;
-  gate.gamma = b->norm2;
-  gate.eps = b->eps;
+  w.norm2.apply(gate, b->eps);
   gate.epilogue = kGemvSwiglu;
-  if (gemvt_takes(T, d, ff, gate.epilogue, true)) {
-    gate.w_t = transposed_twin(&b->gate_up_t, &b->gate_up_t_stale, b->gate_up, d, 2 * ff, stream, b->norm2);
-    gate.w_t_has_gamma = gate.w_t && b->norm2;
+  if (ff && gemvt_takes(T, d, ff, gate.epilogue, gate.norm)) {
+    // (the RMSNorm weights ride in the copy; Dynamic Tanh adds beta behind its own, so they stay outside)
+    const float *ride = gate.norm == kNormRms ? gate.gamma : nullptr;
+    gate.w_t = transposed_twin(&w.gate_up_t, &w.gate_up_t_stale, w.gate_up, d, 2 * ff, stream, ride);
+    gate.w_t_has_gamma = gate.w_t && ride;
   }
-  const AheadRows ahead = {gate.w_t, d, ff};
-  if ((rc = attn_forward_device(l, x, T, b->h.p, n1, x, no_cache, &ahead))) return rc;
+  if (b->latent) {
+    rc = latent_attn_forward(b->latent, x, T, h, n1, x, no_cache);
+  } else {
+    const AheadRows ahead = {gate.w_t, d, ff};
+    rc = attn_forward_device(b->attn, x, T, h, n1, x, no_cache, &ahead);
+  }
+  if (rc || !ff) return rc;
   // hidden = silu(normed2 * gate_proj) * (normed2 * up_proj), normed2 = @norm2.forward(h)
-  if ((rc = l->proj.project(b->h.p, d, b->gate_up, b->hidden.p, T, d, ff, stream, gate))) return rc;
+  if ((rc = proj.project(h, d, w.gate_up, b->hidden.p, T, d, ff, stream, gate))) return rc;
   // out = h + hidden * down_proj
   Fused down;
   down.epilogue = kGemvResidual;
-  down.res = b->h.p;
-  if (gemvt_takes(T, ff, d, down.epilogue, false)) down.w_t = transposed_twin(&b->down_t, &b->down_t_stale, b->down, ff, d, stream);
-  return l->proj.project(b->hidden.p, ff, b->down, out, T, ff, d, stream, down);
+  down.res = h;
+  if (gemvt_takes(T, ff, d, down.epilogue, down.norm)) down.w_t = transposed_twin(&w.down_t, &w.down_t_stale, w.down, ff, d, stream);
+  return proj.project(b->hidden.p, ff, w.down, out, T, ff, d, stream, down);
 }
 
 }  // namespace
@@ -370,32 +413,69 @@ int shainet_llama_block_forward_device(shainet_llama_block *b, const float *x, i
 }
 int shainet_llama_block_buffers(shainet_llama_block *b, LlamaBlockBuffers *out) {
   shainet_llama_attn *l = b->attn;
+  BlockWeights &bw = *b->w;
   const size_t d = (size_t)b->d_model, ff = (size_t)b->ff_hidden;
+  const bool tanh_norm = bw.norm1.kind == kNormDynTanh;
   struct Want {
     float **p;
-    size_t n;
-  } wants[] = {{&l->w_qkv, d * (size_t)(l->q_dim + 2 * l->kv_dim)}, {&l->w_o, (size_t)l->q_dim * d},
-               {&b->gate_up, d * 2 * ff},                            {&b->down, ff * d},
-               {&b->norm1, d},                                       {&b->norm2, d}};
+    size_t n;  // 0: this block has no such buffer
+  } wants[] = {{l ? &l->w_qkv : nullptr, l ? d * (size_t)(l->q_dim + 2 * l->kv_dim) : 0},
+               {l ? &l->w_o : nullptr, l ? (size_t)l->q_dim * d : 0},
+               {&bw.gate_up, d * 2 * ff},
+               {&bw.down, ff * d},
+               {&bw.norm1.gamma, d},
+               {&bw.norm2.gamma, ff ? d : 0},
+               {&bw.norm1.beta, tanh_norm ? d : 0},
+               {&bw.norm2.beta, tanh_norm && ff ? d : 0}};
   for (const Want &w : wants)
-    if (!*w.p && hipMalloc((void **)w.p, w.n * sizeof(float)) != hipSuccess) {
+    if (w.n && !*w.p && hipMalloc((void **)w.p, w.n * sizeof(float)) != hipSuccess) {
       *w.p = nullptr;
       return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
     }
   // (whoever asks for the buffers is about to write the weights: the transposed copies are made again)
-  l->w_o_t_stale = l->w_qkv_t_stale = b->gate_up_t_stale = b->down_t_stale = true;
-  *out = LlamaBlockBuffers{l->w_qkv, l->w_o, b->gate_up, b->down, b->norm1, b->norm2,
-                           b->d_model, l->q_dim, l->kv_dim, b->ff_hidden};
+  bw.gate_up_t_stale = bw.down_t_stale = true;
+  if (l) l->w_o_t_stale = l->w_qkv_t_stale = true;
+  *out = LlamaBlockBuffers{l ? l->w_qkv : nullptr, l ? l->w_o : nullptr, bw.gate_up, bw.down,
+                           &bw.norm1,  &bw.norm2,  b->d_model,  l ? l->q_dim : 0, l ? l->kv_dim : 0, b->ff_hidden};
   return SHAINET_HIP_OK;
 }
+
+int shainet_llama_block_create_latent(shainet_llama_block **out, int d_model, const shainet_latent_config &cfg,
+                                      int ff_hidden, int norm_kind, double eps, const shainet_llama_block *weights_of) {
+  *out = nullptr;
+  if (ff_hidden < 0) return fail(SHAINET_HIP_ERR_ARGUMENT, "ff_hidden must not be negative");
+  if (weights_of && (!weights_of->latent || weights_of->d_model != d_model || weights_of->ff_hidden != ff_hidden ||
+                     weights_of->w->norm1.kind != norm_kind))
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "layers that share weights must have the same mixer, feed-forward and norms");
+  LatentAttn *l = nullptr;
+  if (int rc = latent_attn_create(&l, d_model, cfg, eps, weights_of ? weights_of->latent : nullptr)) return rc;
+  shainet_llama_block *b = new (std::nothrow) shainet_llama_block();
+  if (!b) {
+    latent_attn_destroy(l);
+    return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
+  }
+  b->latent = l;
+  b->d_model = d_model;
+  b->ff_hidden = ff_hidden;
+  b->eps = eps;
+  if (weights_of)
+    b->w = weights_of->w;
+  else
+    b->w->norm1.kind = b->w->norm2.kind = norm_kind;
+  *out = b;
+  return SHAINET_HIP_OK;
+}
+LatentAttn *shainet_llama_block_latent_mixer(shainet_llama_block *b) { return b->latent; }
 
 // One decode step of the whole stack in one launch (step_kernel.hip): where this block's weights,
 // parameters and cache are, with room for one more row made first (ensure_gpu_cache!,
 // llama_block.cr:497-520); *pos = rows cached so far.  The step's kernel appends the row;
 // shainet_llama_block_step_commit counts it afterwards.
 int shainet_llama_block_step_begin(shainet_llama_block *b, StepLayer *out, int *pos) {
+  if (int bad = latent_only(b, "one-launch decode step")) return bad;
   shainet_llama_attn *l = b->attn;
-  if (!l->w_qkv || !l->w_o || !b->gate_up || !b->down) return fail(SHAINET_HIP_ERR_ARGUMENT, "weights not set");
+  const BlockWeights &w = *b->w;
+  if (!l->w_qkv || !l->w_o || !w.gate_up || !w.down) return fail(SHAINET_HIP_ERR_ARGUMENT, "weights not set");
   int rc = ensure_context(l);
   if (rc) return rc;
   const int cap = shainet_kv_cache_capacity(l->cache);
@@ -404,10 +484,10 @@ int shainet_llama_block_step_begin(shainet_llama_block *b, StepLayer *out, int *
   if ((rc = shainet_attn_begin_prepared(l->ctx, l->cache, 1, &where))) return rc;
   out->w_qkv = l->w_qkv;
   out->w_o = l->w_o;
-  out->w_gu = b->gate_up;
-  out->w_down = b->down;
-  out->norm1 = b->norm1;
-  out->norm2 = b->norm2;
+  out->w_gu = w.gate_up;
+  out->w_down = w.down;
+  out->norm1 = w.norm1.gamma;
+  out->norm2 = w.norm2.gamma;
   out->b_q = where.b_q;
   out->b_k = where.b_k;
   out->b_v = where.b_v;
@@ -426,17 +506,20 @@ void shainet_llama_block_step_commit(shainet_llama_block *b) {
   shainet_attn_commit_prepared(l->ctx, l->cache, 1);
   l->cache_len += 1;
 }
-// The block's geometry, for the planner of the step kernel.
-void shainet_llama_block_geometry(const shainet_llama_block *b, int *H, int *KV, int *hd, int *ff, double *qk_eps) {
+// The block's geometry, for the planner of the step kernel (false: the kernel does not know this mixer).
+bool shainet_llama_block_geometry(const shainet_llama_block *b, int *H, int *KV, int *hd, int *ff, double *qk_eps) {
+  if (!b->attn) return false;
   *H = b->attn->num_heads;
   *KV = b->attn->num_kv_heads;
   *hd = b->attn->head_dim;
   *ff = b->ff_hidden;
   *qk_eps = b->attn->qk_norm_eps;
+  return true;
 }
 
 // Forget the cached rows past `len` (generation that ran ahead of a stop token).
 int shainet_llama_block_truncate(shainet_llama_block *b, int len) {
+  if (b->latent) return shainet_kv_cache_truncate(latent_attn_cache(b->latent), 0, len);
   shainet_llama_attn *l = b->attn;
   if (len < 0 || len > l->cache_len) return fail(SHAINET_HIP_ERR_ARGUMENT, "truncate beyond the cached length");
   if (l->cache) {
@@ -448,6 +531,10 @@ int shainet_llama_block_truncate(shainet_llama_block *b, int len) {
 }
 // The model's kernels and its blocks' report a given-up wait into one word, the model's.
 void shainet_llama_block_share_error_word(shainet_llama_block *b, int *word) {
+  if (b->latent) {
+    latent_attn_share_error_word(b->latent, word);
+    return;
+  }
   shainet_llama_attn *l = b->attn;
   l->shared_error = word;
   if (l->ctx) {
@@ -456,9 +543,16 @@ void shainet_llama_block_share_error_word(shainet_llama_block *b, int *word) {
   }
 }
 int shainet_llama_block_set_stream(shainet_llama_block *b, hipStream_t stream) {
-  int rc = ensure_context(b->attn);
+  shainet_attn_ctx *ctx = nullptr;
+  int rc = block_context(b, &ctx);
   if (rc) return rc;
-  return shainet_attn_set_stream(b->attn->ctx, (void *)stream);
+  return shainet_attn_set_stream(ctx, (void *)stream);
+}
+// Room for `positions` positions in all, made ahead (a windowed mixer keeps what its window needs).
+int shainet_llama_block_reserve(shainet_llama_block *b, int positions) {
+  if (b->latent) return latent_attn_reserve(b->latent, positions);
+  const int rc = ensure_context(b->attn);
+  return rc ? rc : shainet_kv_cache_reserve(b->attn->cache, positions);
 }
 
 extern "C" {
@@ -488,8 +582,7 @@ int shainet_llama_block_create(shainet_llama_block **out, int d_model, int num_h
 int shainet_llama_block_destroy(shainet_llama_block *b) {
   if (!b) return SHAINET_HIP_OK;
   shainet_llama_attn_destroy(b->attn);
-  for (float *p : {b->norm1, b->norm2, b->gate_up, b->down, b->gate_up_t, b->down_t})
-    if (p) (void)hipFree(p);
+  latent_attn_destroy(b->latent);
   for (DevF *f : {&b->x, &b->h, &b->hidden, &b->out}) f->release();
   b->x_pin.release();
   b->out_pin.release();
@@ -501,9 +594,10 @@ shainet_llama_attn *shainet_llama_block_attn(shainet_llama_block *b) { return b 
 
 int shainet_llama_block_set_norms(shainet_llama_block *b, const float *norm1, const float *norm2) {
   if (!b) return fail(SHAINET_HIP_ERR_ARGUMENT, "block is null");
+  if (int bad = latent_only(b, "shainet_llama_block_set_norms")) return bad;
   if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
   int rc = SHAINET_HIP_OK;
-  float **dst[2] = {&b->norm1, &b->norm2};
+  float **dst[2] = {&b->w->norm1.gamma, &b->w->norm2.gamma};
   const float *src[2] = {norm1, norm2};
   for (int i = 0; i < 2 && !rc; ++i) {
     if (src[i]) {
@@ -514,28 +608,45 @@ int shainet_llama_block_set_norms(shainet_llama_block *b, const float *norm1, co
     }
   }
   // (the transposed copies of q | k | v and gate | up carry the norm weights)
-  b->attn->w_qkv_t_stale = b->gate_up_t_stale = true;
+  b->attn->w_qkv_t_stale = b->w->gate_up_t_stale = true;
   b->attn->w_qkv_t_gamma = nullptr;
   return rc;
 }
 
 int shainet_llama_block_set_ffn(shainet_llama_block *b, const float *gate, const float *up, const float *down) {
   if (!b || !gate || !up || !down) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
+  if (int bad = latent_only(b, "shainet_llama_block_set_ffn")) return bad;
   if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
   const float *mats[2] = {gate, up};
   const int widths[2] = {b->ff_hidden, b->ff_hidden};
-  int rc = upload_side_by_side(&b->gate_up, mats, widths, 2, b->d_model);
-  if (!rc) rc = upload_floats(&b->down, down, (size_t)b->ff_hidden * b->d_model);
-  b->gate_up_t_stale = b->down_t_stale = true;
+  int rc = upload_side_by_side(&b->w->gate_up, mats, widths, 2, b->d_model);
+  if (!rc) rc = upload_floats(&b->w->down, down, (size_t)b->ff_hidden * b->d_model);
+  b->w->gate_up_t_stale = b->w->down_t_stale = true;
   return rc;
 }
 
 int shainet_llama_block_clear_cache(shainet_llama_block *b) {
   if (!b) return fail(SHAINET_HIP_ERR_ARGUMENT, "block is null");
+  if (b->latent) return shainet_kv_cache_clear(latent_attn_cache(b->latent), -1);
   return shainet_llama_attn_clear_cache(b->attn);
 }
 
-int shainet_llama_block_cache_len(const shainet_llama_block *b) { return b ? b->attn->cache_len : -1; }
+int shainet_llama_block_cache_len(const shainet_llama_block *b) {
+  if (b && b->latent) return shainet_kv_cache_len(latent_attn_cache(b->latent), 0);
+  return b ? b->attn->cache_len : -1;
+}
+
+shainet_kv_cache *shainet_llama_block_cache(shainet_llama_block *b) {
+  if (!b) return nullptr;
+  return b->latent ? latent_attn_cache(b->latent) : b->attn->cache;
+}
+
+int shainet_llama_block_latent_config(shainet_llama_block *b, shainet_latent_config *cfg) {
+  if (!b || !cfg) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
+  if (!b->latent) return fail(SHAINET_HIP_ERR_ARGUMENT, "this block's mixer is not latent attention");
+  *cfg = latent_attn_config(b->latent);
+  return SHAINET_HIP_OK;
+}
 
 static int block_forward_any(shainet_llama_block *b, const float *x, int new_tokens, float *out, int mem, bool no_cache);
 
@@ -552,12 +663,13 @@ static int block_forward_any(shainet_llama_block *b, const float *x, int new_tok
   if (mem != SHAINET_HIP_MEM_HOST && mem != SHAINET_HIP_MEM_DEVICE)
     return fail(SHAINET_HIP_ERR_ARGUMENT, "mem must be SHAINET_HIP_MEM_HOST or SHAINET_HIP_MEM_DEVICE");
   if (mem == SHAINET_HIP_MEM_DEVICE) return block_forward_device(b, x, new_tokens, out, no_cache);
-  int rc = ensure_context(b->attn);
+  shainet_attn_ctx *ctx = nullptr;
+  int rc = block_context(b, &ctx);
   if (rc) return rc;
   const size_t xd = (size_t)new_tokens * b->d_model;
   if (!b->x.reserve(xd) || !b->out.reserve(xd) || !b->x_pin.reserve(xd) || !b->out_pin.reserve(xd))
     return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
-  hipStream_t stream = (hipStream_t)shainet_attn_stream(b->attn->ctx);
+  hipStream_t stream = (hipStream_t)shainet_attn_stream(ctx);
   memcpy(b->x_pin.p, x, xd * sizeof(float));
   if (hipMemcpyAsync(b->x.p, b->x_pin.p, xd * sizeof(float), hipMemcpyHostToDevice, stream) != hipSuccess)
     return fail(SHAINET_HIP_ERR_RUNTIME, "hipMemcpyAsync(x) failed");
@@ -569,7 +681,7 @@ static int block_forward_any(shainet_llama_block *b, const float *x, int new_tok
       hipStreamSynchronize(stream) != hipSuccess)
     return fail(SHAINET_HIP_ERR_RUNTIME, "copying the result back failed");
   memcpy(out, b->out_pin.p, xd * sizeof(float));
-  return check_error_word(shainet_attn_error_word(b->attn->ctx));
+  return check_error_word(shainet_attn_error_word(ctx));
 }
 
 }  // extern "C"

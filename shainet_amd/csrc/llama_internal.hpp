@@ -35,13 +35,30 @@ int *shainet_attn_error_word(shainet_attn_ctx *c);
 
 // Device weight buffers of a block / a model, allocated on first request, for a loader
 // that fills them on the device (llama_block.hip, llama_model.hip).
+namespace shainet {
+struct NormWeights;
+struct LatentAttn;
+}
 struct LlamaBlockBuffers {
-  float *w_qkv, *w_o, *gate_up, *down, *norm1, *norm2;
+  float *w_qkv, *w_o, *gate_up, *down;  // w_qkv, w_o: null where the mixer is latent attention; gate_up, down: where there is no feed-forward
+  shainet::NormWeights *norm1, *norm2;
   int d_model, q_dim, kv_dim, ff_hidden;
 };
 int shainet_llama_block_buffers(shainet_llama_block *b, LlamaBlockBuffers *out);
+// A block whose mixer is latent attention (latent_attn.hpp), its norms of one kind (kNorm*), with a
+// dense feed-forward or none (ff_hidden 0).  weights_of: the block whose weights it uses, or null.
+int shainet_llama_block_create_latent(shainet_llama_block **out, int d_model, const shainet_latent_config &cfg,
+                                      int ff_hidden, int norm_kind, double eps, const shainet_llama_block *weights_of);
+shainet::LatentAttn *shainet_llama_block_latent_mixer(shainet_llama_block *b);  // null: grouped-query attention
+// A model without blocks yet, and one more block for it (which it then owns), for loaders of designs
+// whose layers are not all alike.
+int shainet_llama_model_create_empty(shainet_llama_model **out, int vocab, int d_model, double eps,
+                                     double embedding_scale, int norm_kind);
+int shainet_llama_model_add_block(shainet_llama_model *m, shainet_llama_block *b);
 struct LlamaModelBuffers {
-  float *embedding, *final_norm, *lm_head;
+  float *embedding;
+  shainet::NormWeights *final_norm;
+  float *lm_head;
 };
 int shainet_llama_model_buffers(shainet_llama_model *m, LlamaModelBuffers *out);
 
@@ -68,14 +85,31 @@ struct PinnedF {
 struct Fused {
   int epilogue = 0;            // kGemvPlain, kGemvResidual (y = res + x W) or kGemvSwiglu (W = gate | up, [K, 2N])
   const float *res = nullptr;  // [T, N]
-  bool norm = false;           // RMSNorm the rows of x first
+  int norm = 0;                // kNorm*: applied to the rows of x first
   const float *gamma = nullptr;
+  const float *beta = nullptr;  // kNormDynTanh
+  float alpha = 0.f;            // kNormDynTanh
   double eps = 0.0;
   const GemvPrep *prep = nullptr;  // kGemvQkvPrep: where the head rows go (y may be null); at most 16 rows
   // the same weights transposed ([N, K]; kGemvSwiglu: [2N, K]) or null: one row of x then takes the
   // product that gives a wavefront whole outputs (launch_gemvt) where its shapes allow
   const float *w_t = nullptr;
   bool w_t_has_gamma = false;  // the rows of w_t were made with gamma multiplied in: the norm's factor 1 / rms is all that is left to apply
+};
+
+// The weights of one norm, on the device.
+struct NormWeights {
+  int kind = 1;            // kNorm*
+  float *gamma = nullptr;  // null = ones (kNormRms only)
+  float *beta = nullptr;   // kNormDynTanh
+  float alpha = 0.f;       // kNormDynTanh
+  void apply(Fused &f, double eps) const {  // the norm in front of a product
+    f.norm = kind;
+    f.gamma = gamma;
+    f.beta = beta;
+    f.alpha = alpha;
+    f.eps = eps;
+  }
 };
 
 // y[T,N] = epilogue(norm(x)[T,K] * W), all row-major on the device.  Up to 16 rows

@@ -26,11 +26,12 @@ using namespace shainet;
 // llama_block.hip
 int shainet_llama_block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache);
 int shainet_llama_block_set_stream(shainet_llama_block *b, hipStream_t stream);
+int shainet_llama_block_reserve(shainet_llama_block *b, int positions);
 int shainet_llama_block_truncate(shainet_llama_block *b, int len);
 void shainet_llama_block_share_error_word(shainet_llama_block *b, int *word);
 int shainet_llama_block_step_begin(shainet_llama_block *b, shainet::StepLayer *out, int *pos);
 void shainet_llama_block_step_commit(shainet_llama_block *b);
-void shainet_llama_block_geometry(const shainet_llama_block *b, int *H, int *KV, int *hd, int *ff, double *qk_eps);
+bool shainet_llama_block_geometry(const shainet_llama_block *b, int *H, int *KV, int *hd, int *ff, double *qk_eps);
 
 // What the one-launch decode step (step_kernel.hip) keeps between steps.
 struct ModelStep {
@@ -66,7 +67,8 @@ struct shainet_llama_model {
   double eps = 1e-6;
   std::vector<shainet_llama_block *> blocks;
   float *embedding = nullptr;   // device [vocab, d_model]
-  float *final_norm = nullptr;  // device [d_model]; has_final_norm says whether the step exists (@final_norm)
+  float embedding_scale = 1.f;  // times every embedding row
+  NormWeights final_norm;       // has_final_norm says whether the step exists (@final_norm)
   bool has_final_norm = false;
   float *lm_head = nullptr;     // device [d_model, vocab]
   // lm_head transposed ([vocab, d_model]) for the product of a single row: the embedding table
@@ -80,6 +82,7 @@ struct shainet_llama_model {
   int *error = nullptr;  // pinned host word: set by any kernel of the model that gave up a bounded wait
   Projector proj;
   DevF act[2], logits;
+  DevF row_act, row_logits;  // shainet_llama_model_run_rows: the wanted rows and their logits
   int *d_tokens = nullptr;
   size_t d_tokens_cap = 0;
   bool have_logits = false;
@@ -103,10 +106,11 @@ int shainet_llama_model_buffers(shainet_llama_model *m, LlamaModelBuffers *out) 
     float **p;
     size_t n;
   } wants[] = {{&m->embedding, (size_t)m->vocab * m->d_model},
-               {&m->final_norm, (size_t)m->d_model},
+               {&m->final_norm.gamma, (size_t)m->d_model},
+               {&m->final_norm.beta, m->final_norm.kind == kNormDynTanh ? (size_t)m->d_model : 0},
                {&m->lm_head, (size_t)m->d_model * m->vocab}};
   for (const Want &w : wants)
-    if (!*w.p && hipMalloc((void **)w.p, w.n * sizeof(float)) != hipSuccess) {
+    if (w.n && !*w.p && hipMalloc((void **)w.p, w.n * sizeof(float)) != hipSuccess) {
       *w.p = nullptr;
       return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
     }
@@ -114,7 +118,7 @@ int shainet_llama_model_buffers(shainet_llama_model *m, LlamaModelBuffers *out) 
   m->lm_head_t_stale = true;  // (whoever asks for the buffers is about to write them)
   if (m->lm_bias) (void)hipFree(m->lm_bias);  // the loader's output bias is all zeros (hf_loader.cr:404)
   m->lm_bias = nullptr;
-  *out = LlamaModelBuffers{m->embedding, m->final_norm, m->lm_head};
+  *out = LlamaModelBuffers{m->embedding, &m->final_norm, m->lm_head};
   return SHAINET_HIP_OK;
 }
 
@@ -209,11 +213,12 @@ void plan_model_step(shainet_llama_model *m) {
     const int v = atoi(env);
     if (v >= 1 && v < st.n_wgs) st.n_wgs = v;
   }
-  shainet_llama_block_geometry(m->blocks[0], &st.H, &st.KV, &st.hd, &st.ff, &st.qk_eps);
+  // the step kernel knows embedding rows as they are, grouped-query attention and RMSNorm
+  if (m->embedding_scale != 1.f || !shainet_llama_block_geometry(m->blocks[0], &st.H, &st.KV, &st.hd, &st.ff, &st.qk_eps)) return;
   for (shainet_llama_block *b : m->blocks) {
     int H, KV, hd, ff;
     double qe;
-    shainet_llama_block_geometry(b, &H, &KV, &hd, &ff, &qe);
+    if (!shainet_llama_block_geometry(b, &H, &KV, &hd, &ff, &qe)) return;
     if (H != st.H || KV != st.KV || hd != st.hd || ff != st.ff || qe != st.qk_eps) return;
   }
   const StepPlan p = plan_step(m->d_model, st.H, st.KV, st.hd, st.ff, st.n_wgs);
@@ -303,10 +308,26 @@ int run_step(shainet_llama_model *m, const int *d_token) {
   return SHAINET_HIP_OK;
 }
 
+// logits [n, vocab] = lm_head(final norm(n rows of x)) (+ bias)
+int head_rows(shainet_llama_model *m, const float *x, int n, float *logits) {
+  const int d = m->d_model;
+  Fused fin;
+  if (m->has_final_norm) m->final_norm.apply(fin, m->eps);
+  if (gemvt_takes(n, d, m->vocab, fin.epilogue, fin.norm)) fin.w_t = lm_head_twin(m);
+  if (int rc = m->proj.project(x, d, m->lm_head, logits, n, d, m->vocab, m->stream, fin)) return rc;
+  for (int i = 0; m->lm_bias && i < n; ++i) {
+    const hipError_t e = launch_add_bias_row(logits + (size_t)i * m->vocab, m->lm_bias, m->vocab, m->stream);
+    if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("bias launch: ") + hipGetErrorString(e));
+  }
+  return SHAINET_HIP_OK;
+}
+
 // Network#run on token ids that already sit in device memory; asynchronous.  no_cache: every block's
 // LlamaBlock#forward instead of forward_cached (network_run.cr:199-204 with use_kv_cache off): the
 // rows attend among themselves from position 0 and the caches stay as they are.
-int run_device_tokens(shainet_llama_model *m, const int *d_tokens, int T, bool no_cache = false) {
+// last_block (nullable): receives the last block's output, all T rows, as long as the next run lasts.
+int run_device_tokens(shainet_llama_model *m, const int *d_tokens, int T, bool no_cache = false,
+                      const float **last_block = nullptr) {
   const int d = m->d_model;
   if (!m->act[0].reserve((size_t)T * d) || !m->act[1].reserve((size_t)T * d) || !m->logits.reserve((size_t)m->vocab))
     return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
@@ -319,7 +340,7 @@ int run_device_tokens(shainet_llama_model *m, const int *d_tokens, int T, bool n
       return fail(SHAINET_HIP_ERR_ARGUMENT, "this model's geometry does not fit the one-launch decode step");
   }
   if (rc < 0) {
-    hipError_t e = launch_embed(m->embedding, d_tokens, m->act[0].p, T, d, m->stream);
+    hipError_t e = launch_embed(m->embedding, d_tokens, m->act[0].p, T, d, m->stream, m->embedding_scale);
     if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("embedding launch: ") + hipGetErrorString(e));
     for (shainet_llama_block *b : m->blocks) {
       if ((rc = shainet_llama_block_set_stream(b, m->stream))) return rc;
@@ -327,24 +348,37 @@ int run_device_tokens(shainet_llama_model *m, const int *d_tokens, int T, bool n
       cur ^= 1;
     }
   }
-  hipError_t e = hipSuccess;
   // the final norm runs over every row in the reference; only the last one is used afterwards
-  const float *last = m->act[cur].p + (size_t)(T - 1) * d;
-  Fused fin;
-  fin.norm = m->has_final_norm;
-  fin.gamma = m->final_norm;
-  fin.eps = m->eps;
-  if (gemvt_takes(1, d, m->vocab, fin.epilogue, fin.norm)) fin.w_t = lm_head_twin(m);
-  if ((rc = m->proj.project(last, d, m->lm_head, m->logits.p, 1, d, m->vocab, m->stream, fin))) return rc;
-  if (m->lm_bias) {
-    e = launch_add_bias_row(m->logits.p, m->lm_bias, m->vocab, m->stream);
-    if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("bias launch: ") + hipGetErrorString(e));
-  }
+  if ((rc = head_rows(m, m->act[cur].p + (size_t)(T - 1) * d, 1, m->logits.p))) return rc;
+  if (last_block) *last_block = m->act[cur].p;
   m->have_logits = true;
   return SHAINET_HIP_OK;
 }
 
 }  // namespace
+
+int shainet_llama_model_create_empty(shainet_llama_model **out, int vocab, int d_model, double eps,
+                                     double embedding_scale, int norm_kind) {
+  *out = nullptr;
+  if (vocab < 1 || d_model < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "vocab and d_model must be positive");
+  shainet_llama_model *m = new (std::nothrow) shainet_llama_model();
+  if (!m) return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
+  m->vocab = vocab;
+  m->d_model = d_model;
+  m->eps = eps;
+  m->embedding_scale = (float)embedding_scale;
+  m->final_norm.kind = norm_kind;
+  m->error = alloc_error_word();  // null without a device: said by the first call that needs one
+  m->proj.error = m->error;
+  *out = m;
+  return SHAINET_HIP_OK;
+}
+
+int shainet_llama_model_add_block(shainet_llama_model *m, shainet_llama_block *b) {
+  shainet_llama_block_share_error_word(b, m->error);
+  m->blocks.push_back(b);
+  return SHAINET_HIP_OK;
+}
 
 extern "C" {
 
@@ -353,13 +387,8 @@ int shainet_llama_model_create(shainet_llama_model **out, int vocab, int d_model
   if (!out) return fail(SHAINET_HIP_ERR_ARGUMENT, "out is null");
   *out = nullptr;
   if (vocab < 1 || d_model < 1 || n_layers < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "vocab, d_model and n_layers must be positive");
-  shainet_llama_model *m = new (std::nothrow) shainet_llama_model();
-  if (!m) return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
-  m->vocab = vocab;
-  m->d_model = d_model;
-  m->eps = eps;
-  m->error = alloc_error_word();  // null without a device: said by the first call that needs one
-  m->proj.error = m->error;
+  shainet_llama_model *m = nullptr;
+  if (int rc = shainet_llama_model_create_empty(&m, vocab, d_model, eps, 1.0, kNormRms)) return rc;
   for (int i = 0; i < n_layers; ++i) {
     shainet_llama_block *b = nullptr;
     int rc = shainet_llama_block_create(&b, d_model, num_heads, ff_hidden, eps, rope_theta, num_kv_heads, head_dim);
@@ -367,8 +396,7 @@ int shainet_llama_model_create(shainet_llama_model **out, int vocab, int d_model
       shainet_llama_model_destroy(m);
       return rc;
     }
-    shainet_llama_block_share_error_word(b, m->error);
-    m->blocks.push_back(b);
+    shainet_llama_model_add_block(m, b);
   }
   *out = m;
   return SHAINET_HIP_OK;
@@ -377,7 +405,7 @@ int shainet_llama_model_create(shainet_llama_model **out, int vocab, int d_model
 int shainet_llama_model_destroy(shainet_llama_model *m) {
   if (!m) return SHAINET_HIP_OK;
   for (shainet_llama_block *b : m->blocks) shainet_llama_block_destroy(b);
-  for (float *p : {m->embedding, m->final_norm, m->lm_head, m->lm_bias, m->d_vals, m->lm_head_t_own})
+  for (float *p : {m->embedding, m->final_norm.gamma, m->final_norm.beta, m->lm_head, m->lm_bias, m->d_vals, m->lm_head_t_own})
     if (p) (void)hipFree(p);
   if (m->d_tokens) (void)hipFree(m->d_tokens);
   if (m->d_ids) (void)hipFree(m->d_ids);
@@ -385,10 +413,20 @@ int shainet_llama_model_destroy(shainet_llama_model *m) {
   if (m->topk_scratch) (void)hipFree(m->topk_scratch);
   m->proj.release();
   m->step.release();
-  for (DevF *f : {&m->act[0], &m->act[1], &m->logits}) f->release();
+  for (DevF *f : {&m->act[0], &m->act[1], &m->logits, &m->row_act, &m->row_logits}) f->release();
   if (m->stream) (void)hipStreamDestroy(m->stream);
   free_error_word(m->error);
   delete m;
+  return SHAINET_HIP_OK;
+}
+
+int shainet_llama_model_vocab(const shainet_llama_model *m) { return m ? m->vocab : -1; }
+int shainet_llama_model_d_model(const shainet_llama_model *m) { return m ? m->d_model : -1; }
+
+int shainet_llama_model_reserve(shainet_llama_model *m, int positions) {
+  if (!m || positions < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid arguments");
+  for (shainet_llama_block *b : m->blocks)
+    if (int rc = shainet_llama_block_reserve(b, positions)) return rc;
   return SHAINET_HIP_OK;
 }
 
@@ -408,10 +446,11 @@ int shainet_llama_model_set_embedding(shainet_llama_model *m, const float *table
 
 int shainet_llama_model_set_final_norm(shainet_llama_model *m, const float *gamma) {
   if (!m) return fail(SHAINET_HIP_ERR_ARGUMENT, "model is null");
+  if (m->final_norm.kind != kNormRms) return fail(SHAINET_HIP_ERR_ARGUMENT, "this model's final norm is not an RMSNorm");
   m->has_final_norm = gamma != nullptr;
   if (!gamma) return SHAINET_HIP_OK;
   if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
-  return upload_floats(&m->final_norm, gamma, (size_t)m->d_model);
+  return upload_floats(&m->final_norm.gamma, gamma, (size_t)m->d_model);
 }
 
 int shainet_llama_model_set_lm_head(shainet_llama_model *m, const float *w, const float *bias) {
@@ -449,7 +488,8 @@ int shainet_llama_model_run_full(shainet_llama_model *m, const int *tokens, int 
   return model_run(m, tokens, n_tokens, logits, true);
 }
 
-static int model_run(shainet_llama_model *m, const int *tokens, int n_tokens, float *logits, bool no_cache) {
+// Token ids from the host through the blocks.
+static int run_host_tokens(shainet_llama_model *m, const int *tokens, int n_tokens, bool no_cache, const float **last_block) {
   if (!m || !tokens || n_tokens < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid arguments");
   if (!m->embedding || !m->lm_head) return fail(SHAINET_HIP_ERR_ARGUMENT, "embedding or lm_head not set");
   for (int i = 0; i < n_tokens; ++i)  // an id outside the table raises IndexError in the reference
@@ -463,13 +503,41 @@ static int model_run(shainet_llama_model *m, const int *tokens, int n_tokens, fl
   if (hipMemcpyAsync(m->d_tokens, tokens, (size_t)n_tokens * sizeof(int), hipMemcpyHostToDevice, m->stream) !=
       hipSuccess)
     return fail(SHAINET_HIP_ERR_RUNTIME, "hipMemcpyAsync(tokens) failed");
-  if ((rc = run_device_tokens(m, m->d_tokens, n_tokens, no_cache))) return rc;
-  if (logits) {
-    if (hipMemcpyAsync(logits, m->logits.p, (size_t)m->vocab * sizeof(float), hipMemcpyDeviceToHost, m->stream) !=
-            hipSuccess ||
-        hipStreamSynchronize(m->stream) != hipSuccess)
-      return fail(SHAINET_HIP_ERR_RUNTIME, "copying the logits back failed");
-    return check_error_word(m->error);
+  return run_device_tokens(m, m->d_tokens, n_tokens, no_cache, last_block);
+}
+
+static int copy_logits_back(shainet_llama_model *m, const float *from, size_t n, float *to) {
+  if (hipMemcpyAsync(to, from, n * sizeof(float), hipMemcpyDeviceToHost, m->stream) != hipSuccess ||
+      hipStreamSynchronize(m->stream) != hipSuccess)
+    return fail(SHAINET_HIP_ERR_RUNTIME, "copying the logits back failed");
+  return check_error_word(m->error);
+}
+
+static int model_run(shainet_llama_model *m, const int *tokens, int n_tokens, float *logits, bool no_cache) {
+  if (int rc = run_host_tokens(m, tokens, n_tokens, no_cache, nullptr)) return rc;
+  return logits ? copy_logits_back(m, m->logits.p, (size_t)m->vocab, logits) : SHAINET_HIP_OK;
+}
+
+int shainet_llama_model_run_rows(shainet_llama_model *m, const int *tokens, int n_tokens, const int *rows, int n_rows,
+                                 float *logits) {
+  if (n_rows < 0 || (n_rows > 0 && (!rows || !logits))) return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid arguments");
+  for (int i = 0; i < n_rows; ++i)
+    if (rows[i] < 0 || rows[i] >= n_tokens) return fail(SHAINET_HIP_ERR_ARGUMENT, "wanted row outside the run's tokens");
+  const float *hidden = nullptr;
+  if (int rc = run_host_tokens(m, tokens, n_tokens, false, &hidden)) return rc;
+  if (n_rows == 1 && rows[0] == n_tokens - 1) return copy_logits_back(m, m->logits.p, (size_t)m->vocab, logits);
+  constexpr int kChunk = 512;  // rows of logits on the device at a time
+  for (int i0 = 0; i0 < n_rows; i0 += kChunk) {
+    const int n = n_rows - i0 < kChunk ? n_rows - i0 : kChunk;
+    if (int rc = reserve_ints(&m->d_tokens, &m->d_tokens_cap, (size_t)n)) return rc;
+    if (!m->row_act.reserve((size_t)n * m->d_model) || !m->row_logits.reserve((size_t)n * m->vocab))
+      return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+    if (hipMemcpyAsync(m->d_tokens, rows + i0, (size_t)n * sizeof(int), hipMemcpyHostToDevice, m->stream) != hipSuccess)
+      return fail(SHAINET_HIP_ERR_RUNTIME, "hipMemcpyAsync(rows) failed");
+    const hipError_t e = launch_gather_rows(hidden, m->d_tokens, m->row_act.p, n, m->d_model, m->stream);
+    if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("gather launch: ") + hipGetErrorString(e));
+    if (int rc = head_rows(m, m->row_act.p, n, m->row_logits.p)) return rc;
+    if (int rc = copy_logits_back(m, m->row_logits.p, (size_t)n * m->vocab, logits + (size_t)i0 * m->vocab)) return rc;
   }
   return SHAINET_HIP_OK;
 }

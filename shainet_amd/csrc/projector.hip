@@ -133,12 +133,14 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
   const bool swiglu = f.epilogue == kGemvSwiglu;
   if (f.epilogue == kGemvQkvPrep && (!f.prep || T > 16 || (N & 3)))
     return llama_fail(SHAINET_HIP_ERR_ARGUMENT, "the fused q | k | v epilogue takes at most 16 rows");
-  if (f.w_t && gemvt_takes(T, K, N, f.epilogue, f.norm, f.prep) && !(((uintptr_t)x | (uintptr_t)f.gamma) & 15)) {
+  if (f.w_t && gemvt_takes(T, K, N, f.epilogue, f.norm, f.prep) && !(((uintptr_t)x | (uintptr_t)f.gamma | (uintptr_t)f.beta) & 15)) {
     GemvArgs a = {};
     a.x = x;
     a.x_stride = x_stride;
-    a.norm = f.norm ? 1 : 0;
+    a.norm = f.norm;
     a.gamma = f.w_t_has_gamma ? nullptr : f.gamma;
+    a.beta = f.beta;
+    a.alpha = f.alpha;
     a.eps = f.eps;
     a.w = f.w_t;
     a.res = f.res;
@@ -156,14 +158,14 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
   if (T <= 16 && (N & 3) == 0) {
     const float *xin = x;
     long long xs = x_stride;
-    bool norm = f.norm;
-    if (norm && T > 4) {  // every workgroup would redo the sums of squares of all rows: norm them once instead
+    int norm = f.norm;
+    if (norm == kNormRms && T > 4) {  // every workgroup would redo the sums of squares of all rows: norm them once instead
       if (!normed.reserve((size_t)T * K)) return llama_fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
       hipError_t e = launch_rmsnorm(x, x_stride, f.gamma, normed.p, T, K, f.eps, stream);
       if (e != hipSuccess) return llama_fail(SHAINET_HIP_ERR_RUNTIME, std::string("rmsnorm launch: ") + hipGetErrorString(e));
       xin = normed.p;
       xs = K;
-      norm = false;
+      norm = kNormNone;
     }
     const GemvPlan p = plan_gemv(T, K, N, f.epilogue, f.prep ? f.prep->hd : 0);
     if (!scratch.reserve(p.partial_floats)) return llama_fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
@@ -173,8 +175,10 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
     GemvArgs a = {};
     a.x = xin;
     a.x_stride = xs;
-    a.norm = norm ? 1 : 0;
+    a.norm = norm;
     a.gamma = f.gamma;
+    a.beta = f.beta;
+    a.alpha = f.alpha;
     a.eps = f.eps;
     a.w = w;
     a.res = f.res;
@@ -200,8 +204,9 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
   hipError_t e = hipSuccess;
   if (f.norm) {
     if (!normed.reserve((size_t)T * K)) return llama_fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
-    e = launch_rmsnorm(x, x_stride, f.gamma, normed.p, T, K, f.eps, stream);
-    if (e != hipSuccess) return llama_fail(SHAINET_HIP_ERR_RUNTIME, std::string("rmsnorm launch: ") + hipGetErrorString(e));
+    e = f.norm == kNormDynTanh ? launch_dyn_tanh(x, x_stride, f.gamma, f.beta, f.alpha, normed.p, T, K, stream)
+                               : launch_rmsnorm(x, x_stride, f.gamma, normed.p, T, K, f.eps, stream);
+    if (e != hipSuccess) return llama_fail(SHAINET_HIP_ERR_RUNTIME, std::string("norm launch: ") + hipGetErrorString(e));
     xin = normed.p;
     xs = K;
   }

@@ -113,6 +113,13 @@ _SIGNATURES = {
     "shainet_hf_read_llama_config": (C.c_int, [C.c_char_p, C.c_void_p]),
     "shainet_hf_rope_freqs": (C.c_int, [C.c_void_p, _f32p, C.c_int]),
     "shainet_hf_load_llama": (C.c_int, [C.c_char_p, C.POINTER(C.c_void_p)]),
+    "shainet_hf_load_model": (C.c_int, [C.c_char_p, C.POINTER(C.c_void_p)]),
+    "shainet_llama_block_latent_config": (C.c_int, [C.c_void_p, C.c_void_p]),
+    "shainet_llama_block_cache": (C.c_void_p, [C.c_void_p]),
+    "shainet_llama_model_vocab": (C.c_int, [C.c_void_p]),
+    "shainet_llama_model_d_model": (C.c_int, [C.c_void_p]),
+    "shainet_llama_model_reserve": (C.c_int, [C.c_void_p, C.c_int]),
+    "shainet_llama_model_run_rows": (C.c_int, [C.c_void_p, _i32p, C.c_int, _i32p, C.c_int, _f32p]),
     "shainet_llama_model_create": (C.c_int, [C.POINTER(C.c_void_p), C.c_int, C.c_int, C.c_int, C.c_int, C.c_int,
                                              C.c_int, C.c_int, C.c_double, C.c_double]),
     "shainet_llama_model_destroy": (C.c_int, [C.c_void_p]),
@@ -688,6 +695,61 @@ class LlamaBlock:
         return out
 
 
+class _LatentConfig(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank", "window", "rot_dims")] + \
+               [("rot_base", C.c_double), ("scale", C.c_double)]
+
+
+class LatentBlock:
+    """A block whose mixer is latent attention, owned by the LlamaModel that `HFLoader.load_model` made."""
+
+    def __init__(self, d_model, handle):
+        self.d_model, self._block = d_model, C.c_void_p(handle)
+        cfg = _LatentConfig()
+        _check(lib().shainet_llama_block_latent_config(self._block, C.byref(cfg)))
+        self.config = {name: getattr(cfg, name) for name, _ in _LatentConfig._fields_}
+
+    def close(self):
+        self._block = None
+
+    def clear_cache(self):
+        _check(lib().shainet_llama_block_clear_cache(self._block))
+
+    @property
+    def cache_len(self):
+        return lib().shainet_llama_block_cache_len(self._block)
+
+    @property
+    def cache_capacity(self):
+        """Rows the block's cache has room for; a window keeps it from growing with the sequence."""
+        return lib().shainet_kv_cache_capacity(lib().shainet_llama_block_cache(self._block))
+
+    def cache_rows(self, pos0, n):
+        """Cached rows [n, kv_rank + rot_dim] of positions pos0 .. pos0 + n - 1 (the ones still held)."""
+        import numpy as np
+
+        width = self.config["kv_rank"] + self.config["rot_dim"]
+        out = np.empty((n, (width + 15) // 16 * 16), np.float32)
+        _check(lib().shainet_kv_cache_read(lib().shainet_llama_block_cache(self._block), 0, 0, pos0, n,
+                                           out.ctypes.data_as(_f32p), None))
+        return out[:, :width]
+
+    def forward_cached(self, x, _fn="shainet_llama_block_forward_cached"):
+        """numpy [T, d_model] -> numpy, the rows appended behind the cached ones."""
+        import numpy as np
+
+        x = np.ascontiguousarray(x, np.float32)
+        if x.ndim != 2 or x.shape[1] != self.d_model:
+            raise ArgumentError(f"x must be [T, {self.d_model}]")
+        out = np.empty_like(x)
+        _check(getattr(lib(), _fn)(self._block, x.ctypes.data, x.shape[0], out.ctypes.data, MEM_HOST))
+        return out
+
+    def forward(self, x):
+        """The rows among themselves from position 0; the cache is left as it is."""
+        return self.forward_cached(x, _fn="shainet_llama_block_forward")
+
+
 class LlamaModel:
     """Network#run with use_kv_cache for a LLaMA-family network (network_run.cr:185-226) on the
     device: embedding -> blocks -> final norm -> lm_head (+ bias), logits kept on the device for
@@ -705,6 +767,17 @@ class LlamaModel:
         self.vocab, self.d_model, self.n_layers = vocab, d_model, n_layers
         self.blocks = [LlamaBlock(d_model, num_heads, ff_hidden, eps, rope_theta, num_kv_heads, head_dim,
                                   _borrowed=lib().shainet_llama_model_block(self._h, i)) for i in range(n_layers)]
+
+    @classmethod
+    def _adopt(cls, handle):
+        """A model whose layers the library's loader made, described by the library itself."""
+        self = cls.__new__(cls)
+        self._h = handle
+        L = lib()
+        self.vocab, self.d_model = L.shainet_llama_model_vocab(handle), L.shainet_llama_model_d_model(handle)
+        self.n_layers = L.shainet_llama_model_layers(handle)
+        self.blocks = [LatentBlock(self.d_model, L.shainet_llama_model_block(handle, i)) for i in range(self.n_layers)]
+        return self
 
     def close(self):
         if getattr(self, "_h", None) and lib is not None:
@@ -757,6 +830,21 @@ class LlamaModel:
         _check(lib().shainet_llama_model_run(self._h, ids.ctypes.data_as(C.POINTER(C.c_int)), ids.size,
                                              logits.ctypes.data_as(_f32p) if want_logits else None))
         return logits
+
+    def run_rows(self, tokens, rows):
+        """`run`, and the logits [len(rows), vocab] of the given places among `tokens`."""
+        import numpy as np
+
+        ids = np.ascontiguousarray(tokens, np.int32).reshape(-1)
+        want = np.ascontiguousarray(list(rows), np.int32).reshape(-1)
+        logits = np.empty((want.size, self.vocab), np.float32)
+        _check(lib().shainet_llama_model_run_rows(self._h, ids.ctypes.data_as(_i32p), ids.size,
+                                                  want.ctypes.data_as(_i32p), want.size, logits.ctypes.data_as(_f32p)))
+        return logits
+
+    def reserve(self, positions):
+        """Room for that many positions in every block's cache (they grow on demand otherwise)."""
+        _check(lib().shainet_llama_model_reserve(self._h, positions))
 
     def run_full(self, tokens, want_logits=True):
         """Network#run with use_kv_cache off: the rows attend among themselves from position 0,
@@ -984,3 +1072,20 @@ class HFLoader:
         return LlamaModel(cfg["vocab_size"], cfg["hidden_size"], cfg["num_hidden_layers"], cfg["num_attention_heads"],
                           cfg["intermediate_size"], cfg["rms_norm_eps"], cfg["rope_theta"],
                           cfg["num_key_value_heads"], cfg["head_dim"] or None, _loaded=h)
+
+    @staticmethod
+    def load_model(model_dir):
+        """Any model the library has, chosen by its config.json: LLaMA-family ones by "model_type", other
+        designs by "architecture"."""
+        import json
+
+        try:
+            with open(os.path.join(model_dir, "config.json")) as f:
+                config = json.load(f)
+        except (OSError, ValueError) as e:
+            raise ArgumentError(f"config.json in {model_dir}: {e}") from None
+        if "architecture" not in config:
+            return HFLoader.load_llama(model_dir)
+        h = C.c_void_p()
+        _check(lib().shainet_hf_load_model(os.fsencode(model_dir), C.byref(h)))
+        return LlamaModel._adopt(h)
