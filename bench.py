@@ -414,6 +414,134 @@ def model_decode(sa, np, steps, ctx_len=512):
             "prefill_tflops": 2.0 * (weight_bytes / 4 - d * V) * ctx_len / prefill_s / 1e12}
 
 
+# --tutilorn: the design at a few sizes that resemble a real model's layers, beside a LLaMA-family model of
+# the same width, feed-forward, depth and vocabulary.  name, width, ff, layers, vocab,
+# (heads, dim, rot_dim, vdim, kv_rank, q_rank, window), (q heads, kv heads, head_dim)
+TUTILORN_SIZES = [
+    ("w1024", 1024, 4096, 8, 32000, (16, 64, 32, 64, 256, 384, 1024), (16, 8, 64)),
+    ("w2048", 2048, 8192, 6, 32000, (16, 128, 64, 128, 512, 1024, 4096), (32, 8, 64)),
+    ("w4096", 4096, 8192, 4, 32000, (32, 128, 64, 128, 512, 1536, 4096), (32, 8, 128)),
+]
+TUTILORN_PREFILL = (512, 2048, 8192)
+TUTILORN_DECODE = (512, 4096)
+
+
+def tutilorn_folder(torch, folder, width, ff, layers, vocab, mix):
+    """A checkpoint folder of that size with seeded random weights in bfloat16."""
+    from safetensors.torch import save_file
+
+    H, dim, rd, vd, kr, qr, window = mix
+    gen = torch.Generator(device="cuda").manual_seed(5)
+    w = {}
+
+    def put(name, *shape, g=None):
+        a = torch.randn(shape, generator=gen, device="cuda") * (shape[-1] ** -0.5 if g is None else g)
+        w[name] = a.to(torch.bfloat16).cpu()
+
+    def norm(name, n):
+        w[name] = (1 + 0.1 * torch.randn(n, generator=gen, device="cuda")).to(torch.bfloat16).cpu()
+        put(name + ".b", n, g=0.1)
+        w[name + ".alpha"] = torch.tensor(0.5, dtype=torch.bfloat16)
+
+    put("embed", vocab, width, g=0.02)
+    m = {"heads": H, "dim": dim, "rot_dim": rd, "vdim": vd, "kv_rank": kr, "q_rank": qr, "scale": (dim + rd) ** -0.5,
+         "rot": {"base": 10000.0, "dims": rd}, "mask": {"size": window}}
+    for i in range(layers):
+        p = f"l{i}."
+        norm(p + "norm1", width)
+        norm(p + "norm2", width)
+        for n, o, k in (("dq", qr, width), ("uq", H * (dim + rd), qr), ("dkv", kr + rd, width), ("uk", H * dim, kr),
+                        ("uv", H * vd, kr), ("g", H, width), ("o", width, H * vd)):
+            put(p + "mix." + n, o, k)
+        for n, k in (("dq.norm", qr), ("dkv.norm", kr)):
+            w[p + "mix." + n] = torch.ones(k, dtype=torch.bfloat16)
+        put(p + "mix.sink", H, g=1.0)
+        for n, o, k in (("gate", ff, width), ("up", ff, width), ("down", width, ff)):
+            put(p + "mlp." + n, o, k)
+    norm("final.norm", width)
+    put("head", vocab, width)
+    save_file(w, os.path.join(folder, "model.safetensors"))
+    cfg = {"architecture": "Tutilorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 8.0},
+           "layers": [{"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff}} for _ in range(layers)]}
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    per_layer = (width * (qr + kr + rd + H) + qr * H * (dim + rd) + kr * H * (dim + vd) + H * vd * width + 3 * width * ff)
+    return 4 * (layers * per_layer + width * vocab)
+
+
+def llama_of_size(sa, np, width, ff, layers, vocab, heads):
+    H, KV, hd = heads
+    r = np.random.default_rng(11)
+    m = sa.LlamaModel(vocab, width, layers, H, ff, eps=1e-5, rope_theta=5e5, num_kv_heads=KV, head_dim=hd)
+    m.set_embedding(0.02 * r.standard_normal((vocab, width), dtype=np.float32))
+    m.set_lm_head(0.02 * r.standard_normal((width, vocab), dtype=np.float32))
+    m.set_final_norm(np.ones(width, np.float32))
+    shapes = ((width, H * hd), (width, KV * hd), (width, KV * hd), (H * hd, width), (width, ff), (width, ff), (ff, width))
+    ws = [0.02 * r.standard_normal(sh, dtype=np.float32) for sh in shapes]
+    for b in m.blocks:  # (the same seeded values in every block's own buffers)
+        b.set_weights(*ws[:4])
+        b.set_ffn(*ws[4:])
+        b.set_norms(np.ones(width, np.float32), np.ones(width, np.float32))
+    return m, 4 * (layers * sum(a * b for a, b in shapes) + width * vocab)
+
+
+def model_rates(np, m, vocab, steps, warmup, prefill, decode):
+    """Prompt tokens per second of one run each, and greedy tokens per second behind a prompt."""
+    r = np.random.default_rng(3)
+    out = {}
+    for T in prefill:
+        ids = list(r.integers(0, vocab, T))
+        times = []
+        t_w = time.perf_counter()
+        while len(times) < 3 or time.perf_counter() - t_w < 0.3:
+            m.clear_cache()
+            m.sync()
+            t0 = time.perf_counter()
+            m.run(ids, want_logits=False)
+            m.sync()
+            times.append(time.perf_counter() - t0)
+        times = sorted(times[1:])
+        out["prefill_%d_tokens_per_s" % T] = T / times[len(times) // 2]
+        out["prefill_%d_ms" % T] = times[len(times) // 2] * 1e3
+    for L in decode:
+        m.clear_cache()
+        m.run(list(r.integers(0, vocab, L)), want_logits=False)
+        m.generate_greedy(max(16, warmup))
+        t0 = time.perf_counter()
+        n = len(m.generate_greedy(steps))
+        dt = (time.perf_counter() - t0) / n
+        out["decode_ctx%d_us_per_token" % L] = dt * 1e6
+        out["decode_ctx%d_tokens_per_s" % L] = 1 / dt
+    return out
+
+
+def tutilorn_bench(sa, np, torch, steps, warmup, only):
+    """The --tutilorn line: every size of TUTILORN_SIZES (or those named by --only), both designs."""
+    import tempfile
+
+    sizes = {}
+    for name, width, ff, layers, vocab, mix, heads in TUTILORN_SIZES:
+        if only and name not in only:
+            continue
+        with tempfile.TemporaryDirectory() as folder:
+            nbytes = tutilorn_folder(torch, folder, width, ff, layers, vocab, mix)
+            m = sa.HFLoader.load_model(folder)
+        torch.cuda.empty_cache()
+        res = {"config": {"width": width, "ff": ff, "layers": layers, "vocab": vocab, "window": mix[-1],
+                          "heads_dim_rot_vdim_kvrank_qrank": list(mix[:-1]), "llama_heads_kv_hd": list(heads)}}
+        for key in ("tutilorn", "llama"):
+            if key == "llama":
+                m, nbytes = llama_of_size(sa, np, width, ff, layers, vocab, heads)
+            res[key] = {k: round(v, 2) for k, v in model_rates(np, m, vocab, steps, warmup, TUTILORN_PREFILL, TUTILORN_DECODE).items()}
+            res[key]["weight_bytes_per_token"] = nbytes
+            us = res[key]["decode_ctx%d_us_per_token" % TUTILORN_DECODE[0]]
+            res[key]["decode_frac_of_hbm_peak"] = round(nbytes / us / 1e3 / HBM_PEAK_GBPS, 4)
+            m.close()
+        sizes[name] = res
+        print("size %s done" % name, file=sys.stderr, flush=True)
+    print(json.dumps({"tutilorn": sizes, "steps": steps, "warmup": warmup, "dtype": "f32", "data": "synthetic"}))
+
+
 # The kernels the two roofline objects of the bench line price, and the workloads they are priced on.
 ROOFLINE_KERNELS = {
     "roofline": ("decode_splitk_kernel<128, 4, false, false, false>", "qwen3_8b_decode_b16_ctx2048-8192"),
@@ -520,6 +648,8 @@ def main():
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
     ap.add_argument("--calibrate", action="store_true",
                     help="run only the plain copy/read kernels of known size (counter and bandwidth yardstick)")
+    ap.add_argument("--tutilorn", action="store_true",
+                    help="run only the Tutilorn models and the LLaMA-family models of their sizes (--only: names of sizes)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this path is built and measured on one GPU only (sequences, kv heads and context "
@@ -537,6 +667,10 @@ def main():
 
     if args.calibrate:
         calibrate(torch, sa, 10)
+        return
+
+    if args.tutilorn:
+        tutilorn_bench(sa, np, torch, args.steps, args.warmup, set(filter(None, args.only.split(","))))
         return
 
     K, W = args.steps, args.warmup

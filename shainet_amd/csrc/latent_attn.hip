@@ -26,6 +26,13 @@ constexpr int kInitialCapacity = 256;
 // greedy generation looks at its ids every 16 steps and takes the steps after a stop token back:
 // the rows those positions see must not have been dropped
 constexpr int kTakeBack = 64;
+// which form a call takes: the cheaper one, or (SHAINET_HIP_LATENT_PATH=absorbed|expanded, read when a
+// mixer is made) one of them wherever its shapes allow
+enum { kByCost = 0, kAbsorbed = 1, kExpanded = 2 };
+int path_knob() {
+  const char *env = getenv("SHAINET_HIP_LATENT_PATH");
+  return env && !strcmp(env, "absorbed") ? kAbsorbed : env && !strcmp(env, "expanded") ? kExpanded : kByCost;
+}
 }  // namespace
 
 struct LatentAttn {
@@ -38,7 +45,8 @@ struct LatentAttn {
   shainet_kv_cache *cache = nullptr, *scratch_cache = nullptr;
   int *shared_error = nullptr;
   Projector proj;
-  DevF raw, q, q_abs, partials, heads;
+  int path = kByCost;
+  DevF raw, q, q_abs, kv, partials, heads;
 };
 
 LatentWeights::~LatentWeights() {
@@ -76,6 +84,7 @@ int latent_attn_create(LatentAttn **out, int d_model, const shainet_latent_confi
   l->cfg = c;
   l->eps = eps;
   l->sh = sh;
+  l->path = path_knob();
   int rc = SHAINET_HIP_OK;
   if (weights_of) {
     l->w = weights_of->w;
@@ -116,7 +125,7 @@ void latent_attn_destroy(LatentAttn *l) {
   if (l->cache) shainet_kv_cache_destroy(l->cache);
   if (l->ctx) shainet_attn_destroy(l->ctx);
   l->proj.release();
-  for (DevF *b : {&l->raw, &l->q, &l->q_abs, &l->partials, &l->heads}) b->release();
+  for (DevF *b : {&l->raw, &l->q, &l->q_abs, &l->kv, &l->partials, &l->heads}) b->release();
   delete l;
 }
 
@@ -185,14 +194,30 @@ int latent_attn_forward(LatentAttn *l, const float *x, int T, float *out, const 
   r.rows = cache->k;
   r.start_pos = start_pos;
   r.start_row = start_row;
-  LatentPlan plan;
-  if (!plan_latent_absorbed(sh, T, start_row, plan)) return fail(SHAINET_HIP_ERR_ARGUMENT, "too many rows in one call");
-  if (!l->q_abs.reserve((size_t)T * sh.H * sh.row_w) || !l->partials.reserve(plan.partial_floats))
-    return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
-  hipError_t e = launch_latent_absorb(l->q.p, w.u_kv, r, sh, T, l->q_abs.p, stream);
-  if (e == hipSuccess) e = launch_latent_absorbed(l->q_abs.p, cache->k, l->partials.p, sh, T, start_row, plan, stream);
-  if (e == hipSuccess)
-    e = launch_latent_out(l->partials.p, w.u_kv + (size_t)sh.H * sh.dim * sh.kv_rank, w.sink, r, sh, T, plan, l->heads.p, stream);
+  LatentExpandedPlan ex;
+  hipError_t e;
+  if (l->path != kAbsorbed && plan_latent_expanded(sh, T, start_row, ex) && (ex.pays || l->path == kExpanded)) {
+    const int kvw = sh.H * (sh.dim + sh.vdim);
+    if (!l->kv.reserve((size_t)ex.key_rows * kvw + kLatentKvSlack) || !l->partials.reserve(ex.partial_floats))
+      return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+    e = launch_latent_append(r, sh, T, l->q.p, stream);
+    if (e == hipSuccess) {
+      // keys and values of every position the new rows see
+      if ((rc = l->proj.project(cache->k + (size_t)ex.first_row * sh.row_w, sh.row_w, w.w_ukv, l->kv.p, ex.key_rows,
+                                sh.kv_rank, kvw, stream)))
+        return rc;
+      e = launch_latent_expanded(l->q.p, l->kv.p, w.sink, r, sh, T, ex, l->partials.p, l->heads.p, stream);
+    }
+  } else {
+    LatentPlan plan;
+    if (!plan_latent_absorbed(sh, T, start_row, plan)) return fail(SHAINET_HIP_ERR_ARGUMENT, "too many rows in one call");
+    if (!l->q_abs.reserve((size_t)T * sh.H * sh.row_w) || !l->partials.reserve(plan.partial_floats))
+      return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+    e = launch_latent_absorb(l->q.p, w.u_kv, r, sh, T, l->q_abs.p, stream);
+    if (e == hipSuccess) e = launch_latent_absorbed(l->q_abs.p, cache->k, l->partials.p, sh, T, start_row, plan, stream);
+    if (e == hipSuccess)
+      e = launch_latent_out(l->partials.p, w.u_kv + (size_t)sh.H * sh.dim * sh.kv_rank, w.sink, r, sh, T, plan, l->heads.p, stream);
+  }
   if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("latent attention launch: ") + hipGetErrorString(e));
   if (no_cache) {
     if ((rc = shainet_kv_cache_clear(cache, -1))) return rc;

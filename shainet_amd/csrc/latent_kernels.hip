@@ -8,6 +8,9 @@
 // MFMA 16x16x4 layout (lane l): A[m = l % 16][k = l / 16], B[k = l / 16][n = l % 16],
 // D[m = 4 (l / 16) + r][n = l % 16] for accumulator register r.  The contraction index may be
 // visited in any order as long as A and B agree.
+//
+// Prefill is the expanded form: latent_prefill_kernel, fp32 MFMA 32x32x2 over keys and values that a
+// product made from the cached rows, the rotated key part read from the rows themselves.
 #include "latent_kernels.hpp"
 
 #include <math.h>
@@ -19,6 +22,7 @@ namespace shainet {
 namespace {
 
 typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef float f32x16 __attribute__((ext_vector_type(16)));
 
 constexpr float kLog2e = 1.4426950408889634f;
 
@@ -55,8 +59,22 @@ __device__ __forceinline__ void append_row(const LatentRows &r, const LatentShap
   }
 }
 
-__global__ __launch_bounds__(256) void latent_append_kernel(LatentRows r, LatentShape sh) {
+// q (nullable): the rotated parts of the row's queries turn in place
+__global__ __launch_bounds__(256) void latent_append_kernel(LatentRows r, LatentShape sh, float *q) {
   append_row(r, sh, blockIdx.x);
+  const int half = sh.rot_dims >> 1;
+  if (!q || half == 0) return;
+  const int qd = sh.dim + sh.rot_dim;
+  float *qt = q + (long long)blockIdx.x * sh.H * qd + sh.dim;
+  const float2 *tab = r.rope_tab + (long long)(r.start_pos + blockIdx.x) * half;
+  for (int i = threadIdx.x; i < sh.H * half; i += 256) {
+    const int h = i / half, p = i - h * half;
+    float *v = qt + (long long)h * qd + 2 * p;
+    const float x = v[0], y = v[1];
+    const float2 cs = tab[p];
+    v[0] = x * cs.x - y * cs.y;
+    v[1] = y * cs.x + x * cs.y;
+  }
 }
 
 // Workgroups 0 .. T - 1 append a row each; the others take 64 columns of one head of RT rows: lane =
@@ -328,6 +346,266 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const float *__restrict
   }
 }
 
+// ---- expanded form -----------------------------------------------------------------------------
+//
+// A workgroup owns 128 rows of one head, a wavefront 32 of them; all walk the keys in tiles of 32 that
+// go global memory -> registers -> LDS, the next tile's loads in flight behind the MFMAs of this one
+// (two workgroups share a compute unit, so that one's barriers hide behind the other's MFMAs).
+// S^T = K Q^T, so that the probabilities come out of the accumulator laid out as the B operand of
+// O^T += V^T P^T.  MFMA 32x32x2 layout (lane l): A[m = l % 32][k = l / 32], B[k = l / 32][n = l % 32],
+// D[m = 8 (r / 4) + 4 (l / 32) + r % 4][n = l % 32] for accumulator register r.
+//   scores:  m = key within the tile, n = row; lane half j = l / 32 covers d = 8 i + 4 j + 0..3 of piece i;
+//            d runs over the unrotated dimensions, padded to a multiple of 8, then the rotated ones.
+//   output:  tile t, m: d = NT m + t; step r of lane half j is key 8 (r / 4) + 4 j + r % 4.
+// NK: pieces of 8 query / key dimensions at most; NT: tiles of 32 value dimensions.
+struct LatentPrefillArgs {
+  const float *q;        // [T, H (dim + rot_dim)], rotated (launch_latent_append)
+  const float *kv;       // [key rows, H dim + H vdim]
+  const float *key_rot;  // rotated part of key row 0; rows row_w apart
+  const float *sink;
+  LatentRows r;          // raw (gates), rope_tab, start_pos
+  LatentShape sh;
+  float *out;            // [T, H vdim]
+  float *part_o, *part_ml;  // splits > 1: [blocks][splits][128][32 NT], [..][128][2]
+  int T, first_key;      // row t sees key rows .. first_key + t
+  int items, splits;
+  float c;               // scale * log2(e)
+};
+
+template <int NK, int NT>
+__global__ __launch_bounds__(256, NK <= 24 ? 2 : 1) void latent_prefill_kernel(const LatentPrefillArgs a) {
+  constexpr int KSTR = NK * 8 + 4, VSTR = NT * 32;
+  constexpr int KU = (NK * 2 + 7) / 8, VU = NT;  // float4 of a K (V) tile per thread: 8 threads per row
+  __shared__ __attribute__((aligned(16))) float Ks[32 * KSTR];
+  __shared__ __attribute__((aligned(16))) float Vs[32 * VSTR];
+  const LatentShape &sh = a.sh;
+  // heads fastest: with a multiple of 8 heads an XCD (index % 8) keeps to its own heads' keys and
+  // values; the blocks with the most keys start first
+  const int h = blockIdx.x % sh.H;
+  const int chunk = (blockIdx.x / sh.H) % a.splits;
+  const int item = a.items - 1 - (int)(blockIdx.x / sh.H / a.splits);
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int n = lane & 31, j = lane >> 5;
+  const int dn = sh.dim, dr = sh.rot_dim, dn8 = (dn + 7) / 8 * 8;
+  const int row0 = item * 128, w_row0 = row0 + wave * 32;
+  const bool wave_active = w_row0 < a.T;
+  const int my_row = min(w_row0 + n, a.T - 1);
+  const int my_hi = a.first_key + my_row, my_lo = sh.window ? max(0, my_hi - sh.window + 1) : 0;
+  const int w_first = min(w_row0, a.T - 1), w_last = min(w_row0 + 31, a.T - 1);
+  const int w_hi_min = a.first_key + w_first, w_hi_max = a.first_key + w_last;
+  const int w_lo_min = sh.window ? max(0, w_hi_min - sh.window + 1) : 0;
+  const int w_lo_max = sh.window ? max(0, w_hi_max - sh.window + 1) : 0;
+  const int b_hi = a.first_key + min(row0 + 127, a.T - 1);
+  const int b_lo = sh.window ? max(0, a.first_key + row0 - sh.window + 1) : 0;
+  const int kt_all0 = b_lo >> 5, n_tiles = (b_hi >> 5) + 1 - kt_all0;
+  const int per_chunk = (n_tiles + a.splits - 1) / a.splits;
+  const int kt0 = kt_all0 + chunk * per_chunk, kt1 = min(kt_all0 + n_tiles, kt0 + per_chunk);
+
+  // staging: 8 threads per key row, 16-byte pieces sub, sub + 8, ...; a thread without a piece of its
+  // own repeats the last one (same source, same place), so no load or store is conditional
+  const int srow = threadIdx.x >> 3, sub = threadIdx.x & 7;
+  const unsigned kv_stride = (unsigned)(sh.H * (sh.dim + sh.vdim));
+  const int n_pieces = dn >> 2, r_pieces = dr >> 2;
+  const float *k_src[KU];
+  unsigned k_step[KU];
+  int k_dst[KU];
+#pragma unroll
+  for (int u = 0; u < KU; ++u) {
+    const int p = min(sub + 8 * u, n_pieces + r_pieces - 1);
+    const bool is_rot = p >= n_pieces;
+    k_src[u] = is_rot ? a.key_rot + 4 * (p - n_pieces) : a.kv + h * dn + 4 * p;
+    k_step[u] = is_rot ? (unsigned)sh.row_w : kv_stride;
+    k_dst[u] = srow * KSTR + (is_rot ? dn8 + 4 * (p - n_pieces) : 4 * p);
+  }
+  // (pieces beyond vdim read what follows: the columns they land in are never stored)
+  const float *v_src = a.kv + sh.H * dn + h * sh.vdim + 4 * sub;
+  f32x4 stage[KU > VU ? KU : VU];
+  auto load_k = [&](int kt) {
+    const unsigned key = (unsigned)min(kt * 32 + srow, b_hi);
+#pragma unroll
+    for (int u = 0; u < KU; ++u) stage[u] = *(const f32x4 *)(k_src[u] + (unsigned long long)key * k_step[u]);
+  };
+  auto park_k = [&]() {
+#pragma unroll
+    for (int u = 0; u < KU; ++u) *(f32x4 *)&Ks[k_dst[u]] = stage[u];
+  };
+  auto load_v = [&](int kt) {
+    const float *p = v_src + (unsigned long long)(unsigned)min(kt * 32 + srow, b_hi) * kv_stride;
+#pragma unroll
+    for (int u = 0; u < VU; ++u) stage[u] = *(const f32x4 *)(p + 32 * u);
+  };
+  auto park_v = [&]() {
+#pragma unroll
+    for (int u = 0; u < VU; ++u) *(f32x4 *)&Vs[srow * VSTR + 4 * (sub + 8 * u)] = stage[u];
+  };
+  if (kt0 < kt1) load_k(kt0);
+  // the padding between and behind the two parts of a key: the query is zero there, so anything finite will do
+  for (int i = threadIdx.x; i < 32 * KSTR; i += 256) Ks[i] = 0.f;
+
+  float qr[NK * 4];
+  {
+    const float *qp = a.q + ((long long)my_row * sh.H + h) * (dn + dr);
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int d = 8 * i + 4 * j, e = d - dn8;
+      f32x4 x = {0.f, 0.f, 0.f, 0.f};
+      if (d < dn || (e >= 0 && e < dr)) x = *(const f32x4 *)(qp + (d < dn ? d : dn + e));
+      qr[4 * i + 0] = x.x * a.c;
+      qr[4 * i + 1] = x.y * a.c;
+      qr[4 * i + 2] = x.z * a.c;
+      qr[4 * i + 3] = x.w * a.c;
+    }
+  }
+  f32x16 o[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) o[t][r] = 0.f;
+  float m = -INFINITY, l = 0.f;  // reference value of the row's exponentials (log2 units), this lane half's sum
+  constexpr float kTau = 8.f;    // scores may exceed it by this much before it moves
+
+  // Per tile: the values travel while the scores are computed, the next tile's keys while the
+  // values are used; each set is parked in LDS behind a barrier that says the stage is free.
+  __syncthreads();
+  if (kt0 < kt1) park_k();
+  __syncthreads();
+  for (int kt = kt0; kt < kt1; ++kt) {
+    load_v(kt);
+    const int k_first = kt * 32, k_last = k_first + 31;
+    const bool visible = wave_active && k_first <= w_hi_max && k_last >= w_lo_min;
+    f32x16 s;
+#pragma unroll
+    for (int r = 0; r < 16; ++r) s[r] = 0.f;
+    if (visible) {
+      const float *kl = &Ks[n * KSTR + 4 * j];
+      constexpr int PF = 2;
+      f32x4 kf[NK];
+#pragma unroll
+      for (int i = 0; i < PF && i < NK; ++i) kf[i] = *(const f32x4 *)(kl + 8 * i);
+#pragma unroll
+      for (int i = 0; i < NK; ++i) {
+        if (i + PF < NK) kf[i + PF] = *(const f32x4 *)(kl + 8 * (i + PF));
+        __builtin_amdgcn_sched_barrier(0x7);
+        s = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[i].x, qr[4 * i + 0], s, 0, 0, 0);
+        s = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[i].y, qr[4 * i + 1], s, 0, 0, 0);
+        s = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[i].z, qr[4 * i + 2], s, 0, 0, 0);
+        s = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[i].w, qr[4 * i + 3], s, 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0x7);
+      }
+      if (k_first < w_lo_max || k_last > w_hi_min) {  // an edge of some row's keys lies in the tile
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const int key = k_first + 8 * (r >> 2) + 4 * j + (r & 3);
+          if (key < my_lo || key > my_hi) s[r] = -INFINITY;
+        }
+      }
+      float mx = s[0];
+#pragma unroll
+      for (int r = 1; r < 16; ++r) mx = fmaxf(mx, s[r]);
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      const bool move = mx > (m == -INFINITY ? -INFINITY : m + kTau);
+      if (__builtin_amdgcn_ballot_w64(move) != 0) {
+        const float mnew = move ? mx : m;
+        const float alpha = move && m != -INFINITY ? fast_exp2(m - mnew) : 1.f;  // (nothing to rescale before a row's first key)
+        m = mnew;
+        l *= alpha;
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) o[t][r] *= alpha;
+      }
+      const float mref = m == -INFINITY ? 0.f : m;
+      float psum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        s[r] = fast_exp2(s[r] - mref);
+        psum += s[r];
+      }
+      l += psum;
+    }
+    park_v();
+    __syncthreads();
+    if (kt + 1 < kt1) load_k(kt + 1);
+    if (visible) {
+      constexpr int PF = 2;
+      typedef float vrow_t __attribute__((ext_vector_type(NT)));
+      const float *vl = &Vs[4 * j * VSTR + NT * n];
+      vrow_t vv[16];
+#pragma unroll
+      for (int r = 0; r < PF; ++r) vv[r] = *(const vrow_t *)(vl + (8 * (r >> 2) + (r & 3)) * VSTR);
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        if (r + PF < 16) vv[r + PF] = *(const vrow_t *)(vl + (8 * ((r + PF) >> 2) + ((r + PF) & 3)) * VSTR);
+        __builtin_amdgcn_sched_barrier(0x7);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) o[t] = __builtin_amdgcn_mfma_f32_32x32x2f32(vv[r][t], s[r], o[t], 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0x7);
+      }
+    }
+    if (kt + 1 < kt1) park_k();
+    __syncthreads();
+  }
+
+  l += __shfl_xor(l, 32);
+  if (a.splits > 1) {
+    const long long pbase = (((long long)item * sh.H + h) * a.splits + chunk) * 128 + wave * 32 + n;
+    float *op = a.part_o + pbase * VSTR;
+#pragma unroll
+    for (int r = 0; r < 16; ++r)
+#pragma unroll
+      for (int t = 0; t < NT; t += 2)
+        *(float2 *)(op + NT * (8 * (r >> 2) + 4 * j + (r & 3)) + t) = float2{o[t][r], o[t + 1][r]};
+    if (j == 0) *(float2 *)(a.part_ml + 2 * pbase) = float2{m, l};
+    return;
+  }
+  if (w_row0 + n >= a.T) return;
+  const float sk = a.sink[h] * kLog2e, mf = fmaxf(m, sk);
+  const float f = fast_exp2(m - mf), den = l * f + fast_exp2(sk - mf);
+  const float factor = f / den * sigmoid1(a.r.raw[(long long)my_row * a.r.stride + a.r.gate_off + h]);
+  float *op = a.out + ((long long)my_row * sh.H + h) * sh.vdim;
+#pragma unroll
+  for (int r = 0; r < 16; ++r)
+#pragma unroll
+    for (int t = 0; t < NT; t += 2) {
+      const int d = NT * (8 * (r >> 2) + 4 * j + (r & 3)) + t;
+      if (d < sh.vdim) *(float2 *)(op + d) = float2{o[t][r] * factor, o[t + 1][r] * factor};
+    }
+}
+
+// Merges the key chunks of one (row block, head), sink and gate included; blockIdx.y: 32 of its rows.
+__global__ __launch_bounds__(256) void latent_prefill_combine_kernel(const LatentPrefillArgs a, int vstr) {
+  const LatentShape &sh = a.sh;
+  const int h = blockIdx.x % sh.H, item = blockIdx.x / sh.H, v4 = sh.vdim >> 2;
+  const long long base = ((long long)item * sh.H + h) * a.splits * 128;
+  const float sk = a.sink[h] * kLog2e;
+  for (int i = threadIdx.x; i < 32 * v4; i += 256) {
+    const int rl = blockIdx.y * 32 + i / v4, c = i % v4, row = item * 128 + rl;
+    if (row >= a.T) continue;
+    float mm = sk;
+    for (int s = 0; s < a.splits; ++s) mm = fmaxf(mm, a.part_ml[2 * (base + (long long)s * 128 + rl)]);
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    float den = fast_exp2(sk - mm);
+    for (int s0 = 0; s0 < a.splits; s0 += 4) {
+      f32x4 x[4];
+      float2 ml[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const long long p = base + (long long)min(s0 + u, a.splits - 1) * 128 + rl;
+        x[u] = *(const f32x4 *)(a.part_o + p * vstr + 4 * c);
+        ml[u] = *(const float2 *)(a.part_ml + 2 * p);
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float f = s0 + u < a.splits ? fast_exp2(ml[u].x - mm) : 0.f;  // 0 for a chunk in which the row saw no key
+        acc += f * x[u];
+        den += f * ml[u].y;
+      }
+    }
+    const float g = sigmoid1(a.r.raw[(long long)row * a.r.stride + a.r.gate_off + h]);
+    *(f32x4 *)(a.out + ((long long)row * sh.H + h) * sh.vdim + 4 * c) = acc * (g / den);
+  }
+}
+
 constexpr size_t kMaxLds = 160 * 1024;
 
 bool shape_ok(const LatentShape &sh) {
@@ -343,9 +621,9 @@ bool rows_ok(const LatentRows &r, const LatentShape &sh, int T) {
 
 }  // namespace
 
-hipError_t launch_latent_append(const LatentRows &r, const LatentShape &sh, int T, hipStream_t stream) {
+hipError_t launch_latent_append(const LatentRows &r, const LatentShape &sh, int T, float *q, hipStream_t stream) {
   if (!rows_ok(r, sh, T)) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(latent_append_kernel, dim3((unsigned)T), dim3(256), 0, stream, r, sh);
+  hipLaunchKernelGGL(latent_append_kernel, dim3((unsigned)T), dim3(256), 0, stream, r, sh, q);
   return hipGetLastError();
 }
 
@@ -442,6 +720,81 @@ hipError_t launch_latent_out(const float *partials, const float *uv, const float
   else
     hipLaunchKernelGGL(latent_out_kernel<4>, grid, dim3(256), lds, stream, partials, part_ml, uv, sink, r, sh, T, p.splits,
                        p.v_w, per_wg, out);
+  return hipGetLastError();
+}
+
+bool plan_latent_expanded(const LatentShape &sh, int T, int start_row, LatentExpandedPlan &p) {
+  if (!shape_ok(sh) || T < 1 || start_row < 0) return false;
+  // 16-byte pieces of the query, key and value rows
+  if ((sh.dim | sh.rot_dim | sh.vdim | sh.kv_rank) & 3) return false;
+  const int dk = (sh.dim + 7) / 8 * 8 + (sh.rot_dim + 7) / 8 * 8;
+  if (dk > 256 || sh.vdim > 128) return false;
+  p.nk = dk <= 96 ? 12 : dk <= 128 ? 16 : dk <= 192 ? 24 : 32;
+  p.nt = sh.vdim <= 64 ? 2 : 4;
+  const int back = sh.window && sh.window - 1 < start_row ? sh.window - 1 : start_row;
+  p.first_row = start_row - back;
+  p.key_rows = back + T;
+  p.items = (T + 127) / 128;
+  const long long blocks = (long long)p.items * sh.H;
+  if (blocks > 0x3fffff) return false;
+  int tiles = (p.key_rows + 31) / 32;  // of the row block with the most keys
+  if (sh.window && tiles > (sh.window + 127) / 32 + 2) tiles = (sh.window + 127) / 32 + 2;
+  static const int splits_knob = getenv("SHAINET_HIP_LATENT_SPLITS") ? atoi(getenv("SHAINET_HIP_LATENT_SPLITS")) : 0;
+  int splits = blocks >= 384 ? 1 : (int)((512 + blocks - 1) / blocks);  // two workgroups per compute unit
+  if (splits > tiles / 4) splits = tiles / 4;
+  if (splits > 16) splits = 16;
+  if (splits_knob > 0) splits = splits_knob;
+  p.splits = splits < 1 ? 1 : splits;
+  p.partial_floats = p.splits > 1 ? (size_t)blocks * p.splits * 128 * (p.nt * 32 + 2) : 0;
+  // multiply-adds per (row, key, head): this form's, and its product's share; against the absorbed form's,
+  // whose kernel reaches about half this one's rate
+  const double pairs = (double)T * (sh.window && sh.window < p.key_rows ? sh.window : p.key_rows);
+  const double here = pairs * sh.H * (8 * p.nk + 32 * p.nt) + (double)p.key_rows * sh.kv_rank * sh.H * (sh.dim + sh.vdim);
+  p.pays = T > 16 && here < 2.0 * pairs * sh.H * (sh.row_w + sh.kv_rank);
+  return true;
+}
+
+hipError_t launch_latent_expanded(const float *q, const float *kv, const float *sink, const LatentRows &r,
+                                  const LatentShape &sh, int T, const LatentExpandedPlan &p, float *partials, float *out,
+                                  hipStream_t stream) {
+  LatentExpandedPlan want;
+  if (!rows_ok(r, sh, T) || !q || !kv || !sink || !out || !plan_latent_expanded(sh, T, r.start_row, want) ||
+      want.splits != p.splits || want.key_rows != p.key_rows || (p.splits > 1 && !partials))
+    return hipErrorInvalidValue;
+  if (((uintptr_t)q | (uintptr_t)kv | (uintptr_t)r.rows | (uintptr_t)out | (uintptr_t)partials) & 15) return hipErrorInvalidValue;
+  LatentPrefillArgs a = {};
+  a.q = q;
+  a.kv = kv;
+  a.key_rot = r.rows + (long long)p.first_row * sh.row_w + sh.kv_rank;
+  a.sink = sink;
+  a.r = r;
+  a.sh = sh;
+  a.out = out;
+  a.part_o = partials;
+  a.part_ml = partials ? partials + (size_t)p.items * sh.H * p.splits * 128 * p.nt * 32 : nullptr;
+  a.T = T;
+  a.first_key = r.start_row - p.first_row;
+  a.items = p.items;
+  a.splits = p.splits;
+  a.c = sh.scale * kLog2e;
+  const dim3 grid((unsigned)(p.items * sh.H * p.splits));
+#define SHAINET_LAUNCH_EXPANDED(NK_)                                                               \
+  do {                                                                                             \
+    if (p.nt == 2)                                                                                 \
+      hipLaunchKernelGGL((latent_prefill_kernel<NK_, 2>), grid, dim3(256), 0, stream, a);          \
+    else                                                                                           \
+      hipLaunchKernelGGL((latent_prefill_kernel<NK_, 4>), grid, dim3(256), 0, stream, a);          \
+  } while (0)
+  switch (p.nk) {
+    case 12: SHAINET_LAUNCH_EXPANDED(12); break;
+    case 16: SHAINET_LAUNCH_EXPANDED(16); break;
+    case 24: SHAINET_LAUNCH_EXPANDED(24); break;
+    default: SHAINET_LAUNCH_EXPANDED(32); break;
+  }
+#undef SHAINET_LAUNCH_EXPANDED
+  const hipError_t e = hipGetLastError();
+  if (e != hipSuccess || p.splits == 1) return e;
+  hipLaunchKernelGGL(latent_prefill_combine_kernel, dim3((unsigned)(p.items * sh.H), 4), dim3(256), 0, stream, a, p.nt * 32);
   return hipGetLastError();
 }
 

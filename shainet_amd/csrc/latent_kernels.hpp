@@ -38,8 +38,9 @@ struct LatentRows {
   int start_row;             // its place in `rows`
 };
 
-// rows[start_row + t] = [RMS(c) kv_norm | rotated key part | 0] for T new rows
-hipError_t launch_latent_append(const LatentRows &r, const LatentShape &sh, int T, hipStream_t stream);
+// rows[start_row + t] = [RMS(c) kv_norm | rotated key part | 0] for T new rows; the rotated parts of
+// their queries q [T, H (dim + rot_dim)] turn in place (q nullable)
+hipError_t launch_latent_append(const LatentRows &r, const LatentShape &sh, int T, float *q, hipStream_t stream);
 
 // q [T, H (dim + rot_dim)] -> q_abs [T, H, row_w] = [W_uk,h^T q_h | rotated q_h | 0] * scale * log2(e),
 // and the append of launch_latent_append in the same launch.  uk: [H dim, kv_rank].
@@ -57,7 +58,6 @@ struct LatentPlan {
   size_t lds_bytes;
   size_t partial_floats;  // o and (max, sum) together
 };
-// longest: positions the last of the rows sees
 bool plan_latent_absorbed(const LatentShape &sh, int T, int start_row, LatentPlan &p);
 hipError_t launch_latent_absorbed(const float *q_abs, const float *rows, float *partials, const LatentShape &sh, int T,
                                   int start_row, const LatentPlan &p, hipStream_t stream);
@@ -66,5 +66,22 @@ hipError_t launch_latent_absorbed(const float *q_abs, const float *rows, float *
 // uv: [H vdim, kv_rank]; sink: [H], natural units, counted once per row.
 hipError_t launch_latent_out(const float *partials, const float *uv, const float *sink, const LatentRows &r,
                              const LatentShape &sh, int T, const LatentPlan &p, float *out, hipStream_t stream);
+
+// Attention of T rows over expanded keys and values (q as launch_latent_append leaves it): kv [key_rows, H dim + H vdim] = the latents of cached rows
+// first_row .. first_row + key_rows - 1 (the ones any of the T rows sees) times [W_uk | W_uv].  False: sizes
+// that are no multiple of 4, dim + rot_dim above 256 or vdim above 128 (the absorbed form takes those).
+struct LatentExpandedPlan {
+  int first_row, key_rows;
+  int nk, nt;       // instantiation: pieces of 8 query / key dimensions, tiles of 32 value dimensions
+  int items;        // blocks of 128 rows
+  int splits;       // key chunks per block; > 1 adds the combine kernel
+  size_t partial_floats;
+  bool pays;        // cheaper than the absorbed form
+};
+constexpr int kLatentKvSlack = 128;  // floats behind the last row of kv that the kernel may read (and drops)
+bool plan_latent_expanded(const LatentShape &sh, int T, int start_row, LatentExpandedPlan &p);
+hipError_t launch_latent_expanded(const float *q, const float *kv, const float *sink, const LatentRows &r,
+                                  const LatentShape &sh, int T, const LatentExpandedPlan &p, float *partials, float *out,
+                                  hipStream_t stream);
 
 }  // namespace shainet
