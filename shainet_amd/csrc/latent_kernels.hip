@@ -149,18 +149,22 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restr
   }
 }
 
-// Column c of tile ct is (row, head) pair 16 ct + c = row * H + head.  The workgroup walks its share
-// of the tile's keys in steps of KT: the cached rows go to LDS once and serve as keys (the scores'
-// contraction is shared between the wavefronts) and as values (the wavefronts share the columns of
-// the output, NTW tiles of 16 each).  Row stride row_w + 4 in LDS: 16-byte reads down a column of
-// rows, and reads of 16 neighbours in rows 4 j apart, touch every bank once.
+// Column c of tile ct is (row, head) pair 16 ct + c = row * H + head.  The workgroup (eight wavefronts)
+// walks its share of the tile's keys in steps of KT: the cached rows go to LDS once and serve as keys
+// (the scores' contraction is shared between the wavefronts) and as values (the wavefronts share the
+// columns of the output, NTW tiles of 16 each).  Everything the first step needs is requested at
+// once and the next step's rows while this one's are used: a launch of one new row is one step or two
+// per workgroup, bound by its memory round trips.  Row stride row_w + 4 in LDS: 16-byte reads down a
+// column of rows, and reads of 16 neighbours in rows 4 j apart, touch every bank once.
 template <int KT, int NTW>
-__global__ __launch_bounds__(256) void latent_absorbed_kernel(const float *__restrict__ q_abs,
+__global__ __launch_bounds__(512) void latent_absorbed_kernel(const float *__restrict__ q_abs,
                                                               const float *__restrict__ rows,
                                                               float *__restrict__ part_o, float *__restrict__ part_ml,
                                                               LatentShape sh, int T, int start_row, int splits,
                                                               int tiles_per_split, int v_w) {
-  constexpr int SUB = KT / 16, PARTS = 4 / SUB;
+  constexpr int NTH = 512, SUB = KT / 16, PARTS = 8 / SUB;
+  constexpr int TPR = NTH / KT;                          // threads per key row; 32 per query row
+  constexpr int UK = KT == 32 ? 13 : 10, UQ = KT == 32 ? 7 : 10;  // 16-byte pieces per thread: the widest rows plan_latent_absorbed admits
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int row_w = sh.row_w, ldr = row_w + 4;
   float *qs = smem, *ks = qs + 16 * ldr, *ss = ks + KT * ldr;  // ss: [PARTS][KT][17]
@@ -175,40 +179,58 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(const float *__res
   const int tile0 = sp * tiles_per_split, tile1 = min(n_tiles, tile0 + tiles_per_split);
   const int w4 = row_w >> 2;
 
-  auto stage = [&](float *dst, const float *src, int count, int last) {  // `count` rows, the ones past `last` repeat it
-    constexpr int U = 8;
-    for (int i0 = threadIdx.x; i0 < count * w4; i0 += 256 * U) {
-      f32x4 v[U];
+  // a thread's pieces of its row: sub, sub + TPR, ... (past the end: the last one again, to the same place);
+  // rows past the last key repeat it
+  const int krow = threadIdx.x / TPR, ksub = threadIdx.x % TPR, qrow = threadIdx.x >> 5, qsub = threadIdx.x & 31;
+  f32x4 kv[UK];
+  auto load_keys = [&](int tile) {
+    const float *src = rows + (long long)min(lo + tile * KT + krow, hi) * row_w;
 #pragma unroll
-      for (int u = 0; u < U; ++u) {
-        const int i = min(i0 + 256 * u, count * w4 - 1), rr = i / w4;
-        v[u] = *(const f32x4 *)(src + (long long)min(rr, last) * row_w + 4 * (i - rr * w4));
-      }
+    for (int u = 0; u < UK; ++u)
+      if (TPR * u < w4) kv[u] = *(const f32x4 *)(src + 4 * min(ksub + TPR * u, w4 - 1));
+  };
+  auto park_keys = [&]() {
 #pragma unroll
-      for (int u = 0; u < U; ++u) {
-        const int i = i0 + 256 * u, rr = i / w4;
-        if (i < count * w4) *(f32x4 *)(dst + rr * ldr + 4 * (i - rr * w4)) = v[u];
-      }
-    }
+    for (int u = 0; u < UK; ++u)
+      if (TPR * u < w4) *(f32x4 *)(ks + krow * ldr + 4 * min(ksub + TPR * u, w4 - 1)) = kv[u];
   };
 
   float m = -INFINITY, l = 0.f;
   f32x4 acc[NTW];
 #pragma unroll
   for (int i = 0; i < NTW; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  if (tile0 < tile1) stage(qs, q_abs + (long long)v0 * row_w, 16, v1 - v0);
+  if (tile0 < tile1) {
+    f32x4 qv[UQ];
+    const float *src = q_abs + (long long)min(v0 + qrow, v1) * row_w;
+#pragma unroll
+    for (int u = 0; u < UQ; ++u)
+      if (32 * u < w4) qv[u] = *(const f32x4 *)(src + 4 * min(qsub + 32 * u, w4 - 1));
+    load_keys(tile0);
+#pragma unroll
+    for (int u = 0; u < UQ; ++u)
+      if (32 * u < w4) *(f32x4 *)(qs + qrow * ldr + 4 * min(qsub + 32 * u, w4 - 1)) = qv[u];
+  }
   const int sub = wave % SUB, part = wave / SUB;
   const int steps = row_w >> 4, s_begin = part * steps / PARTS, s_end = (part + 1) * steps / PARTS;
   const int v_tiles = min((v_w - d_first) >> 4, 64);
   for (int tile = tile0; tile < tile1; ++tile) {
     const int k0 = lo + tile * KT;
-    stage(ks, rows + (long long)k0 * row_w, KT, hi - k0);
+    park_keys();
+    if (tile + 1 < tile1) load_keys(tile + 1);
     __syncthreads();
     {
       f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
       const float *kp = ks + (16 * sub + n) * ldr + 4 * j, *qp = qs + n * ldr + 4 * j;
+      // (fragments two steps ahead of the MFMAs that use them; the reads past the end stay inside LDS)
+      f32x4 a1 = *(const f32x4 *)(kp + 16 * s_begin), b1 = *(const f32x4 *)(qp + 16 * s_begin);
+      f32x4 a2 = *(const f32x4 *)(kp + 16 * min(s_begin + 1, steps - 1)), b2 = *(const f32x4 *)(qp + 16 * min(s_begin + 1, steps - 1));
       for (int i = s_begin; i < s_end; ++i) {
-        const f32x4 a = *(const f32x4 *)(kp + 16 * i), b = *(const f32x4 *)(qp + 16 * i);
+        const f32x4 a = a1, b = b1;
+        const int ahead = min(i + 2, steps - 1);
+        a1 = a2;
+        b1 = b2;
+        a2 = *(const f32x4 *)(kp + 16 * ahead);
+        b2 = *(const f32x4 *)(qp + 16 * ahead);
         s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, s0, 0, 0, 0);
         s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, s1, 0, 0, 0);
         s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, s0, 0, 0, 0);
@@ -251,15 +273,13 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(const float *__res
     for (int i = 0; i < NTW; ++i) acc[i] *= alpha;
 #pragma unroll
     for (int i = 0; i < NTW; ++i) {
-      const int vt = wave + 4 * i;
-      if (vt < v_tiles) {
-        const float *vp = ks + 4 * j * ldr + d_first + 16 * vt + n;
+      // (a wavefront without an i-th tile computes the last one again and does not store it)
+      const float *vp = ks + 4 * j * ldr + d_first + 16 * min(wave + 8 * i, v_tiles - 1) + n;
 #pragma unroll
-        for (int u = 0; u < SUB; ++u)
+      for (int u = 0; u < SUB; ++u)
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
-            acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(vp[(16 * u + r) * ldr], p[u][r], acc[i], 0, 0, 0);
-      }
+        for (int r = 0; r < 4; ++r)
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(vp[(16 * u + r) * ldr], p[u][r], acc[i], 0, 0, 0);
     }
     __syncthreads();  // the rows are free for the next step's
   }
@@ -268,81 +288,104 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(const float *__res
   const long long slot = (long long)(v0 + n) * splits + sp;
 #pragma unroll
   for (int i = 0; i < NTW; ++i) {
-    const int vt = wave + 4 * i;
+    const int vt = wave + 8 * i;
     if (vt < v_tiles) *(f32x4 *)(part_o + slot * v_w + d_first + 16 * vt + 4 * j) = acc[i];
   }
   if (wave == 0 && j == 0 && blockIdx.z == 0) *(float2 *)(part_ml + 2 * slot) = float2{m, l};
 }
 
-// blockIdx: x = outputs VB x .. of the head, y = head, z = rows RT z ..: the key ranges' sums of
-// latents are merged into LDS, then a wavefront per output takes its row of W_uv.
+// Sixteen outputs of one head, a wavefront each, for RT rows.  blockIdx.x: head fastest, so that with
+// a multiple of 8 heads the workgroups that merge the same partials sit on one XCD; blockIdx.y: rows.
+// The wavefronts' rows of W_uv and the partials are requested before anything is waited for.
 template <int RT>
-__global__ __launch_bounds__(256) void latent_out_kernel(const float *__restrict__ part_o,
-                                                         const float *__restrict__ part_ml,
-                                                         const float *__restrict__ uv, const float *__restrict__ sink,
-                                                         LatentRows r, LatentShape sh, int T, int splits, int v_w,
-                                                         int per_wg, float *__restrict__ out) {
-  extern __shared__ __attribute__((aligned(16))) float smem[];  // [RT][v_w] latents, then [RT][splits] factors
+__global__ __launch_bounds__(1024) void latent_out_kernel(const float *__restrict__ part_o,
+                                                          const float *__restrict__ part_ml,
+                                                          const float *__restrict__ uv, const float *__restrict__ sink,
+                                                          LatentRows r, LatentShape sh, int T, int splits, int v_w,
+                                                          float *__restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  constexpr int WU = 4;   // 16-byte pieces of a row of W_uv per lane held in registers
+  constexpr int LD = 12;  // partials in flight per thread
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int h = blockIdx.y, t0 = blockIdx.z * RT, nt = min(RT, T - t0);
-  float *lat = smem, *fac = smem + RT * v_w;
-  // the factor of a range: 2^(max - overall max) / denominator, the sink included in both
-  for (int a = wave; a < nt; a += 4) {
-    const float2 *ml = (const float2 *)part_ml + ((long long)(t0 + a) * sh.H + h) * splits;
-    const float sk = sink[h] * kLog2e;
-    float mm = sk;
-    for (int s = lane; s < splits; s += 64) mm = fmaxf(mm, ml[s].x);
+  const int h = blockIdx.x % sh.H, t0 = blockIdx.y * RT, nt = min(RT, T - t0);
+  const int v4 = v_w >> 2, groups = 1024 / v4;  // thread: column of 16 bytes c, ranges g, g + groups, ...
+  const int c = threadIdx.x % v4, g = threadIdx.x / v4;
+  float *lat = smem, *fac = lat + RT * v_w, *red = fac + RT * splits;  // [RT][v_w], [RT][splits], [groups][v_w]
+  const int jj = (int)(blockIdx.x / sh.H) * 16 + wave;
+  const float *wr = uv + ((long long)h * sh.vdim + min(jj, sh.vdim - 1)) * sh.kv_rank;
+  const bool held = (sh.kv_rank & 3) == 0 && sh.kv_rank <= 256 * WU;
+  f32x4 w[WU];
+  if (held) {
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) mm = fmaxf(mm, __shfl_xor(mm, o));
-    float den = 0.f;
-    for (int s = lane; s < splits; s += 64) den += ml[s].y * fast_exp2(ml[s].x - mm);  // (an empty range: 0 * 0)
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) den += __shfl_xor(den, o);
-    const float inv = 1.f / (den + fast_exp2(sk - mm));
-    for (int s = lane; s < splits; s += 64) fac[a * splits + s] = fast_exp2(ml[s].x - mm) * inv;
+    for (int u = 0; u < WU; ++u)
+      if (256 * u < sh.kv_rank) w[u] = *(const f32x4 *)(wr + min(256 * u + 4 * lane, sh.kv_rank - 4));
   }
-  __syncthreads();
-  const int v4 = v_w >> 2;
-  for (int i = threadIdx.x; i < nt * v4; i += 256) {
-    const int a = i / v4, c = i - a * v4;
-    const float *po = part_o + ((long long)(t0 + a) * sh.H + h) * splits * v_w + 4 * c;
+  for (int a = 0; a < nt; ++a) {
+    const long long col = (long long)(t0 + a) * sh.H + h;
+    const float *po = part_o + col * splits * v_w + 4 * c;
+    f32x4 x[LD];
+#pragma unroll
+    for (int u = 0; u < LD; ++u)
+      if (groups * u < splits) x[u] = *(const f32x4 *)(po + (long long)min(g + groups * u, splits - 1) * v_w);
+    // the factor of a range: 2^(max - overall max) / denominator, the sink included in both (an empty
+    // range has max -inf and sum 0: factor 0)
+    if (wave == 0) {
+      const float2 *ml = (const float2 *)part_ml + col * splits;
+      const float sk = sink[h] * kLog2e;
+      float mm = sk;
+      for (int s = lane; s < splits; s += 64) mm = fmaxf(mm, ml[s].x);
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1) mm = fmaxf(mm, __shfl_xor(mm, o));
+      float den = 0.f;
+      for (int s = lane; s < splits; s += 64) den += ml[s].y * fast_exp2(ml[s].x - mm);
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1) den += __shfl_xor(den, o);
+      const float inv = 1.f / (den + fast_exp2(sk - mm));
+      for (int s = lane; s < splits; s += 64) fac[a * splits + s] = fast_exp2(ml[s].x - mm) * inv;
+    }
+    __syncthreads();
     f32x4 sum = {0.f, 0.f, 0.f, 0.f};
-    for (int s0 = 0; s0 < splits; s0 += 8) {
-      f32x4 x[8];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) x[u] = *(const f32x4 *)(po + (long long)min(s0 + u, splits - 1) * v_w);
-#pragma unroll
-      for (int u = 0; u < 8; ++u)
-        if (s0 + u < splits) sum += fac[a * splits + s0 + u] * x[u];
+    for (int u = 0; u < LD; ++u)
+      if (g + groups * u < splits) sum += fac[a * splits + g + groups * u] * x[u];
+    for (int s = g + groups * LD; s < splits; s += groups) sum += fac[a * splits + s] * *(const f32x4 *)(po + (long long)s * v_w);
+    if (g < groups) *(f32x4 *)(red + g * v_w + 4 * c) = sum;
+    __syncthreads();
+    for (int i = threadIdx.x; i < v_w; i += 1024) {
+      float s = red[i];
+      for (int k = 1; k < groups; ++k) s += red[k * v_w + i];
+      lat[a * v_w + i] = s;
     }
-    *(f32x4 *)(lat + a * v_w + 4 * c) = sum;
+    __syncthreads();
   }
-  __syncthreads();
-  const int j1 = min(sh.vdim, ((int)blockIdx.x + 1) * per_wg);
-  for (int jj = blockIdx.x * per_wg + wave; jj < j1; jj += 4) {
-    const float *wr = uv + ((long long)h * sh.vdim + jj) * sh.kv_rank;
-    float s[RT];
+  if (jj >= sh.vdim) return;
+  float s[RT];
 #pragma unroll
-    for (int a = 0; a < RT; ++a) s[a] = 0.f;
-    for (int c0 = lane; c0 < sh.kv_rank; c0 += 64 * 8) {
-      float w[8];
+  for (int a = 0; a < RT; ++a) s[a] = 0.f;
+  if (held) {
 #pragma unroll
-      for (int u = 0; u < 8; ++u) w[u] = wr[min(c0 + 64 * u, sh.kv_rank - 1)];
+    for (int u = 0; u < WU; ++u)
+      if (256 * u + 4 * lane < sh.kv_rank) {
 #pragma unroll
-      for (int u = 0; u < 8; ++u)
-        if (c0 + 64 * u < sh.kv_rank) {
-#pragma unroll
-          for (int a = 0; a < RT; ++a) s[a] += w[u] * lat[a * v_w + c0 + 64 * u];
+        for (int a = 0; a < RT; ++a) {
+          const f32x4 x = *(const f32x4 *)(lat + a * v_w + 256 * u + 4 * lane);
+          s[a] += (w[u].x * x.x + w[u].y * x.y) + (w[u].z * x.z + w[u].w * x.w);
         }
-    }
+      }
+  } else {
+    for (int k = lane; k < sh.kv_rank; k += 64) {
+      const float wv = wr[k];
 #pragma unroll
-    for (int a = 0; a < RT; ++a) {
-#pragma unroll
-      for (int o = 32; o > 0; o >>= 1) s[a] += __shfl_xor(s[a], o);
-      if (lane == 0 && a < nt)
-        out[((long long)(t0 + a) * sh.H + h) * sh.vdim + jj] =
-            s[a] * sigmoid1(r.raw[(long long)(t0 + a) * r.stride + r.gate_off + h]);
+      for (int a = 0; a < RT; ++a) s[a] += wv * lat[a * v_w + k];
     }
+  }
+#pragma unroll
+  for (int a = 0; a < RT; ++a) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) s[a] += __shfl_xor(s[a], o);
+    if (lane == 0 && a < nt)
+      out[((long long)(t0 + a) * sh.H + h) * sh.vdim + jj] =
+          s[a] * sigmoid1(r.raw[(long long)(t0 + a) * r.stride + r.gate_off + h]);
   }
 }
 
@@ -646,19 +689,22 @@ bool plan_latent_absorbed(const LatentShape &sh, int T, int start_row, LatentPla
   if (!shape_ok(sh) || T < 1 || start_row < 0 || (long long)T * sh.H > 0x3fffffff) return false;
   p.v_w = (sh.kv_rank + 15) / 16 * 16;
   p.v_slices = (p.v_w + 1023) / 1024;
-  p.key_tile = sh.row_w <= 320 ? 32 : 16;
+  // (what fits 160 KiB: rows of up to 800 floats in steps of 32, up to 1200 in steps of 16)
+  p.key_tile = sh.row_w <= 800 ? 32 : 16;
   const size_t ldr = (size_t)sh.row_w + 4;
-  p.lds_bytes = ((16 + p.key_tile) * ldr + (size_t)4 * 16 * 17) * sizeof(float);
+  p.lds_bytes = ((16 + p.key_tile) * ldr + (size_t)8 * 16 * 17) * sizeof(float);
   if (p.lds_bytes > kMaxLds) return false;
   p.col_tiles = (T * sh.H + 15) / 16;
-  // the most keys a tile of columns walks: the visible ones of its last row and of the rows before it
-  const int rows_per_tile = (15 + sh.H) / sh.H + 1;
+  // the most keys a tile of columns walks: what the last of its rows sees and the rows before it saw besides
+  int span = (14 + sh.H) / sh.H + 1;  // rows that 16 consecutive (row, head) pairs can touch
+  if (span > T) span = T;
   long long keys = (long long)start_row + T;
-  if (sh.window && keys > sh.window + rows_per_tile) keys = (long long)sh.window + rows_per_tile;
-  const int tiles = (int)((keys + p.key_tile - 1) / p.key_tile) + 1;
+  if (sh.window && keys > (long long)sh.window + span - 1) keys = (long long)sh.window + span - 1;
+  const int tiles = (int)((keys + p.key_tile - 1) / p.key_tile);
   static const int target_knob = getenv("SHAINET_HIP_LATENT_WGS") ? atoi(getenv("SHAINET_HIP_LATENT_WGS")) : 0;
   const int target = target_knob > 0 ? target_knob : 256;
-  int splits = (target + p.col_tiles - 1) / p.col_tiles;
+  int splits = target / p.col_tiles;
+  if (splits > 128) splits = 128;
   if (splits > tiles) splits = tiles;
   if (splits < 1) splits = 1;
   p.tiles_per_split = (tiles + splits - 1) / splits;
@@ -676,13 +722,13 @@ hipError_t launch_latent_absorbed(const float *q_abs, const float *rows, float *
   float *part_o = partials, *part_ml = partials + (size_t)p.col_tiles * 16 * p.splits * p.v_w;
   const dim3 grid((unsigned)p.col_tiles, (unsigned)p.splits, (unsigned)p.v_slices);
   const int slice = p.v_w < 1024 ? p.v_w : 1024;
-  const int ntw = (slice / 16 + 3) / 4;
+  const int ntw = (slice / 16 + 7) / 8;
 #define SHAINET_LAUNCH_ABSORBED(KT_, NTW_)                                                                               \
   do {                                                                                                                   \
     static const hipError_t a_ = hipFuncSetAttribute((const void *)latent_absorbed_kernel<KT_, NTW_>,                           \
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds);                 \
     if (a_ != hipSuccess) return a_;                                                                                    \
-    hipLaunchKernelGGL((latent_absorbed_kernel<KT_, NTW_>), grid, dim3(256), p.lds_bytes, stream, q_abs, rows, part_o,  \
+    hipLaunchKernelGGL((latent_absorbed_kernel<KT_, NTW_>), grid, dim3(512), p.lds_bytes, stream, q_abs, rows, part_o,  \
                        part_ml, sh, T, start_row, p.splits, p.tiles_per_split, p.v_w);                                  \
   } while (0)
 #define SHAINET_LAUNCH_ABSORBED_K(NTW_)  \
@@ -692,14 +738,14 @@ hipError_t launch_latent_absorbed(const float *q_abs, const float *rows, float *
     else                                 \
       SHAINET_LAUNCH_ABSORBED(16, NTW_); \
   } while (0)
-  if (ntw <= 2)
+  if (ntw <= 1)
+    SHAINET_LAUNCH_ABSORBED_K(1);
+  else if (ntw <= 2)
     SHAINET_LAUNCH_ABSORBED_K(2);
   else if (ntw <= 4)
     SHAINET_LAUNCH_ABSORBED_K(4);
-  else if (ntw <= 8)
-    SHAINET_LAUNCH_ABSORBED_K(8);
   else
-    SHAINET_LAUNCH_ABSORBED_K(16);
+    SHAINET_LAUNCH_ABSORBED_K(8);
 #undef SHAINET_LAUNCH_ABSORBED_K
 #undef SHAINET_LAUNCH_ABSORBED
   return hipGetLastError();
@@ -709,17 +755,19 @@ hipError_t launch_latent_out(const float *partials, const float *uv, const float
                              const LatentShape &sh, int T, const LatentPlan &p, float *out, hipStream_t stream) {
   if (!rows_ok(r, sh, T) || !partials || !uv || !sink || !out || sh.H > 65535) return hipErrorInvalidValue;
   const float *part_ml = partials + (size_t)p.col_tiles * 16 * p.splits * p.v_w;
-  const int per_wg = 16;
   const int rt = T == 1 ? 1 : 4;
-  const size_t lds = (size_t)rt * (p.v_w + p.splits) * sizeof(float);
-  if (lds > 64 * 1024 || (T + rt - 1) / rt > 65535) return hipErrorInvalidValue;
-  const dim3 grid((unsigned)((sh.vdim + per_wg - 1) / per_wg), (unsigned)sh.H, (unsigned)((T + rt - 1) / rt));
+  const int v4 = p.v_w / 4;
+  if (v4 > 1024) return hipErrorInvalidValue;
+  const size_t lds = ((size_t)rt * (p.v_w + p.splits) + (size_t)(1024 / v4) * p.v_w) * sizeof(float);
+  const long long wgs = (long long)((sh.vdim + 15) / 16) * sh.H;
+  if (lds > 64 * 1024 || (T + rt - 1) / rt > 65535 || wgs > 0x7fffffffLL) return hipErrorInvalidValue;
+  const dim3 grid((unsigned)wgs, (unsigned)((T + rt - 1) / rt));
   if (rt == 1)
-    hipLaunchKernelGGL(latent_out_kernel<1>, grid, dim3(256), lds, stream, partials, part_ml, uv, sink, r, sh, T, p.splits,
-                       p.v_w, per_wg, out);
+    hipLaunchKernelGGL(latent_out_kernel<1>, grid, dim3(1024), lds, stream, partials, part_ml, uv, sink, r, sh, T, p.splits,
+                       p.v_w, out);
   else
-    hipLaunchKernelGGL(latent_out_kernel<4>, grid, dim3(256), lds, stream, partials, part_ml, uv, sink, r, sh, T, p.splits,
-                       p.v_w, per_wg, out);
+    hipLaunchKernelGGL(latent_out_kernel<4>, grid, dim3(1024), lds, stream, partials, part_ml, uv, sink, r, sh, T, p.splits,
+                       p.v_w, out);
   return hipGetLastError();
 }
 
