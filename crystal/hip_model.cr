@@ -54,6 +54,10 @@ module SHAInet
       HIP.model_fn shainet_llama_model_sample, Model, Int32, Float64, Float64, Pointer(Int32), Int32
       HIP.model_fn shainet_llama_model_generate_greedy, Model, Int32, Pointer(Int32), Int32, Pointer(Int32), Pointer(Int32), Int32
       HIP.model_fn shainet_hf_load_llama, Pointer(UInt8), Pointer(Model), Int32
+      HIP.model_fn shainet_hf_load_model, Pointer(UInt8), Pointer(Model), Int32
+      HIP.model_fn shainet_llama_model_vocab, Model, Int32
+      HIP.model_fn shainet_llama_model_reserve, Model, Int32, Int32
+      HIP.model_fn shainet_llama_model_run_rows, Model, Pointer(Int32), Int32, Pointer(Int32), Int32, Pointer(Float32), Int32
     end
 
     def self.check!(status : Int32)
@@ -73,6 +77,21 @@ module SHAInet
         h = Model.null
         HIP.check!(LibModel.shainet_hf_load_llama(model_dir.to_unsafe, pointerof(h)))
         new(h, vocab)
+      end
+
+      # Any model directory, by its config.json
+      def self.load_model(model_dir : String) : DeviceLlama
+        h = Model.null
+        HIP.check!(LibModel.shainet_hf_load_model(model_dir.to_unsafe, pointerof(h)))
+        new(h, LibModel.shainet_llama_model_vocab(h))
+      end
+
+      # The logits rows of the given places among `ids`
+      def run_rows(ids : Array(Int32), rows : Array(Int32)) : SimpleMatrix
+        logits = SimpleMatrix.new(rows.size, @vocab)
+        HIP.check!(LibModel.shainet_llama_model_run_rows(@handle, ids.to_unsafe, ids.size, rows.to_unsafe, rows.size,
+          logits.data.to_unsafe))
+        logits
       end
 
       def run(ids : Array(Int32)) : SimpleMatrix

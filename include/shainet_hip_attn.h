@@ -317,8 +317,8 @@ int shainet_llama_block_forward(shainet_llama_block *block, const float *x, int 
  * [RMS-normed latent of kv_rank | rotated key part of rot_dim | zeros to a multiple of 16].  Per head, dim
  * unrotated and rot_dim rotated query / key dimensions (pairs (2i, 2i + 1) of the first rot_dims turn by
  * position * rot_base^(-2i / rot_dims)) and vdim value dimensions; scores times `scale`; a learned sink per
- * head in the softmax's denominator; the head's output times a sigmoid gate.  window > 0: a position sees
- * itself and the window - 1 before it, and the cache drops the rows nobody can see any more; 0: all before it. */
+ * head in the softmax's denominator; the head's output times a sigmoid gate.  window > 0: a query
+ * reaches that many rows back, its own included, and the cache drops the rows out of every later reach; 0: no limit. */
 typedef struct {
   int heads, dim, rot_dim, vdim, kv_rank, q_rank, window, rot_dims;
   double rot_base, scale;

@@ -36,8 +36,8 @@ struct shainet_attn_ctx {
   // its V array.  v_hd = hd for grouped-query attention; 0 for latent attention, whose one row per
   // position (KV = 1; hd = the padded row width) serves as key and as value.
   int v_hd;
-  // > 0: a position sees itself and the window - 1 positions before it, so a cache may forget
-  // older rows (shainet_kv_cache_make_room); 0: every position up to its own.
+  // > 0: a query reaches `window` rows back, its own row included, so a cache may forget older ones
+  // (shainet_kv_cache_make_room); 0: all the way to position 0.
   int window = 0;
   // angles of the cos/sin table in fp64, rounded when the table is written (false: the fp32 product
   // position * frequency of llama_block.cr:274-277)

@@ -614,7 +614,7 @@ int shainet_kv_cache_truncate(shainet_kv_cache *kc, int seq, int len) {
   if (len == 0) {
     kc->base[seq] = 0;
   } else if (kc->base[seq] > 0) {
-    // the next position sees window - 1 rows before it
+    // the next position's reach
     const int first = len - (kc->ctx->window - 1);
     if (kc->base[seq] > (first > 0 ? first : 0))
       return fail(SHAINET_HIP_ERR_ARGUMENT, "truncate to %d: the rows before position %d have been dropped", len,

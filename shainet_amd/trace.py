@@ -2,7 +2,7 @@
 
 Steps come as JSON lines on standard input:
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": ["a"]}
+    {"step": 4, "entries": [{"id": "chat-7", "tokens": [81, 2, 2, 640], "want": [3]}], "end": ["chat-7"]}
 
 An entry holds a request's next tokens and the places among them whose logits are wanted; "end" lists the
 requests that are finished after the step.  OUT/<step>.f32 receives the wanted rows as little-endian

@@ -41,7 +41,7 @@ def test_sink_is_a_key_without_a_value():
     assert np.allclose(to.softmax_with_sink(s, mask, -1e9).sum(-1), 1)
 
 
-def test_window_counts_the_position_itself():
+def test_window_includes_its_own_row():
     m = to.window_mask(6, 2)
     assert m.sum() == 11 and m[4].tolist() == [False, False, False, True, True, False]
     assert np.array_equal(to.window_mask(6, None), np.tril(np.ones((6, 6), bool)))

@@ -25,7 +25,7 @@ def rope_interleaved(x, positions, base, dims):
 
 
 def window_mask(T, size):
-    """[T, T], True where query i sees key j: 0 <= i - j < size (size None: every key up to i)."""
+    """[query, key], True for lags 0 .. size - 1 of the key behind the query (size None: any lag)."""
     d = np.arange(T)[:, None] - np.arange(T)[None, :]
     return (d >= 0) & ((d < size) if size else True)
 
