@@ -324,8 +324,22 @@ typedef struct {
   double rot_base, scale;
 } shainet_latent_config;
 int shainet_llama_block_latent_config(shainet_llama_block *block, shainet_latent_config *cfg);
-/* the block's cache, owned by the block (null before a grouped-query block's first call) */
+/* the block's cache, owned by the block (null before a grouped-query block's first call, and where a state
+ * takes its place); a block that attends over another block's keys and values gives that one's */
 shainet_kv_cache *shainet_llama_block_cache(shainet_llama_block *block);
+
+/* The kinds of mixers.  BIASED: grouped-query attention without rotation, a learned value by head and distance
+ * (exact distances first, then logarithmic buckets) added to the scores, value heads of a width of their own.
+ * HGRN2: gated linear attention, S <- diag(f) S + (1 - f) v^T and o = S^T q per head, with a state of dim x vdim
+ * floats per head instead of a cache; it can be cleared, not cut short.  Blocks of the last two kinds norm before
+ * and after each sublayer and convolve a sublayer's input over time, whose last rows are part of their state, too. */
+#define SHAINET_HIP_MIXER_GROUPED 0
+#define SHAINET_HIP_MIXER_LATENT 1
+#define SHAINET_HIP_MIXER_BIASED 2
+#define SHAINET_HIP_MIXER_HGRN2 3
+int shainet_llama_block_mixer(shainet_llama_block *block);
+/* An HGRN2 block's state, [heads, dim, vdim], to the host: n = heads * dim * vdim floats; zeros before the first token. */
+int shainet_llama_block_read_state(shainet_llama_block *block, float *out, long long n);
 
 /* ---- the model around the blocks ----------------------------------------------
  *
@@ -461,7 +475,8 @@ int shainet_hf_rope_freqs(const shainet_hf_llama_config *cfg, float *out, int n)
  * to fp32 and transposed to [in, out] there.  The model is ready for shainet_llama_model_run. */
 int shainet_hf_load_llama(const char *model_dir, shainet_llama_model **out);
 /* Any model this library has, by its config.json: a design named under "architecture" ("Tutilorn": latent
- * attention, Dynamic Tanh norms, dense SwiGLU, its layers listed one by one), else shainet_hf_load_llama. */
+ * attention, Dynamic Tanh norms, dense SwiGLU, its layers listed one by one; "Zabutar": HGRN2 and distance-biased
+ * attention layers, norms around the sublayers, short convolutions, xIELU or experts), else shainet_hf_load_llama. */
 int shainet_hf_load_model(const char *model_dir, shainet_llama_model **out);
 
 /* Kernel timing for benchmarks: while enabled, every shainet_attn_forward call

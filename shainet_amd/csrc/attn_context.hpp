@@ -33,8 +33,8 @@ struct PinBuf {
 struct shainet_attn_ctx {
   int H, KV, g, hd;
   // A cache of this context holds, per position and kv head, hd floats in its K array and v_hd in
-  // its V array.  v_hd = hd for grouped-query attention; 0 for latent attention, whose one row per
-  // position (KV = 1; hd = the padded row width) serves as key and as value.
+  // its V array.  v_hd = hd for rotated grouped-query attention; 0 for latent attention, whose one row
+  // per position (KV = 1; hd = the padded row width) serves as key and as value.
   int v_hd;
   // > 0: a query reaches `window` rows back, its own row included, so a cache may forget older ones
   // (shainet_kv_cache_make_room); 0: all the way to position 0.
@@ -104,6 +104,14 @@ struct shainet_kv_cache {
 // rotated dimensions, angles in fp64.
 int shainet_attn_create_rows(shainet_attn_ctx **out, int num_heads, int row_width, int window, double rope_base,
                              int rope_dims, float scale, int max_positions);
+
+// A context for grouped-query attention without rotation, whose values may have a width of their own.
+int shainet_attn_create_unrotated(shainet_attn_ctx **out, int num_heads, int num_kv_heads, int dim, int v_dim, float scale);
+// Attention of new_tokens queries (as DistanceBias lays them out) at positions start_pos .. over sequence 0 of
+// a cache that holds their rows already.  The cache may be another context's of the same kind; its
+// lengths are neither read nor changed.  Asynchronous on c's stream.
+int shainet_attn_run_biased(shainet_attn_ctx *c, shainet_kv_cache *kc, const float *q, const shainet::DistanceBias &bias,
+                            int start_pos, int new_tokens, float *out);
 
 // Room for new_rows more rows of one sequence: drops rows that no later position can see (windowed
 // contexts), else grows the buffers.  keep_back: rows that a later truncate may take back, at most;

@@ -84,12 +84,14 @@ __device__ __forceinline__ void locate_block(const SeqTable &st, int rank, int &
 // tiles are laid out for: query elements beyond it are zeros (whatever stands in for the keys'
 // there does not reach the scores), output elements beyond it are not stored, and a tile's
 // pieces beyond it repeat the row's first piece (a cache hit, no HBM traffic).
-template <int HD, bool SPLIT, int G, bool PAD>
+// BIAS (with PAD): scores gain a value by distance (DistanceBias), value rows have a width of their own.
+template <int HD, bool SPLIT, int G, bool PAD, bool BIAS>
 __device__ __forceinline__ void prefill_block(const int bid, const float *__restrict__ q_rot,
                                               const float *__restrict__ kc, const float *__restrict__ vc,
                                               float *__restrict__ out, float *__restrict__ part_o,
                                               float *__restrict__ part_ml, const SeqTable &st, const Shape &sh,
-                                              int ns, float c) {
+                                              int ns, float c, const DistanceBias &db) {
+  static_assert(PAD || !BIAS, "sizes of their own come with padding");
   constexpr int NK4 = HD / 8;   // float4 pieces of a K row per lane
   constexpr int NT = HD / 32;   // d tiles of the output
   constexpr int KSTR = HD + 4;  // padded K row stride in LDS: conflict-free 16-byte reads down a column
@@ -138,12 +140,16 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
   const int hd = PAD ? uniform(sh.hd) : HD;  // floats between two rows of q, K, V and the output
   const long long head_base = (long long)st.slot[s] * sh.seq_stride + (long long)kvh * sh.cap * hd;
   const float *kbase = kc + head_base;
-  const float *vbase = vc + head_base;
-  const long long qo_off = ((long long)(st.tok_off[s] + row) * sh.H + kvh * g + hg) * hd;
+  const int vhd = BIAS ? uniform(db.v_hd) : hd;
+  const float *vbase = vc + (BIAS ? ((long long)st.slot[s] * sh.KV + kvh) * sh.cap * vhd : head_base);
+  const long long qo_off = ((long long)(st.tok_off[s] + row) * sh.H + kvh * g + hg) * vhd;  // of the row's result
+  const long long q_off = BIAS ? (st.tok_off[s] + row) * db.q_stride + (long long)(kvh * g + hg) * hd : qo_off;
+  // entry of key row k: bias_row[k]
+  const float *bias_row = BIAS ? db.tab + (long long)(kvh * g + hg) * db.stride + (db.origin - lim) : nullptr;
 
   float qr[HD / 2];
   {
-    const float *qp = q_rot + qo_off + 4 * j;
+    const float *qp = q_rot + q_off + 4 * j;
 #pragma unroll
     for (int i = 0; i < NK4; ++i) {
       // (lanes past the last virtual row repeat the last row: their results are never used,
@@ -200,14 +206,15 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
   }
   // NTHREADS is a multiple of HD / 4
   const unsigned col_bytes = PAD && 4 * (threadIdx.x % (HD / 4)) >= (unsigned)hd ? 0u : 16u * (threadIdx.x % (HD / 4));
+  const unsigned v_col_bytes = PAD && 4 * (threadIdx.x % (HD / 4)) >= (unsigned)vhd ? 0u : 16u * (threadIdx.x % (HD / 4));
   static_assert(NTHREADS % (HD / 4) == 0, "a thread keeps its columns");
   // a scalar base and a 32-bit byte offset per lane (a head's rows span less than 4 GiB: checked
   // at launch); rows past the last one repeat it
-  auto load_tiles = [&](f32x4 (&dst)[LD4], const float *base, int sp) {
+  auto load_tiles = [&](f32x4 (&dst)[LD4], const float *base, int sp, int width, unsigned col) {
     const int first_row = (kt0 + G * sp) * 32;
 #pragma unroll
     for (int u = 0; u < LD4; ++u) {
-      const unsigned off = (unsigned)min(first_row + row_in_step[u], L - 1) * (unsigned)(hd * 4) + col_bytes;
+      const unsigned off = (unsigned)min(first_row + row_in_step[u], L - 1) * (unsigned)(width * 4) + col;
       dst[u] = *(const f32x4 *)((const char *)base + off);
     }
   };
@@ -229,8 +236,8 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
       *(f32x4 *)&Vs[buf][ts][r * HD + 4 * c4] = src[u];
     }
   };
-  auto load_k = [&](int sp) { load_tiles(stage_k, kbase, sp); };
-  auto load_v = [&](int sp) { load_tiles(stage_v, vbase, sp); };
+  auto load_k = [&](int sp) { load_tiles(stage_k, kbase, sp, hd, col_bytes); };
+  auto load_v = [&](int sp) { load_tiles(stage_v, vbase, sp, vhd, v_col_bytes); };
   auto store_k = [&](int buf) { park_k(stage_k, buf); };
   auto store_v = [&](int buf) { park_v(stage_v, buf); };
 
@@ -283,10 +290,10 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
     // the tiles that go to LDS right away: one memory round trip before the first MFMA
     // instead of three
     f32x4 k0[LD4], v0[LD4], k1[LD4];
-    load_tiles(k0, kbase, 0);
-    load_tiles(v0, vbase, 0);
+    load_tiles(k0, kbase, 0, hd, col_bytes);
+    load_tiles(v0, vbase, 0, vhd, v_col_bytes);
     if (n_sp > 1) {
-      load_tiles(k1, kbase, 1);
+      load_tiles(k1, kbase, 1, hd, col_bytes);
       load_v(1);
     }
     if (n_sp > 2) load_k(2);
@@ -330,9 +337,26 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
     if (sp + 2 < n_sp) load_v(sp + 2);
     const bool have_next = kt_next < kt1 && kt_next * 32 <= wave_hi;
     const bool have_cur = kt < kt1 && kt * 32 <= wave_hi;
+    // the tile's values by distance are asked for in front of the next tile's MFMAs; a tile that lies
+    // `reach` or more behind all rows of the wavefront has none
+    f32x4 near_bias[BIAS ? 4 : 1];
+    const bool near = BIAS && have_cur && wave_lo - (kt * 32 + 31) < db.reach;
+    if constexpr (BIAS) {
+      if (near) {
+        struct __attribute__((packed, aligned(4))) Four { f32x4 v; };
+#pragma unroll
+        for (int r = 0; r < 4; ++r) near_bias[r] = ((const Four *)(bias_row + kt * 32 + 8 * r + 4 * j))->v;
+      }
+    }
     if (have_next) nxt = scores(buf ^ 1);
     if (have_cur) {
       f32x16 &sacc = cur;            // scores of tile kt minus m_ref, log2 units; not needed after this step
+      if constexpr (BIAS) {
+        if (near) {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) sacc[r] += near_bias[r >> 2][r & 3];
+        }
+      }
       if (kt * 32 + 31 > wave_lo) {  // tile crosses the diagonal for some row of this wavefront
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
@@ -433,7 +457,7 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int d = NT * (8 * (r >> 2) + 4 * j + (r & 3));
-      if (PAD && d >= hd) continue;  // (hd is a multiple of 4 and d of NT = 2 or 4: a store lies inside or outside as a whole)
+      if (PAD && d >= vhd) continue;  // (the width is a multiple of 4 and d of NT = 2 or 4: a store lies inside or outside as a whole)
       if constexpr (NT == 2) {
         *(float2 *)(op + d) = float2{o[0][r] * inv, o[1][r] * inv};
       } else {
@@ -443,15 +467,15 @@ __device__ __forceinline__ void prefill_block(const int bid, const float *__rest
   }
 }
 
-template <int HD, bool SPLIT, int G, bool PAD>
+template <int HD, bool SPLIT, int G, bool PAD, bool BIAS = false>
 __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void prefill_mfma_kernel(const float *__restrict__ q_rot,
                                                               const float *__restrict__ kc,
                                                               const float *__restrict__ vc,
                                                               float *__restrict__ out,
                                                               float *__restrict__ part_o,
                                                               float *__restrict__ part_ml, SeqTable st,
-                                                              Shape sh, int ns, float c) {
-  prefill_block<HD, SPLIT, G, PAD>(blockIdx.x, q_rot, kc, vc, out, part_o, part_ml, st, sh, ns, c);
+                                                              Shape sh, int ns, float c, DistanceBias db) {
+  prefill_block<HD, SPLIT, G, PAD, BIAS>(blockIdx.x, q_rot, kc, vc, out, part_o, part_ml, st, sh, ns, c, db);
 }
 
 // For launches of two or three row blocks per compute unit: a workgroup takes, in turn, block b
@@ -459,18 +483,18 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void prefill_mfma_kernel(c
 // 2N + b (N workgroups): long, short and shorter ones that add up to about the same work for
 // every workgroup, instead of the dispatcher starting another workgroup where one has ended
 // (3.5 us later, measured).
-template <int HD, int G, bool PAD>
+template <int HD, int G, bool PAD, bool BIAS = false>
 __global__ __launch_bounds__(256 * G, 1) void prefill_turns_kernel(const float *__restrict__ q_rot,
                                                                    const float *__restrict__ kc,
                                                                    const float *__restrict__ vc,
                                                                    float *__restrict__ out, SeqTable st, Shape sh,
-                                                                   int n_blocks, float c) {
+                                                                   int n_blocks, float c, DistanceBias db) {
   const int N = gridDim.x, b = blockIdx.x;
   for (int turn = 0; turn < 3; ++turn) {
     const int bid = (turn & 1) ? (turn + 1) * N - 1 - b : turn * N + b;
     if (bid >= n_blocks) continue;
     if (turn) __syncthreads();  // the LDS stages are free: nobody is still merging the last block's halves
-    prefill_block<HD, false, G, PAD>(bid, q_rot, kc, vc, out, nullptr, nullptr, st, sh, 1, c);
+    prefill_block<HD, false, G, PAD, BIAS>(bid, q_rot, kc, vc, out, nullptr, nullptr, st, sh, 1, c, db);
   }
 }
 
@@ -480,12 +504,12 @@ __global__ __launch_bounds__(256 * G, 1) void prefill_turns_kernel(const float *
 __global__ __launch_bounds__(256) void prefill_combine_kernel(const float *__restrict__ part_o,
                                                               const float *__restrict__ part_ml,
                                                               float *__restrict__ out, SeqTable st, Shape sh,
-                                                              int ns, float c, int tile_hd) {
-  // tile_hd: floats per row of a partial (the head dimension the tiles were laid out for)
+                                                              int ns, float c, int tile_hd, int hd) {
+  // hd: floats per row of the result; tile_hd: floats per row of a partial (the head dimension the tiles were laid out for)
   const int kvh = blockIdx.x % sh.KV, item = blockIdx.x / sh.KV;
   int s, vb;
   locate_block(st, item, s, vb);
-  const int g = sh.g, hd = sh.hd, hd4 = hd >> 2;
+  const int g = sh.g, hd4 = hd >> 2;
   const int VR = st.n_new[s] * g;
   const long long base = ((long long)item * sh.KV + kvh) * ns * 128;
   for (int idx = threadIdx.x; idx < 32 * hd4; idx += 256) {
@@ -526,24 +550,25 @@ __global__ __launch_bounds__(256) void prefill_combine_kernel(const float *__res
 }
 
 // ---------------------------------------------------------------------------
-// Any head_dim up to 256: one wavefront per (row, head), lane = key for the
+// Any head_dim: one wavefront per (row, head) and 256 columns of the values (blockIdx.z), lane = key for the
 // scores, lane = d for the output.
 __global__ __launch_bounds__(64) void generic_attn_kernel(const float *__restrict__ q_rot,
                                                           const float *__restrict__ kc,
                                                           const float *__restrict__ vc,
                                                           float *__restrict__ out, SeqTable st, Shape sh,
-                                                          float scale) {
+                                                          float scale, DistanceBias db) {
   extern __shared__ float smem[];
-  const int hd = sh.hd;
+  const int hd = sh.hd, vhd = db.tab ? db.v_hd : hd;
   float *q_s = smem, *p_s = smem + hd;
-  const int token = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+  const int token = blockIdx.x, h = blockIdx.y, lane = threadIdx.x, v0 = blockIdx.z * 256;
   const int s = find_seq(st, token, st.tok_off);
   const int visible = st.start_pos[s] + (token - st.tok_off[s]) + 1;
   const int kvh = h / sh.g;
-  const long long head_base = (long long)st.slot[s] * sh.seq_stride + (long long)kvh * sh.cap * hd;
-  const float *kbase = kc + head_base, *vbase = vc + head_base;
-  const long long qo = ((long long)token * sh.H + h) * hd;
-  for (int d = lane; d < hd; d += 64) q_s[d] = q_rot[qo + d];
+  const long long head_row = ((long long)st.slot[s] * sh.KV + kvh) * sh.cap;
+  const float *kbase = kc + head_row * hd, *vbase = vc + head_row * vhd;
+  const long long qo = ((long long)token * sh.H + h) * vhd;
+  const float *q = q_rot + (db.tab ? token * db.q_stride + (long long)h * hd : qo);
+  for (int d = lane; d < hd; d += 64) q_s[d] = q[d];
   __syncthreads();
   float acc[4] = {0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
@@ -555,6 +580,8 @@ __global__ __launch_bounds__(64) void generic_attn_kernel(const float *__restric
       float dot = 0.f;
       for (int d = 0; d < hd; ++d) dot += q_s[d] * kr[d];
       sv = dot * scale;
+      const int back = visible - 1 - jj;
+      if (db.tab && back < db.reach) sv += db.tab[(long long)h * db.stride + (db.origin - back)] * 0.6931471805599453f;
     }
     float mx = sv;
     for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
@@ -570,10 +597,10 @@ __global__ __launch_bounds__(64) void generic_attn_kernel(const float *__restric
     const int cnt = min(64, visible - j0);
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
-      const int d = lane + 64 * u;
-      if (d < hd) {
+      const int d = v0 + lane + 64 * u;
+      if (d < vhd) {
         float a = acc[u] * alpha;
-        for (int t = 0; t < cnt; ++t) a += p_s[t] * vbase[(long long)(j0 + t) * hd + d];
+        for (int t = 0; t < cnt; ++t) a += p_s[t] * vbase[(long long)(j0 + t) * vhd + d];
         acc[u] = a;
       }
     }
@@ -581,8 +608,8 @@ __global__ __launch_bounds__(64) void generic_attn_kernel(const float *__restric
   }
 #pragma unroll
   for (int u = 0; u < 4; ++u) {
-    const int d = lane + 64 * u;
-    if (d < hd) out[qo + d] = acc[u] / l;
+    const int d = v0 + lane + 64 * u;
+    if (d < vhd) out[qo + d] = acc[u] / l;
   }
 }
 
@@ -616,15 +643,19 @@ int prefill_tile_head_dim(int hd) {
   return hd <= 64 ? 64 : 128;
 }
 
-Path choose_path(const SeqTable &st, const Shape &sh) {
+static int widest(const Shape &sh, int v_hd) { return v_hd > sh.hd ? v_hd : sh.hd; }
+
+Path choose_path(const SeqTable &st, const Shape &sh, int v_hd) {
   // a few new rows per sequence: rows x heads of a group fit the 16 columns of the split-K
   // kernel's MFMA tiles, which then streams K and V once for all of them; up to twice as many
   // rows go to it as two entries (decode_entries), which still beats the key-chunked prefill.
   // Its tiles take any head dimension up to 256 that is a multiple of 4 (padded to 64, 128 or 256).
   SeqTable tmp;
-  if (decode_tile_head_dim(sh.hd) && decode_entries(st, sh, tmp)) return Path::kDecodeSplitK;
+  const bool v_ok = (v_hd & 3) == 0;  // (0 or the width of the value rows)
+  if (v_ok && decode_tile_head_dim(sh.hd) && decode_tile_head_dim(widest(sh, v_hd)) && decode_entries(st, sh, tmp))
+    return Path::kDecodeSplitK;
   // the MFMA prefill kernel's tiles: head dimensions up to 128 (padded to 64 or 128)
-  if (!prefill_tile_head_dim(sh.hd)) return Path::kGeneric;
+  if (!v_ok || !prefill_tile_head_dim(sh.hd) || !prefill_tile_head_dim(widest(sh, v_hd))) return Path::kGeneric;
   return Path::kPrefillMfma;
 }
 
@@ -683,11 +714,11 @@ int prefill_key_splits(const SeqTable &st, const Shape &sh, int items) {
   return ns < 1 ? 1 : ns;
 }
 
-size_t prefill_partial_floats(const Shape &sh, int items, int ns) {
-  return ns > 1 ? (size_t)items * sh.KV * ns * 128 * (prefill_tile_head_dim(sh.hd) + 2) : 0;
+size_t prefill_partial_floats(const Shape &sh, int items, int ns, int v_hd) {
+  return ns > 1 ? (size_t)items * sh.KV * ns * 128 * (prefill_tile_head_dim(widest(sh, v_hd)) + 2) : 0;
 }
 
-PrefillLaunch plan_prefill_launch(const Shape &sh, int items, int ns, int wgs_per_cu, int groups) {
+PrefillLaunch plan_prefill_launch(const Shape &sh, int items, int ns, int wgs_per_cu, int groups, int v_hd) {
   PrefillLaunch p;
   p.n_wgs = (long long)items * sh.KV * ns;
   // With fewer workgroups than three per compute unit everything is resident at
@@ -695,7 +726,7 @@ PrefillLaunch plan_prefill_launch(const Shape &sh, int items, int ns, int wgs_pe
   // two per SIMD (G = 2).  Larger launches already have several workgroups per unit.
   p.groups = groups == 1 || groups == 2 ? groups : (p.n_wgs <= 768 ? 2 : 1);
   // static LDS of the kernel: two stages of `groups` padded K tiles and V tiles
-  const int tile_hd = prefill_tile_head_dim(sh.hd);
+  const int tile_hd = prefill_tile_head_dim(widest(sh, v_hd));
   const size_t static_lds = (size_t)2 * p.groups * (32 * (tile_hd + 4) + 32 * tile_hd) * sizeof(float);
   p.pad = 0;
   // With fewer workgroups than three per compute unit everything is resident at
@@ -721,11 +752,15 @@ PrefillLaunch plan_prefill_launch(const Shape &sh, int items, int ns, int wgs_pe
 
 hipError_t launch_prefill(const float *q_rot, const float *kc, const float *vc, float *out, float *partials,
                           const SeqTable &st, const Shape &sh, int items, int ns, float scale,
-                          hipStream_t stream, int wgs_per_cu, int groups_wanted, hipEvent_t before, hipEvent_t after) {
-  const int tile_hd = prefill_tile_head_dim(sh.hd);
-  if (!table_ok(st, sh) || !tile_hd || items < 1 || ns < 1 || (ns > 1 && !partials)) return hipErrorInvalidValue;
+                          hipStream_t stream, int wgs_per_cu, int groups_wanted, hipEvent_t before, hipEvent_t after,
+                          const DistanceBias *bias) {
+  const DistanceBias db = bias ? *bias : DistanceBias{};
+  const int v_hd = bias ? db.v_hd : sh.hd;
+  const int tile_hd = prefill_tile_head_dim(widest(sh, v_hd));
+  if (bias && (!db.tab || (v_hd & 3) || (db.q_stride & 3) || v_hd < 4 || (long long)sh.cap * v_hd * 4 > 0xffffffffLL)) return hipErrorInvalidValue;
+  if (!table_ok(st, sh) || !tile_hd || !prefill_tile_head_dim(sh.hd) || items < 1 || ns < 1 || (ns > 1 && !partials)) return hipErrorInvalidValue;
   const bool pad = tile_hd != sh.hd;
-  const PrefillLaunch plan = plan_prefill_launch(sh, items, ns, wgs_per_cu, groups_wanted);
+  const PrefillLaunch plan = plan_prefill_launch(sh, items, ns, wgs_per_cu, groups_wanted, v_hd);
   const long long n_wgs = plan.n_wgs;
   if (n_wgs > 0x7fffffffLL) return hipErrorInvalidValue;
   // the kernels address a row of a (sequence, kv head) by a 32-bit byte offset from its first row
@@ -739,16 +774,20 @@ hipError_t launch_prefill(const float *q_rot, const float *kc, const float *vc, 
   if (plan.turns) {
     const int turns = plan.turns;
     dim3 fewer((unsigned)((n_wgs + turns - 1) / turns));
-#define SHAINET_LAUNCH_TURNS(HD_, PAD_)                                                                          \
-  SHAINET_LAUNCH_TIMED((prefill_turns_kernel<HD_, 2, PAD_>), fewer, dim3(512), 0, stream, before, after, q_rot, kc, \
-                       vc, out, st, sh, (int)n_wgs, c)
+#define SHAINET_LAUNCH_TURNS(HD_, ...)                                                                          \
+  SHAINET_LAUNCH_TIMED((prefill_turns_kernel<HD_, 2, __VA_ARGS__>), fewer, dim3(512), 0, stream, before, after, q_rot, kc, \
+                       vc, out, st, sh, (int)n_wgs, c, db)
     if (tile_hd == 64) {
-      if (pad)
+      if (bias)
+        SHAINET_LAUNCH_TURNS(64, true, true);
+      else if (pad)
         SHAINET_LAUNCH_TURNS(64, true);
       else
         SHAINET_LAUNCH_TURNS(64, false);
     } else {
-      if (pad)
+      if (bias)
+        SHAINET_LAUNCH_TURNS(128, true, true);
+      else if (pad)
         SHAINET_LAUNCH_TURNS(128, true);
       else
         SHAINET_LAUNCH_TURNS(128, false);
@@ -757,29 +796,33 @@ hipError_t launch_prefill(const float *q_rot, const float *kc, const float *vc, 
     return hipGetLastError();
   }
   hipEvent_t main_after = ns == 1 ? after : nullptr;  // with key chunks the combine kernel ends the timed stretch
-#define SHAINET_LAUNCH_PREFILL(HD_, SPLIT_, PAD_)                                                              \
+#define SHAINET_LAUNCH_PREFILL(HD_, SPLIT_, ...)                                                               \
   do {                                                                                                          \
     if (groups == 2)                                                                                            \
-      SHAINET_LAUNCH_TIMED((prefill_mfma_kernel<HD_, SPLIT_, 2, PAD_>), grid, dim3(512), lds_pad, stream, before, \
-                           main_after, q_rot, kc, vc, out, part_o, part_ml, st, sh, ns, c);                     \
+      SHAINET_LAUNCH_TIMED((prefill_mfma_kernel<HD_, SPLIT_, 2, __VA_ARGS__>), grid, dim3(512), lds_pad, stream, before, \
+                           main_after, q_rot, kc, vc, out, part_o, part_ml, st, sh, ns, c, db);                     \
     else                                                                                                        \
-      SHAINET_LAUNCH_TIMED((prefill_mfma_kernel<HD_, SPLIT_, 1, PAD_>), grid, dim3(256), lds_pad, stream, before, \
-                           main_after, q_rot, kc, vc, out, part_o, part_ml, st, sh, ns, c);                     \
+      SHAINET_LAUNCH_TIMED((prefill_mfma_kernel<HD_, SPLIT_, 1, __VA_ARGS__>), grid, dim3(256), lds_pad, stream, before, \
+                           main_after, q_rot, kc, vc, out, part_o, part_ml, st, sh, ns, c, db);                     \
   } while (0)
-#define SHAINET_LAUNCH_PREFILL_HD(HD_, PAD_) \
-  do {                                        \
-    if (ns > 1)                               \
-      SHAINET_LAUNCH_PREFILL(HD_, true, PAD_);   \
-    else                                      \
-      SHAINET_LAUNCH_PREFILL(HD_, false, PAD_);  \
+#define SHAINET_LAUNCH_PREFILL_HD(HD_, ...)             \
+  do {                                                  \
+    if (ns > 1)                                         \
+      SHAINET_LAUNCH_PREFILL(HD_, true, __VA_ARGS__);   \
+    else                                                \
+      SHAINET_LAUNCH_PREFILL(HD_, false, __VA_ARGS__);  \
   } while (0)
   if (tile_hd == 64) {
-    if (pad)
+    if (bias)
+      SHAINET_LAUNCH_PREFILL_HD(64, true, true);
+    else if (pad)
       SHAINET_LAUNCH_PREFILL_HD(64, true);
     else
       SHAINET_LAUNCH_PREFILL_HD(64, false);
   } else {
-    if (pad)
+    if (bias)
+      SHAINET_LAUNCH_PREFILL_HD(128, true, true);
+    else if (pad)
       SHAINET_LAUNCH_PREFILL_HD(128, true);
     else
       SHAINET_LAUNCH_PREFILL_HD(128, false);
@@ -790,17 +833,20 @@ hipError_t launch_prefill(const float *q_rot, const float *kc, const float *vc, 
   if (e != hipSuccess || ns == 1) return e;
   hipEvent_t none = nullptr;
   SHAINET_LAUNCH_TIMED(prefill_combine_kernel, dim3((unsigned)(items * sh.KV), 4), dim3(256), 0, stream, none, after,
-                       part_o, part_ml, out, st, sh, ns, 1.0f, tile_hd);  // the partials' maxima are already in log2 units
+                       part_o, part_ml, out, st, sh, ns, 1.0f, tile_hd, v_hd);  // the partials' maxima are already in log2 units
   return hipGetLastError();
 }
 
 hipError_t launch_generic(const float *q_rot, const float *kc, const float *vc, float *out,
                           const SeqTable &st, const Shape &sh, int total_tokens, float scale,
-                          hipStream_t stream) {
-  if (!table_ok(st, sh) || sh.hd < 1 || sh.hd > 256 || total_tokens < 1) return hipErrorInvalidValue;
+                          hipStream_t stream, const DistanceBias *bias) {
+  const DistanceBias db = bias ? *bias : DistanceBias{};
+  const int v_hd = bias ? db.v_hd : sh.hd;
+  if (!table_ok(st, sh) || sh.hd < 1 || sh.hd > 8192 || v_hd < 1 || v_hd > 8192 || total_tokens < 1 || (bias && !db.tab))
+    return hipErrorInvalidValue;
   const size_t smem = (size_t)(sh.hd + 64) * sizeof(float);
-  hipLaunchKernelGGL(generic_attn_kernel, dim3((unsigned)total_tokens, (unsigned)sh.H), dim3(64), smem, stream,
-                     q_rot, kc, vc, out, st, sh, scale);
+  hipLaunchKernelGGL(generic_attn_kernel, dim3((unsigned)total_tokens, (unsigned)sh.H, (unsigned)((v_hd + 255) / 256)), dim3(64),
+                     smem, stream, q_rot, kc, vc, out, st, sh, scale, db);
   return hipGetLastError();
 }
 

@@ -4,6 +4,8 @@
 #include <hip/hip_runtime.h>
 #include <hip/hip_ext.h>
 
+#include "activation.hpp"
+
 // A kernel launch that hands the kernel's own first and last clock reading to two events when
 // there are any (hipExtLaunchKernel), and is a plain launch, as a caller's stream capture may
 // need it, when there are none.
@@ -37,6 +39,20 @@ struct Shape {
   long long seq_stride;  // floats between two sequences' caches = KV*cap*hd
 };
 
+// Attention whose scores gain a value that depends on the query head and on how far back the key lies, and
+// whose value rows need not be as wide as the keys.  The value of head h at distance n is
+// tab[h * stride + origin - n], so that neighbouring keys are neighbours in memory; it is in log2 units and
+// relative to the value of all distances from `reach` on (a softmax does not see what all keys of a
+// row share), which is why far keys cost nothing.  The table holds kDistancePad entries (finite; nobody
+// uses them) before distance 0 and as many zeros from `reach` on.
+constexpr int kDistancePad = 64;
+struct DistanceBias {
+  const float *tab;    // null: no such call
+  int stride, origin, reach;
+  int v_hd;            // floats per value row
+  long long q_stride;  // floats between the queries of two tokens
+};
+
 struct PrepArgs {
   const float *q, *k, *v;           // [tokens, H*hd], [tokens, KV*hd] x2: projection outputs
   long long q_stride, k_stride, v_stride;  // floats between the rows of two tokens (>= the row width)
@@ -57,7 +73,8 @@ hipError_t launch_prep(const PrepArgs &a, const SeqTable &st, const Shape &sh, i
 
 // Which attention kernel a call uses.
 enum class Path { kDecodeSplitK, kPrefillMfma, kGeneric };
-Path choose_path(const SeqTable &st, const Shape &sh);
+// v_hd: floats per value row (0: as many as sh.hd)
+Path choose_path(const SeqTable &st, const Shape &sh, int v_hd = 0);
 // The sequences as the split-K decode kernel takes them: one entry per sequence with up to
 // 16 / g new rows, two entries (the first 16 / g rows, then the rest, which see the first ones
 // as cached) with up to twice as many.  False when some sequence has more or the entries
@@ -104,7 +121,7 @@ inline int device_plan_slots(int n_seqs, int KV) { return kDevicePlanWorkgroups 
 // error: set to 2 when the step is skipped.
 hipError_t launch_decode_plan(int *lens, int n_seqs, const Shape &sh, int rope_positions, DecodeDevicePlan *out,
                               int *error, hipStream_t stream);
-size_t decode_partial_floats(const Shape &sh, const DecodePlan &p);
+size_t decode_partial_floats(const Shape &sh, const DecodePlan &p, int v_hd = 0);
 // The head dimension the split-K decode kernel lays its tiles out for when the data's is hd: 64,
 // 128 or 256, the first that holds hd (a multiple of 4; the rest of a tile is padding that costs
 // no memory traffic); 0 when none does.
@@ -139,12 +156,12 @@ struct DecodeArgs {
 // slots and the columns; everything that depends on the cached lengths is read from *dev.
 hipError_t launch_decode(const DecodeArgs &d, const SeqTable &st, const Shape &sh, const DecodePlan &p, float scale,
                          hipStream_t stream, hipEvent_t before = nullptr, hipEvent_t after = nullptr,
-                         const DecodeDevicePlan *dev = nullptr);
+                         const DecodeDevicePlan *dev = nullptr, const DistanceBias *bias = nullptr);
 // Key splits of a prefill launch: 1 when the row blocks alone fill the chip, more
 // when they do not (few new rows on a long cached prefix); each split leaves
 // partial rows in `partials` (prefill_partial_floats) and a second kernel merges.
 int prefill_key_splits(const SeqTable &st, const Shape &sh, int items);
-size_t prefill_partial_floats(const Shape &sh, int items, int ns);
+size_t prefill_partial_floats(const Shape &sh, int items, int ns, int v_hd = 0);
 // The head dimension the MFMA prefill kernel lays its tiles out for when the data's is hd: 64 or
 // 128, the first that holds hd (a multiple of 4); 0 when neither does.
 int prefill_tile_head_dim(int hd);
@@ -154,7 +171,7 @@ int prefill_tile_head_dim(int hd);
 hipError_t launch_prefill(const float *q_rot, const float *kc, const float *vc, float *out, float *partials,
                           const SeqTable &st, const Shape &sh, int items, int ns, float scale,
                           hipStream_t stream, int wgs_per_cu = 0, int groups = 0, hipEvent_t before = nullptr,
-                          hipEvent_t after = nullptr);
+                          hipEvent_t after = nullptr, const DistanceBias *bias = nullptr);
 // Which instantiation a prefill launch uses and how it is laid out; launch_prefill follows it.
 struct PrefillLaunch {
   long long n_wgs;   // row blocks x kv heads x key chunks
@@ -163,10 +180,10 @@ struct PrefillLaunch {
   int wgs_per_cu;    // 0: as the kernel's registers and LDS allow; 1..3: LDS padded to that occupancy
   size_t pad;        // bytes of dynamic LDS that enforce wgs_per_cu
 };
-PrefillLaunch plan_prefill_launch(const Shape &sh, int items, int ns, int wgs_per_cu, int groups);
+PrefillLaunch plan_prefill_launch(const Shape &sh, int items, int ns, int wgs_per_cu, int groups, int v_hd = 0);
 hipError_t launch_generic(const float *q_rot, const float *kc, const float *vc, float *out,
                           const SeqTable &st, const Shape &sh, int total_tokens, float scale,
-                          hipStream_t stream);
+                          hipStream_t stream, const DistanceBias *bias = nullptr);
 
 // y[T,N] = epilogue(norm(x)[T,K] * W[K,N]), T <= 16, N % 4 == 0: the projections of a
 // decode step with what surrounds them fused in.
@@ -174,7 +191,7 @@ hipError_t launch_generic(const float *q_rot, const float *kc, const float *vc, 
 //   kNormRms      x / sqrt(mean(x^2) + eps) * gamma (gamma null: ones)
 //   kNormDynTanh  tanh(alpha x) * gamma + beta, element by element, no statistics (gamma, beta not null)
 enum { kNormNone = 0, kNormRms = 1, kNormDynTanh = 2 };
-enum { kGemvPlain = 0, kGemvResidual = 1, kGemvSwiglu = 2, kGemvQkvPrep = 3 };
+enum { kGemvPlain = 0, kGemvResidual = 1, kGemvSwiglu = 2, kGemvQkvPrep = 3, kGemvBias = 4 };
 // kGemvQkvPrep: W = W_q | W_k | W_v and the product's rows never go to memory as
 // they are: each head row gets its bias, QK-norm and rotation where it is summed up
 // and lands in q_rot (query heads) or in the cache of one sequence at positions
@@ -184,7 +201,7 @@ struct GemvPrep {
   const float *b_q, *b_k, *b_v;  // nullable
   const float *q_norm, *k_norm;  // nullable, [hd]
   double eps;
-  const float2 *rope_tab;        // [positions][hd/2] (cos, sin)
+  const float2 *rope_tab;        // [positions][hd/2] (cos, sin); null: nothing is rotated
   float *q_rot;                  // [T, H*hd]
   float *kc, *vc;                // the sequence's cache: [KV, cap, hd]
   int H, KV, hd, cap, start_pos;
@@ -199,6 +216,8 @@ struct GemvArgs {
   double eps;
   const float *w;        // [K, N]; kGemvSwiglu: [K, 2N] = gate_proj | up_proj
   const float *res;      // kGemvResidual: [T, N], y = res + x W
+  const float *bias;     // kGemvBias: [N], y = act(x W + bias)
+  Activation act;
   float *y;              // [T, N]; kGemvSwiglu: silu(x W_gate) * (x W_up)
   float *partials;       // GemvPlan::partial_floats floats when the plan has splits > 1
   unsigned *flags;       // GemvPlan::col_tiles * splits words, zero when allocated; left zero
@@ -234,6 +253,11 @@ hipError_t launch_gemvt(const GemvArgs &a, hipStream_t stream);
 int *alloc_error_word();
 void free_error_word(int *w);
 int check_error_word(int *w);
+
+// The key and value parts of T rows (k_off, v_off floats into rows `stride` floats apart) into the cache of one
+// sequence, kc [KV, cap, dim] and vc [KV, cap, v_dim], as they are, at positions start_pos ..
+hipError_t launch_append_rows(const float *rows, long long stride, long long k_off, long long v_off, int T, float *kc, float *vc,
+                              int KV, int dim, int v_dim, int cap, int start_pos, hipStream_t stream);
 
 hipError_t launch_legacy_append(const float *staging, float *kc, float *vc, int new_tokens, int start_pos,
                                 int num_kv_heads, int head_dim, int capacity, hipStream_t stream);

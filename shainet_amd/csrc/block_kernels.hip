@@ -103,10 +103,12 @@ __global__ __launch_bounds__(256) void swiglu_act_kernel(const float *__restrict
 }
 
 __global__ __launch_bounds__(256) void embed_kernel(const float *__restrict__ table, const int *__restrict__ tokens,
-                                                    float *__restrict__ out, int d_model, float scale) {
+                                                    float *__restrict__ out, int d_model, float scale,
+                                                    const float *__restrict__ positions) {
   const float *src = table + (long long)tokens[blockIdx.x] * d_model;
   float *dst = out + (long long)blockIdx.x * d_model;
-  for (int j = threadIdx.x; j < d_model; j += 256) dst[j] = src[j] * scale;
+  const float *pos = positions + (positions ? (long long)blockIdx.x * d_model : 0);
+  for (int j = threadIdx.x; j < d_model; j += 256) dst[j] = positions ? src[j] * scale + pos[j] : src[j] * scale;
 }
 
 // Dynamic Tanh: no statistics over the row, so a workgroup takes 1024 columns of one row.
@@ -368,7 +370,8 @@ hipError_t launch_dyn_tanh(const float *x, long long x_stride, const float *gamm
 hipError_t launch_gather_rows(const float *x, const int *rows, float *out, int n, int cols, hipStream_t stream) {
   if (!x || !rows || !out || n < 1 || cols < 1) return hipErrorInvalidValue;
   // (a row gather is what the embedding lookup is)
-  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n), dim3(256), 0, stream, x, rows, out, cols, 1.f);
+  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n), dim3(256), 0, stream, x, rows, out, cols, 1.f,
+                     (const float *)nullptr);
   return hipGetLastError();
 }
 
@@ -388,9 +391,10 @@ hipError_t launch_swiglu_act(const float *gate_up, float *hidden, int rows, int 
 }
 
 hipError_t launch_embed(const float *table, const int *tokens, float *out, int n_tokens, int d_model,
-                        hipStream_t stream, float scale) {
+                        hipStream_t stream, float scale, const float *positions) {
   if (n_tokens < 1 || d_model < 1) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n_tokens), dim3(256), 0, stream, table, tokens, out, d_model, scale);
+  hipLaunchKernelGGL(embed_kernel, dim3((unsigned)n_tokens), dim3(256), 0, stream, table, tokens, out, d_model, scale,
+                     positions);
   return hipGetLastError();
 }
 

@@ -23,9 +23,9 @@ hipError_t launch_transposed_differ(const float *a, const float *b, int rows, in
 hipError_t launch_add(const float *a, const float *b, float *out, long long n, hipStream_t stream);
 // hidden[r, j] = silu(gate_up[r, j]) * gate_up[r, ff + j];  gate_up is [rows, 2*ff]
 hipError_t launch_swiglu_act(const float *gate_up, float *hidden, int rows, int ff, hipStream_t stream);
-// out[t, :] = table[tokens[t], :] * scale;  the caller has checked 0 <= tokens[t] < vocab
+// out[t, :] = table[tokens[t], :] * scale (+ positions[t, :]);  the caller has checked 0 <= tokens[t] < vocab
 hipError_t launch_embed(const float *table, const int *tokens, float *out, int n_tokens, int d_model,
-                        hipStream_t stream, float scale = 1.f);
+                        hipStream_t stream, float scale = 1.f, const float *positions = nullptr);
 // out[i, :] = x[rows[i], :], n rows of `cols` floats
 hipError_t launch_gather_rows(const float *x, const int *rows, float *out, int n, int cols, hipStream_t stream);
 // logits[j] += bias[j]

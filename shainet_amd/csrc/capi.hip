@@ -246,15 +246,16 @@ struct Workspace {
 // ws != nullptr: nothing is allocated; the split-K decode path only.
 int run_attention(shainet_attn_ctx *c, const float *q_rot, float *kc, float *vc, float *out, SeqTable &st,
                   const Shape &sh, int total_tokens, float scale, hipStream_t stream, const PrepArgs *prep,
-                  const Workspace *ws = nullptr) {
-  const Path path = choose_path(st, sh);
+                  const Workspace *ws = nullptr, const DistanceBias *bias = nullptr) {
+  const int v_hd = bias ? bias->v_hd : sh.hd;
+  const Path path = choose_path(st, sh, v_hd);
   if (ws && path != Path::kDecodeSplitK)
     return fail(SHAINET_HIP_ERR_ARGUMENT,
                 "the entry point that allocates nothing takes decode calls only: at most %d new rows per sequence "
                 "with this head geometry (head_dim a multiple of 4 up to 256)", 32 / (sh.g < 1 ? 1 : sh.g));
   // the MFMA prefill kernels address the rows of a (sequence, kv head) by a 32-bit byte offset;
   // said before anything is written to the cache
-  if (path == Path::kPrefillMfma && (long long)sh.cap * sh.hd * 4 > 0xffffffffLL)
+  if (path == Path::kPrefillMfma && (long long)sh.cap * (v_hd > sh.hd ? v_hd : sh.hd) * 4 > 0xffffffffLL)
     return fail(SHAINET_HIP_ERR_ARGUMENT,
                 "capacity %d x head_dim %d x 4 bytes is 4 GiB or more: not supported for more than 16/g new rows",
                 sh.cap, sh.hd);
@@ -281,7 +282,7 @@ int run_attention(shainet_attn_ctx *c, const float *q_rot, float *kc, float *vc,
       d.part_flag = ws->flags;
       d.flag_set = c->test_lose_marks ? ws->lost_marks : nullptr;
     } else {
-      int rc = c->partials.reserve(decode_partial_floats(sh, plan));
+      int rc = c->partials.reserve(decode_partial_floats(sh, plan, v_hd));
       if (!rc) rc = ensure_decode_flags(c, decode_flag_words(plan), stream);
       if (rc) return rc;
       d.partials = c->partials.p;
@@ -305,7 +306,7 @@ int run_attention(shainet_attn_ctx *c, const float *q_rot, float *kc, float *vc,
       e = launch_prep(*prep, st, sh, total_tokens, stream);
       if (e != hipSuccess) return hip_fail(e, "prep launch");
     }
-    e = launch_decode(d, att, sh, plan, scale, stream, ev0, ev1);
+    e = launch_decode(d, att, sh, plan, scale, stream, ev0, ev1, nullptr, bias);
   } else {
     if (prep) {
       e = launch_prep(*prep, st, sh, total_tokens, stream);
@@ -314,14 +315,14 @@ int run_attention(shainet_attn_ctx *c, const float *q_rot, float *kc, float *vc,
     if (path == Path::kPrefillMfma) {
       const int items = plan_work(st, sh, path);
       int ns = c->prefill_splits_override > 0 ? c->prefill_splits_override : prefill_key_splits(st, sh, items);
-      int rc = c->partials.reserve(prefill_partial_floats(sh, items, ns));
+      int rc = c->partials.reserve(prefill_partial_floats(sh, items, ns, v_hd));
       if (rc) return rc;
       e = launch_prefill(q_rot, kc, vc, out, c->partials.p, st, sh, items, ns, scale, stream,
-                         c->prefill_wgs_per_cu, c->prefill_groups_override, ev0, ev1);
+                         c->prefill_wgs_per_cu, c->prefill_groups_override, ev0, ev1, bias);
     } else {
       plan_work(st, sh, path);
       if (ev0) (void)hipEventRecord(ev0, stream);
-      e = launch_generic(q_rot, kc, vc, out, st, sh, total_tokens, scale, stream);
+      e = launch_generic(q_rot, kc, vc, out, st, sh, total_tokens, scale, stream, bias);
       if (ev1) (void)hipEventRecord(ev1, stream);
     }
   }
@@ -459,19 +460,21 @@ int shainet_attn_create(shainet_attn_ctx **out, int num_heads, int num_kv_heads,
 
 }  // extern "C"
 
-int shainet_attn_create_rows(shainet_attn_ctx **out, int num_heads, int row_width, int window, double rope_base,
-                             int rope_dims, float scale, int max_positions) {
+static int create_sized(shainet_attn_ctx **out, int num_heads, int num_kv_heads, int k_width, int v_width, int window,
+                        double rope_base, int rope_dims, float scale, int max_positions) {
   *out = nullptr;
   if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
   shainet_attn_ctx *c = new (std::nothrow) shainet_attn_ctx();
   if (!c) return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
-  c->H = c->g = num_heads;
-  c->KV = 1;
-  c->hd = row_width;
-  c->v_hd = 0;
+  c->H = num_heads;
+  c->KV = num_kv_heads;
+  c->g = num_heads / num_kv_heads;
+  c->hd = k_width;
+  c->v_hd = v_width;
   c->window = window;
   c->rope_fp64 = true;
   c->scale = scale;
+  c->test_lose_marks = getenv("SHAINET_HIP_TEST_LOSE_PARTIAL_MARKS") != nullptr;
   c->inv_freq64.resize(rope_dims / 2);
   c->inv_freq.resize(rope_dims / 2);
   for (int i = 0; i < rope_dims / 2; ++i) {
@@ -491,6 +494,31 @@ int shainet_attn_create_rows(shainet_attn_ctx **out, int num_heads, int row_widt
   }
   *out = c;
   return SHAINET_HIP_OK;
+}
+
+int shainet_attn_create_rows(shainet_attn_ctx **out, int num_heads, int row_width, int window, double rope_base,
+                             int rope_dims, float scale, int max_positions) {
+  return create_sized(out, num_heads, 1, row_width, 0, window, rope_base, rope_dims, scale, max_positions);
+}
+
+int shainet_attn_create_unrotated(shainet_attn_ctx **out, int num_heads, int num_kv_heads, int dim, int v_dim, float scale) {
+  return create_sized(out, num_heads, num_kv_heads, dim, v_dim, 0, 1.0, 0, scale, 1);
+}
+
+int shainet_attn_run_biased(shainet_attn_ctx *c, shainet_kv_cache *kc, const float *q, const DistanceBias &bias, int start_pos,
+                            int new_tokens, float *out) {
+  if (!c || !kc || !q || !out || kc->ctx->KV != c->KV || kc->ctx->hd != c->hd || kc->ctx->v_hd != c->v_hd || bias.v_hd != c->v_hd)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "context and cache do not belong together");
+  if (start_pos < 0 || new_tokens < 1 || (long long)start_pos + new_tokens > kc->cap)
+    return fail(SHAINET_HIP_ERR_CAPACITY, "%d cached + %d new rows exceed capacity %d", start_pos, new_tokens, kc->cap);
+  SeqTable st;
+  memset(&st, 0, sizeof st);
+  st.n_seqs = 1;
+  st.start_pos[0] = start_pos;
+  st.n_new[0] = new_tokens;
+  st.tok_off[1] = new_tokens;
+  Shape sh = shape_of(c, kc->cap);
+  return run_attention(c, q, kc->k, kc->v, out, st, sh, new_tokens, c->scale, c->stream, nullptr, nullptr, &bias);
 }
 
 extern "C" {
@@ -565,15 +593,16 @@ int shainet_kv_cache_create(shainet_kv_cache **out, shainet_attn_ctx *ctx, int b
   kc->cap = capacity;
   kc->len.assign(batch, 0);
   kc->base.assign(batch, 0);
-  const size_t bytes = (size_t)batch * ctx->KV * capacity * ctx->hd * sizeof(float);
+  const size_t rows = (size_t)batch * ctx->KV * capacity;
+  const size_t bytes = rows * ctx->hd * sizeof(float), v_bytes = rows * ctx->v_hd * sizeof(float);
   const bool has_v = ctx->v_hd > 0;
   hipError_t e = hipMalloc((void **)&kc->k, bytes);
-  if (e == hipSuccess && has_v) e = hipMalloc((void **)&kc->v, bytes);
+  if (e == hipSuccess && has_v) e = hipMalloc((void **)&kc->v, v_bytes);
   // zero-fill: rows never appended must hold finite values.  On the context's stream and
   // waited for: a fill on the null stream is not ordered with the kernels that append rows
   // (the stream is non-blocking) and could wipe rows written right after this call.
   if (e == hipSuccess) e = hipMemsetAsync(kc->k, 0, bytes, ctx->stream);
-  if (e == hipSuccess && has_v) e = hipMemsetAsync(kc->v, 0, bytes, ctx->stream);
+  if (e == hipSuccess && has_v) e = hipMemsetAsync(kc->v, 0, v_bytes, ctx->stream);
   if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
   if (e != hipSuccess) {
     int rc = hip_fail(e, "kv cache allocation");
@@ -640,20 +669,20 @@ int shainet_kv_cache_reserve(shainet_kv_cache *kc, int capacity) {
   if (capacity <= kc->cap) return SHAINET_HIP_OK;
   if (int rc = refuse_while_lengths_on_device(kc, "shainet_kv_cache_reserve")) return rc;  // growth copies len rows
   shainet_attn_ctx *c = kc->ctx;
-  const size_t row = (size_t)c->hd * sizeof(float);
-  const size_t bytes = (size_t)kc->batch * c->KV * capacity * row;
+  const size_t row = (size_t)c->hd * sizeof(float), v_row = (size_t)c->v_hd * sizeof(float);
+  const size_t bytes = (size_t)kc->batch * c->KV * capacity * row, v_bytes = (size_t)kc->batch * c->KV * capacity * v_row;
   float *nk = nullptr, *nv = nullptr;
   const bool has_v = c->v_hd > 0;
   hipError_t e = hipMalloc((void **)&nk, bytes);
-  if (e == hipSuccess && has_v) e = hipMalloc((void **)&nv, bytes);
+  if (e == hipSuccess && has_v) e = hipMalloc((void **)&nv, v_bytes);
   if (e == hipSuccess) e = hipMemsetAsync(nk, 0, bytes, c->stream);
-  if (e == hipSuccess && has_v) e = hipMemsetAsync(nv, 0, bytes, c->stream);
+  if (e == hipSuccess && has_v) e = hipMemsetAsync(nv, 0, v_bytes, c->stream);
   // one strided copy per tensor: [batch*KV] runs of cap rows into runs of capacity rows
   if (e == hipSuccess)
     e = hipMemcpy2DAsync(nk, (size_t)capacity * row, kc->k, (size_t)kc->cap * row, (size_t)kc->cap * row,
                          (size_t)kc->batch * c->KV, hipMemcpyDeviceToDevice, c->stream);
   if (e == hipSuccess && has_v)
-    e = hipMemcpy2DAsync(nv, (size_t)capacity * row, kc->v, (size_t)kc->cap * row, (size_t)kc->cap * row,
+    e = hipMemcpy2DAsync(nv, (size_t)capacity * v_row, kc->v, (size_t)kc->cap * v_row, (size_t)kc->cap * v_row,
                          (size_t)kc->batch * c->KV, hipMemcpyDeviceToDevice, c->stream);
   if (e == hipSuccess) e = hipStreamSynchronize(c->stream);
   if (e != hipSuccess) {
@@ -675,15 +704,15 @@ int shainet_kv_cache_fill(shainet_kv_cache *kc, int seq, const float *k_rows, co
   if (int rc = refuse_while_lengths_on_device(kc, "shainet_kv_cache_fill")) return rc;
   if (n > kc->cap) return fail(SHAINET_HIP_ERR_CAPACITY, "fill of %d rows exceeds capacity %d", n, kc->cap);
   shainet_attn_ctx *c = kc->ctx;
-  const size_t row = (size_t)c->hd * sizeof(float);
+  const size_t row = (size_t)c->hd * sizeof(float), v_row = (size_t)c->v_hd * sizeof(float);
   const hipMemcpyKind kind = mem == SHAINET_HIP_MEM_HOST ? hipMemcpyHostToDevice : hipMemcpyDeviceToDevice;
   if (n > 0) {
     float *dk = kc->k + (size_t)seq * c->KV * kc->cap * c->hd;
     HIP_TRY(hipMemcpy2DAsync(dk, (size_t)kc->cap * row, k_rows, (size_t)n * row, (size_t)n * row, c->KV, kind,
                              c->stream));
     if (kc->v)
-      HIP_TRY(hipMemcpy2DAsync(kc->v + (size_t)seq * c->KV * kc->cap * c->hd, (size_t)kc->cap * row, v_rows,
-                               (size_t)n * row, (size_t)n * row, c->KV, kind, c->stream));
+      HIP_TRY(hipMemcpy2DAsync(kc->v + (size_t)seq * c->KV * kc->cap * c->v_hd, (size_t)kc->cap * v_row, v_rows,
+                               (size_t)n * v_row, (size_t)n * v_row, c->KV, kind, c->stream));
     HIP_TRY(hipStreamSynchronize(c->stream));
   }
   kc->len[seq] = n;
@@ -696,10 +725,10 @@ int shainet_kv_cache_read(shainet_kv_cache *kc, int seq, int kv_head, int pos0, 
       pos0 - kc->base[seq] + n > kc->cap || (v_out && !kc->v))
     return fail(SHAINET_HIP_ERR_ARGUMENT, "invalid read arguments");
   shainet_attn_ctx *c = kc->ctx;
-  const size_t off = (((size_t)seq * c->KV + kv_head) * kc->cap + (pos0 - kc->base[seq])) * c->hd;
+  const size_t first = ((size_t)seq * c->KV + kv_head) * kc->cap + (pos0 - kc->base[seq]);
   HIP_TRY(hipStreamSynchronize(c->stream));
-  if (k_out && n) HIP_TRY(hipMemcpy(k_out, kc->k + off, (size_t)n * c->hd * sizeof(float), hipMemcpyDeviceToHost));
-  if (v_out && n) HIP_TRY(hipMemcpy(v_out, kc->v + off, (size_t)n * c->hd * sizeof(float), hipMemcpyDeviceToHost));
+  if (k_out && n) HIP_TRY(hipMemcpy(k_out, kc->k + first * c->hd, (size_t)n * c->hd * sizeof(float), hipMemcpyDeviceToHost));
+  if (v_out && n) HIP_TRY(hipMemcpy(v_out, kc->v + first * c->v_hd, (size_t)n * c->v_hd * sizeof(float), hipMemcpyDeviceToHost));
   return SHAINET_HIP_OK;
 }
 
@@ -725,13 +754,13 @@ int shainet_kv_cache_make_room(shainet_kv_cache *kc, int seq, int new_rows, int 
   }
   // the rows that stay move to the front; through a buffer of their own where the ranges overlap
   const int drop = held - keep;
-  const size_t row_floats = (size_t)c->hd, bytes = (size_t)keep * row_floats * sizeof(float);
   if (keep > drop)
-    if (int rc = c->in_k.reserve((size_t)keep * row_floats)) return rc;
+    if (int rc = c->in_k.reserve((size_t)keep * (c->v_hd > c->hd ? c->v_hd : c->hd))) return rc;
   for (float *p : {kc->k, kc->v}) {
+    const size_t row_floats = (size_t)(p == kc->k ? c->hd : c->v_hd), bytes = (size_t)keep * row_floats * sizeof(float);
     for (int h = 0; p && h < c->KV && keep > 0; ++h) {
-      float *first = p + ((size_t)seq * c->KV + h) * kc->cap * c->hd;
-      const float *from = first + (size_t)drop * c->hd;
+      float *first = p + ((size_t)seq * c->KV + h) * kc->cap * row_floats;
+      const float *from = first + (size_t)drop * row_floats;
       if (keep > drop) {
         HIP_TRY(hipMemcpyAsync(c->in_k.p, from, bytes, hipMemcpyDeviceToDevice, c->stream));
         from = c->in_k.p;

@@ -107,7 +107,7 @@ __device__ __forceinline__ void issue_k_tile(const float *kbase, int kb, int las
   }
 }
 
-template <int HD, bool PAD>
+template <int HD, bool PAD>  // hd: floats per row of V
 __device__ __forceinline__ void load_v_tile(const float *vbase, int kb, int last_row, int col, int j,
                                             f32x4 (&v)[4][DecodeCfg<HD>::NVU], int hd) {
 #pragma unroll
@@ -157,7 +157,7 @@ __device__ __forceinline__ int segment_rotation(int n_tiles, unsigned rotate) {
 
 // The segment that starts at tile t of the stream; s: a sequence at or before t's, moved up to it.
 __device__ __forceinline__ Segment segment_at(int t, int t_end, int &s, const SeqTable &st, const Shape &sh, int hd,
-                                              const float *kc, const float *vc, unsigned rotate) {
+                                              int vhd, bool own_v_rows, const float *kc, const float *vc, unsigned rotate) {
   while (s + 1 < st.n_seqs && t >= st.work_off[s + 1]) ++s;
   Segment g;
   g.s = s;
@@ -171,7 +171,7 @@ __device__ __forceinline__ Segment segment_at(int t, int t_end, int &s, const Se
   g.rot = __builtin_amdgcn_readfirstlane(segment_rotation(g.tile1 - g.tile0, rotate));
   const long long head_base = (long long)st.slot[s] * sh.seq_stride + (long long)g.kvh * sh.cap * hd;
   g.kbase = kc + head_base;
-  g.vbase = vc + head_base;
+  g.vbase = vc + (own_v_rows ? ((long long)st.slot[s] * sh.KV + g.kvh) * sh.cap * vhd : head_base);
   g.token = st.tok_off[s];
   return g;
 }
@@ -193,12 +193,15 @@ struct ReadAhead {
 // reads the rows 4 j .. 4 j + 3 and n + the same of ah.w with ordinary loads and drops them, so
 // that the launch that needs them next finds them in its XCD's L2 (a decode step of one sequence
 // leaves the memory system idle while it waits on its chain of dependent loads).
-template <int HD, int NW, bool DEV, bool PAD, bool AHEAD = false>
+// BIAS (with PAD): scores gain a value by distance (DistanceBias), value rows have a width of their own.
+template <int HD, int NW, bool DEV, bool PAD, bool AHEAD = false, bool BIAS = false>
 __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_splitk_kernel(
     const float *__restrict__ q_rot, const float *__restrict__ kc, const float *__restrict__ vc,
     float *__restrict__ out, float *part_o, float *part_ml, unsigned *part_flag, unsigned *flag_set,
     int spin_limit, int *error, SeqTable st_arg, Shape sh, int tiles_per_wg_arg, SpanTable sp_arg, int total_tiles_arg,
-    int n_slots, int pstride, float c, unsigned rotate, const DecodeDevicePlan *__restrict__ dev, ReadAhead ah) {
+    int n_slots, int pstride, float c, unsigned rotate, const DecodeDevicePlan *__restrict__ dev, ReadAhead ah,
+    DistanceBias db) {
+  static_assert(PAD || !BIAS, "sizes of their own come with padding");
   if constexpr (AHEAD) {
     if ((int)blockIdx.x >= ah.first_wg) {
       const int row = 4 * ((int)blockIdx.x - ah.first_wg) + (int)(threadIdx.x >> 6);
@@ -236,6 +239,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
   const int col = lane & 15, j = lane >> 4;
   const int g = sh.g;
   const int hd = PAD ? sh.hd : HD;  // floats between two rows of q, K, V and the output
+  const int vhd = BIAS ? db.v_hd : hd;  // of V and the output
+  const float ce = BIAS ? 1.f : c;      // scores with a bias are kept in log2 units
   const int t_begin = span_begin(blockIdx.x, tiles_per_wg, sp);
   const int t_end = min(total_tiles, span_begin(blockIdx.x + 1, tiles_per_wg, sp));
   if (t_begin >= t_end) return;  // unequal spans can leave the last workgroup without tiles
@@ -246,7 +251,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
   // along them with dependent scalar loads took 2.5 us for a workgroup in the middle of 16
   // sequences).
   int s = (int)__popcll(__ballot(lane + 1 < st.n_seqs && t_begin >= st.work_off[lane + 1 < kMaxSeqs ? lane + 1 : kMaxSeqs]));
-  Segment seg = segment_at(t, t_end, s, st, sh, hd, kc, vc, rotate);
+  Segment seg = segment_at(t, t_end, s, st, sh, hd, vhd, BIAS, kc, vc, rotate);
 
   f32x4 v_next[4][C::NVU];
   float qr[HD / 4];
@@ -255,7 +260,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
   // MFMA column c of a segment is new row c / g, head c % g of the group (R * g <= 16 columns)
   auto load_q = [&](const Segment &sg) {
     const int cq = col < sg.R * g ? col : 0, row = cq / g;
-    const float *qp = q_rot + ((long long)(sg.token + row) * sh.H + sg.kvh * g + (cq - row * g)) * hd + 4 * j;
+    const int head = sg.kvh * g + (cq - row * g);
+    const float *qp = q_rot + (BIAS ? (sg.token + row) * db.q_stride + (long long)head * hd : ((long long)(sg.token + row) * sh.H + head) * hd) + 4 * j;
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
       f32x4 x = {0.f, 0.f, 0.f, 0.f};
@@ -282,7 +288,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
   // start fetching the tile at key row `row` into buffer `which`
   auto fetch = [&](int which, const float *kb_, const float *vb_, int row, int last_row) {
     issue_k_tile<HD, PAD>(kb_, row, last_row, my_lds + which * C::TILE_BYTES, lane, hd);
-    load_v_tile<HD, PAD>(vb_, row, last_row, col, j, v_next, hd);
+    load_v_tile<HD, PAD>(vb_, row, last_row, col, j, v_next, vhd);
   };
   if (first_place(t) < seg.tile1 - seg.tile0) fetch(0, seg.kbase, seg.vbase, tile_at(seg, first_place(t)) * 16, seg.L - 1);
   load_q(seg);
@@ -307,11 +313,17 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
     const float *kbase = seg.kbase, *vbase = seg.vbase;
     const int nc = seg.R * g;                                   // columns in use
     const int Lc = L - (seg.R - 1 - (col < nc ? col : 0) / g);  // keys visible to this lane's column
+    // entry of key row k: bias_row[k]
+    const float *bias_row = nullptr;
+    if constexpr (BIAS) {
+      const int cq = col < nc ? col : 0;
+      bias_row = db.tab + (long long)(seg.kvh * g + cq % g) * db.stride + (db.origin - (Lc - 1));
+    }
     // the segment after this one, if the span has one
     const int t_next = t + (tile1 - seg.tile0);
     const bool more = t_next < t_end;
     Segment nseg = seg;
-    if (more) nseg = segment_at(t_next, t_end, s, st, sh, hd, kc, vc, rotate);
+    if (more) nseg = segment_at(t_next, t_end, s, st, sh, hd, vhd, BIAS, kc, vc, rotate);
     const int nplace = first_place(t_next);
     const bool nhave = more && nplace < nseg.tile1 - nseg.tile0;
     const int ntile = nhave ? tile_at(nseg, nplace) : 0;
@@ -340,6 +352,12 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
       for (int r = 0; r < 4; ++r)
 #pragma unroll
         for (int u = 0; u < C::NVU; ++u) v_cur[r][u] = v_next[r][u];
+      // a tile that lies `reach` or more behind every column's row has no values by distance
+      f32x4 near_bias = {0.f, 0.f, 0.f, 0.f};
+      if constexpr (BIAS) {
+        struct __attribute__((packed, aligned(4))) Four { f32x4 v; };
+        if (L - seg.R - (kb + 15) < db.reach) near_bias = ((const Four *)(bias_row + kb + 4 * j))->v;
+      }
       if (place + NW < n_here)
         fetch(par, kbase, vbase, tile_at(seg, place + NW) * 16, L - 1);
       else if (nhave)
@@ -357,17 +375,18 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
       }
       float sv[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) sv[r] = (kb + 4 * j + r < Lc) ? s0[r] + s1[r] : -INFINITY;
+      for (int r = 0; r < 4; ++r)
+        sv[r] = (kb + 4 * j + r < Lc) ? (BIAS ? (s0[r] + s1[r]) * c + near_bias[r] : s0[r] + s1[r]) : -INFINITY;
       float mx = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
       mx = fmaxf(mx, __shfl_xor(mx, 16));
       mx = fmaxf(mx, __shfl_xor(mx, 32));
       const float mnew = fmaxf(m, mx);
       // with several new rows a column may not see any key of a late tile (-inf so far: 0 stands in)
       const float mref = mnew == -INFINITY ? 0.f : mnew;
-      const float alpha = fast_exp2((m - mref) * c);
+      const float alpha = fast_exp2((m - mref) * ce);
       float p[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) p[r] = fast_exp2((sv[r] - mref) * c);
+      for (int r = 0; r < 4; ++r) p[r] = fast_exp2((sv[r] - mref) * ce);
       l = l * alpha + ((p[0] + p[1]) + (p[2] + p[3]));
       m = mnew;
 #pragma unroll
@@ -423,13 +442,13 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
       float acc = 0.f, ls = 0.f;
 #pragma unroll
       for (int w = 0; w < NW; ++w) {
-        const float f = fast_exp2((sm_m[w][cc] - mref) * c);  // 0 for a wavefront that saw no visible key
+        const float f = fast_exp2((sm_m[w][cc] - mref) * ce);  // 0 for a wavefront that saw no visible key
         acc += f * sm_o[park[w] + cc * HD + d];
         ls += f * sm_l[w][cc];
       }
       if (whole_pair) {
         const int row = cc / g;
-        if (!PAD || d < hd) out[((long long)(seg.token + row) * sh.H + seg.kvh * g + (cc - row * g)) * hd + d] = acc / ls;
+        if (!PAD || d < vhd) out[((long long)(seg.token + row) * sh.H + seg.kvh * g + (cc - row * g)) * vhd + d] = acc / ls;
       } else if (slot < n_slots) {
         const long long pi = (long long)slot * pstride + cc;
         coherent_store(&part_o[pi * HD + d], acc);
@@ -527,7 +546,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
 #pragma unroll
         for (int u = 0; u < 8; ++u) {
           const int i = i0 + u * GROUPS + grp;
-          const float w = i < n_part ? fast_exp2((f[u] - mm) * c) : 0.f;
+          const float w = i < n_part ? fast_exp2((f[u] - mm) * ce) : 0.f;
           acc += w * x[u];
           ls += w * lp[u];
         }
@@ -540,10 +559,10 @@ __global__ __launch_bounds__(64 * NW, NW == 4 && HD <= 128 ? 2 : 1) void decode_
         acc.w += __shfl_xor(acc.w, o2);
         ls += __shfl_xor(ls, o2);
       }
-      if (grp == 0 && (!PAD || 4 * d4 < hd)) {
+      if (grp == 0 && (!PAD || 4 * d4 < vhd)) {
         const float inv = 1.0f / ls;
         const int row = cc / g;
-        *(f32x4 *)&out[((long long)(mseg.token + row) * sh.H + mseg.kvh * g + (cc - row * g)) * hd + 4 * d4] = acc * inv;
+        *(f32x4 *)&out[((long long)(mseg.token + row) * sh.H + mseg.kvh * g + (cc - row * g)) * vhd + 4 * d4] = acc * inv;
       }
     }
   }
@@ -679,8 +698,8 @@ int decode_tile_head_dim(int hd) {
   return hd <= 64 ? 64 : hd <= 128 ? 128 : 256;
 }
 
-size_t decode_partial_floats(const Shape &sh, const DecodePlan &p) {
-  return (size_t)p.n_slots * p.cols * (decode_tile_head_dim(sh.hd) + 2);
+size_t decode_partial_floats(const Shape &sh, const DecodePlan &p, int v_hd) {
+  return (size_t)p.n_slots * p.cols * (decode_tile_head_dim(v_hd > sh.hd ? v_hd : sh.hd) + 2);
 }
 
 hipError_t launch_decode_plan(int *lens, int n_seqs, const Shape &sh, int rope_positions, DecodeDevicePlan *out,
@@ -694,7 +713,9 @@ hipError_t launch_decode_plan(int *lens, int n_seqs, const Shape &sh, int rope_p
 }
 
 hipError_t launch_decode(const DecodeArgs &d, const SeqTable &st, const Shape &sh, const DecodePlan &p, float scale,
-                         hipStream_t stream, hipEvent_t before, hipEvent_t after, const DecodeDevicePlan *dev) {
+                         hipStream_t stream, hipEvent_t before, hipEvent_t after, const DecodeDevicePlan *dev,
+                         const DistanceBias *bias) {
+  const DistanceBias db = bias ? *bias : DistanceBias{};
   if (st.n_seqs < 1 || st.n_seqs > kMaxSeqs || sh.g < 1 || sh.g > 16 || sh.H != sh.KV * sh.g ||
       !decode_tile_head_dim(sh.hd) || p.n_wgs < 1 || !d.partials || !d.part_flag || !d.error)
     return hipErrorInvalidValue;
@@ -709,17 +730,18 @@ hipError_t launch_decode(const DecodeArgs &d, const SeqTable &st, const Shape &s
         return hipErrorInvalidValue;
   }
   if (!d.q_rot) return hipErrorInvalidValue;
+  if (bias && (dev || !db.tab || db.v_hd < 4 || (db.v_hd & 3) || (db.q_stride & 3) || db.v_hd > 256)) return hipErrorInvalidValue;
   unsigned *flag_set = d.flag_set ? d.flag_set : d.part_flag;
   const int spin_limit = d.spin_limit > 0 ? d.spin_limit : kFlagSpinLimit;
   float *part_o = d.partials;
-  const int tile_hd = decode_tile_head_dim(sh.hd);
+  const int tile_hd = decode_tile_head_dim(bias && db.v_hd > sh.hd ? db.v_hd : sh.hd);
   float *part_ml = d.partials + (size_t)p.n_slots * p.cols * tile_hd;
   const float c = scale * kLog2e;
   // before / after (nullable) receive the kernel's own first and last clock reading, not the
   // time at which the stream reached them: what is between two kernels stays out
   dim3 grid((unsigned)p.n_wgs), block(64 * kDecodeWaves);
   ReadAhead ah = {nullptr, 0, 0, 0};
-  if (d.ahead_w && d.ahead_wgs > 0 && !dev && !before && !after && (sh.hd == 64 || sh.hd == 128) && d.ahead_k >= 256 &&
+  if (d.ahead_w && d.ahead_wgs > 0 && !dev && !bias && !before && !after && (sh.hd == 64 || sh.hd == 128) && d.ahead_k >= 256 &&
       (d.ahead_k & 255) == 0 && d.ahead_n > 0) {
     ah.w = d.ahead_w;
     ah.k = d.ahead_k;
@@ -737,7 +759,7 @@ hipError_t launch_decode(const DecodeArgs &d, const SeqTable &st, const Shape &s
 #define SHAINET_DECODE_LAUNCH(HD_, DEV_, PAD_)                                                                      \
   SHAINET_LAUNCH_TIMED((decode_splitk_kernel<HD_, kDecodeWaves, DEV_, PAD_>), grid, block, 0, stream, before,      \
                        after, d.q_rot, d.kc, d.vc, d.out, part_o, part_ml, d.part_flag, flag_set, spin_limit,       \
-                       d.error, st, sh, p.tiles_per_wg, p.spans, p.total_tiles, p.n_slots, p.cols, c, rotate, dev, ah)
+                       d.error, st, sh, p.tiles_per_wg, p.spans, p.total_tiles, p.n_slots, p.cols, c, rotate, dev, ah, db)
 #define SHAINET_DECODE_LAUNCH_HD(HD_, PAD_) \
   do {                                      \
     if (dev)                                \
@@ -745,14 +767,25 @@ hipError_t launch_decode(const DecodeArgs &d, const SeqTable &st, const Shape &s
     else                                    \
       SHAINET_DECODE_LAUNCH(HD_, false, PAD_); \
   } while (0)
-  if (ah.w && sh.hd == 64)
+#define SHAINET_DECODE_LAUNCH_BIAS(HD_)                                                                             \
+  SHAINET_LAUNCH_TIMED((decode_splitk_kernel<HD_, kDecodeWaves, false, true, false, true>), grid, block, 0, stream, \
+                       before, after, d.q_rot, d.kc, d.vc, d.out, part_o, part_ml, d.part_flag, flag_set,           \
+                       spin_limit, d.error, st, sh, p.tiles_per_wg, p.spans, p.total_tiles, p.n_slots, p.cols, c,   \
+                       rotate, dev, ah, db)
+  if (bias && tile_hd == 64)
+    SHAINET_DECODE_LAUNCH_BIAS(64);
+  else if (bias && tile_hd == 128)
+    SHAINET_DECODE_LAUNCH_BIAS(128);
+  else if (bias)
+    SHAINET_DECODE_LAUNCH_BIAS(256);
+  else if (ah.w && sh.hd == 64)
     hipLaunchKernelGGL((decode_splitk_kernel<64, kDecodeWaves, false, false, true>), grid, block, 0, stream, d.q_rot, d.kc,
                        d.vc, d.out, part_o, part_ml, d.part_flag, flag_set, spin_limit, d.error, st, sh, p.tiles_per_wg,
-                       p.spans, p.total_tiles, p.n_slots, p.cols, c, rotate, dev, ah);
+                       p.spans, p.total_tiles, p.n_slots, p.cols, c, rotate, dev, ah, db);
   else if (ah.w)
     hipLaunchKernelGGL((decode_splitk_kernel<128, kDecodeWaves, false, false, true>), grid, block, 0, stream, d.q_rot, d.kc,
                        d.vc, d.out, part_o, part_ml, d.part_flag, flag_set, spin_limit, d.error, st, sh, p.tiles_per_wg,
-                       p.spans, p.total_tiles, p.n_slots, p.cols, c, rotate, dev, ah);
+                       p.spans, p.total_tiles, p.n_slots, p.cols, c, rotate, dev, ah, db);
   else if (sh.hd == 64)
     SHAINET_DECODE_LAUNCH_HD(64, false);
   else if (sh.hd == 128)
@@ -763,6 +796,7 @@ hipError_t launch_decode(const DecodeArgs &d, const SeqTable &st, const Shape &s
     SHAINET_DECODE_LAUNCH_HD(128, true);
   else
     SHAINET_DECODE_LAUNCH_HD(256, true);
+#undef SHAINET_DECODE_LAUNCH_BIAS
 #undef SHAINET_DECODE_LAUNCH_HD
 #undef SHAINET_DECODE_LAUNCH
   return hipGetLastError();

@@ -67,6 +67,8 @@ struct GemmArgs {
   const float *w;
   float *y;
   const float *res;  // nullable: y = res + x W
+  const float *bias;  // nullable: y = act(x W + bias)
+  Activation act;
   float *partials;   // [workgroups][128 * 128]: the piece a workgroup leaves unfinished
   unsigned *flags;   // [workgroups], zero between launches
   unsigned *flag_set;  // where a piece is marked complete: `flags`, or elsewhere in the test of the give-up path
@@ -80,6 +82,12 @@ struct GemmArgs {
   int pieces;           // 0: a workgroup's run of units starts where the one before it ends; > 0: every tile
                         // is cut into this many pieces of `quota` steps, a workgroup each, all left in their slots
 };
+
+// v: four neighbouring columns from `col` on
+__device__ __forceinline__ f32x4 add_bias(const GemmArgs &g, f32x4 v, int col) {
+  const f32x4 b = *(const f32x4 *)(g.bias + col);
+  return f32x4{activate(g.act, v.x + b.x), activate(g.act, v.y + b.y), activate(g.act, v.z + b.z), activate(g.act, v.w + b.w)};
+}
 
 // GUARD: K need not be a multiple of 32 (pieces beyond its end are loaded as zeros); without it
 // every load of the loop is unconditional.
@@ -313,6 +321,7 @@ __global__ __launch_bounds__(256, 2) void sgemm_mfma_kernel(const GemmArgs g) {
         if (row < T) {
           const long long o = (long long)row * N + col;
           f32x4 v = out[r];
+          if (g.bias) v = add_bias(g, v, col);
           if (g.res) v = *(const f32x4 *)(g.res + o) + v;
           *(f32x4 *)(g.y + o) = v;
         }
@@ -338,6 +347,7 @@ __global__ __launch_bounds__(256) void sgemm_reduce_kernel(const GemmArgs g, int
   const int col = (tile / g.tiles_m) * TN + 4 * (lane & 31);
   if (row < g.T && col < g.N) {
     const long long o = (long long)row * g.N + col;
+    if (g.bias) acc = add_bias(g, acc, col);
     if (g.res) acc = *(const f32x4 *)(g.res + o) + acc;
     *(f32x4 *)(g.y + o) = acc;
   }
@@ -347,13 +357,15 @@ __global__ __launch_bounds__(256) void sgemm_reduce_kernel(const GemmArgs g, int
 // coalesced along n.  For the small odd shapes of tests; the MFMA kernel takes everything else.
 __global__ __launch_bounds__(256) void sgemm_plain_kernel(const float *__restrict__ x, long long xs,
                                                           const float *__restrict__ w, float *__restrict__ y,
-                                                          const float *__restrict__ res, int T, int K, int N) {
+                                                          const float *__restrict__ res, int T, int K, int N,
+                                                          const float *__restrict__ bias, Activation act) {
   const int n = blockIdx.x * 256 + threadIdx.x;
   if (n >= N) return;
   for (int t = blockIdx.y; t < T; t += gridDim.y) {  // the grid's second dimension ends at 65535
     const float *xr = x + (long long)t * xs;
     float acc = 0.f;
     for (int k = 0; k < K; ++k) acc += xr[k] * w[(long long)k * N + n];
+    if (bias) acc = activate(act, acc + bias[n]);
     const long long o = (long long)t * N + n;
     y[o] = res ? res[o] + acc : acc;
   }
@@ -411,12 +423,12 @@ GemmPlan plan_gemm(int T, int K, int N, long long x_stride) {
 
 hipError_t launch_gemm(const float *x, long long x_stride, const float *w, float *y, const float *res, float *partials,
                        unsigned *flags, int *error, int T, int K, int N, const GemmPlan &p, hipStream_t stream,
-                       unsigned *flag_set, int spin_limit) {
+                       unsigned *flag_set, int spin_limit, const float *bias, Activation act) {
   if (!x || !w || !y || T < 1 || K < 1 || N < 1 || x_stride < K) return hipErrorInvalidValue;
-  const bool aligned = !(((uintptr_t)x | (uintptr_t)w | (uintptr_t)y | (uintptr_t)res) & 15);
+  const bool aligned = !(((uintptr_t)x | (uintptr_t)w | (uintptr_t)y | (uintptr_t)res | (uintptr_t)bias) & 15);
   if (!p.mfma || !aligned) {
     hipLaunchKernelGGL(sgemm_plain_kernel, dim3((unsigned)((N + 255) / 256), (unsigned)(T < 65535 ? T : 65535)), dim3(256), 0, stream, x,
-                       x_stride, w, y, res, T, K, N);
+                       x_stride, w, y, res, T, K, N, bias, act);
     return hipGetLastError();
   }
   if (p.partial_floats && !partials) return hipErrorInvalidValue;
@@ -427,6 +439,8 @@ hipError_t launch_gemm(const float *x, long long x_stride, const float *w, float
   g.w = w;
   g.y = y;
   g.res = res;
+  g.bias = bias;
+  g.act = act;
   g.partials = partials;
   g.flags = flags;
   g.flag_set = flag_set ? flag_set : flags;

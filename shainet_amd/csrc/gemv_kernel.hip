@@ -47,12 +47,18 @@ __device__ __forceinline__ float swiglu1(float gate, float up) {
   return (float)((g / (1.0 + exp(-g))) * (double)up);
 }
 
-__device__ __forceinline__ f32x4 apply_epilogue(int epi, f32x4 a, f32x4 b, const float *res) {
+// row, col: the place of a.x in y
+__device__ __forceinline__ f32x4 apply_epilogue(const GemvArgs &g, f32x4 a, f32x4 b, int row, int col) {
+  const int epi = g.epilogue;
   if (epi == kGemvSwiglu) return f32x4{swiglu1(a.x, b.x), swiglu1(a.y, b.y), swiglu1(a.z, b.z), swiglu1(a.w, b.w)};
   if (epi == kGemvResidual) {
-    const f32x4 r = *(const f32x4 *)res;
+    const f32x4 r = *(const f32x4 *)(g.res + (long long)row * g.N + col);
     return f32x4{(float)((double)r.x + (double)a.x), (float)((double)r.y + (double)a.y),
                  (float)((double)r.z + (double)a.z), (float)((double)r.w + (double)a.w)};
+  }
+  if (epi == kGemvBias) {
+    const float *v = g.bias + col;  // (one float at a time: no alignment is asked of it)
+    return f32x4{activate(g.act, a.x + v[0]), activate(g.act, a.y + v[1]), activate(g.act, a.z + v[2]), activate(g.act, a.w + v[3])};
   }
   return a;
 }
@@ -85,6 +91,7 @@ __device__ __forceinline__ void prep_tile_row(const GemvPrep &p, const float *ti
       dst = (is_v ? p.vc : p.kc) + row;
       rotate = !is_v;
     }
+    rotate = rotate && p.rope_tab;
     if (bias) {
       x0 = x0 + bias[i];
       x1 = x1 + bias[i + half];
@@ -133,7 +140,8 @@ __device__ __forceinline__ PairTarget prep_pair_begin(const GemvPrep &p, int r, 
   t.has_bias = bias != nullptr;
   t.b0 = bias ? bias[i] : 0.f;
   t.b1 = bias ? bias[i + half] : 0.f;
-  t.cs = p.rope_tab[(long long)pos * half + i];
+  t.rotate = t.rotate && p.rope_tab;
+  t.cs = p.rope_tab ? p.rope_tab[(long long)pos * half + i] : float2{1.f, 0.f};
   return t;
 }
 __device__ __forceinline__ void prep_pair_end(const GemvPrep &p, const PairTarget &t, float x0, float x1) {
@@ -295,8 +303,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(GemvArgs a) {
           prep_tile_row(a.prep, tile_s, blockIdx.x * CW, CW, t, wave, lane);
           __syncthreads();
         } else if (writer) {
-          const float *res = a.res ? a.res + (long long)t * N + col : nullptr;
-          *(f32x4 *)(a.y + (long long)t * N + col) = apply_epilogue(a.epilogue, acc[0][t], acc[NACC - 1][t], res);
+          *(f32x4 *)(a.y + (long long)t * N + col) = apply_epilogue(a, acc[0][t], acc[NACC - 1][t], t, col);
         }
       }
     return;
@@ -393,8 +400,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(GemvArgs a) {
       if constexpr (PREP) {
         *(f32x4 *)(tile_s + cl * 4) = sum[0];
       } else {
-        const float *res = a.res ? a.res + (long long)t * N + col : nullptr;
-        *(f32x4 *)(a.y + (long long)t * N + col) = apply_epilogue(a.epilogue, sum[0], sum[NACC - 1], res);
+        *(f32x4 *)(a.y + (long long)t * N + col) = apply_epilogue(a, sum[0], sum[NACC - 1], t, col);
       }
     }
     if constexpr (PREP) {
@@ -524,7 +530,9 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
   // what the epilogue of the first output reads besides: asked for now, behind the weights
   const bool residual = !PREP && a.epilogue == kGemvResidual;
   float res_first = 0.f;
-  if (residual) res_first = a.res[n0];
+  const bool biased = !PREP && a.epilogue == kGemvBias;
+  const float *beside = residual ? a.res : a.bias;
+  if (residual || biased) res_first = beside[n0];
   PairTarget target = {};
   // (head_dim is a power of two here: gemvt_takes)
   if constexpr (PREP) target = prep_pair_begin(a.prep, n0 >> half_shift, n0 & (half_hd - 1));
@@ -645,6 +653,7 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
       float v = s[0];
       if (a.epilogue == kGemvSwiglu) v = swiglu1(s[0], s[NACC - 1]);
       if (residual) v = (float)((double)res_v + (double)s[0]);
+      if (biased) v = activate(a.act, s[0] + res_v);
       a.y[n] = v;
     }
   };
@@ -656,13 +665,13 @@ __global__ __launch_bounds__(256) void gemvt_kernel(GemvArgs a) {
     for (int n = n0; n < n_end; n += 2) {
       if (n + 1 < n_end) {
         load_row(wb, n + 1);
-        if (residual) res_b = a.res[n + 1];
+        if (residual || biased) res_b = beside[n + 1];
       }
       finish_row(wa, n, res_a);
       if (n + 1 < n_end) {
         if (n + 2 < n_end) {
           load_row(wa, n + 2);
-          if (residual) res_a = a.res[n + 2];
+          if (residual || biased) res_a = beside[n + 2];
         }
         finish_row(wb, n + 1, res_b);
       }
@@ -712,7 +721,7 @@ hipError_t launch_gemv(const GemvArgs &args, const GemvPlan &p, hipStream_t stre
   if (p.rows_per_instr != 1 && p.rows_per_instr != 4) return hipErrorInvalidValue;
   if (p.rows_per_wave < 8 * p.rows_per_instr || p.rows_per_wave % (8 * p.rows_per_instr)) return hipErrorInvalidValue;
   if (p.splits > 1 && (!a.partials || !a.flags || !a.error)) return hipErrorInvalidValue;
-  if (a.epilogue == kGemvResidual && !a.res) return hipErrorInvalidValue;
+  if ((a.epilogue == kGemvResidual && !a.res) || (a.epilogue == kGemvBias && !a.bias)) return hipErrorInvalidValue;
   if (a.norm == kNormDynTanh && (!a.gamma || !a.beta)) return hipErrorInvalidValue;
   if (a.epilogue != kGemvResidual) a.res = nullptr;
   const bool prep = a.epilogue == kGemvQkvPrep;
@@ -720,7 +729,7 @@ hipError_t launch_gemv(const GemvArgs &args, const GemvPlan &p, hipStream_t stre
     const GemvPrep &q = a.prep;
     const int cw = 256 / p.rows_per_instr;
     if (q.hd < 2 || q.hd > 128 || (q.hd & (q.hd - 1)) || cw % q.hd || q.H < 1 || q.KV < 1 ||
-        a.N != (q.H + 2 * q.KV) * q.hd || !q.rope_tab || !q.q_rot || !q.kc || !q.vc || q.start_pos < 0 ||
+        a.N != (q.H + 2 * q.KV) * q.hd || !q.q_rot || !q.kc || !q.vc || q.start_pos < 0 ||
         q.start_pos + a.T > q.cap)
       return hipErrorInvalidValue;
   }
@@ -766,22 +775,22 @@ bool gemvt_takes(int T, int K, int N, int epilogue, int norm, const GemvPrep *pr
     return (K == 1024 || K == 2048 || K == 4096) && N == (prep->H + 2 * prep->KV) * prep->hd;
   }
   // rows of 8192: two wavefronts per output, which leaves out the norm prologue and SwiGLU
-  if (K == 8192) return !norm && !(N & 1) && (epilogue == kGemvPlain || epilogue == kGemvResidual);
+  if (K == 8192) return !norm && !(N & 1) && (epilogue == kGemvPlain || epilogue == kGemvResidual || epilogue == kGemvBias);
   if (K != 1024 && K != 2048 && K != 4096) return false;
-  return epilogue == kGemvPlain || epilogue == kGemvResidual || epilogue == kGemvSwiglu;
+  return epilogue == kGemvPlain || epilogue == kGemvResidual || epilogue == kGemvSwiglu || epilogue == kGemvBias;
 }
 
 hipError_t launch_gemvt(const GemvArgs &args, hipStream_t stream) {
   GemvArgs a = args;
   const bool prep = a.epilogue == kGemvQkvPrep;
   if (!gemvt_takes(a.T, a.K, a.N, a.epilogue, a.norm, &a.prep) || !a.x || !a.w || (!a.y && !prep)) return hipErrorInvalidValue;
-  if (a.epilogue == kGemvResidual && !a.res) return hipErrorInvalidValue;
+  if ((a.epilogue == kGemvResidual && !a.res) || (a.epilogue == kGemvBias && !a.bias)) return hipErrorInvalidValue;
   if (((uintptr_t)a.x | (uintptr_t)a.w | (uintptr_t)a.gamma | (uintptr_t)a.beta) & 15) return hipErrorInvalidValue;
   const bool dyt = a.norm == kNormDynTanh;
   if (dyt && (!a.gamma || !a.beta)) return hipErrorInvalidValue;
   if (prep) {
     const GemvPrep &q = a.prep;
-    if (q.H < 1 || q.KV < 1 || !q.rope_tab || !q.q_rot || !q.kc || !q.vc || q.start_pos < 0 || q.start_pos + 1 > q.cap)
+    if (q.H < 1 || q.KV < 1 || !q.q_rot || !q.kc || !q.vc || q.start_pos < 0 || q.start_pos + 1 > q.cap)
       return hipErrorInvalidValue;
     a.N = a.N / 2;  // pairs, two per workgroup
     a.rows_per_wave = 1;

@@ -15,9 +15,13 @@
 
 #include "../../include/shainet_hip_attn.h"
 #include "attn_kernels.hpp"
+#include "biased_attn.hpp"
+#include "feed_forward.hpp"
+#include "hgrn2.hpp"
 #include "latent_attn.hpp"
 #include "llama_internal.hpp"
 #include "mini_json.hpp"
+#include "residual_kernels.hpp"
 #include "safetensors.hpp"
 
 using namespace shainet;
@@ -582,12 +586,285 @@ int load_tutilorn(const char *model_dir, const Json &j, shainet_llama_model **ou
   return SHAINET_HIP_OK;
 }
 
+// Zabutar: layers of HGRN2 or of attention with a bias by distance (which may use another layer's keys and
+// values), each sublayer between two RMS norms and behind a short convolution over time, feed-forwards with
+// xIELU or of experts, learned positions.
+struct ZabutarLayer {
+  bool recurrent = false;
+  Hgrn2Config hgrn2;
+  BiasedConfig attention;
+  int kv_from = -1;
+  int ff = 0;         // > 0: a dense feed-forward
+  MoeShape moe = {};  // experts > 0: a mixture; neither: no feed-forward
+};
+struct ZabutarConfig {
+  int vocab = 0, width = 0, max_positions = 0, taps = 0;
+  double eps = 0.0;
+  std::vector<ZabutarLayer> layers;
+};
+
+bool given(const Json *obj, const char *key) {
+  const Json *v = obj ? obj->get(key) : nullptr;
+  return v && !v->is_null();
+}
+
+int read_zabutar_mlp(const Json &mlp, const std::string &where, int width, ZabutarLayer &out) {
+  const Json *kind = mlp.get("kind");
+  if (!kind || kind->kind != Json::kString) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json lacks " + where + "kind");
+  Fields f = {&mlp, where, ""};
+  if (kind->str == "dense") {
+    out.ff = f.integer("ff");
+    if (int rc = f.status()) return rc;
+    return out.ff > 0 ? SHAINET_HIP_OK : fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "ff must be positive");
+  }
+  if (kind->str != "moe") return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "kind '" + kind->str + "' is not a feed-forward this library has");
+  MoeShape &m = out.moe;
+  m.d = width;
+  m.groups = m.keep = 1;
+  m.scale = 1.f;
+  Fields expert = {f.object("expert"), where + "expert.", ""}, router = {f.object("router"), where + "router.", ""};
+  if (int rc = f.status()) return rc;
+  m.ff = expert.integer("ff");
+  m.experts = router.integer("experts");
+  m.top = router.integer("top");
+  if (given(router.obj, "identity")) m.identity = router.integer("identity");
+  if (given(router.obj, "scale")) m.scale = (float)router.real("scale");
+  Fields groups = {nullptr, where + "router.groups.", ""}, shared = {nullptr, where + "shared.", ""};
+  if (given(router.obj, "groups")) {
+    groups.obj = router.object("groups");
+    m.groups = groups.integer("count");
+    m.keep = groups.integer("keep");
+  }
+  if (given(&mlp, "shared")) {
+    shared.obj = f.object("shared");
+    m.shared_ff = shared.integer("ff");
+    if (shared.missing.empty() && m.shared_ff < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + shared.where + "ff must be positive");
+  }
+  for (const Fields *x : {&f, &expert, &router, &groups, &shared})
+    if (int rc = x->status()) return rc;
+  if (!moe_shape_ok(m))
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "router: at most 1024 outputs in equal groups, and top at most what the kept groups hold");
+  return SHAINET_HIP_OK;
+}
+
+int read_zabutar_layer(const Json &j, int index, int width, ZabutarLayer &out) {
+  const std::string where = "layers[" + std::to_string(index) + "].";
+  const Json *type = j.get("type");
+  if (!type || type->kind != Json::kString) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json lacks " + where + "type");
+  out.recurrent = type->str == "hgrn2";
+  if (!out.recurrent && type->str != "attention")
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "type '" + type->str + "' is not a mixer this design has");
+  Fields top = {&j, where, ""};
+  Fields f = {top.object("mixer"), where + "mixer.", ""};
+  if (int rc = top.status()) return rc;
+  if (out.recurrent) {
+    out.hgrn2.heads = f.integer("heads");
+    out.hgrn2.dim = f.integer("dim");
+    out.hgrn2.vdim = f.integer("vdim");
+  } else {
+    BiasedConfig &a = out.attention;
+    a.heads = f.integer("heads");
+    a.kv_heads = f.integer("kv_heads");
+    a.dim = f.integer("dim");
+    a.vdim = f.integer("vdim");
+    a.scale = f.real("scale");
+    a.bias_max = f.integer("bias_max");
+    if (given(f.obj, "kv_from")) {
+      out.kv_from = f.integer("kv_from");
+      if (out.kv_from < 0) return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: " + where + "mixer.kv_from is not a layer");
+    }
+  }
+  if (int rc = f.status()) return rc;
+  const Json *mlp = j.get("mlp");
+  return mlp && !mlp->is_null() ? read_zabutar_mlp(*mlp, where + "mlp.", width, out) : SHAINET_HIP_OK;
+}
+
+int read_zabutar_config(const Json &j, ZabutarConfig &c) {
+  Fields f = {&j, "", ""};
+  c.vocab = f.integer("vocab");
+  c.width = f.integer("width");
+  c.max_positions = f.integer("max_positions");
+  Fields norm = {f.object("norm"), "norm.", ""}, canon = {f.object("canon"), "canon.", ""};
+  c.eps = norm.real("eps");
+  c.taps = canon.integer("taps");
+  for (const Fields *x : {&f, &norm, &canon})
+    if (int rc = x->status()) return rc;
+  if (c.vocab < 1 || c.width < 1 || c.max_positions < 1)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: vocab, width and max_positions must be positive");
+  if (c.taps < 1 || c.taps > kMaxConvTaps)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: canon.taps must be in [1, " + std::to_string(kMaxConvTaps) + "]");
+  const Json *layers = j.get("layers");
+  if (!layers || layers->kind != Json::kArray || layers->arr.empty())
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json lacks layers");
+  const int n = (int)layers->arr.size();
+  c.layers.resize(n);
+  for (int i = 0; i < n; ++i) {
+    ZabutarLayer &l = c.layers[i];
+    if (int rc = read_zabutar_layer(layers->arr[i], i, c.width, l)) return rc;
+    if (l.kv_from < 0) continue;
+    const ZabutarLayer *from = l.kv_from < i ? &c.layers[l.kv_from] : nullptr;
+    if (!from || from->recurrent || from->kv_from >= 0 || from->attention.kv_heads != l.attention.kv_heads ||
+        from->attention.dim != l.attention.dim || from->attention.vdim != l.attention.vdim)
+      return fail(SHAINET_HIP_ERR_ARGUMENT, "config.json: layers[" + std::to_string(i) +
+                                                "].mixer.kv_from is not an earlier attention layer with projections of its own and the same heads");
+  }
+  return SHAINET_HIP_OK;
+}
+
+// an RMS norm's weight, stored as the distance from 1
+int load_centred_norm(const shainet_safetensors *st, Stager &stage, const std::string &name, int d, float *dst) {
+  if (int rc = load_plain(st, stage, name, 1, d, dst)) return rc;
+  if (launch_add_one(dst, d, nullptr) != hipSuccess || hipDeviceSynchronize() != hipSuccess)
+    return fail(SHAINET_HIP_ERR_RUNTIME, "converting tensor '" + name + "' failed");
+  return SHAINET_HIP_OK;
+}
+
+int load_hgrn2(const shainet_safetensors *st, Stager &stage, const std::string &p, int d, const Hgrn2Config &c, Hgrn2Weights &w) {
+  const int qw = c.heads * c.dim, vw = c.heads * c.vdim;
+  int rc;
+  if ((rc = load_transposed(st, stage, p + "q", qw, d, w.w_in, w.n_in, 0))) return rc;
+  if ((rc = load_transposed(st, stage, p + "f", qw, d, w.w_in, w.n_in, qw))) return rc;
+  if ((rc = load_transposed(st, stage, p + "v", vw, d, w.w_in, w.n_in, 2 * qw))) return rc;
+  if ((rc = load_plain(st, stage, p + "f.b", 1, qw, w.f_bias))) return rc;
+  if ((rc = load_plain(st, stage, p + "lower", 1, qw, w.lower))) return rc;
+  if ((rc = load_plain(st, stage, p + "norm", 1, c.vdim, w.norm))) return rc;
+  return load_transposed(st, stage, p + "o", d, vw, w.w_o, d, 0);
+}
+
+int load_biased(const shainet_safetensors *st, Stager &stage, const std::string &p, int d, const ZabutarLayer &l, int max_positions,
+                BiasedAttn *mixer) {
+  const BiasedConfig &c = l.attention;
+  BiasedWeights &w = biased_attn_weights(mixer);
+  const int qw = c.heads * c.dim, kw = c.kv_heads * c.dim, vw = c.kv_heads * c.vdim;
+  int rc;
+  if ((rc = load_transposed(st, stage, p + "q", qw, d, w.w_in, w.n_in, 0))) return rc;
+  if (l.kv_from < 0) {
+    if ((rc = load_transposed(st, stage, p + "k", kw, d, w.w_in, w.n_in, qw))) return rc;
+    if ((rc = load_transposed(st, stage, p + "v", vw, d, w.w_in, w.n_in, qw + kw))) return rc;
+  }
+  const StTensor *t = need(st, p + "rel", rc);
+  if (!t) return rc;
+  if (t->shape.size() != 2 || t->shape[0] < 1 || t->shape[1] != c.heads)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "tensor '" + p + "rel' is not [rows, heads]");
+  std::vector<float> rel;
+  if ((rc = read_host_vector(st, p + "rel", rel))) return rc;
+  if ((rc = biased_attn_set_table(mixer, rel, (int)t->shape[0], max_positions))) return rc;
+  return load_transposed(st, stage, p + "o", d, c.heads * c.vdim, w.w_o, d, 0);
+}
+
+int load_xielu(const shainet_safetensors *st, Stager &stage, const std::string &p, int d, int ff, DenseWeights &w) {
+  int rc;
+  if ((rc = load_transposed(st, stage, p + "up", ff, d, w.up, ff, 0))) return rc;
+  if ((rc = load_plain(st, stage, p + "up.b", 1, ff, w.up_bias))) return rc;
+  if ((rc = load_transposed(st, stage, p + "down", d, ff, w.down, d, 0))) return rc;
+  if ((rc = load_plain(st, stage, p + "down.b", 1, d, w.down_bias))) return rc;
+  std::vector<float> act;
+  if ((rc = read_host_vector(st, p + "act", act))) return rc;
+  if (act.size() != 2) return fail(SHAINET_HIP_ERR_ARGUMENT, "tensor '" + p + "act' does not hold two numbers");
+  auto softplus = [](double z) { return z > 0 ? z + log1p(exp(-z)) : log1p(exp(z)); };
+  w.act.kind = kActXielu;
+  w.act.pos = (float)softplus(act[0]);
+  w.act.neg = (float)(0.5 + softplus(act[1]));
+  return SHAINET_HIP_OK;
+}
+
+int load_experts(const shainet_safetensors *st, Stager &stage, const std::string &p, const MoeShape &m, MoeWeights &w) {
+  const int n = m.experts + m.identity;
+  const size_t mat = (size_t)m.ff * m.d;
+  int rc;
+  if ((rc = load_plain(st, stage, p + "router", n, m.d, w.router))) return rc;
+  if ((rc = load_plain(st, stage, p + "correction", 1, n, w.correction))) return rc;
+  for (int e = 0; e < m.experts; ++e) {
+    const std::string pe = p + "e" + std::to_string(e) + ".";
+    if ((rc = load_plain(st, stage, pe + "gate", m.ff, m.d, w.gate_up + 2 * e * mat))) return rc;
+    if ((rc = load_plain(st, stage, pe + "up", m.ff, m.d, w.gate_up + (2 * e + 1) * mat))) return rc;
+    if ((rc = load_plain(st, stage, pe + "down", m.d, m.ff, w.down + e * mat))) return rc;
+  }
+  if (!m.shared_ff) return SHAINET_HIP_OK;
+  const std::string ps = p + "shared.";
+  const int ff = m.shared_ff;
+  if ((rc = load_plain(st, stage, ps + "gate", ff, m.d, w.shared_gate_up))) return rc;
+  if ((rc = load_plain(st, stage, ps + "up", ff, m.d, w.shared_gate_up + (size_t)ff * m.d))) return rc;
+  if ((rc = load_plain(st, stage, ps + "down", m.d, ff, w.shared_down))) return rc;
+  if ((rc = load_transposed(st, stage, ps + "gate", ff, m.d, w.shared_gate_up_in, 2LL * ff, 0))) return rc;
+  if ((rc = load_transposed(st, stage, ps + "up", ff, m.d, w.shared_gate_up_in, 2LL * ff, ff))) return rc;
+  return load_transposed(st, stage, ps + "down", m.d, ff, w.shared_down_in, m.d, 0);
+}
+
+// One layer: its parts made and filled.
+int load_zabutar_layer(const shainet_safetensors *st, Stager &stage, const ZabutarConfig &cfg, int i,
+                       const std::vector<shainet_llama_block *> &before, shainet_llama_block **out) {
+  const ZabutarLayer &l = cfg.layers[i];
+  const int d = cfg.width;
+  const std::string p = "l" + std::to_string(i) + ".";
+  Mixer *mixer = nullptr;
+  FeedForward *ff = nullptr;
+  DenseWeights *dense = nullptr;
+  MoeWeights *moe = nullptr;
+  int rc = l.recurrent ? hgrn2_create(&mixer, d, l.hgrn2, cfg.eps)
+                       : biased_attn_create(&mixer, d, l.attention, l.kv_from < 0 ? nullptr : shainet_llama_block_mixer_of(before[l.kv_from]));
+  if (!rc && l.ff) rc = dense_create(&ff, d, l.ff, &dense);
+  if (!rc && l.moe.experts) rc = moe_create(&ff, l.moe, &moe);
+  if (rc) {
+    delete mixer;
+    return rc;
+  }
+  if ((rc = shainet_llama_block_create_wrapped(out, d, mixer, ff, cfg.taps, cfg.eps))) return rc;
+  const WrappedBlockBuffers b = shainet_llama_block_wrapped_buffers(*out);
+  if ((rc = load_centred_norm(st, stage, p + "norm1", d, b.norm1))) return rc;
+  if ((rc = load_centred_norm(st, stage, p + "norm1b", d, b.post1))) return rc;
+  if ((rc = load_transposed(st, stage, p + "canon1", d, cfg.taps, b.conv1, d, 0))) return rc;
+  rc = l.recurrent ? load_hgrn2(st, stage, p + "mix.", d, l.hgrn2, hgrn2_weights(mixer->hgrn2()))
+                   : load_biased(st, stage, p + "mix.", d, l, cfg.max_positions, mixer->biased());
+  if (rc || !ff) return rc;
+  if ((rc = load_centred_norm(st, stage, p + "norm2", d, b.norm2))) return rc;
+  if ((rc = load_centred_norm(st, stage, p + "norm2b", d, b.post2))) return rc;
+  if ((rc = load_transposed(st, stage, p + "canon2", d, cfg.taps, b.conv2, d, 0))) return rc;
+  return dense ? load_xielu(st, stage, p + "mlp.", d, l.ff, *dense) : load_experts(st, stage, p + "mlp.", l.moe, *moe);
+}
+
+int load_zabutar(const char *model_dir, const Json &j, shainet_llama_model **out) {
+  ZabutarConfig cfg;
+  int rc = read_zabutar_config(j, cfg);
+  if (rc) return rc;
+  if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
+  const int d = cfg.width, n = (int)cfg.layers.size();
+  shainet_safetensors *st = nullptr;
+  if ((rc = shainet_safetensors_open(model_dir, &st))) return rc;
+  shainet_llama_model *m = nullptr;
+  Stager stage;
+  rc = shainet_llama_model_create_empty(&m, cfg.vocab, d, cfg.eps, 1.0, kNormRms);
+  std::vector<shainet_llama_block *> blocks;
+  for (int i = 0; i < n && !rc; ++i) {
+    shainet_llama_block *b = nullptr;
+    rc = load_zabutar_layer(st, stage, cfg, i, blocks, &b);
+    if (!b) break;
+    blocks.push_back(b);
+    shainet_llama_model_add_block(m, b);  // owned by the model from here on
+  }
+  LlamaModelBuffers mb;
+  float *positions = nullptr;
+  if (!rc) rc = shainet_llama_model_buffers(m, &mb);
+  if (!rc) rc = shainet_llama_model_position_buffer(m, cfg.max_positions, &positions);
+  if (!rc) rc = load_plain(st, stage, "embed", cfg.vocab, d, mb.embedding);
+  if (!rc) rc = load_plain(st, stage, "pos", cfg.max_positions, d, positions);
+  if (!rc) rc = load_centred_norm(st, stage, "final.norm", d, mb.final_norm->gamma);
+  if (!rc) rc = load_transposed(st, stage, "head", cfg.vocab, d, mb.lm_head, cfg.vocab, 0);
+  shainet_safetensors_close(st);
+  if (rc) {
+    shainet_llama_model_destroy(m);
+    return rc;
+  }
+  *out = m;
+  return SHAINET_HIP_OK;
+}
+
 // Designs by the name their config.json gives under "architecture".
 struct Design {
   const char *name;
   int (*load)(const char *model_dir, const Json &config, shainet_llama_model **out);
 };
-constexpr Design kDesigns[] = {{"Tutilorn", load_tutilorn}};
+constexpr Design kDesigns[] = {{"Tutilorn", load_tutilorn}, {"Zabutar", load_zabutar}};
 
 }  // namespace
 

@@ -9,9 +9,12 @@
 // The second half of this file adds what LlamaBlock#forward_cached
 // (llama_block.cr:189-196) does around attention: the two RMSNorms, the two
 // residual adds and the dense SwiGLU feed-forward, again all on the device.
-// A block's parts are parameters: its mixer is the attention above or latent
-// attention (latent_attn.hip), its norms RMSNorm or Dynamic Tanh, its feed-forward
-// may be missing, and its weights may be another block's.
+// A block's parts are parameters: its mixer is the attention above or one of those
+// behind the Mixer interface (latent_attn.hip, biased_attn.hip, hgrn2.hip), its norms
+// RMSNorm or Dynamic Tanh, its feed-forward another kind (feed_forward.hip) or
+// missing, and its weights may be another block's.  A block with norms behind its
+// sublayers, too, and convolutions over time in front of them takes a forward pass of
+// its own (wrapped_forward_device).
 #include <hip/hip_runtime.h>
 #include <math.h>
 #include <stdio.h>
@@ -27,8 +30,12 @@
 #include "attn_kernels.hpp"
 #include "attn_context.hpp"
 #include "block_kernels.hpp"
+#include "feed_forward.hpp"
+#include "hgrn2.hpp"
 #include "latent_attn.hpp"
 #include "llama_internal.hpp"
+#include "mixer.hpp"
+#include "residual_kernels.hpp"
 #include "step_kernel.hpp"
 
 using namespace shainet;
@@ -325,15 +332,60 @@ struct BlockWeights {
   float *gate_up = nullptr, *down = nullptr;        // device [d_model, 2*ff] (gate | up) and [ff, d_model]
   float *gate_up_t = nullptr, *down_t = nullptr;    // the same transposed ([2*ff, d_model], [d_model, ff]), like w_o_t
   bool gate_up_t_stale = true, down_t_stale = true;
+  // wrapped blocks: norms behind the sublayers [d_model], convolutions in front of them [taps, d_model], and a
+  // feed-forward of another kind (null: none)
+  float *post1 = nullptr, *post2 = nullptr, *conv1 = nullptr, *conv2 = nullptr;
+  int taps = 0;
+  std::unique_ptr<FeedForward> ff;
   ~BlockWeights() {
-    for (float *p : {norm1.gamma, norm1.beta, norm2.gamma, norm2.beta, gate_up, down, gate_up_t, down_t})
+    for (float *p : {norm1.gamma, norm1.beta, norm2.gamma, norm2.beta, gate_up, down, gate_up_t, down_t, post1, post2, conv1, conv2})
+      if (p) (void)hipFree(p);
+  }
+};
+
+// The latent-attention mixer behind the interface all mixers share.
+struct LatentMixer : Mixer {
+  LatentAttn *l;
+  explicit LatentMixer(LatentAttn *l) : l(l) {}
+  ~LatentMixer() override { latent_attn_destroy(l); }
+  hipStream_t stream() override { return (hipStream_t)shainet_attn_stream(latent_attn_context(l)); }
+  int set_stream(hipStream_t s) override { return shainet_attn_set_stream(latent_attn_context(l), (void *)s); }
+  int *error_word() override { return shainet_attn_error_word(latent_attn_context(l)); }
+  void share_error_word(int *word) override { latent_attn_share_error_word(l, word); }
+  Projector &projector() override { return latent_attn_projector(l); }
+  int forward(const float *x, int T, float *out, const Fused &pre, const float *residual, bool no_cache) override {
+    return latent_attn_forward(l, x, T, out, pre, residual, no_cache);
+  }
+  int reserve(int positions) override { return latent_attn_reserve(l, positions); }
+  int clear() override { return shainet_kv_cache_clear(cache(), -1); }
+  int len() override { return shainet_kv_cache_len(cache(), 0); }
+  int truncate(int len) override { return shainet_kv_cache_truncate(cache(), 0, len); }
+  shainet_kv_cache *cache() override { return latent_attn_cache(l); }
+  LatentAttn *latent() override { return l; }
+};
+
+// What a convolution over time in front of a sublayer keeps of its sequence: the sublayer's last taps - 1
+// inputs, in two buffers that take turns.
+struct ConvState {
+  float *rows[2] = {nullptr, nullptr}, *saved = nullptr;
+  int cur = 0;
+  int allocate(size_t n) {
+    const WantedBuffer wants[] = {{&rows[0], n}, {&rows[1], n}, {&saved, n}};
+    return allocate_buffers(wants, 3);
+  }
+  ~ConvState() {
+    for (float *p : {rows[0], rows[1], saved})
       if (p) (void)hipFree(p);
   }
 };
 
 struct shainet_llama_block {
   shainet_llama_attn *attn = nullptr;  // the mixer: one of the two
-  LatentAttn *latent = nullptr;
+  std::unique_ptr<Mixer> mixer;
+  bool wrapped = false;  // norms behind the sublayers (and convolutions in front)
+  ConvState conv[2];
+  int pos = 0, saved_pos = -1;  // wrapped: positions so far, and where the state was saved last
+  DevF joined, y;               // wrapped: the residual with the block before joined in; a sublayer's result
   int d_model = 0, ff_hidden = 0;                   // ff_hidden 0: no feed-forward
   double eps = 1e-6;                                // RMSNorm eps of @norm1 / @norm2 (llama_block.cr:93-94)
   std::shared_ptr<BlockWeights> w = std::make_shared<BlockWeights>();
@@ -343,19 +395,20 @@ struct shainet_llama_block {
 
 namespace {
 
-// the context behind the block's mixer: stream, error word
-int block_context(shainet_llama_block *b, shainet_attn_ctx **ctx) {
-  if (b->latent) {
-    *ctx = latent_attn_context(b->latent);
+// the stream the block's work runs on, once its mixer is ready
+int block_stream(shainet_llama_block *b, hipStream_t *stream) {
+  if (b->mixer) {
+    *stream = b->mixer->stream();
     return SHAINET_HIP_OK;
   }
   const int rc = ensure_context(b->attn);
-  *ctx = b->attn->ctx;
+  if (!rc) *stream = (hipStream_t)shainet_attn_stream(b->attn->ctx);
   return rc;
 }
+int *block_error_word(shainet_llama_block *b) { return b->mixer ? b->mixer->error_word() : shainet_attn_error_word(b->attn->ctx); }
 
-int latent_only(const shainet_llama_block *b, const char *what) {
-  if (b->latent) return fail(SHAINET_HIP_ERR_ARGUMENT, std::string(what) + ": this block's mixer is latent attention");
+int grouped_only(const shainet_llama_block *b, const char *what) {
+  if (b->mixer) return fail(SHAINET_HIP_ERR_ARGUMENT, std::string(what) + ": this block's mixer is not the grouped-query attention of a LLaMA block");
   return SHAINET_HIP_OK;
 }
 
@@ -363,16 +416,74 @@ int latent_only(const shainet_llama_block *b, const char *what) {
 
 namespace {
 
+// One residual_kernels.hpp launch: (with y) the result y of a sublayer joins x; (with pre) what the next sublayer
+// reads, from conv's state if there is a convolution.
+int join(shainet_llama_block *b, const float *x, const float *y, const float *post, float *x_out, const float *pre,
+         const float *conv_w, ConvState *conv, float *h, int T, bool no_cache, hipStream_t stream) {
+  ResidualArgs a = {};
+  a.x = x;
+  a.y = y;
+  a.post = post;
+  a.x_out = x_out;
+  a.pre = pre;
+  a.h = h;
+  a.T = T;
+  a.d = b->d_model;
+  a.eps = (float)b->eps;
+  if (conv_w) {
+    a.conv = conv_w;
+    a.taps = b->w->taps;
+    if (a.taps > 1 && !no_cache) {
+      a.hist_in = b->pos ? conv->rows[conv->cur] : nullptr;  // (nothing lies before a sequence's first row)
+      a.hist_out = conv->rows[conv->cur ^ 1];
+      conv->cur ^= 1;
+    }
+  }
+  const hipError_t e = launch_residual(a, stream);
+  return e == hipSuccess ? SHAINET_HIP_OK : fail(SHAINET_HIP_ERR_RUNTIME, std::string("residual launch: ") + hipGetErrorString(e));
+}
+
+// x <- x + norm1b(mixer(conv1(norm1(x)))), then x <- x + norm2b(ff(conv2(norm2(x)))), where conv(h) = h + the
+// convolution.  Each arrow and what the next sublayer reads are one launch; carry takes the last one over
+// to the next block (BlockCarry).
+int wrapped_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache, BlockCarry *carry) {
+  BlockWeights &w = *b->w;
+  const size_t n = (size_t)T * b->d_model;
+  hipStream_t stream = b->mixer->stream();
+  if (!w.norm1.gamma || !w.post1) return fail(SHAINET_HIP_ERR_ARGUMENT, "weights not set");
+  if (!b->h.reserve(n) || !b->y.reserve(n) || !b->joined.reserve(n)) return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+  const bool carried = carry && carry->y;
+  int rc = join(b, x, carried ? carry->y : nullptr, carried ? carry->post : nullptr, b->joined.p, w.norm1.gamma, w.conv1, &b->conv[0],
+                b->h.p, T, no_cache, stream);
+  if (carry) carry->y = nullptr;
+  const float *res = carried ? b->joined.p : x;
+  if (!rc) rc = b->mixer->forward(b->h.p, T, b->y.p, Fused(), nullptr, no_cache);
+  if (!rc && !w.ff) rc = join(b, res, b->y.p, w.post1, out, nullptr, nullptr, nullptr, nullptr, T, no_cache, stream);
+  if (!rc && w.ff) {
+    rc = join(b, res, b->y.p, w.post1, out, w.norm2.gamma, w.conv2, &b->conv[1], b->h.p, T, no_cache, stream);
+    if (!rc) rc = w.ff->forward(b->mixer->projector(), b->h.p, T, b->y.p, stream);
+    if (!rc && carry) {
+      carry->y = b->y.p;
+      carry->post = w.post2;
+    } else if (!rc) {
+      rc = join(b, out, b->y.p, w.post2, out, nullptr, nullptr, nullptr, nullptr, T, no_cache, stream);
+    }
+  }
+  if (!rc && !no_cache) b->pos += T;
+  return rc;
+}
+
 // x and out on the device; asynchronous on the block's stream.
-int block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache = false) {
+int block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache = false, BlockCarry *carry = nullptr) {
+  if (b->wrapped) return wrapped_forward_device(b, x, T, out, no_cache, carry);
+  if (carry && carry->y) return fail(SHAINET_HIP_ERR_ARGUMENT, "a block without norms behind its sublayers takes no carried result");
   BlockWeights &w = *b->w;
   const int d = b->d_model, ff = b->ff_hidden;
   if (ff && (!w.gate_up || !w.down)) return fail(SHAINET_HIP_ERR_ARGUMENT, "feed-forward weights not set");
-  shainet_attn_ctx *ctx = nullptr;
-  int rc = block_context(b, &ctx);
+  hipStream_t stream = nullptr;
+  int rc = block_stream(b, &stream);
   if (rc) return rc;
-  hipStream_t stream = (hipStream_t)shainet_attn_stream(ctx);
-  Projector &proj = b->latent ? latent_attn_projector(b->latent) : b->attn->proj;
+  Projector &proj = b->mixer ? b->mixer->projector() : b->attn->proj;
   if (ff && (!b->h.reserve((size_t)T * d) || !b->hidden.reserve((size_t)T * ff)))
     return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
   float *h = ff ? b->h.p : out;  // without a feed-forward the mixer's sum is the block's result
@@ -388,8 +499,8 @@ int block_forward_device(shainet_llama_block *b, const float *x, int T, float *o
     gate.w_t = transposed_twin(&w.gate_up_t, &w.gate_up_t_stale, w.gate_up, d, 2 * ff, stream, ride);
     gate.w_t_has_gamma = gate.w_t && ride;
   }
-  if (b->latent) {
-    rc = latent_attn_forward(b->latent, x, T, h, n1, x, no_cache);
+  if (b->mixer) {
+    rc = b->mixer->forward(x, T, h, n1, x, no_cache);
   } else {
     const AheadRows ahead = {gate.w_t, d, ff};
     rc = attn_forward_device(b->attn, x, T, h, n1, x, no_cache, &ahead);
@@ -408,8 +519,23 @@ int block_forward_device(shainet_llama_block *b, const float *x, int T, float *o
 }  // namespace
 
 // used by the model (llama_model.hip)
-int shainet_llama_block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache) {
-  return block_forward_device(b, x, T, out, no_cache);
+int shainet_llama_block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache, BlockCarry *carry) {
+  return block_forward_device(b, x, T, out, no_cache, b->wrapped ? carry : nullptr);
+}
+int shainet_llama_block_join_carry(shainet_llama_block *b, const BlockCarry &carry, float *x, int T) {
+  return join(b, x, carry.y, carry.post, x, nullptr, nullptr, nullptr, nullptr, T, true, b->mixer->stream());
+}
+bool shainet_llama_block_keeps_state(const shainet_llama_block *b) { return b->wrapped; }
+int shainet_llama_block_save_state(shainet_llama_block *b) {
+  if (!b->wrapped) return SHAINET_HIP_OK;
+  b->saved_pos = -1;
+  if (int rc = b->mixer->save()) return rc;
+  const size_t bytes = (size_t)(b->w->taps > 1 ? b->w->taps - 1 : 0) * b->d_model * sizeof(float);
+  for (ConvState &c : b->conv)
+    if (b->pos && bytes && c.saved && hipMemcpyAsync(c.saved, c.rows[c.cur], bytes, hipMemcpyDeviceToDevice, b->mixer->stream()) != hipSuccess)
+      return fail(SHAINET_HIP_ERR_RUNTIME, "hipMemcpyAsync(state) failed");
+  b->saved_pos = b->pos;
+  return SHAINET_HIP_OK;
 }
 int shainet_llama_block_buffers(shainet_llama_block *b, LlamaBlockBuffers *out) {
   shainet_llama_attn *l = b->attn;
@@ -444,17 +570,17 @@ int shainet_llama_block_create_latent(shainet_llama_block **out, int d_model, co
                                       int ff_hidden, int norm_kind, double eps, const shainet_llama_block *weights_of) {
   *out = nullptr;
   if (ff_hidden < 0) return fail(SHAINET_HIP_ERR_ARGUMENT, "ff_hidden must not be negative");
-  if (weights_of && (!weights_of->latent || weights_of->d_model != d_model || weights_of->ff_hidden != ff_hidden ||
+  if (weights_of && (!weights_of->mixer || !weights_of->mixer->latent() || weights_of->d_model != d_model || weights_of->ff_hidden != ff_hidden ||
                      weights_of->w->norm1.kind != norm_kind))
     return fail(SHAINET_HIP_ERR_ARGUMENT, "layers that share weights must have the same mixer, feed-forward and norms");
   LatentAttn *l = nullptr;
-  if (int rc = latent_attn_create(&l, d_model, cfg, eps, weights_of ? weights_of->latent : nullptr)) return rc;
+  if (int rc = latent_attn_create(&l, d_model, cfg, eps, weights_of ? weights_of->mixer->latent() : nullptr)) return rc;
   shainet_llama_block *b = new (std::nothrow) shainet_llama_block();
   if (!b) {
     latent_attn_destroy(l);
     return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
   }
-  b->latent = l;
+  b->mixer.reset(new LatentMixer(l));
   b->d_model = d_model;
   b->ff_hidden = ff_hidden;
   b->eps = eps;
@@ -465,14 +591,45 @@ int shainet_llama_block_create_latent(shainet_llama_block **out, int d_model, co
   *out = b;
   return SHAINET_HIP_OK;
 }
-LatentAttn *shainet_llama_block_latent_mixer(shainet_llama_block *b) { return b->latent; }
+LatentAttn *shainet_llama_block_latent_mixer(shainet_llama_block *b) { return b->mixer ? b->mixer->latent() : nullptr; }
+
+int shainet_llama_block_create_wrapped(shainet_llama_block **out, int d_model, Mixer *mixer, FeedForward *ff, int taps, double eps) {
+  *out = nullptr;
+  std::unique_ptr<Mixer> owned(mixer);
+  std::unique_ptr<FeedForward> owned_ff(ff);
+  if (taps < 1 || taps > kMaxConvTaps)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "convolution taps must be in [1, " + std::to_string(kMaxConvTaps) + "]");
+  std::unique_ptr<shainet_llama_block> b(new (std::nothrow) shainet_llama_block());
+  if (!b) return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
+  b->mixer = std::move(owned);
+  b->wrapped = true;
+  b->d_model = d_model;
+  b->eps = eps;
+  BlockWeights &w = *b->w;
+  w.taps = taps;
+  w.ff = std::move(owned_ff);
+  const size_t d = (size_t)d_model, conv = (size_t)taps * d;
+  const WantedBuffer wants[] = {{&w.norm1.gamma, d}, {&w.post1, d}, {&w.conv1, conv}, {&w.norm2.gamma, ff ? d : 0},
+                                {&w.post2, ff ? d : 0}, {&w.conv2, ff ? conv : 0}};
+  int rc = allocate_buffers(wants, 6);
+  if (!rc && taps > 1) rc = b->conv[0].allocate(conv - d);
+  if (!rc && taps > 1 && ff) rc = b->conv[1].allocate(conv - d);
+  if (rc) return rc;
+  *out = b.release();
+  return SHAINET_HIP_OK;
+}
+WrappedBlockBuffers shainet_llama_block_wrapped_buffers(shainet_llama_block *b) {
+  BlockWeights &w = *b->w;
+  return WrappedBlockBuffers{w.norm1.gamma, w.post1, w.conv1, w.norm2.gamma, w.post2, w.conv2};
+}
+Mixer *shainet_llama_block_mixer_of(shainet_llama_block *b) { return b->mixer.get(); }
 
 // One decode step of the whole stack in one launch (step_kernel.hip): where this block's weights,
 // parameters and cache are, with room for one more row made first (ensure_gpu_cache!,
 // llama_block.cr:497-520); *pos = rows cached so far.  The step's kernel appends the row;
 // shainet_llama_block_step_commit counts it afterwards.
 int shainet_llama_block_step_begin(shainet_llama_block *b, StepLayer *out, int *pos) {
-  if (int bad = latent_only(b, "one-launch decode step")) return bad;
+  if (int bad = grouped_only(b, "one-launch decode step")) return bad;
   shainet_llama_attn *l = b->attn;
   const BlockWeights &w = *b->w;
   if (!l->w_qkv || !l->w_o || !w.gate_up || !w.down) return fail(SHAINET_HIP_ERR_ARGUMENT, "weights not set");
@@ -519,7 +676,19 @@ bool shainet_llama_block_geometry(const shainet_llama_block *b, int *H, int *KV,
 
 // Forget the cached rows past `len` (generation that ran ahead of a stop token).
 int shainet_llama_block_truncate(shainet_llama_block *b, int len) {
-  if (b->latent) return shainet_kv_cache_truncate(latent_attn_cache(b->latent), 0, len);
+  if (b->wrapped) {
+    if (len == b->pos) return SHAINET_HIP_OK;
+    if (len == 0) return shainet_llama_block_clear_cache(b);
+    if (len != b->saved_pos) return fail(SHAINET_HIP_ERR_ARGUMENT, "a block with state can only go back to where it was saved");
+    if (int rc = b->mixer->truncate(len)) return rc;
+    const size_t bytes = (size_t)(b->w->taps - 1) * b->d_model * sizeof(float);
+    for (ConvState &c : b->conv)
+      if (bytes && c.saved && hipMemcpyAsync(c.rows[c.cur], c.saved, bytes, hipMemcpyDeviceToDevice, b->mixer->stream()) != hipSuccess)
+        return fail(SHAINET_HIP_ERR_RUNTIME, "hipMemcpyAsync(state) failed");
+    b->pos = len;
+    return SHAINET_HIP_OK;
+  }
+  if (b->mixer) return b->mixer->truncate(len);
   shainet_llama_attn *l = b->attn;
   if (len < 0 || len > l->cache_len) return fail(SHAINET_HIP_ERR_ARGUMENT, "truncate beyond the cached length");
   if (l->cache) {
@@ -531,8 +700,8 @@ int shainet_llama_block_truncate(shainet_llama_block *b, int len) {
 }
 // The model's kernels and its blocks' report a given-up wait into one word, the model's.
 void shainet_llama_block_share_error_word(shainet_llama_block *b, int *word) {
-  if (b->latent) {
-    latent_attn_share_error_word(b->latent, word);
+  if (b->mixer) {
+    b->mixer->share_error_word(word);
     return;
   }
   shainet_llama_attn *l = b->attn;
@@ -543,14 +712,13 @@ void shainet_llama_block_share_error_word(shainet_llama_block *b, int *word) {
   }
 }
 int shainet_llama_block_set_stream(shainet_llama_block *b, hipStream_t stream) {
-  shainet_attn_ctx *ctx = nullptr;
-  int rc = block_context(b, &ctx);
-  if (rc) return rc;
-  return shainet_attn_set_stream(ctx, (void *)stream);
+  if (b->mixer) return b->mixer->set_stream(stream);
+  const int rc = ensure_context(b->attn);
+  return rc ? rc : shainet_attn_set_stream(b->attn->ctx, (void *)stream);
 }
 // Room for `positions` positions in all, made ahead (a windowed mixer keeps what its window needs).
 int shainet_llama_block_reserve(shainet_llama_block *b, int positions) {
-  if (b->latent) return latent_attn_reserve(b->latent, positions);
+  if (b->mixer) return b->mixer->reserve(positions);
   const int rc = ensure_context(b->attn);
   return rc ? rc : shainet_kv_cache_reserve(b->attn->cache, positions);
 }
@@ -582,8 +750,7 @@ int shainet_llama_block_create(shainet_llama_block **out, int d_model, int num_h
 int shainet_llama_block_destroy(shainet_llama_block *b) {
   if (!b) return SHAINET_HIP_OK;
   shainet_llama_attn_destroy(b->attn);
-  latent_attn_destroy(b->latent);
-  for (DevF *f : {&b->x, &b->h, &b->hidden, &b->out}) f->release();
+  for (DevF *f : {&b->x, &b->h, &b->hidden, &b->out, &b->joined, &b->y}) f->release();
   b->x_pin.release();
   b->out_pin.release();
   delete b;
@@ -594,7 +761,7 @@ shainet_llama_attn *shainet_llama_block_attn(shainet_llama_block *b) { return b 
 
 int shainet_llama_block_set_norms(shainet_llama_block *b, const float *norm1, const float *norm2) {
   if (!b) return fail(SHAINET_HIP_ERR_ARGUMENT, "block is null");
-  if (int bad = latent_only(b, "shainet_llama_block_set_norms")) return bad;
+  if (int bad = grouped_only(b, "shainet_llama_block_set_norms")) return bad;
   if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
   int rc = SHAINET_HIP_OK;
   float **dst[2] = {&b->w->norm1.gamma, &b->w->norm2.gamma};
@@ -615,7 +782,7 @@ int shainet_llama_block_set_norms(shainet_llama_block *b, const float *norm1, co
 
 int shainet_llama_block_set_ffn(shainet_llama_block *b, const float *gate, const float *up, const float *down) {
   if (!b || !gate || !up || !down) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
-  if (int bad = latent_only(b, "shainet_llama_block_set_ffn")) return bad;
+  if (int bad = grouped_only(b, "shainet_llama_block_set_ffn")) return bad;
   if (!shainet_hip_available()) return fail(SHAINET_HIP_ERR_RUNTIME, "no gfx950 device available");
   const float *mats[2] = {gate, up};
   const int widths[2] = {b->ff_hidden, b->ff_hidden};
@@ -627,24 +794,52 @@ int shainet_llama_block_set_ffn(shainet_llama_block *b, const float *gate, const
 
 int shainet_llama_block_clear_cache(shainet_llama_block *b) {
   if (!b) return fail(SHAINET_HIP_ERR_ARGUMENT, "block is null");
-  if (b->latent) return shainet_kv_cache_clear(latent_attn_cache(b->latent), -1);
+  b->pos = 0;
+  b->saved_pos = -1;
+  if (b->mixer) return b->mixer->clear();
   return shainet_llama_attn_clear_cache(b->attn);
 }
 
 int shainet_llama_block_cache_len(const shainet_llama_block *b) {
-  if (b && b->latent) return shainet_kv_cache_len(latent_attn_cache(b->latent), 0);
+  if (b && b->wrapped) return b->pos;
+  if (b && b->mixer) return b->mixer->len();
   return b ? b->attn->cache_len : -1;
 }
 
 shainet_kv_cache *shainet_llama_block_cache(shainet_llama_block *b) {
   if (!b) return nullptr;
-  return b->latent ? latent_attn_cache(b->latent) : b->attn->cache;
+  return b->mixer ? b->mixer->cache() : b->attn->cache;
 }
 
 int shainet_llama_block_latent_config(shainet_llama_block *b, shainet_latent_config *cfg) {
   if (!b || !cfg) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
-  if (!b->latent) return fail(SHAINET_HIP_ERR_ARGUMENT, "this block's mixer is not latent attention");
-  *cfg = latent_attn_config(b->latent);
+  if (!b->mixer || !b->mixer->latent()) return fail(SHAINET_HIP_ERR_ARGUMENT, "this block's mixer is not latent attention");
+  *cfg = latent_attn_config(b->mixer->latent());
+  return SHAINET_HIP_OK;
+}
+
+int shainet_llama_block_mixer(shainet_llama_block *b) {
+  if (!b) return -1;
+  return !b->mixer             ? SHAINET_HIP_MIXER_GROUPED
+         : b->mixer->latent()  ? SHAINET_HIP_MIXER_LATENT
+         : b->mixer->biased()  ? SHAINET_HIP_MIXER_BIASED
+                               : SHAINET_HIP_MIXER_HGRN2;
+}
+
+int shainet_llama_block_read_state(shainet_llama_block *b, float *out, long long n) {
+  if (!b || !out) return fail(SHAINET_HIP_ERR_ARGUMENT, "null argument");
+  Hgrn2 *l = b->mixer ? b->mixer->hgrn2() : nullptr;
+  if (!l) return fail(SHAINET_HIP_ERR_ARGUMENT, "this block has no recurrent state");
+  const Hgrn2Config &c = hgrn2_config(l);
+  if (n != (long long)c.heads * c.dim * c.vdim)
+    return fail(SHAINET_HIP_ERR_ARGUMENT, "the state holds " + std::to_string((long long)c.heads * c.dim * c.vdim) + " floats");
+  if (b->pos == 0) {
+    memset(out, 0, (size_t)n * sizeof(float));
+    return SHAINET_HIP_OK;
+  }
+  if (hipStreamSynchronize(b->mixer->stream()) != hipSuccess ||
+      hipMemcpy(out, hgrn2_state(l), (size_t)n * sizeof(float), hipMemcpyDeviceToHost) != hipSuccess)
+    return fail(SHAINET_HIP_ERR_RUNTIME, "copying the state back failed");
   return SHAINET_HIP_OK;
 }
 
@@ -663,13 +858,12 @@ static int block_forward_any(shainet_llama_block *b, const float *x, int new_tok
   if (mem != SHAINET_HIP_MEM_HOST && mem != SHAINET_HIP_MEM_DEVICE)
     return fail(SHAINET_HIP_ERR_ARGUMENT, "mem must be SHAINET_HIP_MEM_HOST or SHAINET_HIP_MEM_DEVICE");
   if (mem == SHAINET_HIP_MEM_DEVICE) return block_forward_device(b, x, new_tokens, out, no_cache);
-  shainet_attn_ctx *ctx = nullptr;
-  int rc = block_context(b, &ctx);
+  hipStream_t stream = nullptr;
+  int rc = block_stream(b, &stream);
   if (rc) return rc;
   const size_t xd = (size_t)new_tokens * b->d_model;
   if (!b->x.reserve(xd) || !b->out.reserve(xd) || !b->x_pin.reserve(xd) || !b->out_pin.reserve(xd))
     return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
-  hipStream_t stream = (hipStream_t)shainet_attn_stream(ctx);
   memcpy(b->x_pin.p, x, xd * sizeof(float));
   if (hipMemcpyAsync(b->x.p, b->x_pin.p, xd * sizeof(float), hipMemcpyHostToDevice, stream) != hipSuccess)
     return fail(SHAINET_HIP_ERR_RUNTIME, "hipMemcpyAsync(x) failed");
@@ -681,7 +875,7 @@ static int block_forward_any(shainet_llama_block *b, const float *x, int new_tok
       hipStreamSynchronize(stream) != hipSuccess)
     return fail(SHAINET_HIP_ERR_RUNTIME, "copying the result back failed");
   memcpy(out, b->out_pin.p, xd * sizeof(float));
-  return check_error_word(shainet_attn_error_word(ctx));
+  return check_error_word(block_error_word(b));
 }
 
 }  // extern "C"

@@ -6,6 +6,7 @@
 #include <string>
 
 #include "../../include/shainet_hip_attn.h"
+#include "activation.hpp"
 
 // capi.hip: shainet_attn_forward with the rows of q, k and v at given strides
 int shainet_attn_forward_strided(shainet_attn_ctx *c, shainet_kv_cache *kc, const int *seq_ids,
@@ -38,6 +39,8 @@ int *shainet_attn_error_word(shainet_attn_ctx *c);
 namespace shainet {
 struct NormWeights;
 struct LatentAttn;
+struct Mixer;
+struct FeedForward;
 }
 struct LlamaBlockBuffers {
   float *w_qkv, *w_o, *gate_up, *down;  // w_qkv, w_o: null where the mixer is latent attention; gate_up, down: where there is no feed-forward
@@ -50,6 +53,21 @@ int shainet_llama_block_buffers(shainet_llama_block *b, LlamaBlockBuffers *out);
 int shainet_llama_block_create_latent(shainet_llama_block **out, int d_model, const shainet_latent_config &cfg,
                                       int ff_hidden, int norm_kind, double eps, const shainet_llama_block *weights_of);
 shainet::LatentAttn *shainet_llama_block_latent_mixer(shainet_llama_block *b);  // null: grouped-query attention
+// A block with norms behind its sublayers, too (RMS norms of d_model values), and a causal convolution over time
+// of `taps` taps in front of each; ff may be null.  The block takes over mixer and ff, also on failure.
+// Its buffers are there at once, for a loader to fill: norms [d], convolutions [taps, d], oldest row's tap first.
+int shainet_llama_block_create_wrapped(shainet_llama_block **out, int d_model, shainet::Mixer *mixer, shainet::FeedForward *ff,
+                                       int taps, double eps);
+struct WrappedBlockBuffers {
+  float *norm1, *post1, *conv1, *norm2, *post2, *conv2;  // the last three: null without a feed-forward
+};
+WrappedBlockBuffers shainet_llama_block_wrapped_buffers(shainet_llama_block *b);
+shainet::Mixer *shainet_llama_block_mixer_of(shainet_llama_block *b);  // null: the grouped-query attention of a LLaMA block
+// The result of such a block's last sublayer that has not joined the residual yet: the next block's first launch
+// does it (shainet_llama_block_forward_device), or shainet_llama_block_join_carry behind the last block.
+struct BlockCarry {
+  const float *y = nullptr, *post = nullptr;
+};
 // A model without blocks yet, and one more block for it (which it then owns), for loaders of designs
 // whose layers are not all alike.
 int shainet_llama_model_create_empty(shainet_llama_model **out, int vocab, int d_model, double eps,
@@ -60,6 +78,9 @@ struct LlamaModelBuffers {
   shainet::NormWeights *final_norm;
   float *lm_head;
 };
+// Position vectors [max_positions, d_model] that are added to the embedding rows: the buffer, allocated on first
+// request, for a loader to fill.  A sequence cannot outgrow them.
+int shainet_llama_model_position_buffer(shainet_llama_model *m, int max_positions, float **out);
 int shainet_llama_model_buffers(shainet_llama_model *m, LlamaModelBuffers *out);
 
 namespace shainet {
@@ -83,8 +104,10 @@ struct PinnedF {
 
 // What rides along with a projection y = x W.
 struct Fused {
-  int epilogue = 0;            // kGemvPlain, kGemvResidual (y = res + x W) or kGemvSwiglu (W = gate | up, [K, 2N])
+  int epilogue = 0;            // kGemvPlain, kGemvResidual (y = res + x W), kGemvSwiglu (W = gate | up, [K, 2N]) or kGemvBias
   const float *res = nullptr;  // [T, N]
+  const float *bias = nullptr;  // [N]: y = act(x W + bias)
+  Activation act;
   int norm = 0;                // kNorm*: applied to the rows of x first
   const float *gamma = nullptr;
   const float *beta = nullptr;  // kNormDynTanh
@@ -137,7 +160,7 @@ struct Projector {
   int reserve_flags(size_t n_flags, hipStream_t stream);
   // res != nullptr: y = res + x W
   int gemm(const float *x, long long x_stride, const float *w, float *y, int T, int K, int N, hipStream_t stream,
-           const float *res = nullptr);
+           const float *res = nullptr, const float *bias = nullptr, Activation act = Activation());
 };
 
 // Replace *dst (device, hipMalloc'ed or null) by a copy of n host floats.

@@ -24,7 +24,10 @@
 using namespace shainet;
 
 // llama_block.hip
-int shainet_llama_block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache);
+int shainet_llama_block_forward_device(shainet_llama_block *b, const float *x, int T, float *out, bool no_cache, BlockCarry *carry);
+int shainet_llama_block_join_carry(shainet_llama_block *b, const BlockCarry &carry, float *x, int T);
+bool shainet_llama_block_keeps_state(const shainet_llama_block *b);
+int shainet_llama_block_save_state(shainet_llama_block *b);
 int shainet_llama_block_set_stream(shainet_llama_block *b, hipStream_t stream);
 int shainet_llama_block_reserve(shainet_llama_block *b, int positions);
 int shainet_llama_block_truncate(shainet_llama_block *b, int len);
@@ -68,6 +71,8 @@ struct shainet_llama_model {
   std::vector<shainet_llama_block *> blocks;
   float *embedding = nullptr;   // device [vocab, d_model]
   float embedding_scale = 1.f;  // times every embedding row
+  float *positions = nullptr;   // device [max_positions, d_model], added to the embedding rows; null: none
+  int max_positions = 0;        // with positions: a sequence is at most this long
   NormWeights final_norm;       // has_final_norm says whether the step exists (@final_norm)
   bool has_final_norm = false;
   float *lm_head = nullptr;     // device [d_model, vocab]
@@ -119,6 +124,19 @@ int shainet_llama_model_buffers(shainet_llama_model *m, LlamaModelBuffers *out) 
   if (m->lm_bias) (void)hipFree(m->lm_bias);  // the loader's output bias is all zeros (hf_loader.cr:404)
   m->lm_bias = nullptr;
   *out = LlamaModelBuffers{m->embedding, &m->final_norm, m->lm_head};
+  return SHAINET_HIP_OK;
+}
+
+int shainet_llama_model_position_buffer(shainet_llama_model *m, int max_positions, float **out) {
+  if (max_positions < 1) return fail(SHAINET_HIP_ERR_ARGUMENT, "max_positions must be positive");
+  if (m->positions) (void)hipFree(m->positions);
+  m->positions = nullptr;
+  m->max_positions = max_positions;
+  if (hipMalloc((void **)&m->positions, (size_t)max_positions * m->d_model * sizeof(float)) != hipSuccess) {
+    m->positions = nullptr;
+    return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+  }
+  *out = m->positions;
   return SHAINET_HIP_OK;
 }
 
@@ -214,7 +232,7 @@ void plan_model_step(shainet_llama_model *m) {
     if (v >= 1 && v < st.n_wgs) st.n_wgs = v;
   }
   // the step kernel knows embedding rows as they are, grouped-query attention and RMSNorm
-  if (m->embedding_scale != 1.f || !shainet_llama_block_geometry(m->blocks[0], &st.H, &st.KV, &st.hd, &st.ff, &st.qk_eps)) return;
+  if (m->embedding_scale != 1.f || m->positions || !shainet_llama_block_geometry(m->blocks[0], &st.H, &st.KV, &st.hd, &st.ff, &st.qk_eps)) return;
   for (shainet_llama_block *b : m->blocks) {
     int H, KV, hd, ff;
     double qe;
@@ -340,13 +358,20 @@ int run_device_tokens(shainet_llama_model *m, const int *d_tokens, int T, bool n
       return fail(SHAINET_HIP_ERR_ARGUMENT, "this model's geometry does not fit the one-launch decode step");
   }
   if (rc < 0) {
-    hipError_t e = launch_embed(m->embedding, d_tokens, m->act[0].p, T, d, m->stream, m->embedding_scale);
+    const int start = no_cache ? 0 : shainet_llama_model_cache_len(m);
+    if (m->positions && (long long)start + T > m->max_positions)
+      return fail(SHAINET_HIP_ERR_CAPACITY, std::to_string(start) + " + " + std::to_string(T) + " positions: this model has " +
+                                                std::to_string(m->max_positions));
+    hipError_t e = launch_embed(m->embedding, d_tokens, m->act[0].p, T, d, m->stream, m->embedding_scale,
+                                m->positions ? m->positions + (size_t)start * d : nullptr);
     if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("embedding launch: ") + hipGetErrorString(e));
+    BlockCarry carry;
     for (shainet_llama_block *b : m->blocks) {
       if ((rc = shainet_llama_block_set_stream(b, m->stream))) return rc;
-      if ((rc = shainet_llama_block_forward_device(b, m->act[cur].p, T, m->act[cur ^ 1].p, no_cache))) return rc;
+      if ((rc = shainet_llama_block_forward_device(b, m->act[cur].p, T, m->act[cur ^ 1].p, no_cache, &carry))) return rc;
       cur ^= 1;
     }
+    if (carry.y && (rc = shainet_llama_block_join_carry(m->blocks.back(), carry, m->act[cur].p, T))) return rc;
   }
   // the final norm runs over every row in the reference; only the last one is used afterwards
   if ((rc = head_rows(m, m->act[cur].p + (size_t)(T - 1) * d, 1, m->logits.p))) return rc;
@@ -405,7 +430,7 @@ int shainet_llama_model_create(shainet_llama_model **out, int vocab, int d_model
 int shainet_llama_model_destroy(shainet_llama_model *m) {
   if (!m) return SHAINET_HIP_OK;
   for (shainet_llama_block *b : m->blocks) shainet_llama_block_destroy(b);
-  for (float *p : {m->embedding, m->final_norm.gamma, m->final_norm.beta, m->lm_head, m->lm_bias, m->d_vals, m->lm_head_t_own})
+  for (float *p : {m->embedding, m->final_norm.gamma, m->final_norm.beta, m->lm_head, m->lm_bias, m->d_vals, m->lm_head_t_own, m->positions})
     if (p) (void)hipFree(p);
   if (m->d_tokens) (void)hipFree(m->d_tokens);
   if (m->d_ids) (void)hipFree(m->d_ids);
@@ -560,9 +585,15 @@ int shainet_llama_model_generate_greedy(shainet_llama_model *m, int max_tokens, 
     m->topk_scratch_cap = need;
   }
   int host_ids[kChunk];
+  bool stateful = false;  // steps cannot be dropped from a state: it goes back to the chunk's beginning and takes the others again
+  for (shainet_llama_block *b : m->blocks) stateful = stateful || shainet_llama_block_keeps_state(b);
   while (*n_out < max_tokens) {
     const int steps = max_tokens - *n_out < kChunk ? max_tokens - *n_out : kChunk;
     const int len0 = shainet_llama_model_cache_len(m);
+    if (stateful && n_stop > 0) {
+      for (shainet_llama_block *b : m->blocks)
+        if (int rc = shainet_llama_block_save_state(b)) return rc;
+    }
     for (int i = 0; i < steps; ++i) {
       // best_id = Sampler.greedy(logits) into d_gen[i]; then net.run([best_id]) reading it from there
       hipError_t e = launch_topk(m->logits.p, m->vocab, 1, true, m->topk_scratch, m->d_gen + i, nullptr, nullptr,
@@ -581,9 +612,11 @@ int shainet_llama_model_generate_greedy(shainet_llama_model *m, int max_tokens, 
       if (stop) {
         // the device ran ahead: the caches keep the rows of the i tokens before the stop token
         for (shainet_llama_block *b : m->blocks) {
-          int rc = shainet_llama_block_truncate(b, len0 + i);
+          int rc = shainet_llama_block_truncate(b, stateful ? len0 : len0 + i);
           if (rc) return rc;
         }
+        for (int k = 0; stateful && k < i; ++k)
+          if (int rc = run_device_tokens(m, m->d_gen + k, 1)) return rc;
         m->have_logits = false;  // the row on the device belongs to a later position
         return SHAINET_HIP_OK;
       }

@@ -312,7 +312,31 @@ __global__ void legacy_append_kernel(const float *__restrict__ staging, float *_
   (is_v ? vc : kc)[dst] = staging[idx];
 }
 
+// A workgroup per new row: its key heads, then its value heads.
+__global__ __launch_bounds__(256) void append_rows_kernel(const float *__restrict__ rows, long long stride, long long k_off,
+                                                          long long v_off, float *__restrict__ kc, float *__restrict__ vc,
+                                                          int KV, int dim, int v_dim, int cap, int start_pos) {
+  const float *row = rows + blockIdx.x * stride;
+  const long long pos = start_pos + blockIdx.x;
+  const int nk = KV * dim, nv = KV * v_dim;
+  for (int i = threadIdx.x; i < nk + nv; i += 256) {
+    const bool is_v = i >= nk;
+    const int e = is_v ? i - nk : i, w = is_v ? v_dim : dim, h = e / w;
+    (is_v ? vc : kc)[((long long)h * cap + pos) * w + (e - h * w)] = row[(is_v ? v_off : k_off) + e];
+  }
+}
+
 }  // namespace
+
+hipError_t launch_append_rows(const float *rows, long long stride, long long k_off, long long v_off, int T, float *kc, float *vc,
+                              int KV, int dim, int v_dim, int cap, int start_pos, hipStream_t stream) {
+  if (!rows || !kc || !vc || T < 1 || KV < 1 || dim < 1 || v_dim < 1 || start_pos < 0 || (long long)start_pos + T > cap ||
+      (long long)KV * (dim + v_dim) > 0x7fffffffLL)
+    return hipErrorInvalidValue;
+  hipLaunchKernelGGL(append_rows_kernel, dim3((unsigned)T), dim3(256), 0, stream, rows, stride, k_off, v_off, kc, vc, KV, dim,
+                     v_dim, cap, start_pos);
+  return hipGetLastError();
+}
 
 hipError_t launch_prep(const PrepArgs &a, const SeqTable &st, const Shape &sh, int total_tokens,
                        hipStream_t stream, const DecodeDevicePlan *dev) {

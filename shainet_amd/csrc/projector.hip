@@ -117,13 +117,13 @@ int Projector::reserve_flags(size_t n_flags, hipStream_t stream) {
 
 // y = (res +) x W with the library's own MFMA kernel; res == y is allowed.
 int Projector::gemm(const float *x, long long x_stride, const float *w, float *y, int T, int K, int N,
-                    hipStream_t stream, const float *res) {
+                    hipStream_t stream, const float *res, const float *bias, Activation act) {
   const GemmPlan p = plan_gemm(T, K, N, x_stride);
   if (!scratch.reserve(p.partial_floats)) return llama_fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
   if (int rc = reserve_flags(p.flag_words, stream)) return rc;
   if (p.flag_words && !error) return llama_fail(SHAINET_HIP_ERR_RUNTIME, "the projector has no error word");
   hipError_t e = launch_gemm(x, x_stride, w, y, res, scratch.p, flags, error, T, K, N, p, stream,
-                             lose_marks ? flags + flags_cap : nullptr, lose_marks ? 2000 : 0);
+                             lose_marks ? flags + flags_cap : nullptr, lose_marks ? 2000 : 0, bias, act);
   if (e != hipSuccess) return llama_fail(SHAINET_HIP_ERR_RUNTIME, std::string("gemm launch: ") + hipGetErrorString(e));
   return SHAINET_HIP_OK;
 }
@@ -144,6 +144,8 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
     a.eps = f.eps;
     a.w = f.w_t;
     a.res = f.res;
+    a.bias = f.bias;
+    a.act = f.act;
     a.y = y;
     a.T = T;
     a.K = K;
@@ -182,6 +184,8 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
     a.eps = f.eps;
     a.w = w;
     a.res = f.res;
+    a.bias = f.bias;
+    a.act = f.act;
     a.y = y;
     a.partials = scratch.p;
     a.flags = flags;
@@ -218,7 +222,8 @@ int Projector::project(const float *x, long long x_stride, const float *w, float
     if (e != hipSuccess) return llama_fail(SHAINET_HIP_ERR_RUNTIME, std::string("epilogue launch: ") + hipGetErrorString(e));
     return SHAINET_HIP_OK;
   }
-  return gemm(xin, xs, w, y, T, K, N, stream, f.epilogue == kGemvResidual ? f.res : nullptr);
+  return gemm(xin, xs, w, y, T, K, N, stream, f.epilogue == kGemvResidual ? f.res : nullptr,
+              f.epilogue == kGemvBias ? f.bias : nullptr, f.act);
 }
 
 void Projector::release() {

@@ -115,6 +115,8 @@ _SIGNATURES = {
     "shainet_hf_load_llama": (C.c_int, [C.c_char_p, C.POINTER(C.c_void_p)]),
     "shainet_hf_load_model": (C.c_int, [C.c_char_p, C.POINTER(C.c_void_p)]),
     "shainet_llama_block_latent_config": (C.c_int, [C.c_void_p, C.c_void_p]),
+    "shainet_llama_block_mixer": (C.c_int, [C.c_void_p]),
+    "shainet_llama_block_read_state": (C.c_int, [C.c_void_p, _f32p, C.c_longlong]),
     "shainet_llama_block_cache": (C.c_void_p, [C.c_void_p]),
     "shainet_llama_model_vocab": (C.c_int, [C.c_void_p]),
     "shainet_llama_model_d_model": (C.c_int, [C.c_void_p]),
@@ -700,14 +702,19 @@ class _LatentConfig(C.Structure):
                [("rot_base", C.c_double), ("scale", C.c_double)]
 
 
-class LatentBlock:
-    """A block whose mixer is latent attention, owned by the LlamaModel that `HFLoader.load_model` made."""
+class DesignBlock:
+    """A block of a design that the library's loader made, owned by the LlamaModel `HFLoader.load_model` returns."""
+
+    GROUPED, LATENT, BIASED, HGRN2 = range(4)
 
     def __init__(self, d_model, handle):
         self.d_model, self._block = d_model, C.c_void_p(handle)
-        cfg = _LatentConfig()
-        _check(lib().shainet_llama_block_latent_config(self._block, C.byref(cfg)))
-        self.config = {name: getattr(cfg, name) for name, _ in _LatentConfig._fields_}
+        self.mixer = lib().shainet_llama_block_mixer(self._block)
+
+    @staticmethod
+    def of(d_model, handle):
+        kind = lib().shainet_llama_block_mixer(C.c_void_p(handle))
+        return (LatentBlock if kind == DesignBlock.LATENT else DesignBlock)(d_model, handle)
 
     def close(self):
         self._block = None
@@ -721,21 +728,20 @@ class LatentBlock:
 
     @property
     def cache_capacity(self):
-        """Rows the block's cache has room for; a window keeps it from growing with the sequence."""
-        return lib().shainet_kv_cache_capacity(lib().shainet_llama_block_cache(self._block))
+        """Rows the block's cache has room for (None: a state takes its place)."""
+        cache = lib().shainet_llama_block_cache(self._block)
+        return lib().shainet_kv_cache_capacity(cache) if cache else None
 
-    def cache_rows(self, pos0, n):
-        """Cached rows [n, kv_rank + rot_dim] of positions pos0 .. pos0 + n - 1 (the ones still held)."""
+    def state(self, heads, dim, vdim):
+        """The recurrent state [heads, dim, vdim] of a block whose mixer is HGRN2."""
         import numpy as np
 
-        width = self.config["kv_rank"] + self.config["rot_dim"]
-        out = np.empty((n, (width + 15) // 16 * 16), np.float32)
-        _check(lib().shainet_kv_cache_read(lib().shainet_llama_block_cache(self._block), 0, 0, pos0, n,
-                                           out.ctypes.data_as(_f32p), None))
-        return out[:, :width]
+        out = np.empty((heads, dim, vdim), np.float32)
+        _check(lib().shainet_llama_block_read_state(self._block, out.ctypes.data_as(_f32p), out.size))
+        return out
 
     def forward_cached(self, x, _fn="shainet_llama_block_forward_cached"):
-        """numpy [T, d_model] -> numpy, the rows appended behind the cached ones."""
+        """numpy [T, d_model] -> numpy, the rows behind the ones before."""
         import numpy as np
 
         x = np.ascontiguousarray(x, np.float32)
@@ -746,8 +752,28 @@ class LatentBlock:
         return out
 
     def forward(self, x):
-        """The rows among themselves from position 0; the cache is left as it is."""
+        """The rows among themselves from position 0; what the block keeps is left as it is."""
         return self.forward_cached(x, _fn="shainet_llama_block_forward")
+
+
+class LatentBlock(DesignBlock):
+    """A block whose mixer is latent attention; a window keeps its cache from growing with the sequence."""
+
+    def __init__(self, d_model, handle):
+        super().__init__(d_model, handle)
+        cfg = _LatentConfig()
+        _check(lib().shainet_llama_block_latent_config(self._block, C.byref(cfg)))
+        self.config = {name: getattr(cfg, name) for name, _ in _LatentConfig._fields_}
+
+    def cache_rows(self, pos0, n):
+        """Cached rows [n, kv_rank + rot_dim] of positions pos0 .. pos0 + n - 1 (the ones still held)."""
+        import numpy as np
+
+        width = self.config["kv_rank"] + self.config["rot_dim"]
+        out = np.empty((n, (width + 15) // 16 * 16), np.float32)
+        _check(lib().shainet_kv_cache_read(lib().shainet_llama_block_cache(self._block), 0, 0, pos0, n,
+                                           out.ctypes.data_as(_f32p), None))
+        return out[:, :width]
 
 
 class LlamaModel:
@@ -776,7 +802,7 @@ class LlamaModel:
         L = lib()
         self.vocab, self.d_model = L.shainet_llama_model_vocab(handle), L.shainet_llama_model_d_model(handle)
         self.n_layers = L.shainet_llama_model_layers(handle)
-        self.blocks = [LatentBlock(self.d_model, L.shainet_llama_model_block(handle, i)) for i in range(self.n_layers)]
+        self.blocks = [DesignBlock.of(self.d_model, L.shainet_llama_model_block(handle, i)) for i in range(self.n_layers)]
         return self
 
     def close(self):
