@@ -422,8 +422,8 @@ TUTILORN_SIZES = [
     ("w2048", 2048, 8192, 6, 32000, (16, 128, 64, 128, 512, 1024, 4096), (32, 8, 64)),
     ("w4096", 4096, 8192, 4, 32000, (32, 128, 64, 128, 512, 1536, 4096), (32, 8, 128)),
 ]
-TUTILORN_PREFILL = (512, 2048, 8192)
-TUTILORN_DECODE = (512, 4096)
+DESIGN_PREFILL = (512, 2048, 8192)
+DESIGN_DECODE = (512, 4096)
 
 
 def tutilorn_folder(torch, folder, width, ff, layers, vocab, mix):
@@ -515,31 +515,134 @@ def model_rates(np, m, vocab, steps, warmup, prefill, decode):
     return out
 
 
-def tutilorn_bench(sa, np, torch, steps, warmup, only):
-    """The --tutilorn line: every size of TUTILORN_SIZES (or those named by --only), both designs."""
+# --zabutar: the same for that design.  name, width, dense ff, layers (a period of four: HGRN2 with a dense
+# feed-forward, HGRN2, attention and attention over the layer before's keys with experts), vocab, HGRN2 (heads, dim, vdim),
+# attention (q heads, kv heads, dim, vdim, bias_max, table rows), experts (ff, experts, identity, top, groups, keep, shared ff)
+ZABUTAR_SIZES = [
+    ("w1024", 1024, 4096, 8, 32000, (8, 128, 128), (16, 8, 64, 64, 240, 32), (512, 24, 8, 6, 4, 3, 1024), (16, 8, 64)),
+    ("w2048", 2048, 8192, 8, 32000, (16, 128, 128), (32, 8, 64, 64, 240, 32), (768, 24, 8, 8, 4, 3, 2048), (32, 8, 64)),
+    ("w4096", 4096, 8192, 4, 32000, (32, 128, 128), (32, 8, 128, 128, 240, 32), (1024, 12, 4, 4, 4, 3, 4096), (32, 8, 128)),
+]
+
+
+def zabutar_folder(torch, folder, width, ff, layers, vocab, rec, att, ex):
+    """A checkpoint folder of that size with seeded random weights in bfloat16; weight bytes one token reads (as fp32,
+    with the share of the chosen experts that a uniform router gives real experts)."""
+    from safetensors.torch import save_file
+
+    gen = torch.Generator(device="cuda").manual_seed(6)
+    w = {}
+
+    def put(name, *shape, g=None, plus=0.0):
+        a = torch.randn(shape, generator=gen, device="cuda") * (shape[-1] ** -0.5 if g is None else g) + plus
+        w[name] = a.to(torch.bfloat16).cpu()
+
+    def expert(p, n):
+        for name, o, k in (("gate", n, width), ("up", n, width), ("down", width, n)):
+            put(p + name, o, k)
+
+    rh, rd, rv = rec
+    H, KV, dim, vd, far, rows = att
+    eff, E, ident, top, groups, keep, sff = ex
+    put("embed", vocab, width, g=1.0)
+    put("pos", 16384, width, g=0.5)
+    specs, read = [], width * vocab
+    for i in range(layers):
+        p, kind = f"l{i}.", i % 4
+        for n in ("norm1", "norm2", "norm1b", "norm2b"):
+            put(p + n, width, g=0.1)
+        for n in ("canon1", "canon2"):
+            put(p + n, width, 4, g=0.3)
+        if kind < 2:
+            m = {"heads": rh, "dim": rd, "vdim": rv}
+            for n, o in (("q", rh * rd), ("f", rh * rd), ("v", rh * rv)):
+                put(p + "mix." + n, o, width)
+            put(p + "mix.f.b", rh * rd, g=1.0, plus=2.0)
+            w[p + "mix.lower"] = torch.linspace(0, 0.95, rh * rd).to(torch.bfloat16)
+            put(p + "mix.norm", rv, g=0.1, plus=1.0)
+            put(p + "mix.o", width, rh * rv)
+            read += width * rh * (2 * rd + 2 * rv)
+        else:
+            m = {"heads": H, "kv_heads": KV, "dim": dim, "vdim": vd, "scale": dim ** -0.5, "bias_max": far}
+            if kind == 3:
+                m["kv_from"] = i - 1
+            for n, o in (("q", H * dim), ("k", KV * dim), ("v", KV * vd))[:1 if kind == 3 else 3]:
+                put(p + "mix." + n, o, width)
+                read += o * width
+            put(p + "mix.rel", rows, H, g=1.0)
+            put(p + "mix.o", width, H * vd)
+            read += width * H * vd
+        if kind == 0:
+            mlp = {"kind": "dense", "ff": ff}
+            put(p + "mlp.up", ff, width)
+            put(p + "mlp.down", width, ff)
+            put(p + "mlp.up.b", ff, g=0.1)
+            put(p + "mlp.down.b", width, g=0.1)
+            put(p + "mlp.act", 2, g=0.5)
+            read += 2 * width * ff
+        else:
+            mlp = {"kind": "moe", "expert": {"ff": eff}, "shared": {"ff": sff},
+                   "router": {"experts": E, "identity": ident, "top": top, "scale": 1.5, "groups": {"count": groups, "keep": keep}}}
+            put(p + "mlp.router", E + ident, width)
+            put(p + "mlp.correction", E + ident, g=0.02)
+            for e in range(E):
+                expert(p + f"mlp.e{e}.", eff)
+            expert(p + "mlp.shared.", sff)
+            read += width * (E + ident) + 3 * width * sff + 3 * width * eff * top * E // (E + ident)
+        specs.append({"type": "hgrn2" if kind < 2 else "attention", "mixer": m, "mlp": mlp})
+    put("final.norm", width, g=0.1)
+    put("head", vocab, width)
+    save_file(w, os.path.join(folder, "model.safetensors"))
+    cfg = {"architecture": "Zabutar", "vocab": vocab, "width": width, "max_positions": 16384, "norm": {"eps": 1e-6},
+           "canon": {"taps": 4}, "layers": specs}
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    return 4 * read
+
+
+def zabutar_sizes():
+    for name, width, ff, layers, vocab, rec, att, ex, heads in ZABUTAR_SIZES:
+        info = {"width": width, "ff": ff, "layers": layers, "vocab": vocab, "hgrn2_heads_dim_vdim": list(rec),
+                "attention_heads_kv_dim_vdim_biasmax_rows": list(att), "experts_ff_n_identity_top_groups_keep_sharedff": list(ex),
+                "llama_heads_kv_hd": list(heads)}
+        yield name, info, heads, lambda torch, folder, a=(width, ff, layers, vocab, rec, att, ex): zabutar_folder(torch, folder, *a)
+
+
+def tutilorn_sizes():
+    for name, width, ff, layers, vocab, mix, heads in TUTILORN_SIZES:
+        info = {"width": width, "ff": ff, "layers": layers, "vocab": vocab, "window": mix[-1],
+                "heads_dim_rot_vdim_kvrank_qrank": list(mix[:-1]), "llama_heads_kv_hd": list(heads)}
+        yield name, info, heads, lambda torch, folder, a=(width, ff, layers, vocab, mix): tutilorn_folder(torch, folder, *a)
+
+
+def design_bench(sa, np, torch, design, sizes, steps, warmup, only):
+    """The line of --tutilorn or --zabutar: every size (or those named by --only; "name/design" and "name/llama": one
+    side of it), the design and a LLaMA-family model of the same width, feed-forward, depth and vocabulary."""
     import tempfile
 
-    sizes = {}
-    for name, width, ff, layers, vocab, mix, heads in TUTILORN_SIZES:
-        if only and name not in only:
-            continue
-        with tempfile.TemporaryDirectory() as folder:
-            nbytes = tutilorn_folder(torch, folder, width, ff, layers, vocab, mix)
-            m = sa.HFLoader.load_model(folder)
-        torch.cuda.empty_cache()
-        res = {"config": {"width": width, "ff": ff, "layers": layers, "vocab": vocab, "window": mix[-1],
-                          "heads_dim_rot_vdim_kvrank_qrank": list(mix[:-1]), "llama_heads_kv_hd": list(heads)}}
-        for key in ("tutilorn", "llama"):
+    out = {}
+    for name, info, heads, folder_of in sizes:
+        res = {"config": info}
+        for key in (design, "llama"):
+            if only and name not in only and "%s/%s" % (name, key) not in only:
+                continue
             if key == "llama":
-                m, nbytes = llama_of_size(sa, np, width, ff, layers, vocab, heads)
-            res[key] = {k: round(v, 2) for k, v in model_rates(np, m, vocab, steps, warmup, TUTILORN_PREFILL, TUTILORN_DECODE).items()}
+                m, nbytes = llama_of_size(sa, np, info["width"], info["ff"], info["layers"], info["vocab"], heads)
+            else:
+                with tempfile.TemporaryDirectory() as folder:
+                    nbytes = folder_of(torch, folder)
+                    m = sa.HFLoader.load_model(folder)
+                torch.cuda.empty_cache()
+            print("size %s: %s loaded" % (name, key), file=sys.stderr, flush=True)
+            res[key] = {k: round(v, 2) for k, v in model_rates(np, m, info["vocab"], steps, warmup, DESIGN_PREFILL, DESIGN_DECODE).items()}
             res[key]["weight_bytes_per_token"] = nbytes
-            us = res[key]["decode_ctx%d_us_per_token" % TUTILORN_DECODE[0]]
+            us = res[key]["decode_ctx%d_us_per_token" % DESIGN_DECODE[0]]
             res[key]["decode_frac_of_hbm_peak"] = round(nbytes / us / 1e3 / HBM_PEAK_GBPS, 4)
             m.close()
-        sizes[name] = res
-        print("size %s done" % name, file=sys.stderr, flush=True)
-    print(json.dumps({"tutilorn": sizes, "steps": steps, "warmup": warmup, "dtype": "f32", "data": "synthetic"}))
+            print("size %s: %s done" % (name, key), file=sys.stderr, flush=True)
+        if len(res) > 1:
+            out[name] = res
+    print(json.dumps({design: out, "steps": steps, "warmup": warmup, "dtype": "f32", "data": "synthetic"}))
 
 
 # The kernels the two roofline objects of the bench line price, and the workloads they are priced on.
@@ -650,6 +753,8 @@ def main():
                     help="run only the plain copy/read kernels of known size (counter and bandwidth yardstick)")
     ap.add_argument("--tutilorn", action="store_true",
                     help="run only the Tutilorn models and the LLaMA-family models of their sizes (--only: names of sizes)")
+    ap.add_argument("--zabutar", action="store_true",
+                    help="run only the Zabutar models and the LLaMA-family models of their sizes (--only: names of sizes)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this path is built and measured on one GPU only (sequences, kv heads and context "
@@ -670,7 +775,10 @@ def main():
         return
 
     if args.tutilorn:
-        tutilorn_bench(sa, np, torch, args.steps, args.warmup, set(filter(None, args.only.split(","))))
+        design_bench(sa, np, torch, "tutilorn", tutilorn_sizes(), args.steps, args.warmup, set(filter(None, args.only.split(","))))
+        return
+    if args.zabutar:
+        design_bench(sa, np, torch, "zabutar", zabutar_sizes(), args.steps, args.warmup, set(filter(None, args.only.split(","))))
         return
 
     K, W = args.steps, args.warmup
