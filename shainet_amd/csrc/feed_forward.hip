@@ -40,13 +40,13 @@ struct Dense : FeedForward {
 struct Moe : FeedForward {
   MoeShape m = {};
   MoeWeights w;
-  DevF scratch, hidden;
+  DevF scratch, hidden, logits;
   int *counts = nullptr;
   ~Moe() override {
-    scratch.release();
-    hidden.release();
+    for (DevF *f : {&scratch, &hidden, &logits}) f->release();
     if (counts) (void)hipFree(counts);
-    for (float *p : {w.router, w.correction, w.gate_up, w.down, w.shared_gate_up, w.shared_down, w.shared_gate_up_in, w.shared_down_in})
+    for (float *p : {w.router, w.router_in, w.correction, w.gate_up, w.down, w.shared_gate_up, w.shared_down, w.shared_gate_up_in,
+                     w.shared_down_in})
       if (p) (void)hipFree(p);
   }
   int forward(Projector &proj, const float *h, int T, float *y, hipStream_t stream) override {
@@ -69,8 +69,10 @@ struct Moe : FeedForward {
         if (int rc = proj.project(hp, m.d, w.shared_gate_up_in, hidden.p, n, m.d, m.shared_ff, stream, gate)) return rc;
         if (int rc = proj.project(hidden.p, m.shared_ff, w.shared_down_in, yp, n, m.shared_ff, m.d, stream)) return rc;
       }
-      if (!scratch.reserve(moe_many_floats(m, n))) return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
-      e = launch_moe_many(m, t, hp, yp, m.shared_ff > 0, n, scratch.p, counts, stream);
+      if (!scratch.reserve(moe_many_floats(m, n)) || !logits.reserve((size_t)n * w.n_router))
+        return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+      if (int rc = proj.project(hp, m.d, w.router_in, logits.p, n, m.d, w.n_router, stream)) return rc;
+      e = launch_moe_many(m, t, hp, logits.p, w.n_router, yp, m.shared_ff > 0, n, scratch.p, counts, stream);
       if (e != hipSuccess) return fail(SHAINET_HIP_ERR_RUNTIME, std::string("expert launch: ") + hipGetErrorString(e));
     }
     return SHAINET_HIP_OK;
@@ -105,10 +107,13 @@ int moe_create(FeedForward **out, const MoeShape &m, MoeWeights **weights) {
   if (!f) return fail(SHAINET_HIP_ERR_ALLOC, "out of host memory");
   f->m = m;
   const size_t d = (size_t)m.d, n = (size_t)m.experts + m.identity, e = (size_t)m.experts * d * m.ff, s = d * m.shared_ff;
-  const WantedBuffer wants[] = {{&f->w.router, n * d},        {&f->w.correction, n},  {&f->w.gate_up, 2 * e},
+  f->w.n_router = (int)((n + 3) / 4 * 4);
+  const WantedBuffer wants[] = {{&f->w.router_in, d * f->w.n_router}, {&f->w.router, n * d}, {&f->w.correction, n},  {&f->w.gate_up, 2 * e},
                                 {&f->w.down, e},              {&f->w.shared_gate_up, 2 * s}, {&f->w.shared_down, s},
                                 {&f->w.shared_gate_up_in, 2 * s}, {&f->w.shared_down_in, s}};
-  int rc = allocate_buffers(wants, 8);
+  int rc = allocate_buffers(wants, 9);
+  // (the columns past the last output are never filled by a loader)
+  if (!rc && hipMemset(f->w.router_in, 0, d * f->w.n_router * sizeof(float)) != hipSuccess) rc = fail(SHAINET_HIP_ERR_RUNTIME, "hipMemset failed");
   if (!rc && hipMalloc((void **)&f->counts, (size_t)m.experts * sizeof(int)) != hipSuccess) {
     f->counts = nullptr;
     rc = fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");

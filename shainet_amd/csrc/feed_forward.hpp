@@ -20,10 +20,12 @@ struct DenseWeights {
 };
 int dense_create(FeedForward **out, int d_model, int ff, DenseWeights **weights);
 
-// moe_kernels.hpp; expert and router matrices as [out, in].  The shared expert's are kept both ways round: many
-// tokens take it through the ordinary products.
+// moe_kernels.hpp; expert matrices as [out, in].  The router's and the shared expert's are kept both ways round: many
+// tokens take them through the ordinary products.
 struct MoeWeights {
   float *router = nullptr, *correction = nullptr, *gate_up = nullptr, *down = nullptr;
+  float *router_in = nullptr;                                     // [d, n_router], zero columns up to a multiple of 4
+  int n_router = 0;
   float *shared_gate_up = nullptr, *shared_down = nullptr;        // [2 ff, d], [d, ff]
   float *shared_gate_up_in = nullptr, *shared_down_in = nullptr;  // [d, 2 ff], [ff, d]
 };

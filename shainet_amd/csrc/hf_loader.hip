@@ -773,6 +773,7 @@ int load_experts(const shainet_safetensors *st, Stager &stage, const std::string
   const size_t mat = (size_t)m.ff * m.d;
   int rc;
   if ((rc = load_plain(st, stage, p + "router", n, m.d, w.router))) return rc;
+  if ((rc = load_transposed(st, stage, p + "router", n, m.d, w.router_in, w.n_router, 0))) return rc;
   if ((rc = load_plain(st, stage, p + "correction", 1, n, w.correction))) return rc;
   for (int e = 0; e < m.experts; ++e) {
     const std::string pe = p + "e" + std::to_string(e) + ".";

@@ -21,12 +21,13 @@ constexpr int kMaxLds = 160 * 1024;
 constexpr int kChunksAtOnce = 64;
 
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
-__device__ __forceinline__ float sigmoid1(float z) { return 1.f / (1.f + expf(-z)); }
-__device__ __forceinline__ float silu1(float z) { return z / (1.f + expf(-z)); }
+// (the hardware's reciprocal is good to the last bit or so; the argument is at least 1)
+__device__ __forceinline__ float silu1(float z) { return z * __builtin_amdgcn_rcpf(1.f + expf(-z)); }
 // f and 1 - f, each to full precision
 __device__ __forceinline__ void gate(float z, float l, float &f, float &k) {
-  f = l + (1.f - l) * sigmoid1(z);
-  k = (1.f - l) * sigmoid1(-z);
+  const float e = expf(-fabsf(z)), r = __builtin_amdgcn_rcpf(1.f + e), lo = e * r;  // sigmoid(|z|) and sigmoid(-|z|)
+  f = l + (1.f - l) * (z >= 0.f ? r : lo);
+  k = (1.f - l) * (z >= 0.f ? lo : r);
 }
 
 // ---- one row after the other -------------------------------------------------------------------
@@ -113,14 +114,16 @@ __global__ __launch_bounds__(1024) void hgrn2_step_kernel(const Hgrn2Args a) {
 }
 
 // ---- chunks ------------------------------------------------------------------------------------
-// The gates of one channel over the kSub rows from `first` on: body(i, f, k), f = 1 and k = 0 past the end.
-template <class F>
-__device__ __forceinline__ void walk_gates(const Hgrn2Args &a, int i, int first, F body) {
-  const float *z = a.raw + (long long)a.H * a.dim + i;
-  const float b = a.f_bias[i], l = a.lower[i];
-  float x[kSub];
+// Column `col` of the kSub rows from `first` on (rows past the end repeat the last one).
+__device__ __forceinline__ void load_column(const Hgrn2Args &a, long long col, int first, float (&x)[kSub]) {
 #pragma unroll
-  for (int r = 0; r < kSub; ++r) x[r] = z[(long long)min(first + r, a.T - 1) * a.stride];
+  for (int r = 0; r < kSub; ++r) x[r] = a.raw[(long long)min(first + r, a.T - 1) * a.stride + col];
+}
+
+// The gates of one channel over the kSub rows from `first` on, made of x: body(r, f, k), f = 1 and k = 0 past the end.
+template <class F>
+__device__ __forceinline__ void walk_gates(const Hgrn2Args &a, int i, int first, const float (&x)[kSub], F body) {
+  const float b = a.f_bias[i], l = a.lower[i];
 #pragma unroll
   for (int r = 0; r < kSub; ++r) {
     float f, k;
@@ -145,7 +148,9 @@ __global__ __launch_bounds__(256) void hgrn2_chunk_kernel(const Hgrn2Args a, int
     const int j = it / d32, d = it - j * d32;
     float k_[kSub], f_[kSub];
     if (d < dim) {
-      walk_gates(a, h * dim + d, first + j * kSub, [&](int r, float f, float k) {
+      float x[kSub];
+      load_column(a, (long long)a.H * dim + h * dim + d, first + j * kSub, x);
+      walk_gates(a, h * dim + d, first + j * kSub, x, [&](int r, float f, float k) {
         f_[r] = f;
         k_[r] = k;
       });
@@ -166,14 +171,13 @@ __global__ __launch_bounds__(256) void hgrn2_chunk_kernel(const Hgrn2Args a, int
   }
   __syncthreads();
   const long long at = (long long)c * a.H + h;
-  for (int d = threadIdx.x; d < d32; d += 256) {
+  for (int it = threadIdx.x; it < NS * d32; it += 256) {
+    const int j = it / d32, d = it - j * d32;
     float later = 1.f;
-    for (int j = NS - 1; j >= 0; --j) {
-      if (j < NS - 1)
-        for (int r = 0; r < kSub; ++r) kd[(j * kSub + r) * d32 + d] *= later;
-      later *= tot[j * d32 + d];
-    }
-    if (d < dim) decay[at * dim + d] = later;
+    for (int b = NS - 1; b > j; --b) later *= tot[b * d32 + d];
+#pragma unroll
+    for (int r = 0; r < kSub; ++r) kd[(j * kSub + r) * d32 + d] *= later;
+    if (j == 0 && d < dim) decay[at * dim + d] = later * tot[d];
   }
   __syncthreads();
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -253,8 +257,9 @@ __global__ __launch_bounds__(256) void hgrn2_scan_kernel(float *__restrict__ sta
 
 // The rows of one chunk of one head: eight wavefronts.  In LDS, per row and channel: q, k = 1 - f and L, the
 // log2 of the gates' product from the beginning of the row's sub-chunk of 16 up to the row itself.
-//   within a sub-chunk   P[t][s] = sum_d q_t k_s 2^(L_t - L_s), a thread per pair
-//   between sub-chunks   the same sum as a product of (q_t 2^(L_t + what lies between)) and (k_s 2^(total - L_s))
+//   within eight rows    P[t][s] = sum_d q_t k_s 2^(L_t - L_s), a thread per pair
+//   further apart        the same sum as a product of two matrices, q_t and k_s each decayed to a row between them:
+//                        the end of a sub-chunk's first eight rows, or the end of the key's sub-chunk
 //   o_t = sum_s P[t][s] v_s + (q_t 2^(L_t + what came before)) S, S the state in front of the chunk
 // NT: tiles of 32 value columns per wavefront.
 template <int C, int NT>
@@ -267,13 +272,47 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
   float *qs = smem, *ks = qs + PR * ds, *ls = ks + C * ds, *P = ls + C * ds, *tot = P + PR * PS;  // tot: [NS][d16]
   const int h = blockIdx.x % a.H, c = blockIdx.x / a.H, first = (chunk0 + c) * C;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int n = lane & 31, half = lane >> 5;
+  const int rt = wave % RT, cg = wave / RT, n_vt = (vdim + 31) / 32;
+  const float *start = starts + ((long long)c * a.H + h) * dim * vdim;
+  const float *v0 = a.raw + 2LL * a.H * dim + (long long)h * vdim;
+  // what the last part needs of memory is asked for at the beginning: rows of the state (SB k steps of 8) and of the values
+  constexpr int SB = NT == 1 ? 16 : 4, VB = C / 8;
+  float xs[SB][4], xv[VB][4];
+  auto load_s = [&](float (&y)[4], int col, int k0) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) y[i] = start[(long long)min(k0 + 4 * half + i, dim - 1) * vdim + col];
+  };
+  auto load_tile = [&](int vt) {
+    const int col = min(vt * 32 + n, vdim - 1);
+#pragma unroll
+    for (int b = 0; b < SB; ++b)
+      if (8 * b < d16) load_s(xs[b], col, 8 * b);
+#pragma unroll
+    for (int b = 0; b < VB; ++b)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) xv[b][i] = v0[(long long)min(first + 8 * b + 4 * half + i, a.T - 1) * a.stride + col];
+  };
+  float z[kSub], q[kSub];
+  auto load_gates = [&](int it) {
+    const int j = it / d16, i = h * dim + min(it - j * d16, dim - 1);
+    load_column(a, (long long)a.H * dim + i, first + j * kSub, z);
+    load_column(a, i, first + j * kSub, q);
+  };
+  // (loads come back in order: what is needed first goes first)
+  if ((int)threadIdx.x < NS * d16) load_gates(threadIdx.x);
+  if (cg < n_vt) load_tile(cg);
 
   for (int it = threadIdx.x; it < NS * d16; it += 512) {
     const int j = it / d16, d = it - j * d16;
     float L = 0.f;
+    if (it >= 512) load_gates(it);
+#pragma unroll
+    for (int r = 0; r < kSub; ++r)
+      qs[(j * kSub + r) * ds + d] = d < dim && first + j * kSub + r < a.T ? silu1(q[r]) : 0.f;
     if (d < dim) {
-      walk_gates(a, h * dim + d, first + j * kSub, [&](int r, float f, float k) {
-        L += log2f(fmaxf(f, 0x1p-40f));  // (smaller gates leave nothing of what was there before)
+      walk_gates(a, h * dim + d, first + j * kSub, z, [&](int r, float f, float k) {
+        L += __builtin_amdgcn_logf(fmaxf(f, 0x1p-40f));  // (smaller gates leave nothing of what was there before)
         ks[(j * kSub + r) * ds + d] = k;
         ls[(j * kSub + r) * ds + d] = L;
       });
@@ -282,16 +321,12 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
     }
     tot[it] = L;
   }
-  for (int it = threadIdx.x; it < PR * d16; it += 512) {
-    const int t = it / d16, d = it - t * d16;
-    const bool in = t < C && first + t < a.T && d < dim;
-    qs[t * ds + d] = in ? silu1(a.raw[(long long)(first + t) * a.stride + h * dim + d]) : 0.f;
-  }
+  for (int it = C * ds + threadIdx.x; it < PR * ds; it += 512) qs[it] = 0.f;
   for (int it = threadIdx.x; it < PR * PS; it += 512) P[it] = 0.f;
   __syncthreads();
 
-  for (int p = threadIdx.x; p < NS * kSub * kSub; p += 512) {
-    const int b = p / (kSub * kSub) * kSub, t = b + (p / kSub) % kSub, s = b + p % kSub;
+  for (int p = threadIdx.x; p < C * 8; p += 512) {
+    const int b = p / 64 * 8, t = b + p / 8 % 8, s = b + p % 8;
     if (s > t) continue;
     const f32x4 *qp = (const f32x4 *)(qs + t * ds), *lt = (const f32x4 *)(ls + t * ds), *kp = (const f32x4 *)(ks + s * ds),
                 *lp = (const f32x4 *)(ls + s * ds);
@@ -304,39 +339,45 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
   }
   {
     const int m = lane & 15, j4 = 4 * (lane >> 4);
-    for (int item = wave; item < NS * (NS - 1) / 2; item += 8) {
-      int bi = 1, rest = item;
-      while (rest >= bi) rest -= bi++;
-      const int bj = rest;  // bj < bi
+    for (int item = wave; item < NS * (NS + 1) / 2; item += 8) {
+      int bi = 0, rest = item;
+      while (rest > bi) rest -= ++bi;
+      const int bj = rest;  // bj <= bi; equal: rows 8 .. 15 of the sub-chunk against its first eight
+      const bool half = bi == bj;
       const float *qp = qs + (bi * kSub + m) * ds + j4, *lt = ls + (bi * kSub + m) * ds + j4;
       const float *kp = ks + (bj * kSub + m) * ds + j4, *lp = ls + (bj * kSub + m) * ds + j4;
+      const float *mid = half ? ls + (bj * kSub + 7) * ds + j4 : tot + bj * d16 + j4;  // where both decay to
+      const bool q_in = !half || m >= 8, k_in = !half || m < 8;
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
       for (int i = 0; i < d16; i += 16) {
         f32x4 q = *(const f32x4 *)(qp + i), k = *(const f32x4 *)(kp + i), eq = *(const f32x4 *)(lt + i);
-        const f32x4 ek = *(const f32x4 *)(tot + bj * d16 + j4 + i) - *(const f32x4 *)(lp + i);
+        const f32x4 at = *(const f32x4 *)(mid + i);
+        f32x4 ek = at - *(const f32x4 *)(lp + i);
+        if (half) eq -= at;
         for (int b = bj + 1; b < bi; ++b) eq += *(const f32x4 *)(tot + b * d16 + j4 + i);
-        q *= f32x4{fast_exp2(eq.x), fast_exp2(eq.y), fast_exp2(eq.z), fast_exp2(eq.w)};
-        k *= f32x4{fast_exp2(ek.x), fast_exp2(ek.y), fast_exp2(ek.z), fast_exp2(ek.w)};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          q[e] = q_in ? q[e] * fast_exp2(eq[e]) : 0.f;
+          k[e] = k_in ? k[e] * fast_exp2(ek[e]) : 0.f;
+        }
 #pragma unroll
         for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e], k[e], acc, 0, 0, 0);
       }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) P[(bi * kSub + j4 + r) * PS + bj * kSub + m] = acc[r];
+      for (int r = 0; r < 4; ++r)
+        if (!half || (j4 + r >= 8 && m < 8)) P[(bi * kSub + j4 + r) * PS + bj * kSub + m] = acc[r];
     }
   }
   __syncthreads();
-  for (int it = threadIdx.x; it < C * d16; it += 512) {
-    const int t = it / d16, d = it - t * d16;
-    float e = ls[t * ds + d];
-    for (int b = 0; b < t / kSub; ++b) e += tot[b * d16 + d];
-    qs[t * ds + d] *= fast_exp2(e);
+  for (int it = threadIdx.x; it < NS * d16; it += 512) {
+    const int j = it / d16, d = it - j * d16;
+    float before = 0.f;
+    for (int b = 0; b < j; ++b) before += tot[b * d16 + d];
+#pragma unroll
+    for (int r = 0; r < kSub; ++r) qs[(j * kSub + r) * ds + d] *= fast_exp2(ls[(j * kSub + r) * ds + d] + before);
   }
   __syncthreads();
 
-  const int n = lane & 31, half = lane >> 5;
-  const int rt = wave % RT, cg = wave / RT, n_vt = (vdim + 31) / 32;
-  const float *start = starts + ((long long)c * a.H + h) * dim * vdim;
-  const float *v0 = a.raw + 2LL * a.H * dim + (long long)h * vdim;
   f32x16 acc[NT];
 #pragma unroll
   for (int u = 0; u < NT; ++u) {
@@ -344,50 +385,30 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
     for (int r = 0; r < 16; ++r) acc[u][r] = 0.f;
     const int vt = cg + CW * u;
     if (vt < n_vt) {
+      if (u > 0) {
+        __builtin_amdgcn_sched_barrier(0);  // (the loads of one tile at a time: there are no registers for more)
+        load_tile(vt);
+      }
       const int col = min(vt * 32 + n, vdim - 1);
-      const float *qp = qs + (rt * 32 + n) * ds + 4 * half, *sp = start + col;
-      constexpr int B = 4;  // k steps of 8 in flight
-      float x[B][4];
-      auto load_s = [&](float (&y)[4], int k0) {
+      const float *qp = qs + (rt * 32 + n) * ds + 4 * half;
+      for (int k0 = 0; k0 < d16; k0 += 8 * SB) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) y[i] = sp[(long long)min(k0 + 4 * half + i, dim - 1) * vdim];
-      };
-#pragma unroll
-      for (int b = 0; b < B; ++b) load_s(x[b], 8 * b);
-      for (int k0 = 0; k0 < d16; k0 += 8 * B) {
-#pragma unroll
-        for (int b = 0; b < B; ++b) {
+        for (int b = 0; b < SB; ++b) {
           if (k0 + 8 * b < d16) {
             const f32x4 q = *(const f32x4 *)(qp + k0 + 8 * b);
-            float y[4];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) y[i] = x[b][i];
-            load_s(x[b], k0 + 8 * (b + B));
-#pragma unroll
-            for (int i = 0; i < 4; ++i) acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(q[i], y[i], acc[u], 0, 0, 0);
+            for (int i = 0; i < 4; ++i) acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(q[i], xs[b][i], acc[u], 0, 0, 0);
+            if (k0 + 8 * (b + SB) < d16) load_s(xs[b], col, k0 + 8 * (b + SB));
           }
         }
       }
       const float *pp = P + (rt * 32 + n) * PS + 4 * half;
-      auto load_v = [&](float (&y)[4], int k0) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) y[i] = v0[(long long)min(first + min(k0 + 4 * half + i, C - 1), a.T - 1) * a.stride + col];
-      };
-      // (columns of P behind the row's own 32-row tile are zeros)
-      const int k_end = min(C, rt * 32 + 32);
-      constexpr int BV = C / 8 < B ? C / 8 : B;
+      for (int b = 0; b < VB; ++b) {
+        if (8 * b < rt * 32 + 32) {  // (columns of P behind the row's own 32-row tile are zeros)
+          const f32x4 p = *(const f32x4 *)(pp + 8 * b);
 #pragma unroll
-      for (int b = 0; b < BV; ++b) load_v(x[b], 8 * b);
-      for (int k0 = 0; k0 < k_end; k0 += 8 * BV) {
-#pragma unroll
-        for (int b = 0; b < BV; ++b) {
-          const f32x4 p = *(const f32x4 *)(pp + k0 + 8 * b);
-          float y[4];
-#pragma unroll
-          for (int i = 0; i < 4; ++i) y[i] = x[b][i];
-          load_v(x[b], k0 + 8 * (b + BV));
-#pragma unroll
-          for (int i = 0; i < 4; ++i) acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(p[i], y[i], acc[u], 0, 0, 0);
+          for (int i = 0; i < 4; ++i) acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(p[i], xv[b][i], acc[u], 0, 0, 0);
         }
       }
     }

@@ -385,7 +385,7 @@ struct shainet_llama_block {
   bool wrapped = false;  // norms behind the sublayers (and convolutions in front)
   ConvState conv[2];
   int pos = 0, saved_pos = -1;  // wrapped: positions so far, and where the state was saved last
-  DevF joined, y;               // wrapped: the residual with the block before joined in; a sublayer's result
+  DevF joined, y, factors;      // wrapped: the residual with the block before joined in; a sublayer's result; scratch
   int d_model = 0, ff_hidden = 0;                   // ff_hidden 0: no feed-forward
   double eps = 1e-6;                                // RMSNorm eps of @norm1 / @norm2 (llama_block.cr:93-94)
   std::shared_ptr<BlockWeights> w = std::make_shared<BlockWeights>();
@@ -433,6 +433,7 @@ int join(shainet_llama_block *b, const float *x, const float *y, const float *po
   if (conv_w) {
     a.conv = conv_w;
     a.taps = b->w->taps;
+    a.factors = b->factors.p;
     if (a.taps > 1 && !no_cache) {
       a.hist_in = b->pos ? conv->rows[conv->cur] : nullptr;  // (nothing lies before a sequence's first row)
       a.hist_out = conv->rows[conv->cur ^ 1];
@@ -451,7 +452,7 @@ int wrapped_forward_device(shainet_llama_block *b, const float *x, int T, float 
   const size_t n = (size_t)T * b->d_model;
   hipStream_t stream = b->mixer->stream();
   if (!w.norm1.gamma || !w.post1) return fail(SHAINET_HIP_ERR_ARGUMENT, "weights not set");
-  if (!b->h.reserve(n) || !b->y.reserve(n) || !b->joined.reserve(n)) return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
+  if (!b->h.reserve(n) || !b->y.reserve(n) || !b->joined.reserve(n) || !b->factors.reserve((size_t)T)) return fail(SHAINET_HIP_ERR_ALLOC, "hipMalloc failed");
   const bool carried = carry && carry->y;
   int rc = join(b, x, carried ? carry->y : nullptr, carried ? carry->post : nullptr, b->joined.p, w.norm1.gamma, w.conv1, &b->conv[0],
                 b->h.p, T, no_cache, stream);
@@ -750,7 +751,7 @@ int shainet_llama_block_create(shainet_llama_block **out, int d_model, int num_h
 int shainet_llama_block_destroy(shainet_llama_block *b) {
   if (!b) return SHAINET_HIP_OK;
   shainet_llama_attn_destroy(b->attn);
-  for (DevF *f : {&b->x, &b->h, &b->hidden, &b->out, &b->joined, &b->y}) f->release();
+  for (DevF *f : {&b->x, &b->h, &b->hidden, &b->out, &b->joined, &b->y, &b->factors}) f->release();
   b->x_pin.release();
   b->out_pin.release();
   delete b;

@@ -3,6 +3,7 @@
 
 #include <math.h>
 #include <stdint.h>
+#include <stdlib.h>
 
 namespace shainet {
 
@@ -38,6 +39,55 @@ __device__ __forceinline__ void wave_best(float &v, int &i) {
 __device__ __forceinline__ void choose(const MoeShape &m, const float *logits, const float *correction, float *s, float *c,
                                        float *best, int *ids, float *weights) {
   const int n = m.experts + m.identity, lane = threadIdx.x & 63, per = n / m.groups;
+  if (n <= 64) {
+    // a lane per output: who comes before whom is counted instead of searched for round by round
+    const bool in = lane < n;
+    const float z = in ? logits[lane] : -INFINITY, corr = in ? correction[lane] : 0.f;
+    float top_z = z;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) top_z = fmaxf(top_z, __shfl_xor(top_z, o));
+    const float e = in ? expf(z - top_z) : 0.f;
+    const float p = e / wave_sum(e), x = p + corr;
+    bool open = in;
+    if (m.groups > 1) {
+      if (in) c[lane] = x;
+      __threadfence_block();
+      const int mine = (in ? lane : 0) / per;
+      float gb = -INFINITY;
+#pragma unroll 4
+      for (int i = 0; i < per; ++i) gb = fmaxf(gb, c[mine * per + i]);
+      if (in && lane == mine * per) best[mine] = gb;
+      __threadfence_block();
+      int before = 0;
+#pragma unroll 4
+      for (int g = 0; g < m.groups; ++g) {
+        const float v = best[g];
+        before += v > gb || (v == gb && g < mine) ? 1 : 0;
+      }
+      open = in && before < m.keep;
+    }
+    if (in) s[lane] = open ? x : -INFINITY;
+    __threadfence_block();
+    int before = 0;
+#pragma unroll 8
+    for (int k = 0; k < n; ++k) {
+      const float v = s[k];
+      before += v > x || (v == x && k < lane) ? 1 : 0;
+    }
+    const bool chosen = open && before < m.top;
+    const float total = wave_sum(chosen ? p : 0.f);
+    for (int k = lane; k < m.top; k += 64) {  // (only with logits that are no numbers would an entry stay like this)
+      ids[k] = 0;
+      weights[k] = 0.f;
+    }
+    __threadfence_block();
+    if (chosen) {
+      ids[before] = lane;
+      weights[before] = p / (total + 1e-20f) * m.scale;
+    }
+    __threadfence_block();
+    return;
+  }
   float mx = -INFINITY;
   for (int i = lane; i < n; i += 64) mx = fmaxf(mx, logits[i]);
 #pragma unroll
@@ -148,107 +198,192 @@ __global__ __launch_bounds__(256) void moe_logits_kernel(const float *__restrict
 }
 
 // hidden[t][slot][j] = silu(gate row j . h) * (up row j . h) of the slot's expert; slot `top` is the shared one.
-// Every workgroup works the choice out again from the logits (a launch of its own would take longer);
-// the first one of each token leaves it for moe_down_kernel.
+// A wavefront per output; blockIdx.x: the shared expert's outputs, then slot 0's, slot 1's ...  Every workgroup
+// of a slot works the choice out again from the logits (a launch of its own would take longer) with one
+// wavefront while the others bring h into LDS; the first one leaves it for moe_down_kernel.
 template <bool VEC>
 __global__ __launch_bounds__(256) void moe_up_kernel(MoeShape m, MoeTensors w, const float *__restrict__ h,
                                                      const float *__restrict__ logits, float *__restrict__ hidden,
-                                                     int width, int *__restrict__ ids_out, float *__restrict__ weights_out) {
-  extern __shared__ float smem[];  // s, c, best, weights, then ids
-  const int n = m.experts + m.identity, slot = blockIdx.y, t = blockIdx.z;
+                                                     int width, int shared_blocks, int slot_blocks,
+                                                     int *__restrict__ ids_out, float *__restrict__ weights_out) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];  // h, s, c, best, weights, ids
+  const int n = m.experts + m.identity, t = blockIdx.y;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const bool shared = slot == m.top;
+  const bool shared = (int)blockIdx.x < shared_blocks;
+  const int slot = shared ? m.top : ((int)blockIdx.x - shared_blocks) / slot_blocks;
+  const int j = (shared ? (int)blockIdx.x : ((int)blockIdx.x - shared_blocks) - slot * slot_blocks) * 4 + wave;
   const int ff = shared ? m.shared_ff : m.ff;
-  const int j = blockIdx.x * 4 + wave;
-  const float *gate = w.shared_gate_up;
-  if (!shared) {
-    float *weights = smem + 2 * n + m.groups;
+  const float *row = h + (long long)t * m.d;
+  float *xs = smem;
+  if (wave > 0) {
+    if constexpr (VEC) {
+      for (int i = threadIdx.x - 64; i < m.d >> 2; i += 192) ((f32x4 *)xs)[i] = ((const f32x4 *)row)[i];
+    } else {
+      for (int i = threadIdx.x - 64; i < m.d; i += 192) xs[i] = row[i];
+    }
+  } else if (shared) {
+    // (nothing to choose)
+  } else {
+    float *s = smem + (m.d + 3) / 4 * 4, *weights = s + 2 * n + m.groups;
     int *ids = (int *)(weights + m.top);
-    if (wave == 0) choose(m, logits + (long long)t * n, w.correction, smem, smem + n, smem + 2 * n, ids, weights);
-    __syncthreads();
-    if (blockIdx.x == 0 && slot == 0)
-      for (int k = threadIdx.x; k < m.top; k += 256) {
+    choose(m, logits + (long long)t * n, w.correction, s, s + n, s + 2 * n, ids, weights);
+    if (slot == 0 && j == 0)
+      for (int k = lane; k < m.top; k += 64) {
         ids_out[t * m.top + k] = ids[k];
         weights_out[t * m.top + k] = weights[k];
       }
-    const int e = ids[slot];
+  }
+  __syncthreads();
+  const float *gate = w.shared_gate_up;
+  if (!shared) {
+    const int e = ((const int *)(smem + (m.d + 3) / 4 * 4 + 2 * n + m.groups + m.top))[slot];
     if (e >= m.experts) return;
     gate = w.gate_up + (long long)e * 2 * m.ff * m.d;
   }
   if (j >= ff) return;
-  const float *x = h + (long long)t * m.d;
   float g, u;
   if constexpr (VEC) {  // both rows in flight together
-    const float *gp = gate + (long long)j * m.d, *up = gate + (long long)(ff + j) * m.d;
+    const f32x4 *gp = (const f32x4 *)(gate + (long long)j * m.d), *up = (const f32x4 *)(gate + (long long)(ff + j) * m.d);
     f32x4 ga = {0.f, 0.f, 0.f, 0.f}, ua = ga;
     const int n4 = m.d >> 2;
-    for (int i0 = lane; i0 < n4; i0 += 256) {
-      f32x4 gv[4], uv[4], xv[4];
+    constexpr int U = 8;
+    for (int i0 = lane; i0 < n4; i0 += 64 * U) {
+      f32x4 gv[U], uv[U];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) {
-        const int i = min(i0 + 64 * k, n4 - 1);
-        gv[k] = __builtin_nontemporal_load((const f32x4 *)gp + i);
-        uv[k] = __builtin_nontemporal_load((const f32x4 *)up + i);
-        xv[k] = ((const f32x4 *)x)[i];
-      }
+      for (int k = 0; k < U; ++k)
+        if (i0 - lane + 64 * k < n4) {
+          const int i = min(i0 + 64 * k, n4 - 1);
+          gv[k] = __builtin_nontemporal_load(gp + i);
+          uv[k] = __builtin_nontemporal_load(up + i);
+        }
 #pragma unroll
-      for (int k = 0; k < 4; ++k)
+      for (int k = 0; k < U; ++k)
         if (i0 + 64 * k < n4) {
-          ga += gv[k] * xv[k];
-          ua += uv[k] * xv[k];
+          const f32x4 x = ((const f32x4 *)xs)[i0 + 64 * k];
+          ga += gv[k] * x;
+          ua += uv[k] * x;
         }
     }
     g = (ga.x + ga.y) + (ga.z + ga.w);
     u = (ua.x + ua.y) + (ua.z + ua.w);
   } else {
-    g = dot_lane<false>(gate + (long long)j * m.d, x, m.d);
-    u = dot_lane<false>(gate + (long long)(ff + j) * m.d, x, m.d);
+    g = dot_lane<false>(gate + (long long)j * m.d, xs, m.d);
+    u = dot_lane<false>(gate + (long long)(ff + j) * m.d, xs, m.d);
   }
   g = wave_sum(g);
   u = wave_sum(u);
   if (lane == 0) hidden[((long long)t * (m.top + 1) + slot) * width + j] = swiglu1(g, u);
 }
 
-// y[t][j]: a wavefront per output, over all slots
+// y[t][j]: a wavefront per output, over all slots, four experts' rows in flight together
 template <bool VEC>
 __global__ __launch_bounds__(256) void moe_down_kernel(MoeShape m, MoeTensors w, const float *__restrict__ h,
                                                        const float *__restrict__ hidden, int width,
                                                        const int *__restrict__ ids, const float *__restrict__ weights,
                                                        float *__restrict__ y) {
-  const int j = blockIdx.x * 4 + (threadIdx.x >> 6), t = blockIdx.y;
+  const int j = blockIdx.x * 4 + (threadIdx.x >> 6), t = blockIdx.y, lane = threadIdx.x & 63;
   if (j >= m.d) return;
   const float *hid = hidden + (long long)t * (m.top + 1) * width;
   float s = 0.f, same = 0.f;
-  for (int k = 0; k < m.top; ++k) {
-    const int e = ids[t * m.top + k];
-    const float wk = weights[t * m.top + k];
-    if (e >= m.experts)
-      same += wk;
-    else
-      s += wk * dot_lane<VEC>(w.down + ((long long)e * m.d + j) * m.ff, hid + (long long)k * width, m.ff);
+  if constexpr (VEC) {
+    constexpr int G = 4, U = 4;
+    const int n4 = m.ff >> 2, s4 = m.shared_ff >> 2;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    if (m.shared_ff) {
+      const f32x4 *a = (const f32x4 *)(w.shared_down + (long long)j * m.shared_ff), *b = (const f32x4 *)(hid + (long long)m.top * width);
+      for (int i0 = 0; i0 < s4; i0 += 64 * 8) {
+        f32x4 x[8], v[8];
+#pragma unroll
+        for (int k = 0; k < 8; ++k)
+          if (i0 + 64 * k < s4) {
+            const int i = min(i0 + 64 * k + lane, s4 - 1);
+            x[k] = __builtin_nontemporal_load(a + i);
+            v[k] = b[i];
+          }
+#pragma unroll
+        for (int k = 0; k < 8; ++k)
+          if (i0 + 64 * k + lane < s4) acc += x[k] * v[k];
+      }
+    }
+    for (int k0 = 0; k0 < m.top; k0 += G) {
+      const f32x4 *a[G], *b[G];
+      float wk[G];
+#pragma unroll
+      for (int g = 0; g < G; ++g) {
+        const int k = min(k0 + g, m.top - 1), e = ids[t * m.top + k];
+        const bool real = k0 + g < m.top && e < m.experts;
+        wk[g] = real ? weights[t * m.top + k] : 0.f;
+        if (k0 + g < m.top && e >= m.experts) same += weights[t * m.top + k];
+        a[g] = real ? (const f32x4 *)(w.down + ((long long)e * m.d + j) * m.ff) : nullptr;
+        b[g] = (const f32x4 *)(hid + (long long)k * width);
+      }
+      for (int i0 = 0; i0 < n4; i0 += 64 * U) {
+        f32x4 x[G][U], v[G][U];
+#pragma unroll
+        for (int g = 0; g < G; ++g)
+#pragma unroll
+          for (int u = 0; u < U; ++u)
+            if (a[g] && i0 + 64 * u < n4) {
+              const int i = min(i0 + 64 * u + lane, n4 - 1);
+              x[g][u] = __builtin_nontemporal_load(a[g] + i);
+              v[g][u] = b[g][i];
+            }
+#pragma unroll
+        for (int g = 0; g < G; ++g)
+#pragma unroll
+          for (int u = 0; u < U; ++u)
+            if (a[g] && i0 + 64 * u + lane < n4) acc += wk[g] * (x[g][u] * v[g][u]);
+      }
+    }
+    s = (acc.x + acc.y) + (acc.z + acc.w);
+  } else {
+    for (int k = 0; k < m.top; ++k) {
+      const int e = ids[t * m.top + k];
+      const float wk = weights[t * m.top + k];
+      if (e >= m.experts)
+        same += wk;
+      else
+        s += wk * dot_lane<false>(w.down + ((long long)e * m.d + j) * m.ff, hid + (long long)k * width, m.ff);
+    }
+    if (m.shared_ff) s += dot_lane<false>(w.shared_down + (long long)j * m.shared_ff, hid + (long long)m.top * width, m.shared_ff);
   }
-  if (m.shared_ff)
-    s += dot_lane<VEC>(w.shared_down + (long long)j * m.shared_ff, hid + (long long)m.top * width, m.shared_ff);
   s = wave_sum(s);
-  if ((threadIdx.x & 63) == 0) y[(long long)t * m.d + j] = s + same * h[(long long)t * m.d + j];
+  if (lane == 0) y[(long long)t * m.d + j] = s + same * h[(long long)t * m.d + j];
 }
 
 // ---- many tokens -------------------------------------------------------------------------------
-// A wavefront per token chooses; a chosen expert's counter gives the token's place among its rows.
+// A wavefront chooses for one token after the other; the places of a workgroup's tokens among an expert's rows
+// are counted in LDS, and one addition per expert to the expert's counter gives where they begin.  tokens: per
+// workgroup.
 __global__ __launch_bounds__(256) void moe_select_kernel(MoeShape m, const float *__restrict__ correction,
-                                                         const float *__restrict__ logits, int T, int *__restrict__ ids,
-                                                         float *__restrict__ weights, int *__restrict__ rank, int *counts) {
-  extern __shared__ float smem[];
-  const int n = m.experts + m.identity, wave = threadIdx.x >> 6, t = blockIdx.x * 4 + wave;
-  if (t >= T) return;
-  float *s = smem + wave * (2 * n + m.groups + 2 * m.top), *wl = s + 2 * n + m.groups;
-  int *il = (int *)(wl + m.top);
-  choose(m, logits + (long long)t * n, correction, s, s + n, s + 2 * n, il, wl);
-  for (int k = threadIdx.x & 63; k < m.top; k += 64) {
-    const int e = il[k];
-    ids[t * m.top + k] = e;
-    weights[t * m.top + k] = wl[k];
-    rank[t * m.top + k] = e < m.experts ? atomicAdd(counts + e, 1) : 0;
+                                                         const float *__restrict__ logits, int stride, int T, int tokens,
+                                                         int *__restrict__ ids, float *__restrict__ weights,
+                                                         int *__restrict__ rank, int *counts) {
+  extern __shared__ float smem[];  // per wavefront: s, c, best, weights, ids; then [experts] counts
+  const int n = m.experts + m.identity, wave = threadIdx.x >> 6, per_wave = 2 * n + m.groups + 2 * m.top;
+  float *s = smem + wave * per_wave, *wl = s + 2 * n + m.groups;
+  int *il = (int *)(wl + m.top), *cnt = (int *)(smem + 4 * per_wave);
+  for (int e = threadIdx.x; e < m.experts; e += 256) cnt[e] = 0;
+  __syncthreads();
+  const int t0 = blockIdx.x * tokens;
+  for (int i = wave; i < tokens && t0 + i < T; i += 4) {
+    const int t = t0 + i;
+    choose(m, logits + (long long)t * stride, correction, s, s + n, s + 2 * n, il, wl);
+    for (int k = threadIdx.x & 63; k < m.top; k += 64) {
+      const int e = il[k];
+      ids[t * m.top + k] = e;
+      weights[t * m.top + k] = wl[k];
+      rank[t * m.top + k] = e < m.experts ? atomicAdd(cnt + e, 1) : 0;
+    }
+    __threadfence_block();
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < m.experts; e += 256) cnt[e] = cnt[e] ? atomicAdd(counts + e, cnt[e]) : 0;
+  __syncthreads();
+  const int mine = min(tokens, T - t0) * m.top;
+  for (int i = threadIdx.x; i < mine; i += 256) {  // (ids and ranks of this workgroup's own tokens)
+    const int at = t0 * m.top + i, e = ids[at];
+    if (e < m.experts) rank[at] += cnt[e];
   }
 }
 
@@ -444,18 +579,17 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(MoeShape m, const floa
 size_t up4(size_t n) { return (n + 3) / 4 * 4; }
 
 struct ManyLayout {
-  size_t logits, weights, ids, rank, off, tile_off, rows, hidden, rows_y, total;
+  size_t weights, ids, rank, off, tile_off, rows, hidden, rows_y, total;
 };
 ManyLayout many_layout(const MoeShape &m, int T) {
   ManyLayout l;
-  const size_t n = (size_t)m.experts + m.identity, slots = (size_t)T * m.top;
+  const size_t slots = (size_t)T * m.top;
   size_t at = 0;
   auto take = [&](size_t k) {
     const size_t here = at;
     at += up4(k);
     return here;
   };
-  l.logits = take((size_t)T * n);
   l.weights = take(slots);
   l.ids = take(slots);
   l.rank = take(slots);
@@ -521,21 +655,23 @@ hipError_t launch_moe_few(const MoeShape &m, const MoeTensors &w, const float *h
       !w.down || (m.shared_ff && (!w.shared_gate_up || !w.shared_down)))
     return hipErrorInvalidValue;
   const int n = m.experts + m.identity, most = m.ff > m.shared_ff ? m.ff : m.shared_ff, width = (int)up4(most);
-  const int slots = m.top + (m.shared_ff ? 1 : 0);
   float *logits = scratch, *weights = logits + up4((size_t)T * n);
   int *ids = (int *)(weights + up4((size_t)T * m.top));
   float *hidden = (float *)ids + up4((size_t)T * m.top);
-  const dim3 g1((unsigned)((n + 3) / 4), (unsigned)T), g2((unsigned)((most + 3) / 4), (unsigned)slots, (unsigned)T),
-      g3((unsigned)((m.d + 3) / 4), (unsigned)T);
-  const size_t lds = (size_t)(2 * n + m.groups + 2 * m.top) * sizeof(float);
-  if (slots > 65535) return hipErrorInvalidValue;
+  const int shared_blocks = (m.shared_ff + 3) / 4, slot_blocks = (m.ff + 3) / 4;
+  const long long blocks = (long long)shared_blocks + (long long)m.top * slot_blocks;
+  const dim3 g1((unsigned)((n + 3) / 4), (unsigned)T), g2((unsigned)blocks, (unsigned)T), g3((unsigned)((m.d + 3) / 4), (unsigned)T);
+  const size_t lds = ((size_t)up4(m.d) + 2 * n + m.groups + 2 * m.top) * sizeof(float);
+  if (blocks > 0x7fffffffLL || lds > 64 * 1024) return hipErrorInvalidValue;
   const bool vec_d = (m.d & 3) == 0, vec_ff = ((m.ff | m.shared_ff) & 3) == 0;
   if (vec_d) {
     hipLaunchKernelGGL(moe_logits_kernel<true>, g1, dim3(256), 0, stream, h, w.router, logits, n, m.d);
-    hipLaunchKernelGGL(moe_up_kernel<true>, g2, dim3(256), lds, stream, m, w, h, logits, hidden, width, ids, weights);
+    hipLaunchKernelGGL(moe_up_kernel<true>, g2, dim3(256), lds, stream, m, w, h, logits, hidden, width, shared_blocks, slot_blocks,
+                       ids, weights);
   } else {
     hipLaunchKernelGGL(moe_logits_kernel<false>, g1, dim3(256), 0, stream, h, w.router, logits, n, m.d);
-    hipLaunchKernelGGL(moe_up_kernel<false>, g2, dim3(256), lds, stream, m, w, h, logits, hidden, width, ids, weights);
+    hipLaunchKernelGGL(moe_up_kernel<false>, g2, dim3(256), lds, stream, m, w, h, logits, hidden, width, shared_blocks, slot_blocks,
+                       ids, weights);
   }
   if (vec_ff)
     hipLaunchKernelGGL(moe_down_kernel<true>, g3, dim3(256), 0, stream, m, w, h, hidden, width, ids, weights, y);
@@ -546,31 +682,26 @@ hipError_t launch_moe_few(const MoeShape &m, const MoeTensors &w, const float *h
 
 size_t moe_many_floats(const MoeShape &m, int T) { return many_layout(m, T).total; }
 
-hipError_t launch_moe_many(const MoeShape &m, const MoeTensors &w, const float *h, float *y, bool add_to_y, int T,
-                           float *scratch, int *counts, hipStream_t stream) {
-  if (!moe_shape_ok(m) || T < 1 || (long long)T * m.top > 0x3fffffff || !h || !y || !scratch || !counts || !w.router ||
-      !w.correction || !w.gate_up || !w.down)
+hipError_t launch_moe_many(const MoeShape &m, const MoeTensors &w, const float *h, const float *logits, int stride, float *y,
+                           bool add_to_y, int T, float *scratch, int *counts, hipStream_t stream) {
+  if (!moe_shape_ok(m) || T < 1 || (long long)T * m.top > 0x3fffffff || !h || !y || !logits ||
+      stride < m.experts + m.identity || !scratch || !counts || !w.correction || !w.gate_up || !w.down)
     return hipErrorInvalidValue;
   const ManyLayout l = many_layout(m, T);
   const int n = m.experts + m.identity, slots = T * m.top;
-  float *logits = scratch + l.logits, *weights = scratch + l.weights, *hidden = scratch + l.hidden, *rows_y = scratch + l.rows_y;
+  float *weights = scratch + l.weights, *hidden = scratch + l.hidden, *rows_y = scratch + l.rows_y;
   int *ids = (int *)(scratch + l.ids), *rank = (int *)(scratch + l.rank), *off = (int *)(scratch + l.off),
       *tile_off = (int *)(scratch + l.tile_off), *rows = (int *)(scratch + l.rows);
-  GroupedArgs r = {};
-  r.x = h;
-  r.w = w.router;
-  r.y = logits;
-  r.rows = T;
-  r.groups = 1;
-  r.K = m.d;
-  r.N = n;
-  hipError_t e = launch_product(r, 32, false, stream);
-  if (e != hipSuccess) return e;
-  const size_t lds = (size_t)4 * (2 * n + m.groups + 2 * m.top) * sizeof(float);
+  hipError_t e = hipSuccess;
+  const size_t lds = ((size_t)4 * (2 * n + m.groups + 2 * m.top) + m.experts) * sizeof(float);
   if (lds > 64 * 1024) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(moe_select_kernel, dim3((unsigned)((T + 3) / 4)), dim3(256), lds, stream, m, w.correction, logits, T, ids,
-                     weights, rank, counts);
-  const int per_expert = slots / m.experts, tm = per_expert > 96 ? 128 : per_expert > 32 ? 64 : 32;
+  const int tokens = T <= 4096 ? 4 : 16;
+  hipLaunchKernelGGL(moe_select_kernel, dim3((unsigned)((T + tokens - 1) / tokens)), dim3(256), lds, stream, m, w.correction, logits,
+                     stride, T, tokens, ids, weights, rank, counts);
+  // rows an expert gets if the router spreads them evenly
+  const int per_expert = slots / n, best_tm = per_expert > 1024 ? 128 : per_expert > 32 ? 64 : 32;
+  static const int tile_knob = getenv("SHAINET_HIP_MOE_TILE") ? atoi(getenv("SHAINET_HIP_MOE_TILE")) : 0;  // a tuning knob: 32, 64 or 128
+  const int tm = tile_knob == 32 || tile_knob == 64 || tile_knob == 128 ? tile_knob : best_tm;
   hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(1024), 0, stream, m.experts, tm, counts, off, tile_off);
   hipLaunchKernelGGL(moe_scatter_kernel, dim3((unsigned)((slots + 255) / 256)), dim3(256), 0, stream, slots, m.top, m.experts,
                      ids, rank, off, rows);

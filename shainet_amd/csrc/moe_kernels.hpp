@@ -34,10 +34,11 @@ size_t moe_few_floats(const MoeShape &m, int T);
 hipError_t launch_moe_few(const MoeShape &m, const MoeTensors &w, const float *h, float *y, int T, float *scratch,
                           hipStream_t stream);
 
-// Any number of rows.  y [T, d] holds the shared expert's rows already (add_to_y) or nothing.
+// Any number of rows.  logits: the router's product with h, rows of `stride` floats; y [T, d] holds the shared
+// expert's rows already (add_to_y) or nothing.
 // scratch: moe_many_floats floats; counts: m.experts ints, zero before the first call, left zero.
 size_t moe_many_floats(const MoeShape &m, int T);
-hipError_t launch_moe_many(const MoeShape &m, const MoeTensors &w, const float *h, float *y, bool add_to_y, int T,
-                           float *scratch, int *counts, hipStream_t stream);
+hipError_t launch_moe_many(const MoeShape &m, const MoeTensors &w, const float *h, const float *logits, int stride,
+                           float *y, bool add_to_y, int T, float *scratch, int *counts, hipStream_t stream);
 
 }  // namespace shainet

@@ -29,13 +29,14 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
   return s;
 }
 
-// One row: everything it needs is requested at once and stays in registers.  P: 16-byte pieces per thread.
-template <int P>
+// One row: everything it needs is requested at once and stays in registers.  P: 16-byte pieces per thread;
+// TAPS: taps of the convolution that are asked for ahead (more are read when they are used).
+template <int P, int TAPS>
 __global__ __launch_bounds__(1024) void residual_row_kernel(const ResidualArgs a) {
   __shared__ float red_y[16], red_x[16];
   const int d4 = a.d >> 2, nt = blockDim.x;
   const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-  f32x4 x[P], y[P], post[P], pre[P];
+  f32x4 x[P], y[P], post[P], pre[P], w[P][TAPS], old[P][TAPS];
 #pragma unroll
   for (int p = 0; p < P; ++p) {
     const int i = threadIdx.x + p * nt;
@@ -44,6 +45,11 @@ __global__ __launch_bounds__(1024) void residual_row_kernel(const ResidualArgs a
     y[p] = in && a.y ? ((const f32x4 *)a.y)[i] : zero;
     post[p] = in && a.y ? ((const f32x4 *)a.post)[i] : zero;
     pre[p] = in && a.pre ? ((const f32x4 *)a.pre)[i] : zero;
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) {
+      w[p][k] = in && a.conv && k < a.taps ? ((const f32x4 *)a.conv)[(long long)k * d4 + i] : zero;
+      old[p][k] = in && a.hist_in && k < a.taps - 1 ? ((const f32x4 *)a.hist_in)[(long long)k * d4 + i] : zero;
+    }
   }
   if (a.y) {
     float sq = 0.f;
@@ -58,20 +64,6 @@ __global__ __launch_bounds__(1024) void residual_row_kernel(const ResidualArgs a
     }
   }
   if (!a.pre) return;
-  // (the earlier rows' part of the convolution does not depend on this row's norm)
-  f32x4 c[P], w_own[P];
-#pragma unroll
-  for (int p = 0; p < P; ++p) {
-    c[p] = w_own[p] = zero;
-    const int i = threadIdx.x + p * nt;
-    if (!a.conv || i >= d4) continue;
-    w_own[p] = ((const f32x4 *)a.conv)[(long long)(a.taps - 1) * d4 + i];
-    for (int k = 0; k < a.taps - 1; ++k) {
-      const f32x4 v = a.hist_in ? ((const f32x4 *)a.hist_in)[(long long)k * d4 + i] : zero;
-      c[p] += v * ((const f32x4 *)a.conv)[(long long)k * d4 + i];
-      if (a.hist_out && k > 0) ((f32x4 *)a.hist_out)[(long long)(k - 1) * d4 + i] = v;
-    }
-  }
   float sq = 0.f;
 #pragma unroll
   for (int p = 0; p < P; ++p) sq += sum4(x[p] * x[p]);
@@ -81,142 +73,151 @@ __global__ __launch_bounds__(1024) void residual_row_kernel(const ResidualArgs a
     const int i = threadIdx.x + p * nt;
     if (i >= d4) continue;
     const f32x4 h = x[p] * f * pre[p];
-    if (a.hist_out && a.taps > 1) ((f32x4 *)a.hist_out)[(long long)(a.taps - 2) * d4 + i] = h;
-    ((f32x4 *)a.h)[i] = h + (c[p] + h * w_own[p]);
+    f32x4 c = zero;
+    if (a.conv) {
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) {
+        if (k < a.taps - 1) {
+          c += old[p][k] * w[p][k];
+          if (a.hist_out && k > 0) ((f32x4 *)a.hist_out)[(long long)(k - 1) * d4 + i] = old[p][k];
+        } else if (k == a.taps - 1) {
+          c += h * w[p][k];
+        }
+      }
+      for (int k = TAPS; k < a.taps; ++k) {
+        const f32x4 v = k == a.taps - 1 ? h : a.hist_in ? ((const f32x4 *)a.hist_in)[(long long)k * d4 + i] : zero;
+        c += v * ((const f32x4 *)a.conv)[(long long)k * d4 + i];
+        if (a.hist_out && k < a.taps - 1) ((f32x4 *)a.hist_out)[(long long)(k - 1) * d4 + i] = v;
+      }
+      if (a.hist_out && a.taps > 1) ((f32x4 *)a.hist_out)[(long long)(a.taps - 2) * d4 + i] = h;
+    }
+    ((f32x4 *)a.h)[i] = h + c;
   }
 }
 
-// The two factors of the rows first - back .. first + kRows - 1 that exist, a wavefront per row.
+// Many rows, first launch: a workgroup per row.  Without a convolution h is finished here, with one its factor
+// is left for the second launch.  P: 16-byte pieces per thread (0: any width, element by element).
+template <int P>
+__global__ __launch_bounds__(256) void residual_join_kernel(const ResidualArgs a) {
+  __shared__ float red_y[4], red_x[4];
+  const long long t = blockIdx.x;
+  if constexpr (P > 0) {
+    const int d4 = a.d >> 2;
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    const f32x4 *xr = (const f32x4 *)a.x + t * d4, *yr = a.y ? (const f32x4 *)a.y + t * d4 : nullptr;
+    f32x4 x[P], y[P];
+#pragma unroll
+    for (int p = 0; p < P; ++p) {
+      const int i = threadIdx.x + 256 * p;
+      x[p] = i < d4 ? xr[i] : zero;
+      y[p] = i < d4 && yr ? yr[i] : zero;
+    }
+    if (yr) {
+      float sq = 0.f;
+#pragma unroll
+      for (int p = 0; p < P; ++p) sq += sum4(y[p] * y[p]);
+      const float f = inv_rms(block_sum(sq, red_y), a.d, a.eps);
+#pragma unroll
+      for (int p = 0; p < P; ++p) {
+        const int i = threadIdx.x + 256 * p;
+        if (i >= d4) continue;
+        x[p] += y[p] * f * ((const f32x4 *)a.post)[i];
+        ((f32x4 *)a.x_out)[t * d4 + i] = x[p];
+      }
+    }
+    if (!a.pre) return;
+    float sq = 0.f;
+#pragma unroll
+    for (int p = 0; p < P; ++p) sq += sum4(x[p] * x[p]);
+    const float f = inv_rms(block_sum(sq, red_x), a.d, a.eps);
+    if (a.conv) {
+      if (threadIdx.x == 0) a.factors[t] = f;
+      return;
+    }
+#pragma unroll
+    for (int p = 0; p < P; ++p) {
+      const int i = threadIdx.x + 256 * p;
+      if (i < d4) ((f32x4 *)a.h)[t * d4 + i] = x[p] * f * ((const f32x4 *)a.pre)[i];
+    }
+  } else {
+    const float *xr = a.x + t * a.d;
+    if (a.y) {
+      float sq = 0.f;
+      for (int i = threadIdx.x; i < a.d; i += 256) sq += a.y[t * a.d + i] * a.y[t * a.d + i];
+      const float f = inv_rms(block_sum(sq, red_y), a.d, a.eps);
+      for (int i = threadIdx.x; i < a.d; i += 256) a.x_out[t * a.d + i] = xr[i] + a.y[t * a.d + i] * f * a.post[i];
+      xr = a.x_out + t * a.d;  // (a thread reads what it wrote itself)
+    }
+    if (!a.pre) return;
+    float sq = 0.f;
+    for (int i = threadIdx.x; i < a.d; i += 256) sq += xr[i] * xr[i];
+    const float f = inv_rms(block_sum(sq, red_x), a.d, a.eps);
+    if (a.conv) {
+      if (threadIdx.x == 0) a.factors[t] = f;
+      return;
+    }
+    for (int i = threadIdx.x; i < a.d; i += 256) a.h[t * a.d + i] = xr[i] * f * a.pre[i];
+  }
+}
+
+// Second launch: kRows rows of 256 columns (of 16 bytes) per workgroup; x: the joined rows.  All rows a thread
+// needs are requested before the first is used.
 constexpr int kRows = 8;
-template <bool VEC>
-__device__ __forceinline__ void row_factors(const ResidualArgs &a, int first, int back, float *fy, float *fx) {
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  for (int k = wave; k < back + kRows; k += 4) {
-    const int t = first - back + k;
-    if (t < 0 || t >= a.T) continue;
-    const float *x = a.x + (long long)t * a.d, *y = a.y ? a.y + (long long)t * a.d : nullptr;
-    float f1 = 0.f;
-    if (y) {
-      float sq = 0.f;
-      if (VEC)
-        for (int i = lane; i < a.d >> 2; i += 64) sq += sum4(((const f32x4 *)y)[i] * ((const f32x4 *)y)[i]);
-      else
-        for (int i = lane; i < a.d; i += 64) sq += y[i] * y[i];
-      f1 = inv_rms(wave_sum(sq), a.d, a.eps);
-    }
-    float f2 = 0.f;
-    if (a.pre) {
-      float sq = 0.f;
-      if (VEC) {
-        for (int i = lane; i < a.d >> 2; i += 64) {
-          f32x4 v = ((const f32x4 *)x)[i];
-          if (y) v += ((const f32x4 *)y)[i] * f1 * ((const f32x4 *)a.post)[i];
-          sq += sum4(v * v);
-        }
-      } else {
-        for (int i = lane; i < a.d; i += 64) {
-          float v = x[i];
-          if (y) v += y[i] * f1 * a.post[i];
-          sq += v * v;
-        }
-      }
-      f2 = inv_rms(wave_sum(sq), a.d, a.eps);
-    }
-    if (lane == 0) {
-      fy[k] = f1;
-      fx[k] = f2;
-    }
-  }
-}
-
-// Many rows: a workgroup takes kRows rows and works out again what it needs of the TAPS - 1 rows before
-// them.  A thread walks down its columns with the last TAPS rows' h in registers.
-// x_out == x would let a workgroup read a neighbour's rows after they have changed: the caller passes
-// another buffer when TAPS > 1.
 template <int TAPS>
-__global__ __launch_bounds__(256) void residual_rows_kernel(const ResidualArgs a) {
-  __shared__ float fy[TAPS - 1 + kRows], fx[TAPS - 1 + kRows];
-  const int first = blockIdx.x * kRows, last = min(first + kRows, a.T);
-  row_factors<true>(a, first, TAPS - 1, fy, fx);
-  __syncthreads();
-  const int d4 = a.d >> 2;
+__global__ __launch_bounds__(256) void residual_conv_kernel(const ResidualArgs a, const float *__restrict__ x) {
+  constexpr int BACK = TAPS - 1, N = kRows + BACK;
+  const int d4 = a.d >> 2, i = blockIdx.y * 256 + threadIdx.x, first = blockIdx.x * kRows;
+  if (i >= d4) return;
   const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-  for (int i = threadIdx.x; i < d4; i += 256) {
-    f32x4 post = zero, pre = zero, w[TAPS], win[TAPS];
-    if (a.y) post = ((const f32x4 *)a.post)[i];
-    if (a.pre) pre = ((const f32x4 *)a.pre)[i];
+  f32x4 h[N], w[TAPS];
+  float f[N];
 #pragma unroll
-    for (int k = 0; k < TAPS; ++k) {
-      w[k] = a.conv ? ((const f32x4 *)a.conv)[(long long)k * d4 + i] : zero;
-      win[k] = zero;
+  for (int k = 0; k < N; ++k) {
+    const int t = first - BACK + k;
+    if (t < 0) {
+      h[k] = a.hist_in && t >= -BACK ? ((const f32x4 *)a.hist_in)[(long long)(BACK + t) * d4 + i] : zero;
+      f[k] = 1.f;
+    } else {
+      h[k] = ((const f32x4 *)x)[(long long)min(t, a.T - 1) * d4 + i];
+      f[k] = a.factors[min(t, a.T - 1)];
     }
-    for (int k = 0; k < TAPS - 1 + kRows; ++k) {
-      const int t = first - (TAPS - 1) + k;
-      if (t >= last) break;
-      f32x4 h = zero;
-      if (t < 0) {
-        if (a.hist_in && t >= -(TAPS - 1)) h = ((const f32x4 *)a.hist_in)[(long long)(TAPS - 1 + t) * d4 + i];
-      } else {
-        f32x4 x = ((const f32x4 *)a.x)[(long long)t * d4 + i];
-        if (a.y) {
-          x += ((const f32x4 *)a.y)[(long long)t * d4 + i] * fy[k] * post;
-          if (t >= first) ((f32x4 *)a.x_out)[(long long)t * d4 + i] = x;
-        }
-        h = x * fx[k] * pre;
-      }
+  }
 #pragma unroll
-      for (int j = 0; j + 1 < TAPS; ++j) win[j] = win[j + 1];
-      win[TAPS - 1] = h;
-      if (a.hist_out) {  // the last TAPS - 1 rows of [what came in | this call's]
-        const int slot = t - (a.T - (TAPS - 1));
-        if (slot >= 0 && slot < TAPS - 1 && (t >= first || (t < 0 && blockIdx.x == 0)))
-          ((f32x4 *)a.hist_out)[(long long)slot * d4 + i] = h;
-      }
-      if (t < first || !a.pre) continue;
-      f32x4 c = zero;
+  for (int k = 0; k < TAPS; ++k) w[k] = ((const f32x4 *)a.conv)[(long long)k * d4 + i];
+  const f32x4 pre = ((const f32x4 *)a.pre)[i];
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) c += win[j] * w[j];
-      ((f32x4 *)a.h)[(long long)t * d4 + i] = h + c;
+  for (int k = 0; k < N; ++k) {
+    const int t = first - BACK + k;
+    if (t >= 0) h[k] = h[k] * f[k] * pre;
+    if (a.hist_out && t < a.T && (k >= BACK || (t < 0 && blockIdx.x == 0))) {  // the last rows of [what came in | this call's]
+      const int slot = t - (a.T - BACK);
+      if (slot >= 0 && slot < BACK) ((f32x4 *)a.hist_out)[(long long)slot * d4 + i] = h[k];
     }
+    if (k < BACK || t >= a.T) continue;
+    f32x4 c = zero;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) c += h[k - BACK + j] * w[j];
+    ((f32x4 *)a.h)[(long long)t * d4 + i] = h[k] + c;
   }
 }
 
-// Any width and number of taps: a column per thread, the window in LDS.
-__global__ __launch_bounds__(256) void residual_any_kernel(const ResidualArgs a) {
-  extern __shared__ float win[];  // [taps][256], row t in slot t mod taps
-  __shared__ float fy[kMaxConvTaps - 1 + kRows], fx[kMaxConvTaps - 1 + kRows];
-  const int taps = a.taps, back = taps - 1;
-  const int first = blockIdx.x * kRows, last = min(first + kRows, a.T);
-  row_factors<false>(a, first, back, fy, fx);
-  __syncthreads();
-  for (int i = threadIdx.x; i < a.d; i += 256) {
-    for (int k = 0; k < back + kRows; ++k) {
-      const int t = first - back + k;
-      if (t >= last) break;
-      float h = 0.f;
-      if (t < 0) {
-        if (a.hist_in) h = a.hist_in[(long long)(back + t) * a.d + i];
-      } else {
-        float x = a.x[(long long)t * a.d + i];
-        if (a.y) {
-          x += a.y[(long long)t * a.d + i] * fy[k] * a.post[i];
-          if (t >= first) a.x_out[(long long)t * a.d + i] = x;
-        }
-        if (a.pre) h = x * fx[k] * a.pre[i];
-      }
-      win[(k % taps) * 256 + threadIdx.x] = h;
-      if (a.hist_out) {
-        const int slot = t - (a.T - back);
-        if (slot >= 0 && slot < back && (t >= first || (t < 0 && blockIdx.x == 0)))
-          a.hist_out[(long long)slot * a.d + i] = h;
-      }
-      if (t < first || !a.pre) continue;
-      float c = 0.f;
-      if (a.conv)
-        for (int j = 0; j < taps; ++j) c += win[((k + 1 + j) % taps) * 256 + threadIdx.x] * a.conv[(long long)j * a.d + i];
-      a.h[(long long)t * a.d + i] = h + c;
-    }
-  }
+// Any width and number of taps: an element per thread.
+__global__ __launch_bounds__(256) void residual_conv_any_kernel(const ResidualArgs a, const float *__restrict__ x) {
+  const int back = a.taps - 1, i = blockIdx.y * 256 + threadIdx.x;
+  if (i >= a.d) return;
+  auto row = [&](int t) {
+    if (t < 0) return a.hist_in ? a.hist_in[(long long)(back + t) * a.d + i] : 0.f;
+    return x[(long long)t * a.d + i] * a.factors[t] * a.pre[i];
+  };
+  const int t = blockIdx.x;
+  float c = 0.f;
+  for (int j = 0; j < a.taps; ++j) c += row(t - back + j) * a.conv[(long long)j * a.d + i];
+  const float h = row(t);
+  a.h[(long long)t * a.d + i] = h + c;
+  if (!a.hist_out) return;
+  if (t >= a.T - back) a.hist_out[(long long)(t - (a.T - back)) * a.d + i] = h;
+  if (t == 0)
+    for (int s = 0; s < back - a.T; ++s) a.hist_out[(long long)s * a.d + i] = row(s + a.T - back);
 }
 
 __global__ __launch_bounds__(256) void add_one_kernel(float *x, long long n) {
@@ -245,26 +246,41 @@ hipError_t launch_residual(const ResidualArgs &args, hipStream_t stream) {
     if (threads > 1024) threads = 1024;
     const int p = (d4 + threads - 1) / threads;
     if (p <= 1)
-      hipLaunchKernelGGL(residual_row_kernel<1>, dim3(1), dim3(threads), 0, stream, a);
+      hipLaunchKernelGGL((residual_row_kernel<1, 4>), dim3(1), dim3(threads), 0, stream, a);
     else if (p <= 2)
-      hipLaunchKernelGGL(residual_row_kernel<2>, dim3(1), dim3(threads), 0, stream, a);
+      hipLaunchKernelGGL((residual_row_kernel<2, 2>), dim3(1), dim3(threads), 0, stream, a);
     else
-      hipLaunchKernelGGL(residual_row_kernel<4>, dim3(1), dim3(threads), 0, stream, a);
+      hipLaunchKernelGGL((residual_row_kernel<4, 1>), dim3(1), dim3(threads), 0, stream, a);
     return hipGetLastError();
   }
-  const bool spread = a.taps > 1 && a.T > kRows;  // rows are read by the workgroup behind them, too
-  if (spread && a.y && a.x_out == a.x) return hipErrorInvalidValue;
-  const dim3 grid((unsigned)((a.T + kRows - 1) / kRows));
+  if (a.conv && !a.factors) return hipErrorInvalidValue;
+  const dim3 rows((unsigned)a.T);
+  const int pieces = vec ? (d4 + 255) / 256 : 99;
+  {
+    if (pieces <= 1)
+      hipLaunchKernelGGL(residual_join_kernel<1>, rows, dim3(256), 0, stream, a);
+    else if (pieces <= 2)
+      hipLaunchKernelGGL(residual_join_kernel<2>, rows, dim3(256), 0, stream, a);
+    else if (pieces <= 4)
+      hipLaunchKernelGGL(residual_join_kernel<4>, rows, dim3(256), 0, stream, a);
+    else if (pieces <= 8)
+      hipLaunchKernelGGL(residual_join_kernel<8>, rows, dim3(256), 0, stream, a);
+    else
+      hipLaunchKernelGGL(residual_join_kernel<0>, rows, dim3(256), 0, stream, a);
+  }
+  if (!a.conv) return hipGetLastError();
+  const float *x = a.y ? a.x_out : a.x;
+  const dim3 grid((unsigned)((a.T + kRows - 1) / kRows), (unsigned)((d4 + 255) / 256));
   if (vec && a.taps == 1)
-    hipLaunchKernelGGL(residual_rows_kernel<1>, grid, dim3(256), 0, stream, a);
+    hipLaunchKernelGGL(residual_conv_kernel<1>, grid, dim3(256), 0, stream, a, x);
   else if (vec && a.taps == 2)
-    hipLaunchKernelGGL(residual_rows_kernel<2>, grid, dim3(256), 0, stream, a);
+    hipLaunchKernelGGL(residual_conv_kernel<2>, grid, dim3(256), 0, stream, a, x);
   else if (vec && a.taps == 3)
-    hipLaunchKernelGGL(residual_rows_kernel<3>, grid, dim3(256), 0, stream, a);
+    hipLaunchKernelGGL(residual_conv_kernel<3>, grid, dim3(256), 0, stream, a, x);
   else if (vec && a.taps == 4)
-    hipLaunchKernelGGL(residual_rows_kernel<4>, grid, dim3(256), 0, stream, a);
+    hipLaunchKernelGGL(residual_conv_kernel<4>, grid, dim3(256), 0, stream, a, x);
   else
-    hipLaunchKernelGGL(residual_any_kernel, grid, dim3(256), (size_t)a.taps * 256 * sizeof(float), stream, a);
+    hipLaunchKernelGGL(residual_conv_any_kernel, dim3((unsigned)a.T, (unsigned)((a.d + 255) / 256)), dim3(256), 0, stream, a, x);
   return hipGetLastError();
 }
 

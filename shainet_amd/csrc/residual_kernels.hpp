@@ -3,7 +3,8 @@
 //   x' = x + y / rms(y) * post           the sublayer's result y joins the residual
 //   h  = x' / rms(x') * pre              what the next sublayer reads, before
 //   h' = h + conv(h)                     and after a causal convolution over time on each channel
-// One launch does all of it; every part but the first two inputs can be left out.
+// A single row is one launch.  More rows are two: the first joins y and takes the norms' factors, the second
+// walks the rows of a column for the convolution.  Every part but x can be left out.
 #pragma once
 #include <hip/hip_runtime.h>
 
@@ -22,6 +23,7 @@ struct ResidualArgs {
   const float *hist_in;  // [taps - 1, d] the h of the rows before row 0, oldest first; null: zeros
   float *hist_out;       // [taps - 1, d] the same for the next call, not hist_in; null: not kept
   float *h;              // [T, d]
+  float *factors;        // [T] scratch, with pre and conv
   int T, d;
   float eps;
 };
