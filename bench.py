@@ -519,9 +519,9 @@ def model_rates(np, m, vocab, steps, warmup, prefill, decode):
 # feed-forward, HGRN2, attention and attention over the layer before's keys with experts), vocab, HGRN2 (heads, dim, vdim),
 # attention (q heads, kv heads, dim, vdim, bias_max, table rows), experts (ff, experts, identity, top, groups, keep, shared ff)
 ZABUTAR_SIZES = [
-    ("w1024", 1024, 4096, 8, 32000, (8, 128, 128), (16, 8, 64, 64, 240, 32), (512, 24, 8, 6, 4, 3, 1024), (16, 8, 64)),
-    ("w2048", 2048, 8192, 8, 32000, (16, 128, 128), (32, 8, 64, 64, 240, 32), (768, 24, 8, 8, 4, 3, 2048), (32, 8, 64)),
-    ("w4096", 4096, 8192, 4, 32000, (32, 128, 128), (32, 8, 128, 128, 240, 32), (1024, 12, 4, 4, 4, 3, 4096), (32, 8, 128)),
+    ("w1024", 1024, 4096, 8, 32000, (8, 128, 128), (16, 8, 64, 64, 700, 32), (512, 24, 8, 6, 4, 3, 1024), (16, 8, 64)),
+    ("w2048", 2048, 8192, 8, 32000, (16, 128, 128), (32, 8, 64, 64, 700, 32), (768, 24, 8, 8, 4, 3, 2048), (32, 8, 64)),
+    ("w4096", 4096, 8192, 4, 32000, (32, 128, 128), (32, 8, 128, 128, 700, 32), (1024, 12, 4, 4, 4, 3, 4096), (32, 8, 128)),
 ]
 
 

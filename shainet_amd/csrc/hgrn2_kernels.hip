@@ -21,11 +21,20 @@ constexpr int kMaxLds = 160 * 1024;
 constexpr int kChunksAtOnce = 64;
 
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+// e^-|z|: the part of |z| log2(e) that its rounding leaves out comes back to first order
+__device__ __forceinline__ float exp_neg_abs(float z) {
+  const float y = -fabsf(z), hi = y * 1.44269504f, lo = fmaf(y, 1.44269504f, -hi) + y * 1.925963e-8f;
+  const float e = fast_exp2(hi);
+  return fmaf(e, lo * 0.693147181f, e);
+}
 // (the hardware's reciprocal is good to the last bit or so; the argument is at least 1)
-__device__ __forceinline__ float silu1(float z) { return z * __builtin_amdgcn_rcpf(1.f + expf(-z)); }
+__device__ __forceinline__ float silu1(float z) {
+  const float e = exp_neg_abs(z), r = __builtin_amdgcn_rcpf(1.f + e);
+  return z * (z >= 0.f ? r : e * r);
+}
 // f and 1 - f, each to full precision
 __device__ __forceinline__ void gate(float z, float l, float &f, float &k) {
-  const float e = expf(-fabsf(z)), r = __builtin_amdgcn_rcpf(1.f + e), lo = e * r;  // sigmoid(|z|) and sigmoid(-|z|)
+  const float e = exp_neg_abs(z), r = __builtin_amdgcn_rcpf(1.f + e), lo = e * r;  // sigmoid(|z|) and sigmoid(-|z|)
   f = l + (1.f - l) * (z >= 0.f ? r : lo);
   k = (1.f - l) * (z >= 0.f ? lo : r);
 }
@@ -135,21 +144,40 @@ __device__ __forceinline__ void walk_gates(const Hgrn2Args &a, int i, int first,
 
 // What chunk c leaves of the state and adds to it: decay[c][h][d] = prod f, add[c][h] = sum over its rows s of
 // (prod over later rows of f) (1 - f_s) v_s^T.  blockIdx.x: head fastest.  The decayed (1 - f) go through LDS as
-// the MFMAs' A operand; a wavefront takes DG tiles of 32 channels against one tile of 32 value columns.
+// the MFMAs' A operand; each of eight wavefronts takes DG tiles of 32 channels against one tile of 32 value columns.
 template <int C, int DG>
-__global__ __launch_bounds__(256) void hgrn2_chunk_kernel(const Hgrn2Args a, int chunk0, float *__restrict__ add,
-                                                          float *__restrict__ decay) {
+__global__ __launch_bounds__(512, 4) void hgrn2_chunk_kernel(const Hgrn2Args a, int chunk0, float *__restrict__ add,
+                                                             float *__restrict__ decay) {
   constexpr int NS = C / kSub;
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int dim = a.dim, vdim = a.vdim, d32 = (dim + 31) / 32 * 32;
   float *kd = smem, *tot = kd + C * d32;  // [C][d32], [NS][d32]
   const int h = blockIdx.x % a.H, c = blockIdx.x / a.H, first = (chunk0 + c) * C;
-  for (int it = threadIdx.x; it < NS * d32; it += 256) {
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int n = lane & 31, half = lane >> 5;
+  const int n_vt = (vdim + 31) / 32, n_dt = d32 / 32, n_dg = (n_dt + DG - 1) / DG;
+  // values of a wavefront's item: PB steps of 16 rows are asked for ahead, the first item's together with the gates
+  constexpr int PB = NS < 2 ? 1 : 2;
+  float b[PB][8];
+  auto load_v = [&](int item, int s0) {
+    const float *v = a.raw + 2LL * a.H * dim + (long long)h * vdim + min(item % n_vt * 32 + n, vdim - 1);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) b[s0 / 16 % PB][i] = v[(long long)min(first + s0 + 2 * i + half, a.T - 1) * a.stride];
+  };
+  float x[kSub];
+  auto load_gates = [&](int it) {
+    const int j = it / d32, d = it - j * d32;
+    load_column(a, (long long)a.H * dim + h * dim + min(d, dim - 1), first + j * kSub, x);
+  };
+  if ((int)threadIdx.x < NS * d32) load_gates(threadIdx.x);
+  if (wave < n_vt * n_dg)
+#pragma unroll
+    for (int s0 = 0; s0 < 16 * PB; s0 += 16) load_v(wave, s0);
+  for (int it = threadIdx.x; it < NS * d32; it += 512) {
     const int j = it / d32, d = it - j * d32;
     float k_[kSub], f_[kSub];
+    if (it >= 512) load_gates(it);
     if (d < dim) {
-      float x[kSub];
-      load_column(a, (long long)a.H * dim + h * dim + d, first + j * kSub, x);
       walk_gates(a, h * dim + d, first + j * kSub, x, [&](int r, float f, float k) {
         f_[r] = f;
         k_[r] = k;
@@ -171,7 +199,7 @@ __global__ __launch_bounds__(256) void hgrn2_chunk_kernel(const Hgrn2Args a, int
   }
   __syncthreads();
   const long long at = (long long)c * a.H + h;
-  for (int it = threadIdx.x; it < NS * d32; it += 256) {
+  for (int it = threadIdx.x; it < NS * d32; it += 512) {
     const int j = it / d32, d = it - j * d32;
     float later = 1.f;
     for (int b = NS - 1; b > j; --b) later *= tot[b * d32 + d];
@@ -180,14 +208,10 @@ __global__ __launch_bounds__(256) void hgrn2_chunk_kernel(const Hgrn2Args a, int
     if (j == 0 && d < dim) decay[at * dim + d] = later * tot[d];
   }
   __syncthreads();
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int n = lane & 31, half = lane >> 5;
-  const int n_vt = (vdim + 31) / 32, n_dt = d32 / 32, n_dg = (n_dt + DG - 1) / DG;
   float *dst = add + at * dim * vdim;
-  for (int item = wave; item < n_vt * n_dg; item += 4) {
+  for (int item = wave; item < n_vt * n_dg; item += 8) {
     const int vt = item % n_vt, dt0 = item / n_vt * DG;
     const int col = vt * 32 + n;
-    const float *v = a.raw + 2LL * a.H * dim + (long long)h * vdim + min(col, vdim - 1);
     f32x16 acc[DG];
 #pragma unroll
     for (int u = 0; u < DG; ++u)
@@ -196,20 +220,18 @@ __global__ __launch_bounds__(256) void hgrn2_chunk_kernel(const Hgrn2Args a, int
     const float *kp[DG];
 #pragma unroll
     for (int u = 0; u < DG; ++u) kp[u] = kd + half * d32 + min(dt0 + u, n_dt - 1) * 32 + n;
-    float b[2][8];
-    auto load = [&](float (&x)[8], int s0) {
+    if (item != wave) {
 #pragma unroll
-      for (int i = 0; i < 8; ++i) x[i] = v[(long long)min(first + s0 + 2 * i + half, a.T - 1) * a.stride];
-    };
-    load(b[0], 0);
+      for (int s0 = 0; s0 < 16 * PB; s0 += 16) load_v(item, s0);
+    }
 #pragma unroll
     for (int s0 = 0; s0 < C; s0 += 16) {
-      if (s0 + 16 < C) load(b[(s0 / 16 + 1) & 1], s0 + 16);
 #pragma unroll
       for (int i = 0; i < 8; ++i)
 #pragma unroll
         for (int u = 0; u < DG; ++u)
-          acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(kp[u][(s0 + 2 * i) * d32], b[(s0 / 16) & 1][i], acc[u], 0, 0, 0);
+          acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(kp[u][(s0 + 2 * i) * d32], b[s0 / 16 % PB][i], acc[u], 0, 0, 0);
+      if (s0 + 16 * PB < C) load_v(item, s0 + 16 * PB);
     }
     if (col < vdim) {
 #pragma unroll
@@ -268,6 +290,7 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
   constexpr int PR = C < 32 ? 32 : C;  // rows of P and of q that the 32-row tiles read
   extern __shared__ __attribute__((aligned(16))) float smem[];
   __shared__ float sq_s[8 * NT][32];
+  __shared__ __attribute__((aligned(16))) float inv_s[32 * RT];
   const int dim = a.dim, vdim = a.vdim, d16 = (dim + 15) / 16 * 16, ds = d16 + 4;
   float *qs = smem, *ks = qs + PR * ds, *ls = ks + C * ds, *P = ls + C * ds, *tot = P + PR * PS;  // tot: [NS][d16]
   const int h = blockIdx.x % a.H, c = blockIdx.x / a.H, first = (chunk0 + c) * C;
@@ -302,6 +325,9 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
   // (loads come back in order: what is needed first goes first)
   if ((int)threadIdx.x < NS * d16) load_gates(threadIdx.x);
   if (cg < n_vt) load_tile(cg);
+  float norm[NT];
+#pragma unroll
+  for (int u = 0; u < NT; ++u) norm[u] = a.norm[min((cg + CW * u) * 32 + n, vdim - 1)];
 
   for (int it = threadIdx.x; it < NS * d16; it += 512) {
     const int j = it / d16, d = it - j * d16;
@@ -325,47 +351,92 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
   for (int it = threadIdx.x; it < PR * PS; it += 512) P[it] = 0.f;
   __syncthreads();
 
+  // a wavefront takes eight rows; four lanes, a quarter of the channels each, take two rows against two
   for (int p = threadIdx.x; p < C * 8; p += 512) {
-    const int b = p / 64 * 8, t = b + p / 8 % 8, s = b + p % 8;
-    if (s > t) continue;
-    const f32x4 *qp = (const f32x4 *)(qs + t * ds), *lt = (const f32x4 *)(ls + t * ds), *kp = (const f32x4 *)(ks + s * ds),
-                *lp = (const f32x4 *)(ls + s * ds);
-    f32x4 sum = {0.f, 0.f, 0.f, 0.f};
-    for (int i = 0; i < d16 >> 2; ++i) {
-      const f32x4 e = lt[i] - lp[i];
-      sum += qp[i] * kp[i] * f32x4{fast_exp2(e.x), fast_exp2(e.y), fast_exp2(e.z), fast_exp2(e.w)};
+    const int quarter = p & 3, ti = p >> 4 & 3, si = p >> 2 & 3, b = p / 64 * 8, t = b + 2 * ti, s = b + 2 * si, n4 = d16 >> 4;
+    if (si > ti) continue;
+    const int o = quarter * 4 * n4;
+    const f32x4 *qp[2], *lt[2], *kp[2], *lp[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      qp[u] = (const f32x4 *)(qs + (t + u) * ds + o);
+      lt[u] = (const f32x4 *)(ls + (t + u) * ds + o);
+      kp[u] = (const f32x4 *)(ks + (s + u) * ds + o);
+      lp[u] = (const f32x4 *)(ls + (s + u) * ds + o);
     }
-    P[t * PS + s] = (sum.x + sum.y) + (sum.z + sum.w);
+    f32x4 sum[2][2];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) sum[u >> 1][u & 1] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < n4; ++i) {
+      f32x4 q[2], k[2], x[2], y[2];
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        q[u] = qp[u][i];
+        k[u] = kp[u][i];
+        x[u] = lt[u][i];
+        y[u] = lp[u][i];
+      }
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int v = 0; v < 2; ++v) {
+          const f32x4 e = x[u] - y[v];
+          sum[u][v] += q[u] * k[v] * f32x4{fast_exp2(e.x), fast_exp2(e.y), fast_exp2(e.z), fast_exp2(e.w)};
+        }
+    }
+    float mine = 0.f;  // of the four pairs, the one this lane writes
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const f32x4 x = sum[u >> 1][u & 1];
+      float total = (x.x + x.y) + (x.z + x.w);
+      total += __shfl_xor(total, 1);
+      total += __shfl_xor(total, 2);
+      if (quarter == u) mine = total;
+    }
+    const int row = t + (quarter >> 1), col = s + (quarter & 1);
+    if (col <= row) P[row * PS + col] = mine;
   }
   {
+    // 16 rows against 16: two sub-chunks, or rows 8 .. 15 against the first eight of two sub-chunks at once
+    // (of which the squares across the sub-chunks are not used)
     const int m = lane & 15, j4 = 4 * (lane >> 4);
-    for (int item = wave; item < NS * (NS + 1) / 2; item += 8) {
-      int bi = 0, rest = item;
-      while (rest > bi) rest -= ++bi;
-      const int bj = rest;  // bj <= bi; equal: rows 8 .. 15 of the sub-chunk against its first eight
-      const bool half = bi == bj;
-      const float *qp = qs + (bi * kSub + m) * ds + j4, *lt = ls + (bi * kSub + m) * ds + j4;
-      const float *kp = ks + (bj * kSub + m) * ds + j4, *lp = ls + (bj * kSub + m) * ds + j4;
-      const float *mid = half ? ls + (bj * kSub + 7) * ds + j4 : tot + bj * d16 + j4;  // where both decay to
-      const bool q_in = !half || m >= 8, k_in = !half || m < 8;
+    constexpr int apart = NS * (NS - 1) / 2;
+    for (int item = wave; item < apart + (NS + 1) / 2; item += 8) {
+      int bi = 1, bj = item;
+      const bool within = item >= apart;
+      if (within) {
+        bi = bj = min(2 * (item - apart) + (m >> 3), NS - 1);
+      } else {
+        while (bj >= bi) bj -= bi++;
+      }
+      const int q0 = (bi * kSub + (within ? 8 + (m & 7) : m)) * ds + j4, k0 = (bj * kSub + (within ? m & 7 : m)) * ds + j4;
+      const float *mid = within ? ls + (bj * kSub + 7) * ds + j4 : tot + bj * d16 + j4;  // where both decay to
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
       for (int i = 0; i < d16; i += 16) {
-        f32x4 q = *(const f32x4 *)(qp + i), k = *(const f32x4 *)(kp + i), eq = *(const f32x4 *)(lt + i);
+        f32x4 q = *(const f32x4 *)(qs + q0 + i), k = *(const f32x4 *)(ks + k0 + i), eq = *(const f32x4 *)(ls + q0 + i);
         const f32x4 at = *(const f32x4 *)(mid + i);
-        f32x4 ek = at - *(const f32x4 *)(lp + i);
-        if (half) eq -= at;
-        for (int b = bj + 1; b < bi; ++b) eq += *(const f32x4 *)(tot + b * d16 + j4 + i);
+        const f32x4 ek = at - *(const f32x4 *)(ls + k0 + i);
+        if (within) {
+          eq -= at;
+        } else {
+          for (int b = bj + 1; b < bi; ++b) eq += *(const f32x4 *)(tot + b * d16 + j4 + i);
+        }
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          q[e] = q_in ? q[e] * fast_exp2(eq[e]) : 0.f;
-          k[e] = k_in ? k[e] * fast_exp2(ek[e]) : 0.f;
+          q[e] *= fast_exp2(eq[e]);
+          k[e] *= fast_exp2(ek[e]);
         }
 #pragma unroll
         for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e], k[e], acc, 0, 0, 0);
       }
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (!half || (j4 + r >= 8 && m < 8)) P[(bi * kSub + j4 + r) * PS + bj * kSub + m] = acc[r];
+      for (int r = 0; r < 4; ++r) {
+        const int row = j4 + r;
+        if (!within)
+          P[(bi * kSub + row) * PS + bj * kSub + m] = acc[r];
+        else if (row >> 3 == m >> 3 && 2 * (item - apart) + (m >> 3) < NS)
+          P[(bi * kSub + 8 + (row & 7)) * PS + bi * kSub + (m & 7)] = acc[r];
+      }
     }
   }
   __syncthreads();
@@ -412,29 +483,44 @@ __global__ __launch_bounds__(512) void hgrn2_output_kernel(const Hgrn2Args a, in
         }
       }
     }
-    // squares of this tile, summed over its 32 columns
+    // squares of this tile, summed over its 32 columns: with every exchange a lane keeps half of the rows it has
+    float sq[16];
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      float sq = vt < n_vt && vt * 32 + n < vdim ? acc[u][r] * acc[u][r] : 0.f;
+    for (int r = 0; r < 16; ++r) sq[r] = vt < n_vt && vt * 32 + n < vdim ? acc[u][r] * acc[u][r] : 0.f;
 #pragma unroll
-      for (int x = 16; x > 0; x >>= 1) sq += __shfl_xor(sq, x);
-      if (n == 0) sq_s[wave * NT + u][8 * (r >> 2) + 4 * half + (r & 3)] = sq;
+    for (int x = 16, keep = 8; x > 1; x >>= 1, keep >>= 1) {
+      const bool upper = n & x;
+#pragma unroll
+      for (int r = 0; r < keep; ++r) {
+        const float other = __shfl_xor(upper ? sq[r] : sq[r + keep], x);
+        sq[r] = (upper ? sq[r + keep] : sq[r]) + other;
+      }
     }
+    sq[0] += __shfl_xor(sq[0], 1);
+    if (!(n & 1)) sq_s[wave * NT + u][8 * (n >> 3) + 4 * half + (n >> 1 & 3)] = sq[0];
   }
   __syncthreads();
-#pragma unroll
-  for (int r = 0; r < 16; ++r) {
-    const int lt = 8 * (r >> 2) + 4 * half + (r & 3), t = rt * 32 + lt;
+  if (threadIdx.x < 32 * RT) {
+    const int row_tile = threadIdx.x >> 5;
     float sum = 0.f;
     for (int w = 0; w < CW; ++w)
 #pragma unroll
-      for (int u = 0; u < NT; ++u) sum += sq_s[(w * RT + rt) * NT + u][lt];
-    const float f = 1.f / sqrtf(sum / (float)vdim + a.eps);
-    if (t >= C || first + t >= a.T) continue;
+      for (int u = 0; u < NT; ++u) sum += sq_s[(w * RT + row_tile) * NT + u][n];
+    inv_s[threadIdx.x] = 1.f / sqrtf(sum / (float)vdim + a.eps);
+  }
+  __syncthreads();
 #pragma unroll
-    for (int u = 0; u < NT; ++u) {
-      const int col = (cg + CW * u) * 32 + n;
-      if (col < vdim) a.out[((long long)(first + t) * a.H + h) * vdim + col] = acc[u][r] * f * a.norm[col];
+  for (int r4 = 0; r4 < 4; ++r4) {
+    const int t0 = rt * 32 + 8 * r4 + 4 * half;
+    const f32x4 inv = *(const f32x4 *)(inv_s + t0);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      if (t0 + r >= C || first + t0 + r >= a.T) continue;
+#pragma unroll
+      for (int u = 0; u < NT; ++u) {
+        const int col = (cg + CW * u) * 32 + n;
+        if (col < vdim) a.out[((long long)(first + t0 + r) * a.H + h) * vdim + col] = acc[u][4 * r4 + r] * inv[r] * norm[u];
+      }
     }
   }
 }
@@ -463,11 +549,9 @@ hipError_t launch_chunks(const Hgrn2Args &a, const Hgrn2Plan &p, float *scratch,
   do {                                                                                                           \
     static const hipError_t e_ = allow_lds(hgrn2_chunk_kernel<C, DG_>);                                          \
     if (e_ != hipSuccess) return e_;                                                                             \
-    hipLaunchKernelGGL((hgrn2_chunk_kernel<C, DG_>), grid, dim3(256), lds_a, stream, a, c0, add, decay);         \
+    hipLaunchKernelGGL((hgrn2_chunk_kernel<C, DG_>), grid, dim3(512), lds_a, stream, a, c0, add, decay);         \
   } while (0)
-    if (n_vt >= 4)
-      SHAINET_LAUNCH_CHUNK(4);
-    else if (n_vt >= 2)
+    if ((long long)n_vt * ((d32 / 32 + 1) / 2) >= 8)  // (an item for every wavefront)
       SHAINET_LAUNCH_CHUNK(2);
     else
       SHAINET_LAUNCH_CHUNK(1);
